@@ -42,8 +42,10 @@ class RemoteGenerationMixin:
                 T + pre + max_new_tokens + 1)
         out_tokens = [input_ids]
         try:
-            hidden = self.embed(input_ids)
-            if pe is not None and session.position == 0:
+            fresh = session.position == 0
+            hidden = self.embed(input_ids,
+                                session.position + (pre if fresh else 0))
+            if pe is not None and fresh:
                 p = pe.detach().to(hidden.dtype).unsqueeze(0).expand(B, -1, -1)
                 hidden = torch.cat([p, hidden], dim=1)
             hidden = session.step(
@@ -53,7 +55,7 @@ class RemoteGenerationMixin:
                                   top_p, generator)
             out_tokens.append(next_tok.view(B, 1))
             for _ in range(max_new_tokens - 1):
-                hidden = self.embed(next_tok.view(B, 1))
+                hidden = self.embed(next_tok.view(B, 1), session.position)
                 hidden = session.step(hidden)
                 logits = self.lm_head(self.final_norm(hidden[:, -1:]))[:, -1]
                 next_tok = self._pick(logits, do_sample, temperature, top_k,

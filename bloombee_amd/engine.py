@@ -13,17 +13,22 @@ the same Blocks object serves both local and distributed paths.
 """
 from __future__ import annotations
 
-from typing import List, Optional, Sequence
+from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
 import torch.nn.functional as F
 
-from bloombee_amd.kv.paged import PagedKVCache, SessionHandle
+from bloombee_amd.kv.batch import (DecodeSlots, TokenBatch, lockstep_batch,
+                                   session_batch)
+from bloombee_amd.kv.paged import (AllocationFailed, PagedKVCache,
+                                   SessionHandle)
 from bloombee_amd.models.auto import get_block_class
-from bloombee_amd.models.base import ModelConfig, resolve_config
+from bloombee_amd.models.base import (ModelConfig, get_family,
+                                      resolve_config)
 from bloombee_amd.models.llama.block import RopeTables
 from bloombee_amd.utils.logging import get_logger
 from bloombee_amd import ops
+from bloombee_amd.ops import ragged
 
 logger = get_logger(__name__)
 
@@ -37,7 +42,10 @@ class BlockStack(torch.nn.Module):
         self.config = config
         self.start, self.end = start, end
         block_cls = get_block_class(config.model_type)
-        self.rope = RopeTables(config)
+        self.rope = (None if getattr(block_cls, "token_batched", False)
+                     else RopeTables(config))
+        # blocks that run whole ragged steps (kv/batch.py)
+        self.token_batched = self.rope is None
         self.blocks = torch.nn.ModuleList()
         for i in range(start, end):
             blk = block_cls(config, layer_index=i, rope=self.rope).to(device)
@@ -52,15 +60,24 @@ class BlockStack(torch.nn.Module):
             # bypass Module.__setattr__: a plain reference, not a submodule
             object.__setattr__(self.blocks[j], "prev_block",
                                self.blocks[j - 1])
+        for blk in self.blocks:
+            src = getattr(blk, "kv_source", None)
+            if src is not None and src >= start:
+                object.__setattr__(blk, "train_source",
+                                   self.blocks[src - start])
         self.device = torch.device(device)
 
     def make_kv(self, max_tokens: int) -> PagedKVCache:
-        # per-layer KV geometry hook (gemma-4 heterogeneous head_dim/kv heads)
-        if hasattr(self.config, "kv_geometry"):
+        # per-layer KV geometry hooks (gemma-4 heterogeneous head_dim/kv heads;
+        # kv_layout also names value sizes and shared layers)
+        if hasattr(self.config, "kv_layout"):
+            geometry = self.config.kv_layout(self.start, self.end)
+        elif hasattr(self.config, "kv_geometry"):
             hkv, dims = self.config.kv_geometry(self.start, self.end)
+            geometry = dict(num_kv_heads=hkv, head_dim=dims)
         else:
-            hkv = self.config.num_key_value_heads
-            dims = self.config.head_dim
+            geometry = dict(num_kv_heads=self.config.num_key_value_heads,
+                            head_dim=self.config.head_dim)
         from bloombee_amd.config import get_config
         P = get_config().kv.page_size
         # the decode kernels walk KV in 32-position tiles and require page
@@ -69,8 +86,7 @@ class BlockStack(torch.nn.Module):
             raise ValueError(f"BBAMD_KV_PAGE_SIZE must divide 32, got {P}")
         return PagedKVCache(
             num_layers=len(self.blocks),
-            num_kv_heads=hkv,
-            head_dim=dims,
+            **geometry,
             max_tokens=max_tokens,
             page_size=P,
             device=self.device,
@@ -91,6 +107,19 @@ class BlockStack(torch.nn.Module):
         sp0 = int(start_pos[0]) if deep_prompts is not None else 0
         pre = deep_prompts.shape[1] if deep_prompts is not None else 0
         n_over = min(pre - sp0, hidden.shape[1]) if sp0 < pre else 0
+        if self.token_batched:
+            if tree_mask is not None or position_ids is not None:
+                raise NotImplementedError(
+                    f"{self.config.model_type}: no tree-structured steps")
+            B, T, W = hidden.shape
+            x = hidden.reshape(B * T, W).to(torch.float32, copy=True)
+            hook = None
+            if n_over > 0:
+                def hook(i):
+                    x.view(B, T, W)[:, :n_over] += \
+                        deep_prompts[i, sp0:sp0 + n_over].to(x.dtype)
+            self.forward_batch(x, lockstep_batch(kv, start_pos, B, T), hook)
+            return x.view(B, T, W)
         for i, blk in enumerate(self.blocks):
             if n_over > 0:
                 dp = deep_prompts[i, sp0:sp0 + n_over].to(hidden.dtype)
@@ -101,6 +130,22 @@ class BlockStack(torch.nn.Module):
             else:
                 hidden = blk.forward_inference(hidden, kv, start_pos, position_ids)
         return hidden
+
+    @torch.no_grad()
+    def forward_batch(self, x: torch.Tensor, batch: TokenBatch,
+                      before_block=None) -> torch.Tensor:
+        """One ragged step: x (N, W) f32 through all blocks, in place. A block
+        leaves its sum Pending and the next one's norm folds it in;
+        before_block(i) needs the sum, so it forces the fold."""
+        pending = None
+        for i, blk in enumerate(self.blocks):
+            if before_block is not None:
+                ragged.residual_norm(x, pending)
+                pending = None
+                before_block(i)
+            pending = blk.forward_tokens(x, pending, batch)
+        ragged.residual_norm(x, pending)
+        return x
 
     def forward_train(self, hidden: torch.Tensor, start_pos: int = 0,
                       deep_prompts: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -122,11 +167,40 @@ class LocalEngine:
     """
 
     def __init__(self, config_or_name, device="cpu", seed: int = 0,
-                 kv_max_tokens: int = 1 << 16, quantize_q4: bool = False):
+                 kv_max_tokens: int = 1 << 16, quantize_q4: bool = False,
+                 checkpoint_dir: Optional[str] = None):
         cfg = (config_or_name if isinstance(config_or_name, ModelConfig)
                else resolve_config(config_or_name))
+        # a servable weight folder loads its weights, a preset draws them
+        if checkpoint_dir is None and isinstance(config_or_name, str):
+            from bloombee_amd.server.from_pretrained import is_servable
+            if is_servable(config_or_name):
+                checkpoint_dir = config_or_name
         self.config = cfg
         self.device = torch.device(device)
+        head_cls = get_family(cfg.model_type).head_cls
+        self.head = None
+        if head_cls is not None:
+            self.head = head_cls(cfg, device=device, seed=seed,
+                                 checkpoint_dir=checkpoint_dir)
+        else:
+            self._init_plain_head(cfg, device, seed, checkpoint_dir)
+        self.stack = BlockStack(cfg, 0, cfg.num_hidden_layers, device=device, seed=seed)
+        if checkpoint_dir is not None:
+            from bloombee_amd.server.from_pretrained import load_block_weights
+            for i, blk in enumerate(self.stack.blocks):
+                load_block_weights(blk, checkpoint_dir, i)
+        if quantize_q4:
+            # 4-bit weight-compressed decode (w4_gemm.hip): ~4x less weight
+            # memory + HBM traffic. Used for cheap same-weights draft models
+            # (speculative decoding) and compressed serving.
+            for blk in self.stack.blocks:
+                if hasattr(blk, "quantize_weights_q4"):
+                    blk.quantize_weights_q4()
+        self.kv_pool = self.stack.make_kv(kv_max_tokens)
+        self._decode_graphs: Dict[tuple, "_DecodeGraph"] = {}
+
+    def _init_plain_head(self, cfg, device, seed, checkpoint_dir) -> None:
         gen = torch.Generator().manual_seed(seed)
         dt = cfg.dtype
         # family head shape: bloom/falcon use LayerNorm heads; bloom also
@@ -147,19 +221,23 @@ class LocalEngine:
         else:
             self.lm_head_w = (torch.randn(cfg.vocab_size, cfg.hidden_size, generator=gen)
                               .mul_(0.02).to(dt).to(device))
-        self.stack = BlockStack(cfg, 0, cfg.num_hidden_layers, device=device, seed=seed)
-        if quantize_q4:
-            # 4-bit weight-compressed decode (w4_gemm.hip): ~4x less weight
-            # memory + HBM traffic. Used for cheap same-weights draft models
-            # (speculative decoding) and compressed serving.
-            for blk in self.stack.blocks:
-                if hasattr(blk, "quantize_weights_q4"):
-                    blk.quantize_weights_q4()
-        self.kv_pool = self.stack.make_kv(kv_max_tokens)
+        if checkpoint_dir is not None:
+            from bloombee_amd.server.from_pretrained import load_client_weights
+            cw = load_client_weights(checkpoint_dir)
+            if cw["embed"] is None or cw["final_norm"] is None:
+                raise FileNotFoundError(f"no client weights under {checkpoint_dir}")
+            self.embed.copy_(cw["embed"])
+            self.final_norm_w.copy_(cw["final_norm"])
+            if not cfg.tie_word_embeddings:
+                if cw["lm_head"] is None:
+                    raise FileNotFoundError(f"no lm_head under {checkpoint_dir}")
+                self.lm_head_w.copy_(cw["lm_head"])
 
     @torch.no_grad()
     def logits_for(self, hidden_last: torch.Tensor) -> torch.Tensor:
         """hidden_last: (B, H) -> (B, V)"""
+        if self.head is not None:
+            return self.head.logits(self.head.final_norm(hidden_last))
         if self.ln_final:
             y = ops.layer_norm(hidden_last, self.final_norm_w, self.final_norm_b,
                                self.config.layer_norm_epsilon)
@@ -167,7 +245,16 @@ class LocalEngine:
             y = ops.rms_norm(hidden_last, self.final_norm_w, self.config.rms_norm_eps)
         return F.linear(y, self.lm_head_w)
 
-    def _embed(self, input_ids: torch.Tensor) -> torch.Tensor:
+    def _embed(self, input_ids: torch.Tensor,
+               start: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """(B, T) ids; start (B,): position of each row's first token (learned
+        positions only, default 0)."""
+        if self.head is not None:
+            B, T = input_ids.shape
+            pos = torch.arange(T, dtype=torch.int32, device=self.device)
+            pos = (pos.expand(B, T) if start is None
+                   else start.view(B, 1).int() + pos)
+            return self.head.embed(input_ids.to(self.device), pos)
         h = F.embedding(input_ids.to(self.device), self.embed)
         if self.embed_scale != 1.0:
             h = h * self.embed_scale
@@ -176,6 +263,87 @@ class LocalEngine:
                                self.config.layer_norm_epsilon)
         return h
 
+    # -- ragged steps ------------------------------------------------------
+    @torch.no_grad()
+    def step(self, entries: Sequence[Tuple[SessionHandle, Sequence[int],
+                                           Sequence[int]]],
+             ) -> torch.Tensor:
+        """One step over a mixed batch: entries are (one-sequence session, its
+        next tokens, the places among them whose logits are wanted). Returns
+        (wanted, V) f32 in the order of the entries. Only the new tokens run;
+        each session's cache carries what came before.
+
+        Families without ragged blocks run the entries one after the other."""
+        V, limit = self.config.vocab_size, self.config.max_position_embeddings
+        need = 0
+        P = self.kv_pool.page_size
+        for h, toks, want in entries:
+            n = len(toks)
+            if h.batch_size != 1 or n < 1:
+                raise ValueError("an entry is one sequence with new tokens")
+            if not all(0 <= t < V for t in toks):
+                raise ValueError(f"token id outside [0, {V})")
+            if not all(0 <= w < n for w in want):
+                raise ValueError("wanted place outside the entry's tokens")
+            if h.seqs[0].l_spec + n > min(limit, h.max_length):
+                raise ValueError(f"sequence would exceed "
+                                 f"{min(limit, h.max_length)} positions")
+            need += (h.seqs[0].l_spec + n + P - 1) // P - len(h.seqs[0].pages)
+        if len({id(h) for h, _, _ in entries}) != len(entries):
+            raise ValueError("a sequence can enter a step once")
+        if need > self.kv_pool.free_page_count():
+            raise AllocationFailed(
+                f"step needs {need} pages, "
+                f"{self.kv_pool.free_page_count()} are free")
+        for h, toks, _ in entries:
+            h.extend(len(toks))
+        if self.stack.token_batched:
+            batch = session_batch([(h, len(t)) for h, t, _ in entries])
+            ids = torch.tensor([t for _, toks, _ in entries for t in toks],
+                               dtype=torch.int32).to(self.device)
+            hidden = self.stack.forward_batch(
+                self.head.embed(ids, batch.tok_pos), batch)
+        else:
+            outs = []
+            for h, toks, _ in entries:
+                start = torch.tensor([h.seqs[0].l_spec - len(toks)],
+                                     dtype=torch.int32, device=self.device)
+                ids = torch.tensor([list(toks)])
+                outs.append(self.stack.forward_inference(
+                    self._embed(ids, start), h, start)[0])
+            hidden = torch.cat(outs)
+        rows, at = [], 0
+        for _, toks, want in entries:
+            rows += [at + w for w in want]
+            at += len(toks)
+        if not rows:
+            return torch.empty(0, V, device=self.device)
+        idx = torch.tensor(rows, dtype=torch.long).to(self.device)
+        return self.logits_for(hidden[idx]).float()
+
+    @torch.no_grad()
+    def decode(self, entries: Sequence[Tuple[SessionHandle, int]],
+               ) -> torch.Tensor:
+        """step() for a batch that brings one token per sequence and wants
+        every logit; replays a captured graph where the device allows."""
+        from bloombee_amd.config import get_config
+        n = len(entries)
+        if not (self.stack.token_batched and self.device.type == "cuda"
+                and get_config().use_hip_graphs):
+            return self.step([(h, [t], [0]) for h, t in entries])
+        slots = 1
+        while slots < n:
+            slots *= 2
+        need = max(h.seqs[0].l_spec + 1 for h, _ in entries)
+        limit = min(self.config.max_position_embeddings,
+                    self.kv_pool.max_tokens)
+        if need > limit:
+            raise ValueError(f"sequence would exceed {limit} positions")
+        g = self._decode_graphs.get(slots)
+        if g is None:
+            g = self._decode_graphs[slots] = _DecodeGraph(self, slots, limit)
+        return g.run(entries)
+
     @torch.no_grad()
     def prefill(self, input_ids: torch.Tensor, kv: SessionHandle) -> torch.Tensor:
         """input_ids: (B, T). Returns greedy next token ids (B,)."""
@@ -183,7 +351,7 @@ class LocalEngine:
         start = torch.tensor([s.l_spec for s in kv.seqs], dtype=torch.int32,
                              device=self.device)
         kv.extend(T)
-        hidden = self._embed(input_ids)
+        hidden = self._embed(input_ids, start)
         hidden = self.stack.forward_inference(hidden, kv, start)
         return self.logits_for(hidden[:, -1]).argmax(-1)
 
@@ -193,13 +361,20 @@ class LocalEngine:
         start = torch.tensor([s.l_spec for s in kv.seqs], dtype=torch.int32,
                              device=self.device)
         kv.extend(1)
-        hidden = self._embed(input_ids.view(-1, 1))
+        hidden = self._embed(input_ids.view(-1, 1), start)
         hidden = self.stack.forward_inference(hidden, kv, start)
         return self.logits_for(hidden[:, -1]).argmax(-1)
 
     @torch.no_grad()
     def generate_greedy(self, input_ids: torch.Tensor, max_new_tokens: int) -> torch.Tensor:
         B, T = input_ids.shape
+        if self.stack.token_batched:
+            from bloombee_amd.scheduler import BatchScheduler
+            sched = BatchScheduler(self)
+            reqs = [sched.submit(row, max_new_tokens)
+                    for row in input_ids.tolist()]
+            sched.run()
+            return torch.tensor([r.output for r in reqs], device=self.device)
         kv = self.kv_pool.allocate(B, T + max_new_tokens + 1)
         try:
             toks = [self.prefill(input_ids, kv)]
@@ -235,7 +410,7 @@ class LocalEngine:
         def _body():
             ids = dev_in[0:1].view(1, 1)
             pos = dev_in[1:2].to(torch.int32)
-            h = self._embed(ids)
+            h = self._embed(ids, pos)
             h = self.stack.forward_inference(h, kv, pos)
             logits = self.logits_for(h[:, -1]).float()
             p = torch.softmax(logits[0], -1)
@@ -303,8 +478,8 @@ class LocalEngine:
             cur = dev_in[0:1]
             pos0 = dev_in[1:2]
             for i in range(depth):
-                h = self._embed(cur.view(1, 1))
                 sp = (pos0 + i).to(torch.int32)
+                h = self._embed(cur.view(1, 1), sp)
                 h = self.stack.forward_inference(h, kv, sp)
                 logits = self.logits_for(h[:, -1]).float()
                 p = torch.softmax(logits[0], -1)
@@ -337,3 +512,43 @@ class LocalEngine:
                     [float(p) for p in out_host[1]])
 
         return chain
+
+
+class _DecodeGraph:
+    """A captured decode step for up to `slots` sequences: embedding, blocks,
+    norm and logits replay against the buffers of one DecodeSlots."""
+
+    WARMUP = 2
+
+    def __init__(self, engine: LocalEngine, slots: int, limit: int):
+        self.engine = engine
+        self.slots = DecodeSlots(engine.kv_pool, slots, limit)
+        self.graph = None
+        self.calls = 0
+        self.logits: Optional[torch.Tensor] = None
+
+    def _body(self) -> torch.Tensor:
+        eng, b = self.engine, self.slots.batch
+        x = eng.stack.forward_batch(eng.head.embed(self.slots.ids, b.tok_pos), b)
+        return eng.logits_for(x)
+
+    def run(self, entries) -> torch.Tensor:
+        """The result is the graph's buffer: used up before the next call."""
+        for h, _ in entries:
+            h.extend(1)
+        seqs = [h.seqs[0] for h, _ in entries]
+        self.slots.fill([t for _, t in entries], [s.l_spec - 1 for s in seqs],
+                        [s.pages for s in seqs])
+        n = len(entries)
+        if self.graph is None and self.calls < self.WARMUP:
+            self.calls += 1
+            return self._body()[:n]
+        if self.graph is None:
+            self.graph = torch.cuda.CUDAGraph()
+            with torch.cuda.graph(self.graph,
+                                  capture_error_mode="thread_local"):
+                self.logits = self._body()
+            logger.info("ragged decode step of %d slots captured as hipGraph",
+                        self.slots.B)
+        self.graph.replay()
+        return self.logits[:n]

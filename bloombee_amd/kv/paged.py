@@ -65,19 +65,28 @@ class PagedKVCache:
         device: torch.device | str = "cpu",
         dtype: torch.dtype = torch.bfloat16,
         layout=None,
+        v_head_dim=None,
+        shares=None,
     ):
         """num_kv_heads / head_dim may be ints (uniform) or per-layer lists —
         gemma-4 style heterogeneous KV geometry (sliding layers D=256, full
         layers D=512; ref server/backend.py:291-306 per-block KV descriptor
         dispatch). `layout[l]` may be "kv" (default) or "k" — k-only layers
         (gemma-4 attention_k_eq_v full-attention layers) allocate no V plane.
+        v_head_dim: value size where it differs from head_dim (int or per-layer
+        list). `shares[l]` = j makes layer l read layer j's planes (cross-layer
+        KV sharing): it owns no storage, and copies skip it.
         """
         self.num_layers = num_layers
         as_list = (lambda v: list(v) if isinstance(v, (list, tuple))
                    else [v] * num_layers)
         self.num_kv_heads_per_layer = as_list(num_kv_heads)
         self.head_dim_per_layer = as_list(head_dim)
+        self.v_head_dim_per_layer = (list(self.head_dim_per_layer)
+                                     if v_head_dim is None
+                                     else as_list(v_head_dim))
         self.layout = as_list(layout if layout is not None else "kv")
+        self.shares = as_list(shares)
         self.num_kv_heads = self.num_kv_heads_per_layer[0]
         self.head_dim = self.head_dim_per_layer[0]
         self.page_size = page_size
@@ -91,10 +100,22 @@ class PagedKVCache:
         self.pools = []
         for l in range(num_layers):
             hkv, d = self.num_kv_heads_per_layer[l], self.head_dim_per_layer[l]
+            if self.shares[l] is not None:
+                j = self.shares[l]
+                if not (0 <= j < l) or self.shares[j] is not None:
+                    raise PagedKVError(
+                        f"layer {l} cannot share the KV of layer {j}")
+                self.pools.append(self.pools[j])
+                continue
             k = torch.zeros(self.n_pages, hkv, page_size, d,
                             device=self.device, dtype=dtype)
-            v = k if self.layout[l] == "k" else torch.zeros_like(k)
+            v = k if self.layout[l] == "k" else torch.zeros(
+                self.n_pages, hkv, page_size, self.v_head_dim_per_layer[l],
+                device=self.device, dtype=dtype)
             self.pools.append((k, v))
+        # layers that own storage: every copy of KV data loops over these
+        self.own_layers = [l for l in range(num_layers)
+                           if self.shares[l] is None]
         self._free_pages: List[int] = list(range(self.n_pages - 1, -1, -1))
         self._reserved_tokens = 0  # admission-control reservation
         self._lock = threading.Condition()
@@ -127,7 +148,8 @@ class PagedKVCache:
         if self.layout[layer] == "k":
             raise PagedKVError(f"layer {layer} is k-only (v aliases k)")
         v = self.pools[layer][1]
-        hkv, d = self.num_kv_heads_per_layer[layer], self.head_dim_per_layer[layer]
+        hkv = self.num_kv_heads_per_layer[layer]
+        d = self.v_head_dim_per_layer[layer]
         return v.view(self.n_pages, hkv, d, self.page_size)
 
     # -- admission --------------------------------------------------------
@@ -170,6 +192,19 @@ class PagedKVCache:
             self._next_handle += 1
             return handle
 
+    def open_elastic(self, max_length: int) -> "SessionHandle":
+        """A one-sequence session without a reservation: it pays for pages as
+        its tokens arrive and extend() fails at once when the pool is short.
+        For callers that know the live total themselves (the batch scheduler's
+        admission, trace replay) and cannot name a length in advance."""
+        with self._lock:
+            handle = SessionHandle(self, self._next_handle, 1,
+                                   min(max_length, self.max_tokens), 0,
+                                   elastic=True)
+            self._handles[self._next_handle] = handle
+            self._next_handle += 1
+            return handle
+
     def _release(self, handle: "SessionHandle") -> None:
         with self._lock:
             if handle.handle_id not in self._handles:
@@ -205,8 +240,10 @@ class SessionHandle:
     speculative extension, commit/rollback, and a device page table."""
 
     def __init__(self, cache: PagedKVCache, handle_id: int, batch_size: int,
-                 max_length: int, reserved_tokens: int):
+                 max_length: int, reserved_tokens: int,
+                 elastic: bool = False):
         self.cache = cache
+        self.elastic = elastic
         self.handle_id = handle_id
         self.batch_size = batch_size
         self.max_length = max_length
@@ -266,6 +303,8 @@ class SessionHandle:
         if self.is_swapped:
             raise PagedKVError("extend on a swapped-out session; swap_in first")
         P = self.cache.page_size
+        if self.elastic:
+            timeout = 0.0
         deadline = None if timeout is None else time.monotonic() + timeout
         while True:
             with self._meta_lock:
@@ -289,7 +328,7 @@ class SessionHandle:
                              if need_total else [])
                 except AllocationFailed:
                     if (deadline is not None
-                            and time.monotonic() > deadline):
+                            and time.monotonic() >= deadline):
                         raise
                     pages = None
                 if pages is not None:
@@ -357,7 +396,7 @@ class SessionHandle:
                                        "inside the speculative region")
                 pg_s = int(self._page_table_host[b, src // P])
                 pg_d = int(self._page_table_host[b, dst // P])
-                for l in range(self.cache.num_layers):
+                for l in self.cache.own_layers:
                     kp = self.cache.k_pages(l)
                     kp[pg_d, :, dst % P, :] = kp[pg_s, :, src % P, :]
                     if self.cache.layout[l] != "k":
@@ -396,6 +435,9 @@ class SessionHandle:
                                      device=cache.device)
                 per_layer = []
                 for l in range(cache.num_layers):
+                    if cache.shares[l] is not None:
+                        per_layer.append((None, None))
+                        continue
                     k = cache.k_pages(l)[pages]
                     kh = torch.empty_like(k, device="cpu",
                                           pin_memory=on_gpu)
@@ -421,7 +463,8 @@ class SessionHandle:
             for per_layer in snap:
                 cl = []
                 for kh, vh in per_layer:
-                    kq = _ops.quant4_pack(kh.float().reshape(-1, 64)) + (kh.shape, kh.dtype)
+                    kq = (None if kh is None else
+                          _ops.quant4_pack(kh.float().reshape(-1, 64)) + (kh.shape, kh.dtype))
                     vq = (None if vh is None else
                           _ops.quant4_pack(vh.float().reshape(-1, 64)) + (vh.shape, vh.dtype))
                     cl.append((kq, vq))
@@ -467,7 +510,7 @@ class SessionHandle:
                     self._page_table_host[b, j] = pg
                 idx = torch.tensor(new_pages, dtype=torch.long,
                                    device=cache.device)
-                for l in range(cache.num_layers):
+                for l in cache.own_layers:
                     kh, vh = snap[b][l]
                     cache.k_pages(l)[idx] = kh.to(cache.device,
                                                   non_blocking=on_gpu)
@@ -563,8 +606,12 @@ class SessionHandle:
         counts = self._swapped_counts
         host: List[tuple] = []
         for l in range(cache.num_layers):
+            if cache.shares[l] is not None:
+                host.append(host[cache.shares[l]])
+                continue
             hkv = cache.num_kv_heads_per_layer[l]
             d = cache.head_dim_per_layer[l]
+            dv = cache.v_head_dim_per_layer[l]
             P = cache.page_size
             ks, vs = [], []
             for b in range(self.batch_size):
@@ -575,7 +622,7 @@ class SessionHandle:
                 else:
                     # (npages, Hkv, D, P) -> (Hkv, D, npages*P) -> (Hkv, S, D)
                     v_flat = (vh.permute(1, 2, 0, 3)
-                              .reshape(hkv, d, -1)[:, :, :S]
+                              .reshape(hkv, dv, -1)[:, :, :S]
                               .transpose(1, 2).contiguous())
                 ks.append(k_flat)
                 vs.append(v_flat)
@@ -628,6 +675,9 @@ class SessionHandle:
             for b, npages, ids in work:
                 per_layer = []
                 for l in range(cache.num_layers):
+                    if cache.shares[l] is not None:
+                        per_layer.append((None, None))
+                        continue
                     k = cache.k_pages(l)[ids]
                     kh = torch.empty_like(k, device="cpu", pin_memory=on_gpu)
                     kh.copy_(k, non_blocking=on_gpu)
@@ -703,7 +753,7 @@ class SessionHandle:
                 n_copy = min(n_snap, len(pages))
                 idx = torch.tensor(pages[:n_copy], dtype=torch.long,
                                    device=cache.device)
-                for l in range(cache.num_layers):
+                for l in cache.own_layers:
                     kh, vh = per_layer[l]
                     cache.k_pages(l)[idx] = kh[:n_copy].to(
                         cache.device, non_blocking=on_gpu)

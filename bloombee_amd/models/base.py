@@ -55,6 +55,11 @@ class ModelConfig:
         return getattr(torch, os.environ.get("BBAMD_TORCH_DTYPE",
                                              self.torch_dtype))
 
+    @property
+    def hidden_dtype(self) -> torch.dtype:
+        """Type of the hidden states between blocks and on the wire."""
+        return self.dtype
+
     @classmethod
     def from_dict(cls, d: dict) -> "ModelConfig":
         d = dict(d)
@@ -93,6 +98,10 @@ class FamilyEntry:
     causal_lm_cls: Optional[type] = None   # client DistributedModelForCausalLM
     speculative_cls: Optional[type] = None # client ForSpeculativeGeneration
     seq_cls_cls: Optional[type] = None     # client ForSequenceClassification
+    # embeddings + final norm + vocabulary projection as one module, for
+    # families whose client side differs from the plain one
+    head_cls: Optional[type] = None
+    architecture: Optional[str] = None     # config.json "architecture" key
     presets: Dict[str, dict] = field(default_factory=dict)
 
 
@@ -114,6 +123,16 @@ def get_family(model_type: str) -> FamilyEntry:
     return _FAMILIES[model_type]
 
 
+def model_type_of(d: dict) -> str:
+    """Family of a config.json: its model_type, else its architecture name."""
+    if "model_type" not in d and "architecture" in d:
+        for name, entry in _FAMILIES.items():
+            if entry.architecture == d["architecture"]:
+                return name
+        raise KeyError(f"unknown architecture {d['architecture']!r}")
+    return d.get("model_type", "llama")
+
+
 def resolve_config(name_or_path: str) -> ModelConfig:
     """Resolve a model name or local path to a ModelConfig.
 
@@ -125,7 +144,7 @@ def resolve_config(name_or_path: str) -> ModelConfig:
     if os.path.isfile(cfg_path):
         with open(cfg_path) as f:
             d = json.load(f)
-        family = get_family(d.get("model_type", "llama"))
+        family = get_family(model_type_of(d))
         return family.config_cls.from_dict(d)
     key = name_or_path.lower()
     if key in _PRESETS:

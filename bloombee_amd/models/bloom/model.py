@@ -24,7 +24,7 @@ class DistributedBloomModel(DistributedLlamaModel):
         self.norm_b = torch.nn.Parameter(
             torch.zeros(cfg.hidden_size, dtype=dt, device=dev), requires_grad=False)
 
-    def embed(self, input_ids: torch.Tensor) -> torch.Tensor:
+    def embed(self, input_ids: torch.Tensor, start_pos: int = 0) -> torch.Tensor:
         h = F.embedding(input_ids.to(self.device_), self.embed_tokens)
         return ops.layer_norm(h, self.embed_ln_w, self.embed_ln_b,
                               self.config.layer_norm_epsilon)

@@ -13,7 +13,7 @@ from bloombee_amd.models.llama.model import (DistributedLlamaForCausalLM,
 
 
 class DistributedGemma4Model(DistributedLlamaModel):
-    def embed(self, input_ids: torch.Tensor) -> torch.Tensor:
+    def embed(self, input_ids: torch.Tensor, start_pos: int = 0) -> torch.Tensor:
         h = F.embedding(input_ids.to(self.device_), self.embed_tokens)
         return h * math.sqrt(self.config.hidden_size)
 

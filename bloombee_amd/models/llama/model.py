@@ -77,7 +77,8 @@ class DistributedLlamaModel(torch.nn.Module):
         else:
             self.deep_prompts = None
 
-    def embed(self, input_ids: torch.Tensor) -> torch.Tensor:
+    def embed(self, input_ids: torch.Tensor, start_pos: int = 0) -> torch.Tensor:
+        """start_pos: position of the first token (learned positions only)."""
         h = F.embedding(input_ids.to(self.device_), self.embed_tokens)
         return h
 
@@ -97,7 +98,7 @@ class DistributedLlamaModel(torch.nn.Module):
 
     def forward(self, input_ids: torch.Tensor) -> torch.Tensor:
         """Training-path full forward (no KV): returns final hidden states."""
-        h = self.embed(input_ids)
+        h = self.embed(input_ids, self.pre_seq_len)
         if self.prompt_embeds is not None:
             B = h.shape[0]
             p = self.prompt_embeds.to(h.dtype).unsqueeze(0).expand(B, -1, -1)
@@ -158,8 +159,8 @@ class DistributedLlamaForCausalLM(RemoteGenerationMixin, torch.nn.Module):
     def remote(self) -> RemoteSequential:
         return self.transformer.remote
 
-    def embed(self, input_ids):
-        return self.transformer.embed(input_ids)
+    def embed(self, input_ids, start_pos: int = 0):
+        return self.transformer.embed(input_ids, start_pos)
 
     def final_norm(self, hidden):
         return self.transformer.final_norm(hidden)
@@ -182,8 +183,8 @@ class DistributedLlamaForCausalLM(RemoteGenerationMixin, torch.nn.Module):
         # a converted checkpoint directory serves real client weights
         # (ref client/from_pretrained.py: the client loads only its share)
         if "checkpoint_dir" not in kw:
-            from bloombee_amd.server.from_pretrained import is_converted
-            if is_converted(name_or_path):
+            from bloombee_amd.server.from_pretrained import is_servable
+            if is_servable(name_or_path):
                 kw["checkpoint_dir"] = name_or_path
         return cls(cfg, ccfg, model_name=name_or_path, seed=seed,
                    device=device, **kw)

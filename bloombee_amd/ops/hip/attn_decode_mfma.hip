@@ -31,8 +31,6 @@
 
 static constexpr int DKVBLK = 32;  // positions per KV tile
 
-typedef __attribute__((ext_vector_type(4))) short short4v;  // 4 x bf16 = 8 B
-
 // Reduce across the four 16-lane subgroups: lanes {l, l+16, l+32, l+48}.
 DEVINL float quad16_reduce_max(float x) {
   x = fmaxf(x, __shfl_xor(x, 16));

@@ -79,7 +79,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_kernel(
   }
 
   // C layout: row = t*16 + hi*4 + reg, col = n0 + li.
-  if (ksplit == 1) {
+  if (Cpart == nullptr) {
 #pragma unroll
     for (int t = 0; t < MT; ++t)
 #pragma unroll
@@ -319,7 +319,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
 
   if (norm_mode == 2) reduce_invr();
 
-  if (ksplit == 1) {
+  if (Cpart == nullptr) {
     if (ssout == nullptr) {
 #pragma unroll
       for (int t = 0; t < MT; ++t)

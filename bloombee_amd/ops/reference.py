@@ -430,3 +430,97 @@ def moe_gemm_grouped(A: torch.Tensor, W: torch.Tensor, off: torch.Tensor,
             y = y * scale[slots].float().unsqueeze(1)
         C[slots] = y.to(A.dtype)
     return C
+
+
+# ---------------------------------------------------------------------------
+# Ragged batches (ops/ragged.py): the CPU forms of its kernels
+# ---------------------------------------------------------------------------
+
+def grouped_rms_norm(x: torch.Tensor, weight: torch.Tensor, groups: int,
+                     eps: float) -> torch.Tensor:
+    """RMS norm of `groups` equal consecutive parts of the last dim, each by
+    its own mean square; fp32 in and out."""
+    xf = x.float()
+    g = xf.reshape(*xf.shape[:-1], groups, -1)
+    g = g * torch.rsqrt(g.pow(2).mean(-1, keepdim=True) + eps)
+    return g.reshape(xf.shape) * weight.float()
+
+
+def distance_slopes(n_heads: int) -> torch.Tensor:
+    """Per-head linear distance penalties 2^(-8 (h+1) / n_heads). Equal to
+    alibi_slopes where n_heads is a power of two, and only there."""
+    h = torch.arange(1, n_heads + 1, dtype=torch.float64)
+    return torch.pow(2.0, -8.0 * h / n_heads).float()
+
+
+def xielu(z: torch.Tensor, pos: float, neg: float) -> torch.Tensor:
+    """pos z^2 + z/2 above zero, neg (e^z - 1 - z) + z/2 below; pos and neg
+    are the positive curvatures (softplus already applied)."""
+    below = neg * (torch.expm1(z.clamp(max=0.0)) - z)
+    return torch.where(z > 0, pos * z * z, below) + 0.5 * z
+
+
+def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
+               top: int, scale: float):
+    """Softmax scores; the choice adds `correction`, the weights do not and
+    are not renormalized. Outputs from `experts` on are identity experts.
+    Returns ids (N, top) int32 with -1 for identity choices, weights (N, top)
+    and the identity experts' summed weight (N,)."""
+    s = torch.softmax(logits.float(), dim=-1)
+    # stable sort: the lowest index wins a tie
+    ids = torch.sort(s + correction.float(), dim=-1, descending=True,
+                     stable=True).indices[:, :top]
+    w = torch.gather(s, 1, ids) * scale
+    ident = ids >= experts
+    idw = (w * ident).sum(-1)
+    return torch.where(ident, -1, ids).int(), w, idw
+
+
+def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
+                window: int = 0, slopes=None, gate=None) -> torch.Tensor:
+    """Paged attention of a ragged batch: q (N, H, >= dim) -> (N, H * vdim).
+    Row n sees positions j of its own sequence with 0 <= pos - j (< window);
+    score = q.k * scale - slope_h * (pos - j); out *= sigmoid(gate)."""
+    N, H = q.shape[0], q.shape[1]
+    G = k_pages.shape[1]
+    out = torch.zeros(N, H, vdim, dtype=torch.float32, device=q.device)
+    for s in range(batch.page_table.shape[0]):
+        rows = ((batch.tok_seq == s) & (batch.tok_pos >= 0)).nonzero()[:, 0]
+        if rows.numel() == 0:
+            continue
+        pos = batch.tok_pos[rows].long()
+        ctx = int(pos.max()) + 1
+        k, v = kv_gather(k_pages, v_pages, batch.page_table, ctx, s)
+        k = k[..., :dim].float().repeat_interleave(H // G, dim=0)
+        v = v[..., :vdim].float().repeat_interleave(H // G, dim=0)
+        sc = torch.matmul(q[rows, :, :dim].float().transpose(0, 1),
+                          k.transpose(1, 2)) * scale          # (H, R, ctx)
+        dist = pos.view(-1, 1) - torch.arange(ctx, device=q.device).view(1, -1)
+        if slopes is not None:
+            sc = sc - slopes.view(-1, 1, 1) * dist.float()
+        seen = dist >= 0
+        if window > 0:
+            seen &= dist < window
+        p = torch.softmax(sc.masked_fill(~seen, float("-inf")), dim=-1)
+        out[rows] = torch.matmul(p, v).transpose(0, 1)
+    out = out.reshape(N, H * vdim)
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())
+    return out.to(q.dtype)
+
+
+def moe_experts(h, gate_up, down, ids, wts) -> torch.Tensor:
+    """y (N, top, W): wts * down(silu(gate h) * up h) of every chosen expert;
+    rows of skipped choices (id < 0) are zero."""
+    N, top = ids.shape
+    y = torch.zeros(N, top, down.shape[1], dtype=torch.float32, device=h.device)
+    for e in range(gate_up.shape[0]):
+        t, k = (ids == e).nonzero(as_tuple=True)
+        if t.numel() == 0:
+            continue
+        x = h[t].float()
+        g = x @ gate_up[e, 0].float().t()
+        u = x @ gate_up[e, 1].float().t()
+        a = (g * torch.sigmoid(g) * u).to(h.dtype).float()
+        y[t, k] = (a @ down[e].float().t()) * wts[t, k, None]
+    return y.to(h.dtype)

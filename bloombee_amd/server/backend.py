@@ -233,8 +233,8 @@ class StackBackend:
                         " disable BBAMD_MIXED_ATTN for this workload")
                 start_pos = start_pos - handle.pos_offset
             h = hidden.to(self.device, non_blocking=True)
-            if h.dtype != self.config.dtype:
-                h = h.to(self.config.dtype)
+            if h.dtype != self.config.hidden_dtype:
+                h = h.to(self.config.hidden_dtype)
             deep = None
             if prompts is not None:
                 p = prompts.to(h.device)
@@ -384,7 +384,7 @@ class StackBackend:
 
         def run():
             from bloombee_amd.utils.peft import using_adapter
-            h = hidden.to(self.device).to(self.config.dtype)
+            h = hidden.to(self.device).to(self.config.hidden_dtype)
             dp = prompts.to(self.device) if prompts is not None else None
             with torch.no_grad(), using_adapter(adapter):
                 return self.stack.forward_train(h, deep_prompts=dp)
@@ -401,7 +401,7 @@ class StackBackend:
 
         def run():
             from bloombee_amd.utils.peft import using_adapter
-            h = hidden_in.to(self.device).to(self.config.dtype)
+            h = hidden_in.to(self.device).to(self.config.hidden_dtype)
             h = h.detach().requires_grad_(True)
             dp = None
             if prompts is not None:

@@ -11,6 +11,7 @@ bf16 has no numpy dtype, so bf16 tensors are stored as uint16 views with a
 """
 from __future__ import annotations
 
+import json
 import os
 from pathlib import Path
 from typing import Dict, Optional
@@ -19,6 +20,43 @@ import numpy as np
 import torch
 
 SENTINEL = ".bloombee_np_converted"
+
+
+class NativeCheckpoint:
+    """A folder whose model.safetensors the family reads under its own tensor
+    names (no conversion step): blocks and heads pull what they need."""
+
+    def __init__(self, path: str):
+        from safetensors import safe_open
+
+        self._file = safe_open(os.path.join(path, "model.safetensors"),
+                               framework="pt", device="cpu")
+
+    def get(self, name: str) -> torch.Tensor:
+        return self._file.get_tensor(name)
+
+    def layer(self, index: int):
+        return lambda name: self._file.get_tensor(f"l{index}.{name}")
+
+
+def is_native(path: str) -> bool:
+    """True for a checkpoint folder of a family with native tensor names."""
+    from bloombee_amd.models.base import get_family, model_type_of
+
+    cfg, st = Path(path) / "config.json", Path(path) / "model.safetensors"
+    if not (cfg.is_file() and st.is_file()):
+        return False
+    with open(cfg) as f:
+        try:
+            family = get_family(model_type_of(json.load(f)))
+        except KeyError:
+            return False
+    return hasattr(family.block_cls, "load_tensors")
+
+
+def is_servable(path: str) -> bool:
+    """True if `path` itself is a weight folder servers and clients load."""
+    return is_converted(path) or is_native(path)
 
 # our flat parameter names -> reference file-name stems (per block)
 _BLOCK_PARAM_MAP = {
@@ -67,6 +105,8 @@ def load_block_weights(block: torch.nn.Module, ckpt_dir: str, index: int) -> int
     """Load one block's tensors from the npy layout; returns #tensors loaded.
     Supports the fused qkv/gate_up layout directly and falls back to
     concatenating the reference's split q/k/v and gate/up files."""
+    if hasattr(block, "load_tensors"):
+        return block.load_tensors(NativeCheckpoint(ckpt_dir).layer(index))
     d = Path(ckpt_dir)
     loaded = 0
     for pname, stem in _BLOCK_PARAM_MAP.items():
@@ -174,6 +214,8 @@ def convert_hf_checkpoint(hf_dir: str, out_dir: Optional[str] = None,
     import json as _json
     import shutil
 
+    if is_native(hf_dir):
+        return str(hf_dir)     # served as it is
     d = Path(hf_dir)
     out = Path(out_dir) if out_dir else Path(str(d).rstrip("/") + "-np")
     if is_converted(str(out)) and not force:

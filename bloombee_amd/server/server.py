@@ -61,8 +61,8 @@ class Server:
                                          else self.config.model_type)
         # serving a converted real checkpoint: the model path IS the weight dir
         if checkpoint_dir is None and isinstance(model, str):
-            from bloombee_amd.server.from_pretrained import is_converted
-            if is_converted(model):
+            from bloombee_amd.server.from_pretrained import is_servable
+            if is_servable(model):
                 checkpoint_dir = model
         self.device = device
         # persistent identity (ref --identity_path): keeps routing history,

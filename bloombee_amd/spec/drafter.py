@@ -99,7 +99,7 @@ class MultiDrafter:
             start = torch.full((1,), self._kv_len, dtype=torch.int32,
                                device=eng.device)
             kv.extend(new.shape[1])
-            hidden = eng.stack.forward_inference(eng._embed(new), kv, start)
+            hidden = eng.stack.forward_inference(eng._embed(new, start), kv, start)
             probs0 = torch.softmax(
                 eng.logits_for(hidden[:, -1]).float()[0], -1)
         self._kv_len = history.numel()
@@ -181,9 +181,9 @@ class MultiDrafter:
                         t, pr, p = gstep(chain_tok, pos)
                         dist = p.clone() if self.collect_dists else None
                     else:
-                        h = eng._embed(torch.tensor([[chain_tok]]))
                         sp = torch.tensor([pos], dtype=torch.int32,
                                           device=eng.device)
+                        h = eng._embed(torch.tensor([[chain_tok]]), sp)
                         h = eng.stack.forward_inference(h, kv, sp)
                         lg = eng.logits_for(h[:, -1]).float()[0]
                         p = torch.softmax(lg, -1)

@@ -1,8 +1,8 @@
 """Build the bloombee_amd gfx950 HIP extension in-tree.
 
 Invokes hipcc directly (native HIP source — no hipify pass, no CUDA
-compatibility layer). The built .so lands at bloombee_amd/ops/_hip_ops.so so
-it travels with the repo snapshot to the GPU box (gpurun ships in-tree .so
+compatibility layer). The built .so files land in bloombee_amd/ops/ so
+they travel with the repo snapshot to the GPU box (gpurun ships in-tree .so
 files; a JIT cache under ~/.cache would not).
 
 Usage:
@@ -16,7 +16,9 @@ from pathlib import Path
 
 ROOT = Path(__file__).resolve().parent
 HIP_DIR = ROOT / "bloombee_amd" / "ops" / "hip"
-OUT_SO = ROOT / "bloombee_amd" / "ops" / "_hip_ops.so"
+OPS_DIR = ROOT / "bloombee_amd" / "ops"
+# module -> source. _hip_ragged holds all that ragged-batch models need.
+MODULES = {"_hip_ops": "ext.hip", "_hip_ragged": "ext_ragged.hip"}
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 
@@ -27,15 +29,21 @@ def torch_paths():
     return tdir / "include", tdir / "lib"
 
 
-def build(verbose: bool = True) -> Path:
+def _compile(module: str, source: str, verbose: bool) -> Path:
+    """One extension module from one source file."""
     tinc, tlib = torch_paths()
     py_inc = sysconfig.get_paths()["include"]
-    src = HIP_DIR / "ext.hip"
-    obj = HIP_DIR / "ext.o"
+    out = OPS_DIR / f"{module}.so"
+    # private names until the finished file is moved into place: a second
+    # process that builds or loads meanwhile never sees a half-written one
+    obj = HIP_DIR / f"{source}.{os.getpid()}.o"
+    part = OPS_DIR / f".{module}.{os.getpid()}.so"
     compile_cmd = [
         "/opt/rocm/bin/hipcc",
         f"--offload-arch={ARCH}",
         "-O3", "-std=c++17", "-fPIC", "-fno-gpu-rdc",
+        # packed FP32 instructions off: some of their forms are unreliable
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
         "-I", str(tinc),
         "-I", str(tinc / "torch" / "csrc" / "api" / "include"),
         "-I", "/opt/rocm/include",
@@ -43,22 +51,35 @@ def build(verbose: bool = True) -> Path:
         "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1", "-DHIPBLAS_V2",
         "-DCUDA_HAS_FP16=1", "-D__HIP_NO_HALF_OPERATORS__=1",
         "-D__HIP_NO_HALF_CONVERSIONS__=1", "-DHIP_ENABLE_WARP_SYNC_BUILTINS=1",
-        "-DTORCH_API_INCLUDE_EXTENSION_H", "-DTORCH_EXTENSION_NAME=_hip_ops",
-        "-c", str(src), "-o", str(obj),
+        "-DTORCH_API_INCLUDE_EXTENSION_H", f"-DTORCH_EXTENSION_NAME={module}",
+        "-c", str(HIP_DIR / source), "-o", str(obj),
     ]
     link_cmd = [
         "g++", "-shared", str(obj),
         "-L", str(tlib), "-L", "/opt/rocm/lib",
         "-lc10", "-ltorch", "-ltorch_cpu", "-ltorch_python",
         "-lamdhip64", "-lc10_hip", "-ltorch_hip", "-lz",
-        "-o", str(OUT_SO),
+        "-o", str(part),
     ]
-    for cmd in (compile_cmd, link_cmd):
-        if verbose:
-            print("+", " ".join(cmd), file=sys.stderr)
-        subprocess.run(cmd, check=True)
-    obj.unlink(missing_ok=True)
-    return OUT_SO
+    try:
+        for cmd in (compile_cmd, link_cmd):
+            if verbose:
+                print("+", " ".join(cmd), file=sys.stderr)
+            subprocess.run(cmd, check=True)
+        os.replace(part, out)
+    finally:
+        obj.unlink(missing_ok=True)
+        part.unlink(missing_ok=True)
+    return out
+
+
+def build(modules=None, verbose: bool = True) -> list:
+    """Compile the named extension modules (default: all), side by side."""
+    from concurrent.futures import ThreadPoolExecutor
+
+    names = list(modules or MODULES)
+    with ThreadPoolExecutor(len(names)) as ex:
+        return list(ex.map(lambda m: _compile(m, MODULES[m], verbose), names))
 
 
 if __name__ == "__main__":
