@@ -194,6 +194,95 @@ def run_swarm(args):
         dist.destroy_process_group()
 
 
+# (model, closest family of equal layer size); both run LAYERS blocks
+LAYER_PAIRS = [("mubasun-8b-4l", "llama-3-8b"),
+               ("mubasun-8x7b-4l", "mixtral-8x7b-4l"),
+               ("mubasun-64e-4l", None)]
+LAYERS = 4
+
+
+def _layer_numbers(model: str, args) -> dict:
+    """Prefill and decode throughput of LAYERS blocks of `model` (random
+    weights, lockstep sessions, decode replayed from a captured graph where the
+    family's step can be captured)."""
+    from bloombee_amd.engine import BlockStack
+    from bloombee_amd.models.base import resolve_config
+
+    cfg = resolve_config(model)
+    dev = args.device or ("cuda:0" if torch.cuda.is_available() else "cpu")
+    on_gpu = dev.startswith("cuda")
+    stack = BlockStack(cfg, 0, LAYERS, device=dev, seed=0)
+    W = cfg.hidden_size
+    gen = torch.Generator().manual_seed(1)
+    sync = torch.cuda.synchronize if on_gpu else (lambda: None)
+    out = {}
+
+    def timed(fn):
+        for _ in range(args.warmup):
+            fn()
+        sync()
+        t0 = time.monotonic()
+        for _ in range(args.steps):
+            fn()
+        sync()
+        return (time.monotonic() - t0) / args.steps
+
+    for B, T in ((1, 512), (1, 2048), (8, 512)):
+        kv = stack.make_kv(B * T).allocate(B, T)
+        x = (torch.randn(B, T, W, generator=gen).to(cfg.hidden_dtype).to(dev))
+        pos = torch.zeros(B, dtype=torch.int32, device=dev)
+        kv.extend(T)
+        t = timed(lambda: stack.forward_inference(x, kv, pos))
+        out[f"prefill {B}x{T}"] = round(B * T / t, 1)
+        kv.close()
+
+    for B, ctx in ((1, 1024), (32, 1024), (32, 4096), (128, 1024)):
+        kv = stack.make_kv(B * (ctx + 16)).allocate(B, ctx + 16)
+        kv.extend(ctx)
+        x = torch.randn(B, 1, W, generator=gen).to(cfg.hidden_dtype).to(dev)
+        pos = torch.full((B,), ctx - 1, dtype=torch.int32, device=dev)
+        kv.page_table()
+        step = lambda: stack.forward_inference(x, kv, pos)
+        step()
+        # mixtral's routing (bincount) cannot be captured: it runs eagerly
+        if on_gpu and cfg.model_type != "mixtral":
+            step()
+            sync()
+            graph = torch.cuda.CUDAGraph()
+            with torch.cuda.graph(graph):
+                step()
+            step = graph.replay
+        t = timed(step)
+        out[f"decode B{B} ctx{ctx}"] = round(B / t, 1)
+        kv.close()
+    return out
+
+
+def run_layers(args):
+    """Tokens/s through LAYERS blocks: a model beside its closest relative of
+    equal layer size, on the same inputs."""
+    rows = {}
+    for model, like in LAYER_PAIRS:
+        if args.pair and args.pair not in model:
+            continue
+        rows[model] = _layer_numbers(model, args)
+        if like:
+            rows[like] = _layer_numbers(like, args)
+            rows[f"{model} / {like}"] = {
+                k: round(rows[model][k] / rows[like][k], 3)
+                for k in rows[model]}
+        if torch.cuda.is_available():
+            torch.cuda.empty_cache()
+    first = next(iter(rows.values()))
+    print(json.dumps({
+        "metric": f"decode tokens/sec through {LAYERS} layers, B32 ctx1024",
+        "value": first["decode B32 ctx1024"], "unit": "tokens/s",
+        "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "higher_is_better": True, "vs_baseline": None, "dtype": "bf16",
+        "data": "synthetic", "config": {"mode": "layers", "layers": LAYERS},
+        "rows": rows}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -210,14 +299,21 @@ def main():
     ap.add_argument("--tp-mode", default="tensor", choices=["tensor", "expert"],
                     help="what the intra-stage group shards: tensor dims "
                          "(llama TP) or MoE experts (mixtral EP)")
-    ap.add_argument("--mode", default="pipeline", choices=["pipeline", "swarm"],
+    ap.add_argument("--mode", default="pipeline", choices=["pipeline", "swarm", "layers"],
                     help="pipeline = raw RCCL pipeline stages (flagship); "
                          "swarm = the full decentralized serving stack "
-                         "(DHT + sessions + handler) over the same device plane")
+                         "(DHT + sessions + handler) over the same device plane; "
+                         "layers = mubasun layers beside the closest family's")
+    ap.add_argument("--pair", default=None,
+                    help="layers mode: only pairs whose model name contains this")
     args = ap.parse_args()
 
     if args.mode == "swarm":
         run_swarm(args)
+        return
+
+    if args.mode == "layers":
+        run_layers(args)
         return
 
     import torch.distributed as dist

@@ -92,7 +92,7 @@ DEVINL void split_bf16(const float* p, bf16x8& hi, bf16x8& lo) {
 // ---------------------------------------------------------------------------
 
 template <int DK, int DV, int QC>  // QC: 16-row column tiles per wave
-__global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
+__global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefill_kernel(AttnArgs a) {
   constexpr int KT = 64;                 // keys per tile
   constexpr int KROW = DK * 2 + 16;      // bytes
   constexpr int VROW = KT * 2 + 16;
@@ -113,7 +113,8 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
   const int base = blockIdx.x * (64 * QC);
   if (base >= R) return;
   const int tid = threadIdx.x;
-  const int wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int* table = a.table + (long)s * a.maxp;
   const unsigned short* kpool = (const unsigned short*)a.kp;
@@ -137,6 +138,7 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
       qf[c][kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
   }
   const float sc2 = a.scale * LOG2E;
+  const int wlim = a.window > 0 ? a.window : 0x7fffffff;
 
   // visible keys of the workgroup and of this wave
   const int last = min(base + 64 * QC, R) - 1;
@@ -206,6 +208,13 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
     if (kb > whi || kb + KT <= wlo) continue;  // nothing here for this wave
     const bool inside = kb >= flo && kb + KT - 1 <= fhi;
 
+    int d0[QC];
+    float b0[QC];
+#pragma unroll
+    for (int c = 0; c < QC; ++c) {
+      d0[c] = qpos[c] - kb - hi * 8;
+      b0[c] = sl2[c] * (float)d0[c];
+    }
     float p[QC][2][8];
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf)
@@ -223,17 +232,27 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
             st[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[c][kk],
                                                             st[c], 0, 0, 0);
         }
+        // bias: -slope * (distance to the lane's first key - key offset)
 #pragma unroll
         for (int c = 0; c < QC; ++c)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int dist = qpos[c] - (kb + hf * 32 + hi * 8 + n * 4 + r);
-            float v = st[c][r] * sc2 - sl2[c] * (float)dist;
-            if (!inside && (dist < 0 || (a.window > 0 && dist >= a.window)))
-              v = NEG_BIG;
-            p[c][hf][n * 4 + r] = v;
-          }
+          for (int r = 0; r < 4; ++r)
+            p[c][hf][n * 4 + r] = fmaf(
+                st[c][r], sc2, fmaf(sl2[c], (float)(hf * 32 + n * 4 + r), -b0[c]));
       }
+    if (!inside) {
+      // a row that has seen nothing yet piles up weights of one here; its
+      // first visible key scales them by exp2(-1e30) = 0
+#pragma unroll
+      for (int c = 0; c < QC; ++c)
+#pragma unroll
+        for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const int dist = d0[c] - (hf * 32 + j);
+            if (dist < 0 || dist >= wlim) p[c][hf][j] = NEG_BIG;
+          }
+    }
 #pragma unroll
     for (int c = 0; c < QC; ++c) {
       float rm = NEG_BIG;
@@ -250,11 +269,8 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
       for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          // a masked score stays a zero weight while nothing was visible yet
-          const float e = p[c][hf][j] <= NEG_BIG ? 0.f
-                                                 : fast_exp2(p[c][hf][j] - mn);
-          p[c][hf][j] = e;
-          ps += e;
+          p[c][hf][j] = fast_exp2(p[c][hf][j] - mn);
+          ps += p[c][hf][j];
         }
       ps += __shfl_xor(ps, 16);
       ps += __shfl_xor(ps, 32);
@@ -307,7 +323,7 @@ __global__ __launch_bounds__(256) void attn_ragged_prefill_kernel(AttnArgs a) {
 // ---------------------------------------------------------------------------
 
 template <int DK, int DV>
-__global__ __launch_bounds__(256) void attn_ragged_decode_kernel(AttnArgs a) {
+__global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_decode_kernel(AttnArgs a) {
   constexpr int NKK = DK / 32, ND = DV / 16;
   constexpr int MROW = DV + 4;  // f32 per column of the merge buffer
   __shared__ __attribute__((aligned(16))) float merge[3][16 * MROW];
@@ -322,7 +338,8 @@ __global__ __launch_bounds__(256) void attn_ragged_decode_kernel(AttnArgs a) {
   const int row = a.cu[s];
   const int pos = a.tok_pos[row];
   const int tid = threadIdx.x;
-  const int wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int* table = a.table + (long)s * a.maxp;
   const unsigned short* kpool = (const unsigned short*)a.kp;
@@ -401,7 +418,7 @@ __global__ __launch_bounds__(256) void attn_ragged_decode_kernel(AttnArgs a) {
     float ps = 0.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      p[j] = p[j] <= NEG_BIG ? 0.f : fast_exp2(p[j] - mn);
+      p[j] = fast_exp2(p[j] - mn);  // every tile has a visible key
       ps += p[j];
     }
     ps += __shfl_xor(ps, 16);

@@ -155,6 +155,7 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
     a.nw = nw->data_ptr<float>();
     a.h = h->data_ptr();
     a.ldh = h->size(1);
+    vec = vec && a.ldh % 4 == 0;
   }
   if (N == 0) return;
   const size_t lds = 4 * (((W + 3) & ~3) + (size_t)a.groups + 32);
@@ -168,7 +169,8 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
           allow_lds(k, lds);
           k<<<N, decltype(blk)::value, lds, cur_stream()>>>(a);
         };
-        if (W > 2048) go(std::integral_constant<int, 1024>{});
+        // few rows: more waves on each; many: more rows at a time
+        if (W > 2048 && N <= 256) go(std::integral_constant<int, 1024>{});
         else go(std::integral_constant<int, 256>{});
       });
     });
@@ -288,7 +290,7 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
   bool vec = true;
   for (int v : {a.ldp, a.q_off, a.k_off, a.g_off, a.u_off, a.u2_off, a.dim,
                 a.vdim, a.ff, a.act_col, a.lda2})
-    vec = vec && v % 4 == 0;
+    vec = vec && (v < 0 || v % 4 == 0);  // -1: no such section
   const int cols = (a.gate ? HV : 0) + a.lda2 - HV;
   const dim3 grid(N, 3 + (cols + POST_CHUNK - 1) / POST_CHUNK);
   const size_t lds = 4 * (size_t)std::max({a.H * a.dim, a.G * a.dim,
@@ -549,11 +551,11 @@ Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
   }
 
   const int BM = ta == at::kBFloat16 && S / E >= 96 ? 128 : 64;
-  const int max_tiles = S / BM + std::min(S, E);
+  const int max_tiles = S / BM + std::min(S, E);  // the count goes behind
   auto iopt = ids.options();
   auto off = torch::empty({E + 1}, iopt);
   auto sorted = torch::empty({S}, iopt);
-  auto tiles = torch::empty({max_tiles, 2}, iopt);
+  auto tiles = torch::empty({max_tiles + 1, 2}, iopt);
   int* offp = off.data_ptr<int>();
   int* sp = sorted.data_ptr<int>();
   int* tp = tiles.data_ptr<int>();
@@ -572,13 +574,16 @@ Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
   }
   auto tile = [&](auto bm) {
     constexpr int B = decltype(bm)::value;
-    moe_tile_kernel<B, true><<<dim3(F / 64, max_tiles), 256, 0, st>>>(
+    const int nu = (F + 127) / 128, nd = (Wp + 255) / 256;
+    moe_tile_kernel<B, true><<<nu * max_tiles, 256, 0, st>>>(
         (const bf16_bits*)h.data_ptr(), (const bf16_bits*)gate_up.data_ptr(),
-        offp, sp, tp, wp, (bf16_bits*)act.data_ptr(), top, F, K, K, F);
+        offp, sp, tp, wp, (bf16_bits*)act.data_ptr(), max_tiles, nu, top, F, K,
+        K, F);
     check_launch();
-    moe_tile_kernel<B, false><<<dim3((Wp + 127) / 128, max_tiles), 256, 0, st>>>(
+    moe_tile_kernel<B, false><<<nd * max_tiles, 256, 0, st>>>(
         (const bf16_bits*)act.data_ptr(), (const bf16_bits*)down.data_ptr(),
-        offp, sp, tp, wp, (bf16_bits*)y.data_ptr(), top, Wp, F, F, Wp);
+        offp, sp, tp, wp, (bf16_bits*)y.data_ptr(), max_tiles, nd, top, Wp, F,
+        F, Wp);
     check_launch();
   };
   if (BM == 128) tile(std::integral_constant<int, 128>{});

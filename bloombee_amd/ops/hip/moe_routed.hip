@@ -13,7 +13,7 @@
 //    once; a workgroup finds its expert's slots by scanning the ids itself, so
 //    a decode step needs no sort.
 //  * moe_sort_kernel + moe_tile_kernel — longer batches: expert-sorted slots,
-//    128-wide MFMA tiles staged through LDS.
+//    MFMA tiles of 64 or 128 rows staged through LDS.
 //  * moe_simple_kernel — f32 arithmetic on f32 data.
 
 #pragma once
@@ -32,8 +32,8 @@ DEVINL int xcd_order(int id, int n) {
 // sort: one workgroup of 1024
 // ---------------------------------------------------------------------------
 
-// off (E+1), sorted (S) slots, tiles (max_tiles, 2): expert (-1 = unused) and
-// first sorted position of every BM-row tile.
+// off (E+1), sorted (S) slots, tiles (max_tiles + 1, 2): expert (-1 = unused)
+// and first sorted position of every BM-row tile; then the number of tiles.
 __global__ __launch_bounds__(1024) void moe_sort_kernel(
     const int* __restrict__ ids, int* __restrict__ off,
     int* __restrict__ sorted, int* __restrict__ tiles, int S, int E, int BM,
@@ -71,6 +71,7 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(
     }
   }
   if (tid == E - 1) off[E] = scan[tid];
+  if (tid == 0) tiles[2 * max_tiles] = min(tscan[MOE_MAX_E - 1], max_tiles);
   for (int i = tscan[MOE_MAX_E - 1] + tid; i < max_tiles; i += 1024)
     tiles[2 * i] = -1;
   cnt[tid] = first;
@@ -218,7 +219,7 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// tile: grid (tiles of N, row tiles); K % 64 == 0
+// tile: grid of column tiles * row tiles; K % 64 == 0
 // ---------------------------------------------------------------------------
 
 typedef const __attribute__((address_space(1))) void* gptr_t;
@@ -229,47 +230,57 @@ DEVINL void copy16_to_lds(const unsigned short* g, unsigned char* l) {
 }
 
 // UP: A row = sorted slot / top, out row = sorted position, N = activations
-//     (64 per tile: 64 gate rows and 64 up rows of W).
-// else: A row = sorted position, out row = slot, 128 columns per tile.
+//     (128 per tile: 128 gate rows and 128 up rows of W).
+// else: A row = sorted position, out row = slot, 256 columns per tile.
+//
+// A BM x 256 tile per workgroup; each of the four waves holds all BM rows of
+// 64 columns, so a W fragment read from LDS feeds BM / 16 MFMAs. LDS rows are
+// 64 B (32 of K) in four 16 B pieces, piece c of row r at c ^ (r / 4 % 4).
 template <int BM, bool UP>
-__global__ __launch_bounds__(256) void moe_tile_kernel(
+__global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
     const unsigned short* __restrict__ A, const unsigned short* __restrict__ W,
     const int* __restrict__ off, const int* __restrict__ sorted,
     const int* __restrict__ tiles, const float* __restrict__ wts,
-    unsigned short* __restrict__ C, int top, int N, int K, int lda, int ldc) {
-  constexpr int BK = 64, RB = BK * 2;  // LDS row bytes; 16 B pieces swizzled
-  constexpr int AI = BM * 8 / 256, BI = 4;  // 16 B pieces per thread
-  constexpr int MT = BM / 32, NT = 4;       // 16-wide tiles per wave
-  __shared__ __attribute__((aligned(16))) unsigned char
-      lds[2][(BM + 128) * RB];
+    unsigned short* __restrict__ C, int max_tiles, int ntn, int top, int N,
+    int K, int lda, int ldc) {
+  constexpr int BK = 32, RB = BK * 2, BN = 256, HN = BN / 2;
+  constexpr int AI = BM * 4 / 256, BI = BN * 4 / 256;  // 16 B pieces per thread
+  constexpr int MT = BM / 16, NT = 4;
+  __shared__ __attribute__((aligned(16))) unsigned char lds[2][(BM + BN) * RB];
 
-  const int total = gridDim.x * gridDim.y;
-  const int id = xcd_order(blockIdx.y * gridDim.x + blockIdx.x, total);
-  const int nt = id % gridDim.x, rt = id / gridDim.x;
+  // eight row tiles by all column tiles at a time: the workgroups that run
+  // together share both operands
+  const int nrt = tiles[2 * max_tiles];
+  const int total = nrt * ntn;
+  if ((int)blockIdx.x >= total) return;
+  const int id = xcd_order(blockIdx.x, total);
+  const int grp = id / (8 * ntn), in_grp = id % (8 * ntn);
+  const int gsz = min(8, nrt - grp * 8);
+  const int rt = grp * 8 + in_grp % gsz, nt = in_grp / gsz;
   const int e = tiles[2 * rt];
-  if (e < 0) return;
   const int p0 = tiles[2 * rt + 1];
   const int cnt = min(BM, off[e + 1] - p0);
-  const int n0 = nt * (UP ? 64 : 128);
-  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int n0 = nt * (UP ? HN : BN);
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  const int lane = threadIdx.x & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
-  const int wm = wave >> 1, wn = wave & 1;
 
   const unsigned short* ap[AI];
   const unsigned short* bp[BI];
 #pragma unroll
   for (int i = 0; i < AI; ++i) {
     const int ch = (i * 4 + wave) * 64 + lane;
-    const int r = ch / 8, c = (ch % 8) ^ (r & 7);
+    const int r = ch / 4, c = (ch % 4) ^ ((r >> 2) & 3);
     const int p = p0 + min(r, cnt - 1);
     ap[i] = A + (long)(UP ? sorted[p] / top : p) * lda + c * 8;
   }
 #pragma unroll
   for (int i = 0; i < BI; ++i) {
     const int ch = (i * 4 + wave) * 64 + lane;
-    const int r = ch / 8, c = (ch % 8) ^ (r & 7);
-    const long wrow = UP ? ((long)e * 2 + (r >> 6)) * N + n0 + (r & 63)
-                         : (long)e * N + min(n0 + r, N - 1);
+    const int r = ch / 4, c = (ch % 4) ^ ((r >> 2) & 3);
+    const long wrow =
+        UP ? ((long)e * 2 + r / HN) * N + min(n0 + r % HN, N - 1)
+           : (long)e * N + min(n0 + r, N - 1);
     bp[i] = W + wrow * K + c * 8;
   }
   auto issue = [&](int k, int buf) {
@@ -280,11 +291,12 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(
     for (int i = 0; i < BI; ++i)
       copy16_to_lds(bp[i] + k, lds[buf] + BM * RB + (i * 4 + wave) * 1024);
   };
-  // W rows of this wave's four column tiles
+  // W rows of this wave's four column tiles: UP pairs gate and up columns
   int brow[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n)
-    brow[n] = UP ? (n >> 1) * 64 + wn * 32 + (n & 1) * 16 : wn * 64 + n * 16;
+    brow[n] = (UP ? (n >> 1) * HN + wave * 32 + (n & 1) * 16
+                  : wave * 64 + n * 16) + li;
 
   f32x4 acc[MT][NT];
 #pragma unroll
@@ -297,27 +309,20 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(
   int buf = 0;
   for (int k = 0; k < K; k += BK) {
     if (k + BK < K) issue(k + BK, buf ^ 1);
+    bf16x8 wf[NT];
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      bf16x8 af[MT], wf[NT];
+    for (int n = 0; n < NT; ++n)
+      wf[n] = as_bf16x8(*reinterpret_cast<const short8*>(
+          lds[buf] + (BM + brow[n]) * RB + ((hi ^ ((brow[n] >> 2) & 3)) * 16)));
 #pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        const int r = wm * (BM / 2) + m * 16 + li;
-        af[m] = as_bf16x8(*reinterpret_cast<const short8*>(
-            lds[buf] + r * RB + (((kk * 4 + hi) ^ (r & 7)) * 16)));
-      }
+    for (int m = 0; m < MT; ++m) {
+      const int r = m * 16 + li;
+      const bf16x8 af = as_bf16x8(*reinterpret_cast<const short8*>(
+          lds[buf] + r * RB + ((hi ^ ((r >> 2) & 3)) * 16)));
 #pragma unroll
-      for (int n = 0; n < NT; ++n) {
-        const int r = brow[n] + li;
-        wf[n] = as_bf16x8(*reinterpret_cast<const short8*>(
-            lds[buf] + BM * RB + r * RB + (((kk * 4 + hi) ^ (r & 7)) * 16)));
-      }
-#pragma unroll
-      for (int m = 0; m < MT; ++m)
-#pragma unroll
-        for (int n = 0; n < NT; ++n)
-          acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[n], af[m],
-                                                              acc[m][n], 0, 0, 0);
+      for (int n = 0; n < NT; ++n)
+        acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[n], af,
+                                                            acc[m][n], 0, 0, 0);
     }
     __syncthreads();
     buf ^= 1;
@@ -326,25 +331,27 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(
   // a lane holds columns hi*4..hi*4+3 of row li in every tile
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
-    const int r = wm * (BM / 2) + m * 16 + li;
+    const int r = m * 16 + li;
     if (r >= cnt) continue;
     if constexpr (UP) {
 #pragma unroll
       for (int n = 0; n < 2; ++n) {
+        const int col = n0 + wave * 32 + n * 16 + hi * 4;
+        if (col >= N) continue;
         float v[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const float z = acc[m][n][j];
           v[j] = z * sigmoid_f(z) * acc[m][n + 2][j];
         }
-        stv<4>(C + (long)(p0 + r) * ldc + n0 + wn * 32 + n * 16 + hi * 4, v);
+        stv<4>(C + (long)(p0 + r) * ldc + col, v);
       }
     } else {
       const int sl = sorted[p0 + r];
       const float w = wts[sl];
 #pragma unroll
       for (int n = 0; n < NT; ++n) {
-        const int col = n0 + wn * 64 + n * 16 + hi * 4;
+        const int col = n0 + wave * 64 + n * 16 + hi * 4;
         if (col >= N) continue;
         float v[4];
 #pragma unroll

@@ -149,15 +149,20 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
   }
   __syncthreads();
   T* hr = (T*)a.h + t * (long)a.ldh;
-  for (int i = threadIdx.x; i < a.ldh; i += BLOCK) {
-    float v = 0.f;
-    if (i < W) {
-      const int g = i / gs;
-      float ss = 0.f;
-      for (int k = 0; k < subs; ++k) ss += stat[g * subs + k];
-      v = lds_row[i] * (1.f / sqrtf(ss / (float)gs + a.eps)) * a.nw[i];
-    }
-    stf(hr + i, v);
+  // one scale per group, in place of its first partial sum
+  for (int g = threadIdx.x; g < a.groups; g += BLOCK) {
+    float ss = 0.f;
+    for (int k = 0; k < subs; ++k) ss += stat[g * subs + k];
+    stat[g * subs] = 1.f / sqrtf(ss / (float)gs + a.eps);
+  }
+  __syncthreads();
+  for (int i = threadIdx.x * V; i < a.ldh; i += BLOCK * V) {
+    float v[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+      v[j] = i + j < W ? lds_row[i + j] * stat[(i + j) / gs * subs] * a.nw[i + j]
+                       : 0.f;
+    stv<V>(hr + i, v);
   }
 }
 
