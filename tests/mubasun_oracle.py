@@ -174,8 +174,15 @@ def tensor_shapes(cfg):
 
 
 def random_weights(cfg, seed=0):
-    """bf16-representable float32 weights of a lively scale."""
+    """bf16-representable float32 weights of a lively scale.
+
+    Routing must not hang on a rounding, or a 16-bit run would rightly differ
+    from the oracle. So the last norm group (the last sixth, if there is one
+    group) carries a code of +-1 per token: nothing writes to it after the
+    embedding, and the routers read nothing else."""
     gen = torch.Generator().manual_seed(seed)
+    W, groups = cfg["width"], cfg["norm"]["groups"]
+    code = slice(W - (W // groups if groups > 1 else W // 6), W)
     w = {}
     for name, shape in tensor_shapes(cfg).items():
         t = torch.randn(*shape, generator=gen)
@@ -186,9 +193,17 @@ def random_weights(cfg, seed=0):
         elif name == "pos":
             t = 0.3 * t
         elif name.endswith("router"):
-            # logits well apart: no choice hangs on a rounding
             t = t * (4.0 / math.sqrt(shape[-1]))
+            t[:, :code.start] = 0
         elif name != "embed":
             t = t / math.sqrt(shape[-1])
+        if name == "embed":
+            t[:, code] = torch.sign(t[:, code])
+        elif name == "pos":
+            t[:, code] = 0
+        elif name.endswith("norm1"):
+            t[code] = 1
+        elif name.endswith(".o") or name.endswith(".down"):
+            t[code] = 0
         w[name] = t.bfloat16().float()
     return w
