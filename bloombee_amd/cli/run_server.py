@@ -72,7 +72,8 @@ def main():
                     help="max sequences per inference session")
     ap.add_argument("--torch-dtype", default=None,
                     choices=["bfloat16", "float32"],
-                    help="serve dtype (kernels are bf16; float32 = CPU path)")
+                    help="serve dtype (kernels are bf16; float32 runs on CPU, "
+                         "and on the GPU for ragged-batch families)")
     ap.add_argument("--quant-type", default="none",
                     choices=["none", "nf4"],
                     help="nf4 maps to the 4-bit host weight tier "

@@ -51,11 +51,13 @@ def ensure_built(token_batched: bool) -> None:
             mod = importlib.util.module_from_spec(spec)
             spec.loader.exec_module(mod)
             mod.build(missing, verbose=False)
-    # the dispatch modules looked for the extensions when they were imported
-    import importlib
+    if not token_batched:
+        # this module was looked for when its dispatch layer was imported
+        import importlib
 
-    from bloombee_amd.ops import interface, ragged
-    importlib.reload(ragged if token_batched else interface)
+        from bloombee_amd.ops import interface
+        importlib.reload(interface)
+        importlib.reload(_ops)
 
 
 class TraceReplay:

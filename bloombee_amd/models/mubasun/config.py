@@ -63,8 +63,9 @@ MUBASUN_PRESETS = {
         layers=[_layer(6, 2, 32, 24, vdim=48, dense=320),
                 _layer(6, 2, 32, 33, vdim=48, experts=6, top=3, ff=80,
                        identity=2, shared=112, router_scale=1.5),
+                _layer(6, 2, 32, 24, vdim=48),
                 _layer(6, 2, 32, 24, vdim=48, experts=6, top=3, ff=80,
-                       identity=2, kv_from=1)]),
+                       identity=2, kv_from=2)]),
 }
 
 

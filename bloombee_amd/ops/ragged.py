@@ -17,7 +17,7 @@ residual, norms, routing and attention weights are f32 in both.
 from __future__ import annotations
 
 import importlib
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 from typing import Optional, Tuple
 
 import torch
@@ -25,13 +25,7 @@ import torch.nn.functional as F
 
 from bloombee_amd.ops import reference as ref
 
-try:
-    hip_ragged = importlib.import_module("bloombee_amd.ops._hip_ragged")
-    HAVE_HIP_RAGGED = True
-except ImportError as e:  # pragma: no cover
-    hip_ragged = None
-    HAVE_HIP_RAGGED = False
-    _import_error = e
+_hip_ragged = None   # loaded by the first device call
 
 # head sizes the MFMA attention kernels are compiled for; pages and q are
 # padded to the next one with zeros
@@ -40,12 +34,16 @@ SKINNY_ROWS = 32   # up to here a GEMM is a weight stream (split-K kernel)
 
 
 def _ext():
-    if not HAVE_HIP_RAGGED:
-        raise RuntimeError(
-            "the _hip_ragged extension is not built but a tensor is on GPU. "
-            "Run `python setup.py hip` (PYTORCH_ROCM_ARCH=gfx950). "
-            f"Import error was: {_import_error}")
-    return hip_ragged
+    global _hip_ragged
+    if _hip_ragged is None:
+        try:
+            _hip_ragged = importlib.import_module("bloombee_amd.ops._hip_ragged")
+        except ImportError as e:
+            raise RuntimeError(
+                "the _hip_ragged extension is not built but a tensor is on "
+                "GPU. Run `python setup.py hip` (PYTORCH_ROCM_ARCH=gfx950). "
+                f"Import error was: {e}") from e
+    return _hip_ragged
 
 
 def round_up(n: int, m: int) -> int:

@@ -26,7 +26,7 @@ import torch.nn.functional as F
 from bloombee_amd.engine import BlockStack
 from bloombee_amd.kv.paged import PagedKVCache
 from bloombee_amd.kv.views import SessionView
-from bloombee_amd.models.base import ModelConfig, resolve_config
+from bloombee_amd.models.base import ModelConfig, get_family, resolve_config
 from bloombee_amd.utils.logging import get_logger
 
 logger = get_logger(__name__)
@@ -86,6 +86,9 @@ class PipelineStage:
         logger.info(f"rank {self.rank}/{self.world} (pp {self.pp_stage} tp "
                     f"{self.tp_rank}): layers [{start}, {end})")
         self.tp_mode = tp_mode
+        if tp > 1 and get_family(cfg.model_type).head_cls is not None:
+            raise ValueError(f"{cfg.model_type} has no {tp_mode}-parallel "
+                             f"form: use pipeline stages (tp=1)")
         if tp > 1 and tp_mode == "context":
             # context parallelism: full weights on every rank; PREFILL
             # shards the sequence with ring attention (cp_prefill_llama)
@@ -120,9 +123,14 @@ class PipelineStage:
         self.kv = self.kv_pool.allocate(global_batch, max_session_len)
 
         self.is_client = self.rank == 0
+        self.head = None
         if self.is_client:
             gen = torch.Generator().manual_seed(seed)
             dt = cfg.dtype
+            head_cls = get_family(cfg.model_type).head_cls
+            if head_cls is not None:
+                self.head = head_cls(cfg, device=self.device, seed=seed)
+        if self.is_client and self.head is None:
             self.embed = (torch.randn(cfg.vocab_size, cfg.hidden_size, generator=gen)
                           .mul_(0.02).to(dt).to(self.device))
             self.final_norm_w = torch.ones(cfg.hidden_size, dtype=dt, device=self.device)
@@ -135,7 +143,7 @@ class PipelineStage:
         self.prev_rank = ((self.pp_stage - 1) % self.pp_world) * tp
         self.is_leader = self.tp_rank == 0
         # persistent recv buffers per micro-batch
-        self._recv_buf = [torch.empty(self.mb, 1, cfg.hidden_size, dtype=cfg.dtype,
+        self._recv_buf = [torch.empty(self.mb, 1, cfg.hidden_size, dtype=cfg.hidden_dtype,
                                       device=self.device) for _ in range(self.M)]
         # hipGraph decode capture (single-rank fast path): the whole decode
         # step — embed, 32 blocks, LM head, argmax, position bump — replays as
@@ -150,6 +158,15 @@ class PipelineStage:
         self._eager_steps = 0
 
     # ------------------------------------------------------------------
+    def _embed(self, ids: torch.Tensor, start: Optional[torch.Tensor]):
+        """(B, T) ids; start (B,): first positions (learned positions only)."""
+        ids = ids.to(self.device)
+        if self.head is None:
+            return F.embedding(ids, self.embed)
+        pos = torch.arange(ids.shape[1], dtype=torch.int32, device=self.device)
+        pos = pos.expand(*ids.shape) if start is None else start.view(-1, 1) + pos
+        return self.head.embed(ids, pos)
+
     def _run_local(self, hidden: torch.Tensor, view, start_pos: torch.Tensor):
         return self.stack.forward_inference(hidden, view, start_pos)
 
@@ -164,16 +181,9 @@ class PipelineStage:
         """Whole decode step on persistent buffers (graph-capturable: every
         host-varying quantity lives in a device tensor)."""
         B = self.global_batch
-        hid = F.embedding(self._ids_buf.view(B, 1), self.embed)
+        hid = self._embed(self._ids_buf.view(B, 1), self._pos_buf)
         h = self.stack.forward_inference(hid, self.kv, self._pos_buf)
-        from bloombee_amd import ops
-
-        y = ops.rms_norm(h[:, -1], self.final_norm_w, self.config.rms_norm_eps)
-        # vocab projection stays on hipBLASLt: at N=128k it streams the
-        # 1.05 GB weight at 5.5 TB/s vs 5.3 for the skinny kernel (measured
-        # — the skinny kernel only wins the small-N decode shapes)
-        nxt = F.linear(y, self.lm_head_w).float().argmax(-1)
-        self._ids_buf.copy_(nxt)
+        self._ids_buf.copy_(self._lm_head(h[:, -1]))
         self._pos_buf += 1
 
     def _decode_round_single(self, ids: torch.Tensor) -> torch.Tensor:
@@ -221,9 +231,9 @@ class PipelineStage:
 
         if self.pp_stage == 0:
             if self.is_client:
-                hid = F.embedding(ids.view(B, 1).to(self.device), self.embed)
+                hid = self._embed(ids.view(B, 1), start_all)
             else:
-                hid = torch.empty(B, 1, cfg.hidden_size, dtype=cfg.dtype,
+                hid = torch.empty(B, 1, cfg.hidden_size, dtype=cfg.hidden_dtype,
                                   device=self.device)
             if self.tp > 1:
                 dist.broadcast(hid, src=0, group=self.tp_group)
@@ -275,11 +285,11 @@ class PipelineStage:
         B = self.global_batch
         assert self.kv.seqs[0].l_spec == 0, "CP prefill is one-shot"
         assert T % self.tp == 0, "prompt length must divide by cp degree"
-        hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.dtype,
+        hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
                           device=self.device)
         if self.pp_stage == 0:
             if self.is_client:
-                hid = F.embedding(ids.to(self.device), self.embed)
+                hid = self._embed(ids, None)
         elif self.is_leader:
             dist.recv(hid, self.prev_rank)
         if self.tp > 1 and dist.is_initialized():
@@ -324,13 +334,13 @@ class PipelineStage:
         self.kv.extend(T)
         views = self._views()
         pending = []
-        bufs = [torch.empty(mb, T, cfg.hidden_size, dtype=cfg.dtype,
+        bufs = [torch.empty(mb, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
                             device=self.device) for _ in range(M)]
         if self.pp_stage == 0:
             if self.is_client:
-                hid = F.embedding(ids.to(self.device), self.embed)
+                hid = self._embed(ids, start_all)
             else:
-                hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.dtype,
+                hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
                                   device=self.device)
             if self.tp > 1:
                 dist.broadcast(hid, src=0, group=self.tp_group)
@@ -369,7 +379,12 @@ class PipelineStage:
     def _lm_head(self, hidden_last: torch.Tensor) -> torch.Tensor:
         from bloombee_amd import ops
 
+        if self.head is not None:
+            return self.head.logits(self.head.final_norm(hidden_last)).argmax(-1)
         y = ops.rms_norm(hidden_last, self.final_norm_w, self.config.rms_norm_eps)
+        # vocab projection stays on hipBLASLt: at N=128k it streams the
+        # 1.05 GB weight at 5.5 TB/s vs 5.3 for the skinny kernel (measured
+        # — the skinny kernel only wins the small-N decode shapes)
         return F.linear(y, self.lm_head_w).float().argmax(-1)
 
 

@@ -18,7 +18,10 @@ def _free_port():
         return s.getsockname()[1]
 
 
-def _worker(rank, world, q, port):
+MODELS = {"llama-tiny": 1000, "mubasun-tiny": 320}   # name -> vocab
+
+
+def _worker(rank, world, q, port, model):
     os.environ["MASTER_ADDR"] = "127.0.0.1"
     os.environ["MASTER_PORT"] = str(port)
     os.environ["RANK"] = str(rank)
@@ -27,11 +30,11 @@ def _worker(rank, world, q, port):
     try:
         from bloombee_amd.parallel.pipeline import PipelineStage
 
-        stage = PipelineStage("llama-tiny", "cpu", global_batch=4,
+        stage = PipelineStage(model, "cpu", global_batch=4,
                               micro_batches=2, seed=0, kv_max_tokens=8192,
                               max_session_len=64)
         gen = torch.Generator().manual_seed(7)
-        prompt = torch.randint(0, 1000, (4, 10), generator=gen)
+        prompt = torch.randint(0, MODELS[model], (4, 10), generator=gen)
         ids = stage.prefill_round(prompt if rank == 0 else None, 10)
         toks = []
         for _ in range(5):
@@ -45,11 +48,12 @@ def _worker(rank, world, q, port):
 
 
 @pytest.mark.timeout(180)
-def test_pipeline_matches_local_engine():
+@pytest.mark.parametrize("model", list(MODELS))
+def test_pipeline_matches_local_engine(model):
     ctx = mp.get_context("spawn")
     q = ctx.Queue()
     port = _free_port()
-    procs = [ctx.Process(target=_worker, args=(r, 2, q, port)) for r in range(2)]
+    procs = [ctx.Process(target=_worker, args=(r, 2, q, port, model)) for r in range(2)]
     for p in procs:
         p.start()
     got = q.get(timeout=150)
@@ -57,9 +61,9 @@ def test_pipeline_matches_local_engine():
         p.join(timeout=60)
         assert p.exitcode == 0
 
-    eng = LocalEngine("llama-tiny", device="cpu", seed=0, kv_max_tokens=8192)
+    eng = LocalEngine(model, device="cpu", seed=0, kv_max_tokens=8192)
     gen = torch.Generator().manual_seed(7)
-    prompt = torch.randint(0, 1000, (4, 10), generator=gen)
+    prompt = torch.randint(0, MODELS[model], (4, 10), generator=gen)
     kv = eng.kv_pool.allocate(4, 64)
     ids = eng.prefill(prompt, kv)
     expect = []
@@ -72,18 +76,19 @@ def test_pipeline_matches_local_engine():
 
 
 @pytest.mark.timeout(120)
-def test_single_rank_pipeline_matches_local():
+@pytest.mark.parametrize("model", list(MODELS))
+def test_single_rank_pipeline_matches_local(model):
     """world=1 PipelineStage (no dist) == LocalEngine."""
     from bloombee_amd.parallel.pipeline import PipelineStage
 
-    stage = PipelineStage("llama-tiny", "cpu", global_batch=4, seed=0,
+    stage = PipelineStage(model, "cpu", global_batch=4, seed=0,
                           kv_max_tokens=8192, max_session_len=64)
     gen = torch.Generator().manual_seed(7)
-    prompt = torch.randint(0, 1000, (4, 10), generator=gen)
+    prompt = torch.randint(0, MODELS[model], (4, 10), generator=gen)
     ids = stage.prefill_round(prompt, 10)
     toks = [ids]
 
-    eng = LocalEngine("llama-tiny", device="cpu", seed=0, kv_max_tokens=8192)
+    eng = LocalEngine(model, device="cpu", seed=0, kv_max_tokens=8192)
     kv = eng.kv_pool.allocate(4, 64)
     ids2 = eng.prefill(prompt, kv)
     assert torch.equal(toks[0], ids2)
