@@ -368,7 +368,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_decode
 #pragma unroll
   for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
 
-  bf16x8 k0[2][NKK], v0[ND], k1[2][NKK], v1[ND];
+  bf16x8 k0[2][NKK], v0[ND];
   auto load = [&](bf16x8 (&kf)[2][NKK], bf16x8 (&vf)[ND], int tile) {
     const int vpos = tile * 32 + hi * 8;
     const bool live = vpos <= pos;
@@ -440,17 +440,25 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_decode
     }
   };
 
-  // two named buffers: the next tile's loads fly behind this tile's compute
   int t = t_lo + wave;
-  if (t < t_hi) load(k0, v0, t);
-  for (; t < t_hi; t += 8) {
-    if (t + 4 < t_hi) load(k1, v1, t + 4);
-    __builtin_amdgcn_sched_barrier(0);
-    compute(k0, v0, t);
-    if (t + 4 >= t_hi) break;
-    if (t + 8 < t_hi) load(k0, v0, t + 8);
-    __builtin_amdgcn_sched_barrier(0);
-    compute(k1, v1, t + 4);
+  if constexpr (DK + DV > 256) {   // no registers for a second buffer
+    for (; t < t_hi; t += 4) {
+      load(k0, v0, t);
+      compute(k0, v0, t);
+    }
+  } else {
+    // two named buffers: the next tile's loads fly behind this one's compute
+    bf16x8 k1[2][NKK], v1[ND];
+    if (t < t_hi) load(k0, v0, t);
+    for (; t < t_hi; t += 8) {
+      if (t + 4 < t_hi) load(k1, v1, t + 4);
+      __builtin_amdgcn_sched_barrier(0);
+      compute(k0, v0, t);
+      if (t + 4 >= t_hi) break;
+      if (t + 8 < t_hi) load(k0, v0, t + 8);
+      __builtin_amdgcn_sched_barrier(0);
+      compute(k1, v1, t + 4);
+    }
   }
 
   // fold waves 1..3 into wave 0

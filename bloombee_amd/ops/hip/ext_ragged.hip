@@ -290,7 +290,7 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
   bool vec = true;
   for (int v : {a.ldp, a.q_off, a.k_off, a.g_off, a.u_off, a.u2_off, a.dim,
                 a.vdim, a.ff, a.act_col, a.lda2})
-    vec = vec && (v < 0 || v % 4 == 0);  // -1: no such section
+    vec = vec && (v < 0 || v % 8 == 0);  // -1: no such section
   const int cols = (a.gate ? HV : 0) + a.lda2 - HV;
   const dim3 grid(N, 3 + (cols + POST_CHUNK - 1) / POST_CHUNK);
   const size_t lds = 4 * (size_t)std::max({a.H * a.dim, a.G * a.dim,
@@ -299,7 +299,7 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
     by_type(ta, [&](auto t) {
       by_bool(vec, [&](auto v) {
         auto k = proj_post_kernel<decltype(p), decltype(t),
-                                  decltype(v)::value ? 4 : 1>;
+                                  decltype(v)::value ? 8 : 1>;
         allow_lds(k, lds);
         k<<<grid, POST_BLOCK, lds, cur_stream()>>>(a);
       });

@@ -18,15 +18,21 @@
 
 DEVINL float ldf(const unsigned short* p) { return bf2f(*p); }
 DEVINL float ldf(const float* p) { return *p; }
-DEVINL void stf(unsigned short* p, float v) { *p = f2bf(v); }
+// round to nearest even in hardware
+DEVINL unsigned short cvt_bf(float v) {
+  return __builtin_bit_cast(unsigned short, (__bf16)v);
+}
+DEVINL void stf(unsigned short* p, float v) { *p = cvt_bf(v); }
 DEVINL void stf(float* p, float v) { *p = v; }
 
 typedef __attribute__((ext_vector_type(4))) unsigned short ushort4v;
 
-// V consecutive elements as f32. V = 4 needs 4-element alignment.
+// V (1, 4 or 8) consecutive elements as f32, aligned to V elements.
 template <int V>
 DEVINL void ldv(const unsigned short* p, float* o) {
-  if constexpr (V == 4) {
+  if constexpr (V == 8) {
+    load_bf16x8(p, o);
+  } else if constexpr (V == 4) {
     const ushort4v u = *reinterpret_cast<const ushort4v*>(p);
 #pragma unroll
     for (int j = 0; j < 4; ++j) o[j] = bf2f(u[j]);
@@ -36,7 +42,10 @@ DEVINL void ldv(const unsigned short* p, float* o) {
 }
 template <int V>
 DEVINL void ldv(const float* p, float* o) {
-  if constexpr (V == 4) {
+  if constexpr (V == 8) {
+    ldv<4>(p, o);
+    ldv<4>(p + 4, o + 4);
+  } else if constexpr (V == 4) {
     const f32x4 u = *reinterpret_cast<const f32x4*>(p);
 #pragma unroll
     for (int j = 0; j < 4; ++j) o[j] = u[j];
@@ -46,18 +55,26 @@ DEVINL void ldv(const float* p, float* o) {
 }
 template <int V>
 DEVINL void stv(unsigned short* p, const float* v) {
-  if constexpr (V == 4) {
+  if constexpr (V == 8) {
+    short8 u;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) u[j] = (short)cvt_bf(v[j]);
+    *reinterpret_cast<short8*>(p) = u;
+  } else if constexpr (V == 4) {
     ushort4v u;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) u[j] = f2bf(v[j]);
+    for (int j = 0; j < 4; ++j) u[j] = cvt_bf(v[j]);
     *reinterpret_cast<ushort4v*>(p) = u;
   } else {
-    *p = f2bf(v[0]);
+    *p = cvt_bf(v[0]);
   }
 }
 template <int V>
 DEVINL void stv(float* p, const float* v) {
-  if constexpr (V == 4) {
+  if constexpr (V == 8) {
+    stv<4>(p, v);
+    stv<4>(p + 4, v + 4);
+  } else if constexpr (V == 4) {
     f32x4 u;
 #pragma unroll
     for (int j = 0; j < 4; ++j) u[j] = v[j];
@@ -67,7 +84,19 @@ DEVINL void stv(float* p, const float* v) {
   }
 }
 
-DEVINL float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+DEVINL float sigmoid_f(float z) {
+  return __builtin_amdgcn_rcpf(1.f + fast_exp2(-z * LOG2E));
+}
+
+// e^z - 1 - z for z <= 0. Near zero the series, where the difference would
+// cancel.
+DEVINL float exp_minus_1_minus(float z) {
+  const float far = fast_exp2(z * LOG2E) - 1.f - z;
+  const float t = 1.f + z * (1.f / 6) * (1.f + z * (1.f / 7) * (1.f + z * (1.f / 8)));
+  const float near = 0.5f * z * z *
+      (1.f + z * (1.f / 3) * (1.f + z * (1.f / 4) * (1.f + z * (1.f / 5) * t)));
+  return z > -0.5f ? near : far;
+}
 
 // ---------------------------------------------------------------------------
 
@@ -385,7 +414,7 @@ __global__ __launch_bounds__(POST_BLOCK) void proj_post_kernel(PostArgs a) {
 #pragma unroll
         for (int j = 0; j < V; ++j) {
           const float z = v[j];
-          v[j] = (z > 0.f ? a.xp * z * z : a.xq * (expm1f(z) - z)) + 0.5f * z;
+          v[j] = (z > 0.f ? a.xp * z * z : a.xq * exp_minus_1_minus(z)) + 0.5f * z;
         }
       } else {
         float u[V];
