@@ -733,13 +733,17 @@ torch::Tensor gemm_skinny(torch::Tensor A, torch::Tensor W,
     pp = part.data_ptr<float>();
   }
   dim3 grid(N / 64, ksplit);
+  auto launch_v2 = [&](auto mt, auto stage_norm) {
+    gemm_skinny_v2_kernel<decltype(mt)::value, decltype(stage_norm)::value>
+        <<<grid, 256, 0, cur_stream()>>>(
+            bf_ptr(A), bf_ptr(W), ksplit == 1 ? rp : nullptr,
+            ksplit == 1 ? bp : nullptr, bf_ptr_mut(C), pp, M, N, K, kchunk,
+            ksplit, nwp, (float)eps, norm_mode, ssinp, nstripes,
+            ksplit == 1 ? ssoutp : nullptr);
+  };
   auto launch = [&](auto mt) {
-    if (v2)
-      gemm_skinny_v2_kernel<decltype(mt)::value><<<grid, 256, 0, cur_stream()>>>(
-          bf_ptr(A), bf_ptr(W), ksplit == 1 ? rp : nullptr,
-          ksplit == 1 ? bp : nullptr, bf_ptr_mut(C), pp, M, N, K, kchunk, ksplit,
-          nwp, (float)eps, norm_mode, ssinp, nstripes,
-          ksplit == 1 ? ssoutp : nullptr);
+    if (v2 && norm_mode == 1) launch_v2(mt, std::true_type{});
+    else if (v2) launch_v2(mt, std::false_type{});
     else {
       TORCH_CHECK(!norm_mode && (!ssoutp || ksplit > 1),
                   "fused norm / ss_out need the v2 (K%256) kernel");

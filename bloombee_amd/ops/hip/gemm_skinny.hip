@@ -116,7 +116,9 @@ __global__ __launch_bounds__(256) void gemm_skinny_kernel(
 //    to LDS once per stage with full-line loads and A fragments come from
 //    conflict-free padded ds_read_b128.
 // Host guarantees (k1 - k0) % 256 == 0 so the set pairing needs no tail.
-template <int MT>
+// STAGE_NORM: norm mode 1 as an instantiation of its own — its per-element
+// scaling, though never run, slows the other modes' pipeline by 7%.
+template <int MT, bool STAGE_NORM = false>
 __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
     const unsigned short* __restrict__ A,   // (M, K) bf16
     const unsigned short* __restrict__ W,   // (N, K) bf16
@@ -186,7 +188,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
       const int row = min(flat / 32, M - 1);
       const int off = (flat % 32) * 8;
       aregs[j] = *reinterpret_cast<const short8*>(A + (long)row * K + ks + off);
-      if (norm_mode == 1)
+      if (STAGE_NORM)
         nregs[j] = *reinterpret_cast<const short8*>(nw + ks + off);
     }
   };
@@ -195,7 +197,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
     for (int j = 0; j < 4; ++j) {
       const int flat = threadIdx.x + j * 256;
       short8 v = aregs[j];
-      if (norm_mode == 1) {
+      if (STAGE_NORM) {
         const float ir = invr[flat / 32 >= M ? M - 1 : flat / 32];
 #pragma unroll
         for (int e = 0; e < 8; ++e)
@@ -286,7 +288,7 @@ __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
     }
   };
 
-  if (norm_mode == 1) {
+  if (STAGE_NORM) {
     // mode 1 scales A as it stages: invr must exist BEFORE the pipeline.
     // Issue the first W-register set first so the stream is in flight.
     issue0(k0);
@@ -305,10 +307,14 @@ __global__ __launch_bounds__(256) void gemm_skinny_v2_kernel(
     __syncthreads();
   }
   for (int k = k0; k < k1; k += KSTEP) {
+    // the barriers keep the scheduler from sinking a set's loads down to
+    // their first use
     if (k + KSTEP < k1) load_a(k + KSTEP);
     issue1(k + 128);
+    __builtin_amdgcn_sched_barrier(0);
     mfma_set(bB0, 0);
     if (k + KSTEP < k1) issue0(k + KSTEP);
+    __builtin_amdgcn_sched_barrier(0);
     mfma_set(bB1, 1);
     if (k + KSTEP < k1) {
       __syncthreads();  // everyone done reading stage s

@@ -193,8 +193,10 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
     const bool more = k + KSTEP < K;
     if (more) load_a(k + KSTEP);
     load_w(b1, k + 128);
+    __builtin_amdgcn_sched_barrier(0);
     mma(b0, 0);
     if (more) load_w(b0, k + KSTEP);
+    __builtin_amdgcn_sched_barrier(0);
     mma(b1, 1);
     if (more) {
       __syncthreads();
