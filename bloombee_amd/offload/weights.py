@@ -97,7 +97,8 @@ class OffloadedBlockStack:
                              if self.on_gpu else None)
         self._events: Dict[int, torch.cuda.Event] = {}
         self._done_events: Dict[int, torch.cuda.Event] = {}  # slot -> event
-        self._arena: List[Dict[str, torch.Tensor]] = [{}, {}]
+        self._arena: List[torch.Tensor] = []
+        self._layout: Dict[int, Dict[str, tuple]] = {}
         self._arena_owner = [-1, -1]
         self._host: Dict[int, Dict[str, _HostParam]] = {}
 
@@ -113,23 +114,34 @@ class OffloadedBlockStack:
                     params[name] = _HostParam(p.data, policy.pin_weight,
                                               policy.compress_weight, use_disk)
                 self._host[i] = params
-            # arena buffers shaped like block[resident] (uniform block shapes)
-            proto = stack.blocks[self.resident]
-            for slot in range(2):
-                self._arena[slot] = {
-                    name: torch.empty_like(p.data)
-                    for name, p in proto.named_parameters()}
+            # two byte arenas that fit the largest offloaded block; a block's
+            # parameters are views into one of them (blocks may differ)
+            size = 0
+            for i in range(self.resident, n):
+                at, layout = 0, {}
+                for name, p in stack.blocks[i].named_parameters():
+                    nbytes = p.numel() * p.element_size()
+                    layout[name] = (at, nbytes, p.dtype, tuple(p.shape))
+                    at = (at + nbytes + 255) // 256 * 256
+                self._layout[i] = layout
+                size = max(size, at)
+            self._arena = [torch.empty(size, dtype=torch.uint8,
+                                       device=self.device) for _ in range(2)]
             # drop offloaded device copies
             for i in range(self.resident, n):
-                for name, p in stack.blocks[i].named_parameters():
-                    p.data = self._arena[0][name]  # placeholder binding
+                self._bind(i, 0)  # placeholder binding
             logger.info("offload: %d/%d blocks resident, %d on disk, "
                         "compress=%s", self.resident, n, ndisk,
                         policy.compress_weight)
 
     # ------------------------------------------------------------------
+    def _views(self, i: int, slot: int) -> Dict[str, torch.Tensor]:
+        flat = self._arena[slot]
+        return {name: flat[at:at + nbytes].view(dtype).view(shape)
+                for name, (at, nbytes, dtype, shape) in self._layout[i].items()}
+
     def _fill(self, i: int, slot: int) -> None:
-        arena = self._arena[slot]
+        arena = self._views(i, slot)
         if self.on_gpu:
             with torch.cuda.stream(self._copy_stream):
                 # don't overwrite a slot whose previous block may still have
@@ -139,9 +151,9 @@ class OffloadedBlockStack:
                     self._copy_stream.wait_event(done)
                 for name, hp in self._host[i].items():
                     hp.copy_into(arena[name])
-                    # arena tensors were allocated on the default stream; tell
-                    # the caching allocator they are used on the copy stream
-                    arena[name].record_stream(self._copy_stream)
+                # the arena was allocated on the default stream; tell the
+                # caching allocator it is used on the copy stream
+                self._arena[slot].record_stream(self._copy_stream)
                 ev = torch.cuda.Event()
                 ev.record(self._copy_stream)
                 self._events[i] = ev
@@ -152,7 +164,7 @@ class OffloadedBlockStack:
 
     def _bind(self, i: int, slot: int) -> None:
         blk = self.stack.blocks[i]
-        arena = self._arena[slot]
+        arena = self._views(i, slot)
         for name, p in blk.named_parameters():
             p.data = arena[name]
 

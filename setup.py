@@ -1,9 +1,9 @@
 """Build the bloombee_amd gfx950 HIP extension in-tree.
 
 Invokes hipcc directly (native HIP source — no hipify pass, no CUDA
-compatibility layer). The built .so files land in bloombee_amd/ops/ so
-they travel with the repo snapshot to the GPU box (gpurun ships in-tree .so
-files; a JIT cache under ~/.cache would not).
+compatibility layer). The built .so files land in bloombee_amd/ops/, inside the
+tree, so that a copy of the tree carries them (a JIT cache under ~/.cache would
+stay behind).
 
 Usage:
     python setup.py build_ext --inplace     # or: python setup.py hip

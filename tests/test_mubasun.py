@@ -67,7 +67,7 @@ CONFIGS = {
         (attn(5, 5, 18, 18, 31), dense(77)),
         (attn(3, 1, 30, 21, 40, kv_from=0), dense(50))], eps=1e-3),
     # windows beyond the context, many heads on one key head, one group
-    "wide": model(256, 512, 1, [
+    "wide": model(320, 517, 1, [
         (attn(20, 1, 32, 64, 5000), dense(512)),
         (attn(2, 1, 128, 128, 96), moe(16, 64, 4, 0, 1.0))]),
 }
@@ -542,6 +542,32 @@ def test_block_range_must_hold_the_shared_layer(models, monkeypatch):
     BlockStack(cfg, 1, 3).make_kv(64)
     with pytest.raises(RuntimeError, match="KV of layer 1"):
         BlockStack(cfg, 2, 4).make_kv(64)
+
+
+@pytest.mark.parametrize("dev", ["cpu", pytest.param("cuda:0", marks=GPU)])
+def test_offloaded_blocks(models, dev, monkeypatch):
+    """Blocks of unlike shapes stream through one arena."""
+    monkeypatch.setenv("BBAMD_TORCH_DTYPE", "float32")
+    from bloombee_amd.offload import OffloadPolicy
+    from bloombee_amd.offload.weights import OffloadedBlockStack
+    from bloombee_amd.server.from_pretrained import load_block_weights
+    path, w, cfg = models["full"]
+    stack = BlockStack(resolve_config(path), 0, 5, device=dev)
+    for i, blk in enumerate(stack.blocks):
+        load_block_weights(blk, path, i)
+    off = OffloadedBlockStack(stack, OffloadPolicy(weight_gpu_percent=20.0))
+    toks = prompt(cfg, 50, 5)
+    col = []
+    oracle.forward(torch.tensor(toks), w, cfg, col)
+    x = (w["embed"][toks] + w["pos"][:50]).float()[None].to(dev)
+    kv = off.make_kv(128).allocate(1, 50)
+    out = []
+    for a, b in ((0, 31), (31, 49), (49, 50)):
+        kv.extend(b - a)
+        out.append(off.forward_inference(
+            x[:, a:b], kv, torch.tensor([a], dtype=torch.int32, device=dev)))
+    got = torch.cat(out, 1)[0].cpu().double()
+    torch.testing.assert_close(got, col[-1], rtol=1e-4, atol=1e-4)
 
 
 def test_training_path(models, monkeypatch):
