@@ -137,12 +137,11 @@ def linear_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     """x (M, K) @ w (N, K)^T with an f32 result, a few rows at a time (vocab
-    projection of the rows that are sampled)."""
+    projection of the rows that are sampled). One split: a vocabulary is wide,
+    and a library sum over splits may not be capturable."""
     if x.is_cuda and x.dtype == torch.bfloat16:
-        outs = []
-        for xs in x.split(SKINNY_ROWS):
-            p = _ext().gemm_parts(xs.contiguous(), w, 0)
-            outs.append(p[0] if p.shape[0] == 1 else p.sum(0))
+        outs = [_ext().gemm_parts(xs.contiguous(), w, 1)[0]
+                for xs in x.split(SKINNY_ROWS)]
         return outs[0] if len(outs) == 1 else torch.cat(outs)
     return F.linear(x.float(), w.float())
 

@@ -512,25 +512,27 @@ def test_trace_replay(models, name, dev, dt, tmp_path, monkeypatch, capsys):
         check(raw.view(-1, cfg["vocab"]), w, dt, k)
 
 
-def test_swarm_generation(models, monkeypatch):
+@kinds
+def test_swarm_generation(models, dev, dt, monkeypatch):
     """A server and a client on one checkpoint folder, hidden states in 32 bits."""
     from bloombee_amd.client.config import ClientConfig
     from bloombee_amd.models import auto
     from bloombee_amd.net.dht import Dht
     from bloombee_amd.server import Server
-    monkeypatch.setenv("BBAMD_TORCH_DTYPE", "float32")
+    monkeypatch.setenv("BBAMD_TORCH_DTYPE", dt)
     path, _, cfg = models["odd"]
     boot = Dht()
     srv = Server(path, initial_peers=[boot.endpoint], block_indices=(0, 3),
-                 update_period=5.0)
+                 update_period=5.0, device=dev)
     srv.run_in_background()
     try:
         m = auto.AutoDistributedModelForCausalLM.from_pretrained(
-            path, client_config=ClientConfig(initial_peers=[boot.endpoint]))
+            path, client_config=ClientConfig(initial_peers=[boot.endpoint]),
+            device=dev)
         p = prompt(cfg, 12, 4)
         out = m.generate(torch.tensor([p]), max_new_tokens=8)[0].tolist()
         assert out[:12] == p
-        agree(out[12:], models, "odd", p, "float32")
+        agree(out[12:], models, "odd", p, dt)
     finally:
         srv.shutdown()
         boot.shutdown()
