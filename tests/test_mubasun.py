@@ -530,7 +530,8 @@ def test_swarm_generation(models, dev, dt, monkeypatch):
             path, client_config=ClientConfig(initial_peers=[boot.endpoint]),
             device=dev)
         p = prompt(cfg, 12, 4)
-        out = m.generate(torch.tensor([p]), max_new_tokens=8)[0].tolist()
+        out = m.generate(torch.tensor([p], device=dev),
+                         max_new_tokens=8)[0].tolist()
         assert out[:12] == p
         agree(out[12:], models, "odd", p, dt)
     finally:
