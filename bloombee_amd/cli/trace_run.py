@@ -13,7 +13,8 @@ continuing from its request's cache. `want` names the places whose logits go
 to OUT/<step>.f32 (32-bit floats, [wanted, vocab], entry order); `end` frees
 requests. After every step a line "done <step>" is printed. Nothing is sampled.
 
-The KV pool holds --max-tokens, so pages of ended requests are used again.
+The KV pool holds --max-tokens and state slots for --max-requests, so pages and
+slots of ended requests are used again.
 Steps in which every entry brings one token and wants its logits replay the
 engine's captured decode graph, as generation does.
 """
@@ -24,20 +25,17 @@ import json
 import os
 import sys
 
-# families whose blocks run on _hip_ragged alone need no other module
-_MODULES = {True: ["_hip_ragged"], False: ["_hip_ops"]}
-
-
-def ensure_built(token_batched: bool) -> None:
-    """Compile the extension modules this model runs on, if they are missing.
-    A lock file lets concurrent first calls share one compilation."""
+def ensure_built(block_cls) -> None:
+    """Compile the extension modules this model's blocks run on, if they are
+    missing: hip_modules of ragged-batch blocks, _hip_ops for the others. A
+    lock file lets concurrent first calls share one compilation."""
     import fcntl
 
     from bloombee_amd import ops as _ops
 
     ops_dir = os.path.dirname(os.path.abspath(_ops.__file__))
     root = os.path.dirname(os.path.dirname(ops_dir))
-    need = _MODULES[token_batched]
+    need = getattr(block_cls, "hip_modules", ("_hip_ops",))
     path = lambda m: os.path.join(ops_dir, m + ".so")
     if all(os.path.exists(path(m)) for m in need):
         return
@@ -51,7 +49,7 @@ def ensure_built(token_batched: bool) -> None:
             mod = importlib.util.module_from_spec(spec)
             spec.loader.exec_module(mod)
             mod.build(missing, verbose=False)
-    if not token_batched:
+    if "_hip_ops" in need:
         # this module was looked for when its dispatch layer was imported
         import importlib
 
@@ -96,6 +94,9 @@ def main(argv=None) -> int:
     ap.add_argument("--out", required=True, help="folder for <step>.f32")
     ap.add_argument("--max-tokens", type=int, required=True,
                     help="KV tokens that live requests hold at any time")
+    ap.add_argument("--max-requests", type=int, default=4,
+                    help="requests live at any time (state slots of models "
+                         "with recurrent layers)")
     ap.add_argument("--device", default="cuda:0")
     args = ap.parse_args(argv)
 
@@ -110,8 +111,7 @@ def main(argv=None) -> int:
         if not torch.cuda.is_available():
             print("trace_run: no GPU", file=sys.stderr)
             return 2
-        ensure_built(getattr(get_block_class(cfg.model_type),
-                             "token_batched", False))
+        ensure_built(get_block_class(cfg.model_type))
     # 32-bit products stay 32-bit
     torch.backends.cuda.matmul.allow_tf32 = False
     torch.set_float32_matmul_precision("highest")
@@ -119,7 +119,8 @@ def main(argv=None) -> int:
     from bloombee_amd.engine import LocalEngine
 
     replay = TraceReplay(LocalEngine(args.model, device=args.device,
-                                     kv_max_tokens=args.max_tokens))
+                                     kv_max_tokens=args.max_tokens,
+                                     max_seqs=args.max_requests))
     for text in sys.stdin:
         if not text.strip():
             continue

@@ -46,6 +46,8 @@ class KVConfig:
     # Fraction of free device memory the KV pool may claim when the budget is
     # not set explicitly (the reference sizes from --attn_cache_tokens).
     max_tokens: Optional[int] = field(default_factory=lambda: _env("KV_MAX_TOKENS", None, int))
+    # state slots of models with recurrent layers: sequences live at a time
+    max_seqs: int = field(default_factory=lambda: _env("KV_MAX_SEQS", 128))
     alloc_timeout: float = field(default_factory=lambda: _env("KV_ALLOC_TIMEOUT", 60.0))
     # BBAMD_MIXED_ATTN: host-swapped sessions resume DECODING with their
     # committed KV left in host memory (mixed-device attention, exact

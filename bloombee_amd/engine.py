@@ -67,7 +67,9 @@ class BlockStack(torch.nn.Module):
                                    self.blocks[src - start])
         self.device = torch.device(device)
 
-    def make_kv(self, max_tokens: int) -> PagedKVCache:
+    def make_kv(self, max_tokens: int,
+                max_seqs: Optional[int] = None) -> PagedKVCache:
+        """max_seqs: state slots of recurrent layers (default: configured)."""
         # per-layer KV geometry hooks (gemma-4 heterogeneous head_dim/kv heads;
         # kv_layout also names value sizes and shared layers)
         if hasattr(self.config, "kv_layout"):
@@ -79,7 +81,8 @@ class BlockStack(torch.nn.Module):
             geometry = dict(num_kv_heads=self.config.num_key_value_heads,
                             head_dim=self.config.head_dim)
         from bloombee_amd.config import get_config
-        P = get_config().kv.page_size
+        kvc = get_config().kv
+        P = kvc.page_size
         # the decode kernels walk KV in 32-position tiles and require page
         # boundaries to align (attn_decode_mfma.hip: "P | 32")
         if 32 % P != 0:
@@ -91,6 +94,7 @@ class BlockStack(torch.nn.Module):
             page_size=P,
             device=self.device,
             dtype=self.config.dtype,
+            max_seqs=max_seqs or kvc.max_seqs,
         )
 
     @torch.no_grad()
@@ -135,16 +139,17 @@ class BlockStack(torch.nn.Module):
     def forward_batch(self, x: torch.Tensor, batch: TokenBatch,
                       before_block=None) -> torch.Tensor:
         """One ragged step: x (N, W) f32 through all blocks, in place. A block
-        leaves its sum Pending and the next one's norm folds it in;
-        before_block(i) needs the sum, so it forces the fold."""
-        pending = None
+        may leave something to the next one (its sum, for that one's norm to
+        fold in); before_block(i) needs the sum, so it forces the fold."""
+        left = None
         for i, blk in enumerate(self.blocks):
             if before_block is not None:
-                ragged.residual_norm(x, pending)
-                pending = None
+                if left is not None:
+                    left.settle(x)
+                left = None
                 before_block(i)
-            pending = blk.forward_tokens(x, pending, batch)
-        ragged.residual_norm(x, pending)
+            left = blk.forward_tokens(x, left, batch)
+        left.settle(x)
         return x
 
     def forward_train(self, hidden: torch.Tensor, start_pos: int = 0,
@@ -168,7 +173,8 @@ class LocalEngine:
 
     def __init__(self, config_or_name, device="cpu", seed: int = 0,
                  kv_max_tokens: int = 1 << 16, quantize_q4: bool = False,
-                 checkpoint_dir: Optional[str] = None):
+                 checkpoint_dir: Optional[str] = None,
+                 max_seqs: Optional[int] = None):
         cfg = (config_or_name if isinstance(config_or_name, ModelConfig)
                else resolve_config(config_or_name))
         # a servable weight folder loads its weights, a preset draws them
@@ -197,7 +203,7 @@ class LocalEngine:
             for blk in self.stack.blocks:
                 if hasattr(blk, "quantize_weights_q4"):
                     blk.quantize_weights_q4()
-        self.kv_pool = self.stack.make_kv(kv_max_tokens)
+        self.kv_pool = self.stack.make_kv(kv_max_tokens, max_seqs)
         self._decode_graphs: Dict[tuple, "_DecodeGraph"] = {}
 
     def _init_plain_head(self, cfg, device, seed, checkpoint_dir) -> None:
@@ -538,7 +544,7 @@ class _DecodeGraph:
             h.extend(1)
         seqs = [h.seqs[0] for h, _ in entries]
         self.slots.fill([t for _, t in entries], [s.l_spec - 1 for s in seqs],
-                        [s.pages for s in seqs])
+                        [s.pages for s in seqs], [s.slot for s in seqs])
         n = len(entries)
         if self.graph is None and self.calls < self.WARMUP:
             self.calls += 1

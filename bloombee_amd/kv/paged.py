@@ -49,6 +49,7 @@ class _SeqState:
     pages: List[int] = field(default_factory=list)
     l_acc: int = 0    # committed tokens
     l_spec: int = 0   # committed + speculative tokens (>= l_acc)
+    slot: int = -1    # row of the recurrent states, -1 = no recurrent layers
 
 
 class PagedKVCache:
@@ -67,15 +68,23 @@ class PagedKVCache:
         layout=None,
         v_head_dim=None,
         shares=None,
+        state_shapes=None,
+        max_seqs: int = 128,
     ):
         """num_kv_heads / head_dim may be ints (uniform) or per-layer lists —
         gemma-4 style heterogeneous KV geometry (sliding layers D=256, full
         layers D=512; ref server/backend.py:291-306 per-block KV descriptor
         dispatch). `layout[l]` may be "kv" (default) or "k" — k-only layers
-        (gemma-4 attention_k_eq_v full-attention layers) allocate no V plane.
+        (gemma-4 attention_k_eq_v full-attention layers, latent attention)
+        allocate no V plane, "none" layers (recurrent ones) no plane at all.
         v_head_dim: value size where it differs from head_dim (int or per-layer
         list). `shares[l]` = j makes layer l read layer j's planes (cross-layer
         KV sharing): it owns no storage, and copies skip it.
+        `state_shapes[l]` gives layer l a recurrent state of that shape (f32)
+        for each of `max_seqs` sequences. A session holds a state slot per
+        sequence for as long as it lives, host-offloaded or not: the state is
+        small and does not grow. A sequence that starts at position 0 starts
+        from a zero state, so slots are not cleared when they change hands.
         """
         self.num_layers = num_layers
         as_list = (lambda v: list(v) if isinstance(v, (list, tuple))
@@ -99,10 +108,14 @@ class PagedKVCache:
         # aliased to K for "k" layout). A page id indexes every layer's plane.
         self.pools = []
         for l in range(num_layers):
+            if self.layout[l] == "none":
+                self.pools.append(None)
+                continue
             hkv, d = self.num_kv_heads_per_layer[l], self.head_dim_per_layer[l]
             if self.shares[l] is not None:
                 j = self.shares[l]
-                if not (0 <= j < l) or self.shares[j] is not None:
+                if (not (0 <= j < l) or self.shares[j] is not None
+                        or self.layout[j] == "none"):
                     raise PagedKVError(
                         f"layer {l} cannot share the KV of layer {j}")
                 self.pools.append(self.pools[j])
@@ -115,7 +128,15 @@ class PagedKVCache:
             self.pools.append((k, v))
         # layers that own storage: every copy of KV data loops over these
         self.own_layers = [l for l in range(num_layers)
-                           if self.shares[l] is None]
+                           if self.shares[l] is None
+                           and self.layout[l] != "none"]
+        self.states = [
+            None if shape is None else torch.zeros(
+                max_seqs, *shape, device=self.device, dtype=torch.float32)
+            for shape in as_list(state_shapes)]
+        self.has_state = any(t is not None for t in self.states)
+        self.max_seqs = max_seqs
+        self._free_slots: List[int] = list(range(max_seqs - 1, -1, -1))
         self._free_pages: List[int] = list(range(self.n_pages - 1, -1, -1))
         self._reserved_tokens = 0  # admission-control reservation
         self._lock = threading.Condition()
@@ -152,7 +173,20 @@ class PagedKVCache:
         d = self.v_head_dim_per_layer[layer]
         return v.view(self.n_pages, hkv, d, self.page_size)
 
+    def state(self, layer: int) -> torch.Tensor:
+        """Recurrent states of a layer, (max_seqs, *shape) f32."""
+        return self.states[layer]
+
     # -- admission --------------------------------------------------------
+    def _take_slots(self, n: int) -> List[int]:
+        """State slots of n sequences (caller holds the lock and has checked)."""
+        if not self.has_state:
+            return [-1] * n
+        return [self._free_slots.pop() for _ in range(n)]
+
+    def _slots_short(self, n: int) -> bool:
+        return self.has_state and n > len(self._free_slots)
+
     def allocate(
         self, batch_size: int, max_length: int, timeout: Optional[float] = None,
         resident_batch: Optional[int] = None,
@@ -174,7 +208,11 @@ class PagedKVCache:
             * pages_per_seq * self.page_size
         deadline = None if timeout is None else time.monotonic() + timeout
         with self._lock:
-            while self.max_tokens - self._reserved_tokens < need:
+            if self.has_state and batch_size > self.max_seqs:
+                raise AllocationFailed(
+                    f"{batch_size} sequences > {self.max_seqs} state slots")
+            while (self.max_tokens - self._reserved_tokens < need
+                   or self._slots_short(batch_size)):
                 if need > self.max_tokens:
                     raise AllocationFailed(
                         f"requested {need} KV tokens > pool capacity {self.max_tokens}"
@@ -184,10 +222,14 @@ class PagedKVCache:
                     raise AllocationFailed(
                         f"timed out waiting for {need} KV tokens "
                         f"({self.max_tokens - self._reserved_tokens} available)"
+                        + (f" and {batch_size} state slots "
+                           f"({len(self._free_slots)} free)"
+                           if self.has_state else "")
                     )
                 self._lock.wait(timeout=remaining)
             self._reserved_tokens += need
-            handle = SessionHandle(self, self._next_handle, batch_size, max_length, need)
+            handle = SessionHandle(self, self._next_handle, batch_size, max_length,
+                                   need, slots=self._take_slots(batch_size))
             self._handles[self._next_handle] = handle
             self._next_handle += 1
             return handle
@@ -198,9 +240,12 @@ class PagedKVCache:
         For callers that know the live total themselves (the batch scheduler's
         admission, trace replay) and cannot name a length in advance."""
         with self._lock:
+            if self._slots_short(1):
+                raise AllocationFailed(
+                    f"all {self.max_seqs} state slots are in use")
             handle = SessionHandle(self, self._next_handle, 1,
                                    min(max_length, self.max_tokens), 0,
-                                   elastic=True)
+                                   elastic=True, slots=self._take_slots(1))
             self._handles[self._next_handle] = handle
             self._next_handle += 1
             return handle
@@ -213,6 +258,9 @@ class PagedKVCache:
             for seq in handle.seqs:
                 self._free_pages.extend(seq.pages)
                 seq.pages.clear()
+                if seq.slot >= 0:
+                    self._free_slots.append(seq.slot)
+                    seq.slot = -1
             self._reserved_tokens -= handle.reserved_tokens
             self._lock.notify_all()
 
@@ -241,14 +289,16 @@ class SessionHandle:
 
     def __init__(self, cache: PagedKVCache, handle_id: int, batch_size: int,
                  max_length: int, reserved_tokens: int,
-                 elastic: bool = False):
+                 elastic: bool = False, slots: Optional[List[int]] = None):
         self.cache = cache
         self.elastic = elastic
         self.handle_id = handle_id
         self.batch_size = batch_size
         self.max_length = max_length
         self.reserved_tokens = reserved_tokens
-        self.seqs = [_SeqState() for _ in range(batch_size)]
+        self.seqs = [_SeqState(slot=n) for n in slots or [-1] * batch_size]
+        self._slots = None if not cache.has_state else torch.tensor(
+            [s.slot for s in self.seqs], dtype=torch.int32).to(cache.device)
         self._max_pages = (max_length + cache.page_size - 1) // cache.page_size
         self._page_table = torch.zeros(
             batch_size, self._max_pages, device=cache.device, dtype=torch.int32
@@ -302,6 +352,9 @@ class SessionHandle:
         lock is NOT held while waiting — swap_out_rows needs it to free)."""
         if self.is_swapped:
             raise PagedKVError("extend on a swapped-out session; swap_in first")
+        if speculative and self.cache.has_state:
+            raise PagedKVError("recurrent layers cannot take back tokens: "
+                               "no speculative steps")
         P = self.cache.page_size
         if self.elastic:
             timeout = 0.0
@@ -435,7 +488,7 @@ class SessionHandle:
                                      device=cache.device)
                 per_layer = []
                 for l in range(cache.num_layers):
-                    if cache.shares[l] is not None:
+                    if l not in cache.own_layers:
                         per_layer.append((None, None))
                         continue
                     k = cache.k_pages(l)[pages]
@@ -598,6 +651,8 @@ class SessionHandle:
         if not self.is_swapped:
             return
         cache = self.cache
+        if cache.has_state:
+            raise PagedKVError("no mixed-device decode of recurrent layers")
         S = self.seqs[0].l_acc
         if any(s.l_acc != S or s.l_spec != S for s in self.seqs):
             raise PagedKVError("mixed-device restore needs lockstep, "
@@ -675,7 +730,7 @@ class SessionHandle:
             for b, npages, ids in work:
                 per_layer = []
                 for l in range(cache.num_layers):
-                    if cache.shares[l] is not None:
+                    if l not in cache.own_layers:
                         per_layer.append((None, None))
                         continue
                     k = cache.k_pages(l)[ids]
@@ -777,9 +832,13 @@ class SessionHandle:
     def truncate(self, new_lengths: List[int]) -> None:
         """Failover / history-replay support: cut sequences back to
         `new_lengths` committed tokens (ref inference_session.py:802-831)."""
-        for b, (s, n) in enumerate(zip(self.seqs, new_lengths)):
+        for s, n in zip(self.seqs, new_lengths):
             if n > s.l_acc:
                 raise PagedKVError("truncate can only shrink")
+            if self.cache.has_state and n not in (0, s.l_acc):
+                raise PagedKVError("recurrent layers cannot go back: only to "
+                                   "the start of a sequence")
+        for s, n in zip(self.seqs, new_lengths):
             s.l_acc = n
         self.rollback()
 
@@ -793,6 +852,10 @@ class SessionHandle:
 
     def page_table_host(self) -> torch.Tensor:
         return self._page_table_host
+
+    def state_slots(self) -> Optional[torch.Tensor]:
+        """(B,) int32 rows of the recurrent states, None without any."""
+        return self._slots
 
     def k_pages(self, layer: int) -> torch.Tensor:
         return self.cache.k_pages(layer)

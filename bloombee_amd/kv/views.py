@@ -26,6 +26,10 @@ class SessionView:
     def page_table(self) -> torch.Tensor:
         return self.handle.page_table()[self.b0:self.b1]
 
+    def state_slots(self):
+        slots = self.handle.state_slots()
+        return None if slots is None else slots[self.b0:self.b1]
+
     def k_pages(self, layer: int) -> torch.Tensor:
         return self.handle.k_pages(layer)
 

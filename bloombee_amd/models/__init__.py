@@ -14,3 +14,4 @@ import bloombee_amd.models.qwen3  # noqa: F401,E402
 import bloombee_amd.models.mixtral  # noqa: F401,E402
 import bloombee_amd.models.gemma4  # noqa: F401,E402
 import bloombee_amd.models.mubasun  # noqa: F401,E402
+import bloombee_amd.models.risepel  # noqa: F401,E402

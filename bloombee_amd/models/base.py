@@ -13,7 +13,7 @@ import dataclasses
 import json
 import os
 from dataclasses import dataclass, field
-from typing import Any, Dict, Optional, Type
+from typing import Any, Callable, Dict, Optional, Type
 
 import torch
 
@@ -79,6 +79,10 @@ class ModelConfig:
         cfg.extras.update(extras)
         return cfg
 
+    def adopt_shapes(self, shape_of: Callable[[str], tuple]) -> None:
+        """Sizes that only the checkpoint's tensors give. shape_of(name) is a
+        tensor's shape as its file's header states it."""
+
     def to_dict(self) -> dict:
         d = dataclasses.asdict(self)
         d.update(d.pop("extras"))
@@ -88,6 +92,21 @@ class ModelConfig:
     def from_json(cls, path: str) -> "ModelConfig":
         with open(path) as f:
             return cls.from_dict(json.load(f))
+
+
+def kv_shares(source: Callable[[int], Optional[int]], start: int,
+              end: int) -> list:
+    """`shares` of the cache of layers [start, end): source(i) is the layer
+    whose keys layer i reads, None = its own. Both must be in the range."""
+    out = []
+    for i in range(start, end):
+        j = source(i)
+        if j is not None and j < start:
+            raise RuntimeError(
+                f"layer {i} reads the KV of layer {j}: both must be in "
+                f"one server block range (got [{start}, {end}))")
+        out.append(None if j is None else j - start)
+    return out
 
 
 @dataclass
@@ -145,7 +164,12 @@ def resolve_config(name_or_path: str) -> ModelConfig:
         with open(cfg_path) as f:
             d = json.load(f)
         family = get_family(model_type_of(d))
-        return family.config_cls.from_dict(d)
+        cfg = family.config_cls.from_dict(d)
+        if hasattr(family.block_cls, "load_tensors") and os.path.isfile(
+                os.path.join(name_or_path, "model.safetensors")):
+            from bloombee_amd.server.from_pretrained import NativeCheckpoint
+            cfg.adopt_shapes(NativeCheckpoint(name_or_path).shape)
+        return cfg
     key = name_or_path.lower()
     if key in _PRESETS:
         model_type, d = _PRESETS[key]

@@ -29,6 +29,7 @@ from bloombee_amd.ops.ragged import Pending, ProjSpec, pad_k, round_up
 
 class MubasunBlock(torch.nn.Module):
     token_batched = True   # BlockStack hands whole steps to forward_tokens
+    hip_modules = ("_hip_ragged",)
 
     def __init__(self, config: MubasunConfig, layer_index: int = 0, rope=None):
         super().__init__()

@@ -14,7 +14,7 @@ from typing import Optional
 
 import torch
 
-from bloombee_amd.models.base import ModelConfig
+from bloombee_amd.models.base import ModelConfig, kv_shares
 from bloombee_amd.ops.ragged import pad_head
 
 
@@ -126,6 +126,10 @@ class MubasunConfig(ModelConfig):
         return self.extras["layers"]
 
     @property
+    def learned_positions(self) -> bool:
+        return True
+
+    @property
     def norm_groups(self) -> int:
         return int(self.extras["norm"]["groups"])
 
@@ -141,16 +145,8 @@ class MubasunConfig(ModelConfig):
     def kv_layout(self, start: int, end: int) -> dict:
         """PagedKVCache geometry of layers [start, end)."""
         mixers = [self.layers[i]["mixer"] for i in range(start, end)]
-        shares = []
-        for i in range(start, end):
-            j = self.kv_source(i)
-            if j is not None and j < start:
-                raise RuntimeError(
-                    f"layer {i} reads the KV of layer {j}: both must be in "
-                    f"one server block range (got [{start}, {end}))")
-            shares.append(None if j is None else j - start)
         return dict(
             num_kv_heads=[m["kv_heads"] for m in mixers],
             head_dim=[pad_head(m["dim"]) for m in mixers],
             v_head_dim=[pad_head(m["vdim"]) for m in mixers],
-            shares=shares)
+            shares=kv_shares(self.kv_source, start, end))

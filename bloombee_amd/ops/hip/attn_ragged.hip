@@ -1,8 +1,9 @@
 // Paged attention over ragged batches: rows of many sequences, each with its
 // own position, with a sliding window, a linear distance bias
 // (score - slope_h * (i - j)), separate key and value sizes, grouped key/value
-// heads and a sigmoid output gate in the epilogue. Every one of these is a
-// parameter; window 0, null slopes and a null gate switch them off.
+// heads, a sink (one more score per head, unscaled and without a value) and a
+// sigmoid output gate in the epilogue. Every one of these is a parameter;
+// window 0, null slopes, null sinks and a null gate switch them off.
 //
 // Two MFMA kernels and one plain kernel:
 //  * attn_ragged_prefill_kernel: sequences that bring two tokens or more. The
@@ -12,7 +13,8 @@
 //    heads of the group; only the visible range [i - window + 1, i] is walked
 //    and split over waves and workgroups.
 //  * attn_ragged_simple_kernel: one wave per (row, head), f32 arithmetic on
-//    any element type and any head size.
+//    any element type and any head size. Without value pages the values are
+//    the first vdim elements of the keys.
 //
 // Both MFMA kernels compute S^T = K Q^T and O^T = V^T P^T. The rows of a
 // 32-key tile are handed to the two score MFMAs in the order
@@ -31,7 +33,7 @@
 struct AttnArgs {
   const void* q;        // (N, H, dkp)
   const void* kp;       // (np, G, P, dkp)
-  const void* vp;       // (np, G, dvp, P)
+  const void* vp;       // (np, G, dvp, P) or null: values are key prefixes
   const int* table;     // (S, maxp)
   const int* tok_seq;   // (N,)
   const int* tok_pos;   // (N,) -1 = empty slot
@@ -39,6 +41,7 @@ struct AttnArgs {
   const int* q_start;   // (S,)
   const int* list;      // sequences of this launch
   const float* slopes;  // (H,) or null
+  const float* sinks;   // (H,) or null
   const void* gate;     // row stride ldg, (H*vdim) columns; or null
   void* out;            // row stride ldo, (H*vdim) columns
   float* pml;           // decode splits: (units, 16, 2) max and sum
@@ -50,6 +53,15 @@ struct AttnArgs {
 
 DEVINL int first_key(int pos, int window) {
   return window > 0 ? max(0, pos - window + 1) : 0;
+}
+
+// Takes a sink (log2 units) into a row's softmax: returns the factor of its
+// accumulated values.
+DEVINL float add_sink(float sink2, float m2, float& l) {
+  const float mn = fmaxf(m2, sink2);
+  const float c = fast_exp2(m2 - mn);
+  l = l * c + fast_exp2(sink2 - mn);
+  return c;
 }
 
 // Four consecutive output columns of one row, gated.
@@ -306,7 +318,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefil
 #pragma unroll
   for (int c = 0; c < QC; ++c) {
     if (base + (wave * QC + c) * 16 + li >= R) continue;
-    const float inv = l[c] > 0.f ? 1.f / l[c] : 0.f;
+    const float sc = a.sinks ? add_sink(a.sinks[head[c]] * LOG2E, m2[c], l[c]) : 1.f;
+    const float inv = l[c] > 0.f ? sc / l[c] : 0.f;
 #pragma unroll
     for (int n = 0; n < ND; ++n) {
       float o[4];
@@ -502,7 +515,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_decode
           acc[n];
     return;
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float sc = a.sinks ? add_sink(a.sinks[h] * LOG2E, m2, l) : 1.f;
+  const float inv = l > 0.f ? sc / l : 0.f;
 #pragma unroll
   for (int n = 0; n < ND; ++n) {
     float o[4];
@@ -530,7 +544,9 @@ __global__ __launch_bounds__(256) void attn_ragged_combine_kernel(AttnArgs a) {
   for (int i = 0; i < a.n_split; ++i)
     l += a.pml[((u0 + i) * 16 + col) * 2 + 1] *
          fast_exp2(a.pml[((u0 + i) * 16 + col) * 2] - m);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float sc =
+      a.sinks ? add_sink(a.sinks[g * Hg + h0 + col] * LOG2E, m, l) : 1.f;
+  const float inv = l > 0.f ? sc / l : 0.f;
   for (int d = (threadIdx.x % 16) * 4; d < a.vdim; d += 64) {
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     for (int i = 0; i < a.n_split; ++i) {
@@ -550,7 +566,7 @@ __global__ __launch_bounds__(256) void attn_ragged_combine_kernel(AttnArgs a) {
 // plain: grid (N, H), one wave
 // ---------------------------------------------------------------------------
 
-static constexpr int SIMPLE_MAXD = 512;
+static constexpr int SIMPLE_MAXD = 1024;
 
 template <typename T>
 __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
@@ -562,7 +578,8 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
   const int pos = a.tok_pos[row];
   const int* table = a.table + (long)a.tok_seq[row] * a.maxp;
   const T* kpool = (const T*)a.kp;
-  const T* vpool = (const T*)a.vp;
+  const T* vpool = a.vp ? (const T*)a.vp : kpool;
+  const long vstep = a.vp ? a.P : 1;  // between a value's elements
   for (int d = lane; d < a.dim; d += 64)
     q_lds[d] = ldf((const T*)a.q + ((long)row * a.H + h) * a.dkp + d);
   __syncthreads();
@@ -580,7 +597,8 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
       float dot = 0.f;
       for (int d = 0; d < a.dim; ++d) dot += q_lds[d] * ldf(kr + d);
       sc = dot * a.scale - slope * (float)(pos - key);
-      v_lds[lane] = pg * a.dvp * a.P + key % a.P;
+      v_lds[lane] = a.vp ? pg * a.dvp * a.P + key % a.P
+                         : (pg * a.P + key % a.P) * a.dkp;
     }
     const float mn = fmaxf(m, wave_reduce_max(sc));
     const float corr = expf(m - mn);
@@ -595,12 +613,18 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
       const int d = lane + i * 64;
       if (d >= a.vdim) break;
       float s = 0.f;
-      for (int j = 0; j < n; ++j) s += p_lds[j] * ldf(vpool + v_lds[j] + (long)d * a.P);
+      for (int j = 0; j < n; ++j) s += p_lds[j] * ldf(vpool + v_lds[j] + d * vstep);
       acc[i] = acc[i] * corr + s;
     }
     __syncthreads();
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float sc = 1.f;
+  if (a.sinks) {
+    const float mn = fmaxf(m, a.sinks[h]);
+    sc = expf(m - mn);
+    l = l * sc + expf(a.sinks[h] - mn);
+  }
+  const float inv = l > 0.f ? sc / l : 0.f;
 #pragma unroll
   for (int i = 0; i < SIMPLE_MAXD / 64; ++i) {
     const int d = lane + i * 64;

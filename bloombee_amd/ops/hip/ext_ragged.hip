@@ -5,74 +5,23 @@
 //
 // Host side: shape checks, template dispatch, launch shapes.
 
-#include <torch/extension.h>
-#include <c10/hip/HIPStream.h>
-#include <hip/hip_runtime.h>
-
+#include "host.h"
 #include "common.h"
 #include "rows.hip"
 #include "attn_ragged.hip"
 #include "moe_routed.hip"
 #include "gemm_skinny.hip"
 
-using torch::Tensor;
-using OptTensor = c10::optional<Tensor>;
-typedef unsigned short bf16_bits;
-
-static hipStream_t cur_stream() {
-  return c10::hip::getCurrentHIPStream().stream();
-}
-
-#define CHECK_T(x, st)                                                        \
-  TORCH_CHECK((x).is_cuda() && (x).is_contiguous() &&                         \
-                  (x).scalar_type() == (st),                                  \
-              #x " must be a contiguous device tensor of ", toString(st))
-#define CHECK_I32(x) CHECK_T(x, at::kInt)
-#define CHECK_F32(x) CHECK_T(x, at::kFloat)
-
-static void check_launch() {
-  const hipError_t e = hipGetLastError();
-  TORCH_CHECK(e == hipSuccess, "kernel launch: ", hipGetErrorString(e));
-}
-
-static void check_act(const Tensor& t) {
-  TORCH_CHECK(t.is_cuda() && (t.scalar_type() == at::kBFloat16 ||
-                              t.scalar_type() == at::kFloat),
-              "activations must be bf16 or f32 on the device");
-}
-
-// f(element tag) with unsigned short for bf16, float for f32.
-template <typename F>
-static void by_type(at::ScalarType st, F f) {
-  if (st == at::kBFloat16) f((bf16_bits)0);
-  else f(0.f);
-}
-
-template <typename F>
-static void by_bool(bool b, F f) {
-  if (b) f(std::true_type{});
-  else f(std::false_type{});
-}
-
-template <typename K>
-static void allow_lds(K kernel, size_t bytes) {
-  TORCH_CHECK(bytes <= 160 * 1024, "row too long for LDS: ", bytes, " bytes");
-  if (bytes > 64 * 1024)
-    TORCH_CHECK(hipFuncSetAttribute(
-                    reinterpret_cast<const void*>(kernel),
-                    hipFuncAttributeMaxDynamicSharedMemorySize,
-                    (int)bytes) == hipSuccess,
-                "cannot reserve ", bytes, " bytes of LDS");
-}
-
-Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, Tensor pos_table) {
+Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table) {
   CHECK_I32(ids);
   CHECK_I32(pos);
   check_act(table);
-  CHECK_T(pos_table, table.scalar_type());
   TORCH_CHECK(table.is_contiguous() && table.dim() == 2 &&
-              pos_table.dim() == 2 && table.size(1) == pos_table.size(1) &&
               ids.numel() == pos.numel());
+  if (pos_table.has_value()) {
+    CHECK_T((*pos_table), table.scalar_type());
+    TORCH_CHECK(pos_table->dim() == 2 && table.size(1) == pos_table->size(1));
+  }
   const long N = ids.numel();
   auto x = torch::empty({N, table.size(1)}, table.options().dtype(at::kFloat));
   if (N == 0) return x;
@@ -80,8 +29,9 @@ Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, Tensor pos_table) {
     using T = decltype(t);
     embed_rows_kernel<T><<<N, 256, 0, cur_stream()>>>(
         ids.data_ptr<int>(), pos.data_ptr<int>(), (const T*)table.data_ptr(),
-        (const T*)pos_table.data_ptr(), x.data_ptr<float>(),
-        (int)table.size(1), (int)table.size(0), (int)pos_table.size(0));
+        pos_table.has_value() ? (const T*)pos_table->data_ptr() : nullptr,
+        x.data_ptr<float>(), (int)table.size(1), (int)table.size(0),
+        pos_table.has_value() ? (int)pos_table->size(0) : 0);
   });
   check_launch();
   return x;
@@ -93,7 +43,8 @@ Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, Tensor pos_table) {
 
 void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
                    OptTensor idw, OptTensor hprev, OptTensor nw, long groups,
-                   double eps, OptTensor h) {
+                   double eps, OptTensor h, double alpha, OptTensor bias,
+                   bool post) {
   CHECK_F32(x);
   TORCH_CHECK(x.dim() == 2);
   const long N = x.size(0);
@@ -103,6 +54,14 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
   a.W = W;
   a.eps = (float)eps;
   a.groups = (int)groups;
+  a.alpha = (float)alpha;
+  a.post = post;
+  TORCH_CHECK(!post || nw.has_value(), "a norm after the sum needs its weight");
+  if (bias.has_value()) {
+    CHECK_F32((*bias));
+    TORCH_CHECK(parts.has_value() && bias->numel() == W);
+    a.bias = bias->data_ptr<float>();
+  }
   bool vec = W % 4 == 0;
   at::ScalarType tp = at::kFloat, ta = at::kFloat;
   if (parts.has_value()) {
@@ -175,6 +134,62 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
       });
     });
   });
+  check_launch();
+}
+
+// [gate | up] GEMM output -> clamped gated product, (N, ldo).
+void clamped_glu(Tensor parts, long g_off, long u_off, long ff, OptTensor gb,
+                 OptTensor ub, double limit, double slope, Tensor out) {
+  check_act(parts);
+  check_act(out);
+  TORCH_CHECK(parts.dim() == 3 && parts.is_contiguous() && out.dim() == 2 &&
+              out.is_contiguous() && out.size(0) == parts.size(1) &&
+              out.size(1) >= ff && ff >= 1);
+  GluArgs a{};
+  const long N = parts.size(1);
+  a.parts = parts.data_ptr();
+  a.ks = parts.size(0);
+  a.ldp = parts.size(2);
+  a.pstride = N * (long)a.ldp;
+  a.g_off = (int)g_off;
+  a.u_off = (int)u_off;
+  a.ff = (int)ff;
+  a.out = out.data_ptr();
+  a.ldo = out.size(1);
+  a.limit = (float)limit;
+  a.slope = (float)slope;
+  TORCH_CHECK(g_off >= 0 && u_off >= 0 && g_off + ff <= a.ldp &&
+              u_off + ff <= a.ldp);
+  for (const OptTensor* b : {&gb, &ub})
+    if (b->has_value()) {
+      CHECK_F32((**b));
+      TORCH_CHECK((*b)->numel() == ff);
+    }
+  if (gb.has_value()) a.gb = gb->data_ptr<float>();
+  if (ub.has_value()) a.ub = ub->data_ptr<float>();
+  if (N == 0) return;
+  bool vec = true;
+  for (int v : {a.ldp, a.g_off, a.u_off, a.ff, a.ldo}) vec = vec && v % 8 == 0;
+  by_type(parts.scalar_type(), [&](auto p) {
+    by_type(out.scalar_type(), [&](auto t) {
+      by_bool(vec, [&](auto v) {
+        constexpr int V = decltype(v)::value ? 8 : 1;
+        clamped_glu_kernel<decltype(p), decltype(t), V>
+            <<<dim3(N, (a.ldo + 256 * V - 1) / (256 * V)), 256, 0,
+               cur_stream()>>>(a);
+      });
+    });
+  });
+  check_launch();
+}
+
+void softcap(Tensor z, double cap) {
+  CHECK_F32(z);
+  TORCH_CHECK(cap > 0);
+  const long n = z.numel();
+  if (n == 0) return;
+  softcap_kernel<<<std::min<long>((n + 255) / 256, 2048), 256, 0,
+                   cur_stream()>>>(z.data_ptr<float>(), n, (float)cap);
   check_launch();
 }
 
@@ -413,11 +428,11 @@ static void launch_mfma(AttnArgs& a, const Tensor& pre, const Tensor& dec,
   }
 }
 
-void attn_ragged(Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
-                 Tensor tok_pos, Tensor cu, Tensor q_start, Tensor pre,
-                 Tensor dec, long max_new, long max_ctx, long dim, long vdim,
-                 double scale, long window, OptTensor slopes, OptTensor gate,
-                 Tensor out) {
+void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
+                 Tensor tok_seq, Tensor tok_pos, Tensor cu, Tensor q_start,
+                 Tensor pre, Tensor dec, long max_new, long max_ctx, long dim,
+                 long vdim, double scale, long window, OptTensor slopes,
+                 OptTensor sinks, OptTensor gate, Tensor out) {
   check_act(q);
   const auto ta = q.scalar_type();
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
@@ -425,16 +440,21 @@ void attn_ragged(Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
   const long N = q.size(0);
   a.H = q.size(1);
   a.dkp = q.size(2);
-  TORCH_CHECK(kp.dim() == 4 && vp.dim() == 4);
+  TORCH_CHECK(kp.dim() == 4);
   a.G = kp.size(1);
   a.P = kp.size(2);
-  a.dvp = vp.size(2);
+  a.dvp = a.dkp;
   a.dim = (int)dim;
   a.vdim = (int)vdim;
-  TORCH_CHECK(a.H % a.G == 0 && kp.size(3) == a.dkp && vp.size(1) == a.G &&
-              vp.size(3) == a.P && vp.size(0) == kp.size(0) && dim >= 1 &&
-              vdim >= 1 && dim <= a.dkp && vdim <= a.dvp);
-  for (const Tensor& t : {kp, vp})
+  if (vp.has_value()) {
+    TORCH_CHECK(vp->dim() == 4 && vp->size(1) == a.G && vp->size(3) == a.P &&
+                vp->size(0) == kp.size(0));
+    a.dvp = vp->size(2);
+    a.vp = vp->data_ptr();
+  }
+  TORCH_CHECK(a.H % a.G == 0 && kp.size(3) == a.dkp && dim >= 1 && vdim >= 1 &&
+              dim <= a.dkp && vdim <= a.dvp);
+  for (const Tensor& t : {kp, vp.value_or(kp)})
     TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == ta,
                 "pages must have the element type of q");
   for (const Tensor& t : {table, tok_seq, tok_pos, cu, q_start, pre, dec})
@@ -450,6 +470,11 @@ void attn_ragged(Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
     TORCH_CHECK(slopes->numel() == a.H);
     a.slopes = slopes->data_ptr<float>();
   }
+  if (sinks.has_value()) {
+    CHECK_F32((*sinks));
+    TORCH_CHECK(sinks->numel() == a.H);
+    a.sinks = sinks->data_ptr<float>();
+  }
   if (gate.has_value()) {
     TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->size(0) == N &&
                 gate->stride(1) == 1 && gate->scalar_type() == ta &&
@@ -460,7 +485,6 @@ void attn_ragged(Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
   if (N == 0) return;
   a.q = q.data_ptr();
   a.kp = kp.data_ptr();
-  a.vp = vp.data_ptr();
   a.table = table.data_ptr<int>();
   a.maxp = table.size(1);
   a.tok_seq = tok_seq.data_ptr<int>();
@@ -474,15 +498,19 @@ void attn_ragged(Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
   a.n_split = 1;
 
   auto size_ok = [](int d) { return d == 32 || d == 64 || d == 128 || d == 256; };
-  if (ta == at::kBFloat16 && size_ok(a.dkp) && size_ok(a.dvp) && a.P % 8 == 0 &&
-      32 % a.P == 0) {
+  if (ta == at::kBFloat16 && a.vp && (size_ok(a.dkp) || a.dkp == 192) &&
+      size_ok(a.dvp) && a.P % 8 == 0 && 32 % a.P == 0) {
     auto by_dim = [](int d, auto f) {
       if (d == 32) f(std::integral_constant<int, 32>{});
       else if (d == 64) f(std::integral_constant<int, 64>{});
       else if (d == 128) f(std::integral_constant<int, 128>{});
       else f(std::integral_constant<int, 256>{});
     };
-    by_dim(a.dkp, [&](auto dk) {
+    auto by_key = [&](int d, auto f) {
+      if (d == 192) f(std::integral_constant<int, 192>{});
+      else by_dim(d, f);
+    };
+    by_key(a.dkp, [&](auto dk) {
       by_dim(a.dvp, [&](auto dv) {
         launch_mfma<decltype(dk)::value, decltype(dv)::value>(
             a, pre, dec, max_new, max_ctx, q);
@@ -594,6 +622,8 @@ Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_rows", &embed_rows);
   m.def("residual_norm", &residual_norm);
+  m.def("clamped_glu", &clamped_glu);
+  m.def("softcap", &softcap);
   m.def("proj_post", &proj_post);
   m.def("router_gemm", &router_gemm);
   m.def("gemm_parts", &gemm_parts);

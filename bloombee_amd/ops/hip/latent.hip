@@ -1,0 +1,552 @@
+// Latent attention over ragged batches: what a token leaves in the cache is one
+// normed latent c and one rotated key part shared by all heads, [c | r] in one
+// key page plane. Per-head keys and values are linear in c.
+//
+//  latent_post_kernel    norms the query latent, norms c, rotates r, writes
+//                        the page slot.
+//  latent_rope_kernel    queries of prompt rows: [unrotated | rotated].
+//  latent_scatter_kernel keys and values of a context, made from its latents by
+//                        one GEMM, into pages of the prompt attention kernel.
+//  latent_absorb_kernel  queries of decoded rows, taken into the latent space:
+//                        q_lat = W_uk^T q, beside the rotated part. One head's
+//                        query then meets [c | r] itself.
+//  attn_latent_decode_kernel  decoded rows: every key tile is read once, for the
+//                        scores by rows and for the values by columns
+//                        (transposing LDS reads).
+//  latent_output_kernel  folds the splits and the sink, applies W_uv and the
+//                        sigmoid output gate.
+//
+// Rotary pairs are (i, i + dims/2). Angles are reduced in double, in turns.
+
+#pragma once
+#include "common.h"
+#include "rows.hip"
+
+// A GEMM output that may lie in split-K partials.
+struct Parts {
+  const void* p;  // (ks, N, ld)
+  long stride;    // elements between splits
+  int ks, ld;
+};
+
+template <typename TP, int V>
+DEVINL void fold_parts(const Parts& a, long t, int c, float* o) {
+  const TP* row = (const TP*)a.p + t * (long)a.ld + c;
+  ldv<V>(row, o);
+  for (int s = 1; s < a.ks; ++s) {
+    float u[V];
+    ldv<V>(row + s * a.stride, u);
+#pragma unroll
+    for (int j = 0; j < V; ++j) o[j] += u[j];
+  }
+}
+
+// turns: frequency / 2 pi
+DEVINL void rotation(int pos, double turns, float& c, float& s) {
+  double r = (double)pos * turns;
+  r -= rint(r);
+  sincospif(2.f * (float)r, &s, &c);
+}
+
+struct LatentPostArgs {
+  Parts y;              // [query latent | c | r | gate] columns
+  const float* qn;      // (q_rank,)
+  const float* cn;      // (rank,)
+  const double* turns;  // (rdims / 2,)
+  void* cq;             // (N, ldq), zero beyond q_rank
+  void* gate;           // (N, gn) or null
+  void* kp;             // (np, 1, P, ck)
+  const int* table;
+  const int* tok_seq;
+  const int* tok_pos;
+  int q_off, c_off, g_off, q_rank, rank, rot, rdims, rp, ck, ldq, gn, P, maxp;
+  int has_kv;
+  float eps;
+};
+
+// Section of n columns into LDS; returns 1 / rms.
+template <typename TP, int V>
+DEVINL float stage_norm(const Parts& y, long t, int off, int n, float eps,
+                        float* lds, float* red) {
+  float ss = 0.f;
+  for (int i = threadIdx.x * V; i < n; i += 256 * V) {
+    float v[V];
+    fold_parts<TP, V>(y, t, off + i, v);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      lds[i + j] = v[j];
+      ss += v[j] * v[j];
+    }
+  }
+  ss = wave_reduce_sum(ss);
+  if ((threadIdx.x & (WAVE - 1)) == 0) red[threadIdx.x / WAVE] = ss;
+  __syncthreads();
+  return 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)n + eps);
+}
+
+// grid (N, 2 + gate chunks of 2048): y = 0 query latent, 1 page slot, 2.. gate
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
+  extern __shared__ float lds_sec[];
+  __shared__ float red[4];
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x;
+  if (blockIdx.y == 0) {
+    const float inv = stage_norm<TP, V>(a.y, t, a.q_off, a.q_rank, a.eps,
+                                        lds_sec, red);
+    T* o = (T*)a.cq + t * (long)a.ldq;
+    for (int i = tid; i < a.ldq; i += 256)
+      stf(o + i, i < a.q_rank ? lds_sec[i] * inv * a.qn[i] : 0.f);
+    return;
+  }
+  if (blockIdx.y == 1) {
+    const int pos = a.tok_pos[t];
+    if (!a.has_kv || pos < 0) return;
+    const float inv = stage_norm<TP, V>(a.y, t, a.c_off, a.rank, a.eps,
+                                        lds_sec, red);
+    const long page = a.table[(long)a.tok_seq[t] * a.maxp + pos / a.P];
+    T* o = (T*)a.kp + (page * a.P + pos % a.P) * a.ck;
+    for (int i = tid; i < a.rp; i += 256)
+      stf(o + i, i < a.rank ? lds_sec[i] * inv * a.cn[i] : 0.f);
+    const int half = a.rdims / 2;
+    for (int i = tid; i < a.ck - a.rp; i += 256) {
+      float v[1] = {0.f};
+      if (i < a.rot) fold_parts<TP, 1>(a.y, t, a.c_off + a.rank + i, v);
+      if (i < a.rdims) {
+        const int k = i % half;
+        float w[1], c, s;
+        fold_parts<TP, 1>(a.y, t, a.c_off + a.rank + (i < half ? i + half : k), w);
+        rotation(pos, a.turns[k], c, s);
+        v[0] = i < half ? v[0] * c - w[0] * s : v[0] * c + w[0] * s;
+      }
+      stf(o + a.rp + i, v[0]);
+    }
+    return;
+  }
+  const int base = (blockIdx.y - 2) * 2048;
+  const int end = min(base + 2048, a.gn);
+  for (int i = base + tid * V; i < end; i += 256 * V) {
+    float v[V];
+    fold_parts<TP, V>(a.y, t, a.g_off + i, v);
+    stv<V>((T*)a.gate + t * (long)a.gn + i, v);
+  }
+}
+
+struct LatentQueryArgs {
+  Parts y;              // (N, H * (dim + rot))
+  const double* turns;
+  const int* tok_pos;
+  const int* cu;        // decoded rows: row = cu[list[i]]
+  const int* list;
+  const void* wk;       // (H, rp, dimp): W_uk^T, zero padded
+  void* q;              // rope: (N, H, ldq); absorb: (n_list, H, ck)
+  int n_list, H, dim, rot, rdims, rp, ck, dimp, ldq;
+};
+
+// Element e of a head's rotated part for one row.
+template <typename TP>
+DEVINL float rotated(const LatentQueryArgs& a, long t, int pos, int col, int e) {
+  float v[1];
+  fold_parts<TP, 1>(a.y, t, col + e, v);
+  if (e >= a.rdims) return v[0];
+  const int half = a.rdims / 2, k = e % half;
+  float w[1], c, s;
+  fold_parts<TP, 1>(a.y, t, col + (e < half ? e + half : k), w);
+  rotation(pos, a.turns[k], c, s);
+  return e < half ? v[0] * c - w[0] * s : v[0] * c + w[0] * s;
+}
+
+// grid N: a row's queries, [dim unrotated | rot rotated | zeros] per head
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(256) void latent_rope_kernel(LatentQueryArgs a) {
+  extern __shared__ float lds_cs[];  // cos, sin of every pair
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, half = a.rdims / 2;
+  const int pos = max(a.tok_pos[t], 0);
+  for (int k = tid; k < half; k += 256)
+    rotation(pos, a.turns[k], lds_cs[k], lds_cs[half + k]);
+  __syncthreads();
+  T* q = (T*)a.q + t * (long)a.H * a.ldq;
+  const int per = a.ldq / V;
+  for (int idx = tid; idx < a.H * per; idx += 256) {
+    const int h = idx / per, d = (idx % per) * V;
+    const int col = h * (a.dim + a.rot);
+    float v[V];
+    if (d + V <= a.dim) {
+      fold_parts<TP, V>(a.y, t, col + d, v);
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const int e = d + j - a.dim;  // may straddle the border
+        v[j] = 0.f;
+        if (e >= a.rot) continue;
+        float x[1], w[1];
+        fold_parts<TP, 1>(a.y, t, col + d + j, x);
+        v[j] = x[0];
+        if (e < 0 || e >= a.rdims) continue;
+        const int k = e % half;
+        fold_parts<TP, 1>(a.y, t, col + a.dim + (e < half ? e + half : k), w);
+        const float c = lds_cs[k], s = lds_cs[half + k];
+        v[j] = e < half ? x[0] * c - w[0] * s : x[0] * c + w[0] * s;
+      }
+    }
+    stv<V>(q + (long)h * a.ldq + d, v);
+  }
+}
+
+// grid (rp / 64 + 1, H, rows / 32): 32 listed rows of one head times W_uk^T;
+// the last x block writes the rotated part and the zero columns.
+template <typename TP>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(LatentQueryArgs a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned short lds_q[];
+  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 32;
+  const int M = min(32, a.n_list - m0);
+  const int col = h * (a.dim + a.rot);
+  unsigned short* out = (unsigned short*)a.q;
+  if (blockIdx.x == gridDim.x - 1) {
+    const int n = a.ck - a.rp;
+    for (int idx = tid; idx < M * n; idx += 256) {
+      const int m = idx / n, e = idx % n;
+      const long row = a.cu[a.list[m0 + m]];
+      float v = 0.f;
+      if (e < a.rot)
+        v = rotated<TP>(a, row, max(a.tok_pos[row], 0), col + a.dim, e);
+      out[((long)(m0 + m) * a.H + h) * a.ck + a.rp + e] = cvt_bf(v);
+    }
+    return;
+  }
+  const int ldr = a.dimp + 8;
+  for (int idx = tid; idx < 32 * a.dimp; idx += 256) {
+    const int m = idx / a.dimp, d = idx % a.dimp;
+    float v[1] = {0.f};
+    if (m < M && d < a.dim)
+      fold_parts<TP, 1>(a.y, a.cu[a.list[m0 + m]], col + d, v);
+    lds_q[m * ldr + d] = cvt_bf(v[0]);
+  }
+  __syncthreads();
+  const int wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int li = lane & 15, hi = lane >> 4;
+  const int n0 = blockIdx.x * 64 + wave * 16;
+  if (n0 >= a.rp) return;
+  const unsigned short* w = (const unsigned short*)a.wk +
+                            ((long)h * a.rp + n0 + li) * a.dimp + hi * 8;
+  f32x4 acc[2];
+  acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < a.dimp; k += 32) {
+    const bf16x8 wf = as_bf16x8(*reinterpret_cast<const short8*>(w + k));
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const bf16x8 qf = as_bf16x8(*reinterpret_cast<const short8*>(
+          lds_q + (m * 16 + li) * ldr + k + hi * 8));
+      acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf, wf, acc[m], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < 2; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = m * 16 + hi * 4 + r;
+      if (row < M)
+        out[((long)(m0 + row) * a.H + h) * a.ck + n0 + li] = cvt_bf(acc[m][r]);
+    }
+}
+
+struct LatentScatterArgs {
+  const unsigned short* y;    // (npg * P, ldy): [H x dim keys | H x vdim values]
+  const unsigned short* ctx;  // (npg, P, ck) page copies, for the rotated part
+  const int* valid;           // (npg,) tokens in use of every page
+  unsigned short* k;          // (npg, H, P, dkp)
+  unsigned short* v;          // (npg, H, dvp, P)
+  int ldy, H, dim, rot, vdim, rp, ck, dkp, dvp, P;
+};
+
+// grid (npg, H)
+template <int V>
+__global__ __launch_bounds__(256) void latent_scatter_kernel(LatentScatterArgs a) {
+  const long pg = blockIdx.x;
+  const int h = blockIdx.y, tid = threadIdx.x;
+  const int n = a.valid[pg];
+  const unsigned short* y = a.y + pg * a.P * a.ldy;
+  unsigned short* k = a.k + (pg * a.H + h) * (long)a.P * a.dkp;
+  const int per = a.dkp / V;
+  for (int idx = tid; idx < a.P * per; idx += 256) {
+    const int r = idx / per, d = (idx % per) * V;
+    float v[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    if (d + V <= a.dim) {
+      ldv<V>(y + (long)r * a.ldy + h * a.dim + d, v);
+    } else {
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const int e = d + j - a.dim;
+        if (e < 0) v[j] = bf2f(y[(long)r * a.ldy + h * a.dim + d + j]);
+        else if (e < a.rot) v[j] = bf2f(a.ctx[(pg * a.P + r) * a.ck + a.rp + e]);
+      }
+    }
+    stv<V>(k + (long)r * a.dkp + d, v);
+  }
+  unsigned short* vo = a.v + (pg * a.H + h) * (long)a.dvp * a.P;
+  const unsigned short* vy = y + a.H * a.dim + h * a.vdim;
+  for (int idx = tid; idx < a.dvp * (a.P / 8); idx += 256) {
+    const int d = idx % a.dvp, r0 = idx / a.dvp * 8;
+    short8 o = short8{};
+    if (d < a.vdim)
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (r0 + j < n) o[j] = (short)vy[(long)(r0 + j) * a.ldy + d];
+    *reinterpret_cast<short8*>(vo + (long)d * a.P + r0) = o;
+  }
+}
+
+struct LatentDecodeArgs {
+  const unsigned short* q;   // (n_list, H, ck)
+  const unsigned short* kp;  // (np, 1, P, ck)
+  const int* table;
+  const int* tok_pos;
+  const int* cu;
+  const int* list;
+  float* pml;   // (units, n_split, 16, 2): max (log2 units) and sum
+  float* pacc;  // (units, n_split, 16, rp)
+  int H, P, maxp, window, n_split;
+  float scale;
+};
+
+typedef __attribute__((address_space(3))) short4v lds_short4;
+
+// 4 rows of 16-bit elements by columns: lane i of 16 gets column i of the rows
+// whose pieces of four the lanes point at (lane j*4 + c: row j, columns c*4..).
+DEVINL short4v read_columns(const unsigned short* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)p);
+}
+
+// Fragment of 8 rows x 16 columns, rows r0.. of a tile with row stride ld:
+// lane (li, hi) gets column perm-of-li, rows r0 + hi*8 .. +7. col points this
+// lane's group of four columns at its place in the row.
+DEVINL bf16x8 column_frag(const unsigned short* tile, int ld, int r0, int col,
+                          int li, int hi) {
+  const unsigned short* p = tile + (r0 + hi * 8 + li / 4) * ld + col;
+  const short4v a = read_columns(p), b = read_columns(p + 4 * ld);
+  short8 v;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    v[j] = a[j];
+    v[j + 4] = b[j];
+  }
+  return as_bf16x8(v);
+}
+
+// grid (n_list * chunks of 16 heads, n_split). ck = ND * 64 + NR * 32; a wave
+// owns every fourth 16-column tile of the values.
+template <int ND, int NR>
+__global__ __launch_bounds__(256) void attn_latent_decode_kernel(LatentDecodeArgs a) {
+  constexpr int KT = 64, RP = ND * 64, CK = RP + NR * 32, NKK = CK / 32;
+  constexpr int LDK = CK + 8, LDS_S = KT + 4;
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds_dec[];
+  unsigned short* kt = (unsigned short*)lds_dec;
+  float* sc = (float*)(lds_dec + KT * LDK * 2);
+
+  const int nch = (a.H + 15) / 16;
+  const int unit = blockIdx.x, i = unit / nch, h0 = unit % nch * 16;
+  const int Hl = min(16, a.H - h0);
+  const int s = a.list[i];
+  const int pos = a.tok_pos[a.cu[s]];
+  const int tid = threadIdx.x;
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lane = tid & (WAVE - 1);
+  const int li = lane & 15, hi = lane >> 4;
+  const int* table = a.table + (long)s * a.maxp;
+
+  bf16x8 qf[NKK];
+  const unsigned short* qp =
+      a.q + ((long)i * a.H + h0 + min(li, Hl - 1)) * CK + hi * 8;
+#pragma unroll
+  for (int kk = 0; kk < NKK; ++kk)
+    qf[kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
+
+  const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int t_beg = lo / KT;
+  const int t_all = pos < 0 ? 0 : pos / KT + 1 - t_beg;
+  const int per = (t_all + a.n_split - 1) / a.n_split;
+  const int t_lo = t_beg + blockIdx.y * per;
+  const int t_hi = min(t_beg + t_all, t_lo + per);
+
+  float m2 = NEG_BIG, l = 0.f;
+  f32x4 acc[ND];
+#pragma unroll
+  for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const float sc2 = a.scale * LOG2E;
+
+  short8 reg[NKK];  // this thread's 16 B pieces of the next tile
+  auto fetch = [&](int t) {
+#pragma unroll
+    for (int n = 0; n < NKK; ++n) {
+      const int idx = tid + n * 256;
+      const int key = min(t * KT + idx / (CK / 8), pos);
+      reg[n] = __builtin_nontemporal_load(reinterpret_cast<const short8*>(
+          a.kp + ((long)table[key / a.P] * a.P + key % a.P) * CK +
+          idx % (CK / 8) * 8));
+    }
+  };
+  if (t_lo < t_hi) fetch(t_lo);
+  for (int t = t_lo; t < t_hi; ++t) {
+    __syncthreads();  // the last tile is read
+#pragma unroll
+    for (int n = 0; n < NKK; ++n) {
+      const int idx = tid + n * 256;
+      *reinterpret_cast<short8*>(kt + idx / (CK / 8) * LDK + idx % (CK / 8) * 8) =
+          reg[n];
+    }
+    __syncthreads();
+    if (t + 1 < t_hi) fetch(t + 1);
+    f32x4 st = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kk = 0; kk < NKK; ++kk) {
+      const bf16x8 kf = as_bf16x8(*reinterpret_cast<const short8*>(
+          kt + (wave * 16 + li) * LDK + kk * 32 + hi * 8));
+      st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[kk], st, 0, 0, 0);
+    }
+    *reinterpret_cast<f32x4*>(sc + li * LDS_S + wave * 16 + hi * 4) = st;
+    __syncthreads();
+    // every wave takes the softmax of the whole tile
+    float p[2][8];
+    float rm = NEG_BIG;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int key = t * KT + hf * 32 + hi * 8 + j;
+        const float v = sc[li * LDS_S + hf * 32 + hi * 8 + j] * sc2;
+        p[hf][j] = (key < lo || key > pos) ? NEG_BIG : v;
+        rm = fmaxf(rm, p[hf][j]);
+      }
+    rm = fmaxf(rm, __shfl_xor(rm, 16));
+    rm = fmaxf(rm, __shfl_xor(rm, 32));
+    const float mn = fmaxf(m2, rm);  // every tile has a visible key
+    const float corr = fast_exp2(m2 - mn);
+    float ps = 0.f;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        p[hf][j] = fast_exp2(p[hf][j] - mn);
+        ps += p[hf][j];
+      }
+    ps += __shfl_xor(ps, 16);
+    ps += __shfl_xor(ps, 32);
+    l = l * corr + ps;
+    m2 = mn;
+#pragma unroll
+    for (int n = 0; n < ND; ++n)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc[n][r] *= corr;
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      // weights as two bf16, so that their rounding does not show
+      bf16x8 ph, pl;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        ph[j] = (__bf16)p[hf][j];
+        pl[j] = (__bf16)(p[hf][j] - (float)ph[j]);
+      }
+#pragma unroll
+      for (int n = 0; n < ND; ++n) {
+        const bf16x8 vf = column_frag(kt, LDK, hf * 32,
+                                      (n * 4 + wave) * 16 + (li & 3) * 4, li, hi);
+        acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, acc[n], 0, 0, 0);
+        acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, acc[n], 0, 0, 0);
+      }
+    }
+  }
+  if (li >= Hl) return;
+  const long u = ((long)unit * a.n_split + blockIdx.y) * 16 + li;
+  if (wave == 0 && hi == 0) {
+    a.pml[u * 2] = m2;
+    a.pml[u * 2 + 1] = l;
+  }
+#pragma unroll
+  for (int n = 0; n < ND; ++n)
+    *reinterpret_cast<f32x4*>(a.pacc + u * RP + (n * 4 + wave) * 16 + hi * 4) =
+        acc[n];
+}
+
+struct LatentOutputArgs {
+  const float* pml;
+  const float* pacc;
+  const float* sinks;        // (H,) or null
+  const unsigned short* wv;  // (H, vp, rp): W_uv, zero padded
+  const unsigned short* gate;  // row stride ldg, or null
+  unsigned short* out;         // row stride ldo
+  const int* cu;
+  const int* list;
+  long ldg, ldo;
+  int n_list, H, rp, vdim, vp, n_split;
+};
+
+// grid (vp / 64, H, rows / 16)
+__global__ __launch_bounds__(256) void latent_output_kernel(LatentOutputArgs a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned short lds_o[];
+  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 16;
+  const int M = min(16, a.n_list - m0);
+  const int nch = (a.H + 15) / 16, c = h / 16, hl = h % 16;
+  const int ldr = a.rp + 8;
+  {
+    // 16 threads a row
+    const int m = tid / 16;
+    float f = 0.f, mx = NEG_BIG;
+    const long u0 = ((long)(m0 + m) * nch + c) * a.n_split;
+    if (m < M) {
+      float l = 0.f;
+      for (int i = 0; i < a.n_split; ++i)
+        mx = fmaxf(mx, a.pml[((u0 + i) * 16 + hl) * 2]);
+      for (int i = 0; i < a.n_split; ++i)
+        l += a.pml[((u0 + i) * 16 + hl) * 2 + 1] *
+             fast_exp2(a.pml[((u0 + i) * 16 + hl) * 2] - mx);
+      f = 1.f;
+      if (a.sinks) {
+        const float s2 = a.sinks[h] * LOG2E, mn = fmaxf(mx, s2);
+        f = fast_exp2(mx - mn);
+        l = l * f + fast_exp2(s2 - mn);
+      }
+      f = l > 0.f ? f / l : 0.f;
+    }
+    for (int d = tid % 16 * 4; d < a.rp; d += 64) {
+      float o[4] = {0.f, 0.f, 0.f, 0.f};
+      if (m < M) {
+        for (int i = 0; i < a.n_split; ++i) {
+          const float w = fast_exp2(a.pml[((u0 + i) * 16 + hl) * 2] - mx);
+          const f32x4 v = *reinterpret_cast<const f32x4*>(
+              a.pacc + ((u0 + i) * 16 + hl) * a.rp + d);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o[r] += v[r] * w;
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] *= f;
+      }
+      stv<4>(lds_o + m * ldr + d, o);
+    }
+  }
+  __syncthreads();
+  const int wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int li = lane & 15, hi = lane >> 4;
+  const int n0 = blockIdx.x * 64 + wave * 16;
+  const unsigned short* w = a.wv + ((long)h * a.vp + n0 + li) * a.rp + hi * 8;
+  f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < a.rp; k += 32) {
+    const bf16x8 wf = as_bf16x8(*reinterpret_cast<const short8*>(w + k));
+    const bf16x8 of = as_bf16x8(
+        *reinterpret_cast<const short8*>(lds_o + li * ldr + k + hi * 8));
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(of, wf, acc, 0, 0, 0);
+  }
+  const int d = n0 + li;
+  if (d >= a.vdim) return;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int m = hi * 4 + r;
+    if (m >= M) continue;
+    const long row = a.cu[a.list[m0 + m]];
+    float v = acc[r];
+    if (a.gate) v *= sigmoid_f(bf2f(a.gate[row * a.ldg + h * a.vdim + d]));
+    a.out[row * a.ldo + h * a.vdim + d] = cvt_bf(v);
+  }
+}

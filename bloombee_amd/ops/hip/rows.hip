@@ -3,11 +3,14 @@
 // residual_norm_kernel — folds everything a layer left pending (split-K
 //     partials of its output GEMM, routed expert rows, identity-expert
 //     weights) into the 32-bit residual and emits the next layer's grouped
-//     RMS norm, in one pass per row.
+//     RMS norm, in one pass per row. For norms after the sum the residual is
+//     scaled first and the normed row takes its place.
 // proj_post_kernel — everything between the fused input GEMM and attention:
 //     folds split-K partials, RMS-norms q and k over the whole projection,
 //     writes K/V into the pages, hands on the output gate, applies the
 //     feed-forward activation and routes the token to its experts.
+// clamped_glu_kernel — bias, clamps, gate and product of a gated feed-forward.
+// softcap_kernel — cap * tanh(z / cap), in place.
 // router_gemm_kernel — f32 router logits where the input GEMM emits bf16.
 //
 // T is the activation element (unsigned short = bf16 bits, or float), TP the
@@ -108,10 +111,12 @@ struct ResidualArgs {
   const int* ids;      // (N, top): < 0 = no routed row for this choice
   const float* idw;    // (N,) weight of the layer's own input, or null
   const void* hprev;   // (N, ldhp) that input
+  const float* bias;   // (W,) of the pending GEMM, or null
   const float* nw;     // (W,) norm weight; null = fold only
   void* h;             // (N, ldh) normed row, zero beyond W
   int W, ks, ldp, top, ldr, ldhp, ldh, groups;
-  float eps;
+  int post;            // the normed row becomes the residual
+  float eps, alpha;    // alpha scales x before the sum
 };
 
 // LDS: W floats (the row) + groups * subs partial sums.
@@ -130,6 +135,8 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
   for (int i = threadIdx.x * V; i < W; i += BLOCK * V) {
     float v[V], u[V];
     ldv<V>(xr + i, v);
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] *= a.alpha;
     if (a.parts) {
       float d[V];
       ldv<V>(pr + i, d);
@@ -151,9 +158,14 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
 #pragma unroll
         for (int j = 0; j < V; ++j) d[j] += iw * u[j];
       }
+      if (a.bias) {
+        ldv<V>(a.bias + i, u);
+#pragma unroll
+        for (int j = 0; j < V; ++j) d[j] += u[j];
+      }
 #pragma unroll
       for (int j = 0; j < V; ++j) v[j] += d[j];
-      stv<V>(xr + i, v);
+      if (!a.post) stv<V>(xr + i, v);
     }
 #pragma unroll
     for (int j = 0; j < V; ++j) lds_row[i + j] = v[j];
@@ -192,10 +204,60 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
       v[j] = i + j < W ? lds_row[i + j] * stat[(i + j) / gs * subs] * a.nw[i + j]
                        : 0.f;
     stv<V>(hr + i, v);
+    if (a.post && i < W) stv<V>(xr + i, v);
   }
 }
 
-// x[n] = table[ids[n]] + pos_table[pos[n]] in f32; indices are clamped.
+struct GluArgs {
+  const void* parts;  // (ks, N, ldp) [gate | up] columns
+  long pstride;
+  const float* gb;    // (ff,) biases, or null
+  const float* ub;
+  void* out;          // (N, ldo), zero beyond ff
+  int ks, ldp, g_off, u_off, ff, ldo;
+  float limit, slope;
+};
+
+// g = min(gate, limit), u = clamp(up, -limit, limit):
+// out = g * sigmoid(slope * g) * (u + 1). grid (N, chunks of 256 * V columns)
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(GluArgs a) {
+  const long t = blockIdx.x;
+  const int i = (blockIdx.y * 256 + threadIdx.x) * V;
+  if (i >= a.ldo) return;
+  float g[V], u[V], w[V];
+#pragma unroll
+  for (int j = 0; j < V; ++j) g[j] = 0.f;
+  if (i < a.ff) {
+    const TP* row = (const TP*)a.parts + t * (long)a.ldp;
+    ldv<V>(row + a.g_off + i, g);
+    ldv<V>(row + a.u_off + i, u);
+    for (int s = 1; s < a.ks; ++s) {
+      ldv<V>(row + s * a.pstride + a.g_off + i, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) g[j] += w[j];
+      ldv<V>(row + s * a.pstride + a.u_off + i, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += w[j];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const float gj = fminf(g[j] + (a.gb ? a.gb[i + j] : 0.f), a.limit);
+      const float uj = fminf(fmaxf(u[j] + (a.ub ? a.ub[i + j] : 0.f), -a.limit),
+                             a.limit);
+      g[j] = gj * sigmoid_f(a.slope * gj) * (uj + 1.f);
+    }
+  }
+  stv<V>((T*)a.out + t * (long)a.ldo + i, g);
+}
+
+__global__ __launch_bounds__(256) void softcap_kernel(float* __restrict__ z,
+                                                      long n, float cap) {
+  for (long i = blockIdx.x * 256L + threadIdx.x; i < n; i += gridDim.x * 256L)
+    z[i] = cap * tanhf(z[i] / cap);
+}
+
+// x[n] = table[ids[n]] (+ pos_table[pos[n]]) in f32; indices are clamped.
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(
     const int* __restrict__ ids, const int* __restrict__ pos,
@@ -203,6 +265,10 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(
     float* __restrict__ x, int W, int vocab, int max_pos) {
   const long n = blockIdx.x;
   const T* a = table + (long)min(max(ids[n], 0), vocab - 1) * W;
+  if (!pos_table) {
+    for (int i = threadIdx.x; i < W; i += 256) x[n * W + i] = ldf(a + i);
+    return;
+  }
   const T* b = pos_table + (long)min(max(pos[n], 0), max_pos - 1) * W;
   for (int i = threadIdx.x; i < W; i += 256) x[n * W + i] = ldf(a + i) + ldf(b + i);
 }

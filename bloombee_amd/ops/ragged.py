@@ -1,6 +1,7 @@
-"""Fused steps of parallel-residual blocks over ragged batches.
+"""Fused steps of blocks over ragged batches.
 
-The pieces, in the order a layer runs them (N rows, one per token):
+The pieces, in the order a parallel-residual layer runs them (N rows, one per
+token):
 
   residual_norm  x += what the previous layer left pending; h = norm(x)
   linear_parts   h @ W^T, as split-K f32 partials on decode-sized batches
@@ -9,6 +10,9 @@ The pieces, in the order a layer runs them (N rows, one per token):
   moe_experts    routed experts
   attn_ragged    attention + output gate
   linear_parts   [attention | activation] @ [W_o | W_down]^T, left Pending
+
+Layers with a norm after every sum use sum_norm instead, and clamped_glu for
+their feed-forward; other mixers are in ops/mixers.py.
 
 Device tensors run the _hip_ragged extension and fail loudly without it; CPU
 tensors run the forms in ops/reference.py. Activations are bf16 or f32; the
@@ -81,6 +85,19 @@ class Pending:
     routing: Optional[Routing] = None
     h: Optional[torch.Tensor] = None         # (N, >= W)
 
+    def settle(self, x: torch.Tensor) -> None:
+        residual_norm(x, self)
+
+
+@dataclass
+class Carried:
+    """A layer that ends with a norm owes nothing; what it hands on is the
+    residual's rows in the activation type, the next layer's input."""
+    h: torch.Tensor                          # (N, stored inner size)
+
+    def settle(self, x: torch.Tensor) -> None:
+        pass
+
 
 def residual_norm(x: torch.Tensor, pending: Optional[Pending],
                   weight: Optional[torch.Tensor] = None, groups: int = 1,
@@ -99,7 +116,7 @@ def residual_norm(x: torch.Tensor, pending: Optional[Pending],
             x, p.parts if p else None,
             p.routed if p and p.routed is not None else None,
             rt.ids if rt else None, rt.idw if rt else None,
-            p.h if rt else None, weight, groups, eps, h)
+            p.h if rt else None, weight, groups, eps, h, 1.0, None, False)
         return h
     if p is not None:
         d = p.parts.float().sum(0)[:, :W]
@@ -114,13 +131,67 @@ def residual_norm(x: torch.Tensor, pending: Optional[Pending],
     return F.pad(y, (0, (cols or W) - W))
 
 
+def sum_norm(x: torch.Tensor, parts: torch.Tensor,
+             bias: Optional[torch.Tensor], weight: torch.Tensor, alpha: float,
+             eps: float, cols: int, dtype: torch.dtype) -> torch.Tensor:
+    """Norm after the sum: x (N, W) f32 <- rms(alpha x + sum of parts + bias)
+    * weight, in place; returns its rows as (N, cols) in dtype with zero
+    columns beyond W. parts (ks, N, >= W)."""
+    N, W = x.shape
+    if x.is_cuda:
+        h = torch.empty(N, cols, dtype=dtype, device=x.device)
+        _ext().residual_norm(x, parts, None, None, None, None, weight, 1, eps,
+                             h, alpha, bias, True)
+        return h
+    y = alpha * x + parts.float().sum(0)[:, :W]
+    if bias is not None:
+        y = y + bias
+    x.copy_(ref.grouped_rms_norm(y, weight, 1, eps))
+    return input_rows(x, cols, dtype)
+
+
+def input_rows(x: torch.Tensor, cols: int, dtype: torch.dtype) -> torch.Tensor:
+    """x (N, W) f32 as (N, cols) in dtype, zero columns beyond W."""
+    return F.pad(x.to(dtype), (0, cols - x.shape[1])).contiguous()
+
+
+def clamped_glu(parts: torch.Tensor, g_off: int, u_off: int, ff: int,
+                gate_b: Optional[torch.Tensor], up_b: Optional[torch.Tensor],
+                limit: float, slope: float, cols: int,
+                dtype: torch.dtype) -> torch.Tensor:
+    """Gated feed-forward activation of a [gate | up] GEMM output in parts:
+    g = min(gate, limit), u = clamp(up, -limit, limit),
+    g * sigmoid(slope * g) * (u + 1), as (N, cols) with zeros beyond ff."""
+    if parts.is_cuda:
+        out = torch.empty(parts.shape[1], cols, dtype=dtype,
+                          device=parts.device)
+        _ext().clamped_glu(parts, g_off, u_off, ff, gate_b, up_b, limit, slope,
+                           out)
+        return out
+    y = parts.float().sum(0)
+    a = ref.clamped_glu(y[:, g_off:g_off + ff], y[:, u_off:u_off + ff], gate_b,
+                        up_b, limit, slope)
+    return F.pad(a.to(dtype), (0, cols - ff))
+
+
+def softcap_(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """z <- cap * tanh(z / cap), f32, in place."""
+    if z.is_cuda:
+        _ext().softcap(z, cap)
+        return z
+    return z.div_(cap).tanh_().mul_(cap)
+
+
 def embed_rows(ids: torch.Tensor, positions: torch.Tensor,
-               table: torch.Tensor, pos_table: torch.Tensor) -> torch.Tensor:
-    """table[ids] + pos_table[positions] in f32, (..., W)."""
+               table: torch.Tensor, pos_table: Optional[torch.Tensor],
+               ) -> torch.Tensor:
+    """table[ids] (+ pos_table[positions]) in f32, (..., W)."""
     if table.is_cuda:
         x = _ext().embed_rows(ids.reshape(-1).int(),
                               positions.reshape(-1).int(), table, pos_table)
         return x.view(*ids.shape, -1)
+    if pos_table is None:
+        return F.embedding(ids.long(), table).float()
     pos = positions.long().clamp(min=0)
     return (F.embedding(ids.long(), table).float()
             + F.embedding(pos, pos_table).float())
@@ -283,19 +354,27 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
     return ref.moe_experts(h, gate_up, down, rt.ids, rt.wts)
 
 
-def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
+def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor,
+                v_pages: Optional[torch.Tensor],
                 batch, out: torch.Tensor, dim: int, vdim: int, scale: float,
                 window: int = 0, slopes: Optional[torch.Tensor] = None,
-                gate: Optional[torch.Tensor] = None) -> None:
+                gate: Optional[torch.Tensor] = None,
+                sinks: Optional[torch.Tensor] = None,
+                table: Optional[torch.Tensor] = None,
+                portions_only: bool = False) -> None:
     """Attention of a ragged batch into out[:, :H*vdim] (see
-    reference.attn_ragged)."""
+    reference.attn_ragged). Without v_pages the values are the first vdim
+    elements of the keys. table: page table of pages that are not the
+    cache's; portions_only leaves the rows of single tokens alone (where the
+    sizes are those of the tiled kernels)."""
+    table = batch.page_table if table is None else table
     if q.is_cuda:
+        dec = batch.dec_list[:0] if portions_only else batch.dec_list
         _ext().attn_ragged(
-            q, k_pages, v_pages, batch.page_table, batch.tok_seq,
-            batch.tok_pos, batch.cu, batch.q_start, batch.pre_list,
-            batch.dec_list, batch.max_new, batch.max_ctx, dim, vdim, scale,
-            window, slopes, gate, out)
+            q, k_pages, v_pages, table, batch.tok_seq, batch.tok_pos, batch.cu,
+            batch.q_start, batch.pre_list, dec, batch.max_new, batch.max_ctx,
+            dim, vdim, scale, window, slopes, sinks, gate, out)
         return
     n = q.shape[1] * vdim
     out[:, :n] = ref.attn_ragged(q, k_pages, v_pages, batch, dim, vdim, scale,
-                                 window, slopes, gate)
+                                 window, slopes, gate, sinks)

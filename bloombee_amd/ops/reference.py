@@ -29,6 +29,7 @@ import math
 from typing import Optional, Tuple
 
 import torch
+import torch.nn.functional as F
 
 
 # ---------------------------------------------------------------------------
@@ -477,10 +478,13 @@ def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
 
 
 def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
-                window: int = 0, slopes=None, gate=None) -> torch.Tensor:
+                window: int = 0, slopes=None, gate=None,
+                sinks=None) -> torch.Tensor:
     """Paged attention of a ragged batch: q (N, H, >= dim) -> (N, H * vdim).
     Row n sees positions j of its own sequence with 0 <= pos - j (< window);
-    score = q.k * scale - slope_h * (pos - j); out *= sigmoid(gate)."""
+    score = q.k * scale - slope_h * (pos - j); sinks_h is one more score that
+    has no value; out *= sigmoid(gate). Without v_pages the values are the
+    first vdim elements of the keys."""
     N, H = q.shape[0], q.shape[1]
     G = k_pages.shape[1]
     out = torch.zeros(N, H, vdim, dtype=torch.float32, device=q.device)
@@ -490,7 +494,8 @@ def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
             continue
         pos = batch.tok_pos[rows].long()
         ctx = int(pos.max()) + 1
-        k, v = kv_gather(k_pages, v_pages, batch.page_table, ctx, s)
+        k, v = kv_gather(k_pages, v_pages if v_pages is not None
+                         else k_pages.transpose(2, 3), batch.page_table, ctx, s)
         k = k[..., :dim].float().repeat_interleave(H // G, dim=0)
         v = v[..., :vdim].float().repeat_interleave(H // G, dim=0)
         sc = torch.matmul(q[rows, :, :dim].float().transpose(0, 1),
@@ -501,7 +506,11 @@ def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
         seen = dist >= 0
         if window > 0:
             seen &= dist < window
-        p = torch.softmax(sc.masked_fill(~seen, float("-inf")), dim=-1)
+        sc = sc.masked_fill(~seen, float("-inf"))
+        if sinks is not None:
+            sc = torch.cat([sc, sinks.float().view(-1, 1, 1).expand(
+                -1, sc.shape[1], 1)], -1)
+        p = torch.softmax(sc, dim=-1)[..., :ctx]
         out[rows] = torch.matmul(p, v).transpose(0, 1)
     out = out.reshape(N, H * vdim)
     if gate is not None:
@@ -524,3 +533,43 @@ def moe_experts(h, gate_up, down, ids, wts) -> torch.Tensor:
         a = (g * torch.sigmoid(g) * u).to(h.dtype).float()
         y[t, k] = (a @ down[e].float().t()) * wts[t, k, None]
     return y.to(h.dtype)
+
+
+def clamped_glu(gate, up, gate_b, up_b, limit: float, slope: float):
+    """g = min(gate + b, limit), u = clamp(up + b, -limit, limit);
+    g * sigmoid(slope * g) * (u + 1), fp32."""
+    g = gate if gate_b is None else gate + gate_b
+    u = up if up_b is None else up + up_b
+    g = g.clamp(max=limit)
+    return g * torch.sigmoid(slope * g) * (u.clamp(-limit, limit) + 1)
+
+
+def rotate_half(x: torch.Tensor, positions: torch.Tensor,
+                turns: torch.Tensor) -> torch.Tensor:
+    """Rotary positions on the first 2 * len(turns) elements of the last axis,
+    element i with element i + len(turns). x (N, ..., D), positions (N,);
+    turns: frequencies / 2 pi in float64, angles are reduced in float64."""
+    half = turns.numel()
+    r = positions.double().clamp(min=0)[:, None] * turns
+    ang = ((r - r.round()) * (2 * math.pi)).reshape(
+        r.shape[0], *[1] * (x.dim() - 2), half)
+    c, s = torch.cos(ang).to(x.dtype), torch.sin(ang).to(x.dtype)
+    u, v = x[..., :half], x[..., half:2 * half]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
+
+
+def channel_decays(a1, a2, a2_b, tau: float) -> torch.Tensor:
+    """sigmoid(a1 @ a2 + b)^(1 / tau), fp32. a2 (r, channels)."""
+    z = a1.float() @ a2.float() + a2_b.float()
+    return torch.exp(F.logsigmoid(z) / tau)
+
+
+def gla_scan(q, k, v, alpha, state):
+    """Gated linear attention of one sequence, token by token: q, k, alpha
+    (T, H, D), v (T, H, V), state (H, D, V) -> o (T, H, V), new state."""
+    out = []
+    for t in range(q.shape[0]):
+        state = (alpha[t].unsqueeze(-1) * state
+                 + k[t].unsqueeze(-1) * v[t].unsqueeze(-2))
+        out.append((state * q[t].unsqueeze(-1)).sum(-2))
+    return torch.stack(out), state

@@ -35,6 +35,10 @@ class NativeCheckpoint:
     def get(self, name: str) -> torch.Tensor:
         return self._file.get_tensor(name)
 
+    def shape(self, name: str) -> tuple:
+        """From the file's header, no data is read."""
+        return tuple(self._file.get_slice(name).get_shape())
+
     def layer(self, index: int):
         return lambda name: self._file.get_tensor(f"l{index}.{name}")
 

@@ -17,8 +17,10 @@ from pathlib import Path
 ROOT = Path(__file__).resolve().parent
 HIP_DIR = ROOT / "bloombee_amd" / "ops" / "hip"
 OPS_DIR = ROOT / "bloombee_amd" / "ops"
-# module -> source. _hip_ragged holds all that ragged-batch models need.
-MODULES = {"_hip_ops": "ext.hip", "_hip_ragged": "ext_ragged.hip"}
+# module -> source. _hip_ragged holds what all ragged-batch models need,
+# _hip_mixers latent attention and gated linear attention.
+MODULES = {"_hip_ops": "ext.hip", "_hip_ragged": "ext_ragged.hip",
+           "_hip_mixers": "ext_mixers.hip"}
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 
