@@ -159,3 +159,67 @@ def forward(tokens, w, cfg, collect=None):
             collect.append(x)
     y = zero_norm(x, w["final.norm"], eps) @ w["head"].T
     return softcap(y, cfg["logit_softcap"])
+
+
+# ---------------------------------------------------------------------------
+# small random models
+# ---------------------------------------------------------------------------
+
+def tensor_shapes(cfg, rank=lambda layer: 3 + 4 * layer):
+    """rank(layer): rows of a recurrent layer's decay projection, which the
+    configuration does not name."""
+    W = cfg["width"]
+    s = {"embed": (cfg["vocab"], W), "final.norm": (W,), "head": (cfg["vocab"], W)}
+    for i, layer in enumerate(cfg["layers"]):
+        mx, mlp, p = layer["mixer"], layer["mlp"], f"l{i}."
+        H, D, V = mx["heads"], mx["dim"], mx["vdim"]
+        s[p + "norm1"] = (W,)
+        m = p + "mix."
+        s[m + "g"], s[m + "o"] = (H * V, W), (W, H * V)
+        if layer["type"] == "gla":
+            s[m + "q"] = s[m + "k"] = (H * D, W)
+            s[m + "v"], s[m + "norm"] = (H * V, W), (V,)
+            s[m + "a1"], s[m + "a2"] = (rank(i), W), (H * D, rank(i))
+            s[m + "a2.b"] = (H * D,)
+        else:
+            Q, R, E = mx["q_rank"], mx["kv_rank"], mx["rot_dim"]
+            s[m + "dq"], s[m + "dq.norm"] = (Q, W), (Q,)
+            s[m + "uq"] = (H * (D + E), Q)
+            s[m + "uk"], s[m + "uv"], s[m + "sink"] = (H * D, R), (H * V, R), (H,)
+            if mx.get("kv_from") is None:
+                s[m + "dkv"], s[m + "dkv.norm"] = (R + E, W), (R,)
+        if mlp is not None:
+            F = mlp["ff"]
+            s[p + "norm2"] = (W,)
+            for n in ("gate", "up"):
+                s[p + f"mlp.{n}"], s[p + f"mlp.{n}.b"] = (F, W), (F,)
+            s[p + "mlp.down"], s[p + "mlp.down.b"] = (W, F), (W,)
+    return s
+
+
+def random_weights(cfg, seed=0, **kw):
+    """bf16-representable float32 weights of a lively scale: sharp attention,
+    decays from a few tokens to hundreds, logits that meet their cap."""
+    gen = torch.Generator().manual_seed(seed)
+    w = {}
+    for name, shape in tensor_shapes(cfg, **kw).items():
+        t = torch.randn(*shape, generator=gen)
+        last = name.rsplit(".", 1)[-1]
+        if name.endswith(("norm1", "norm2", "final.norm")):
+            t = 0.2 * t
+        elif last == "norm":
+            t = 1 + 0.2 * t
+        elif last == "sink":
+            t = 1 + t
+        elif name.endswith("a2.b"):
+            t = 1.5 + 1.5 * t
+        elif last == "b":
+            t = 0.2 * t
+        elif name != "embed":
+            t = t / math.sqrt(shape[-1])
+            if last in ("uq", "uk"):
+                t = 1.5 * t
+            elif last == "head":
+                t = 0.6 * cfg["logit_softcap"] * t
+        w[name] = t.bfloat16().float()
+    return w
