@@ -197,7 +197,10 @@ def run_swarm(args):
 # (model, closest family of equal layer size); both run LAYERS blocks
 LAYER_PAIRS = [("mubasun-8b-4l", "llama-3-8b"),
                ("mubasun-8x7b-4l", "mixtral-8x7b-4l"),
-               ("mubasun-64e-4l", None)]
+               ("mubasun-64e-4l", None),
+               ("risepel-8b-latent-4l", "mubasun-8b-4l"),
+               ("risepel-8b-gla-4l", "mubasun-8b-4l"),
+               ("risepel-8b-4l", "llama-3-8b")]
 LAYERS = 4
 
 
@@ -266,8 +269,9 @@ def run_layers(args):
         if args.pair and args.pair not in model:
             continue
         rows[model] = _layer_numbers(model, args)
-        if like:
+        if like and like not in rows:
             rows[like] = _layer_numbers(like, args)
+        if like:
             rows[f"{model} / {like}"] = {
                 k: round(rows[model][k] / rows[like][k], 3)
                 for k in rows[model]}
@@ -303,7 +307,8 @@ def main():
                     help="pipeline = raw RCCL pipeline stages (flagship); "
                          "swarm = the full decentralized serving stack "
                          "(DHT + sessions + handler) over the same device plane; "
-                         "layers = mubasun layers beside the closest family's")
+                         "layers = mubasun and risepel layers beside the "
+                         "closest family's")
     ap.add_argument("--pair", default=None,
                     help="layers mode: only pairs whose model name contains this")
     args = ap.parse_args()

@@ -177,12 +177,16 @@ void latent_scatter(Tensor y, Tensor ctx, Tensor valid, long dim, long rot,
 }
 
 template <int ND, int NR>
-static void launch_decode(LatentDecodeArgs& a, long units) {
+static void launch_decode(LatentDecodeArgs& a, long n) {
   constexpr int CK = ND * 64 + NR * 32;
-  constexpr size_t lds = 64 * (CK + 8) * 2 + 16 * 68 * 4;
-  auto k = attn_latent_decode_kernel<ND, NR>;
-  allow_lds(k, lds);
-  k<<<dim3(units, a.n_split), 256, lds, cur_stream()>>>(a);
+  by_bool(a.H > 16, [&](auto two) {
+    constexpr int HG = decltype(two)::value ? 2 : 1;
+    constexpr size_t lds = 64 * (CK + 8) * 2 + HG * 16 * 68 * 4;
+    auto k = attn_latent_decode_kernel<ND, NR, HG>;
+    allow_lds(k, lds);
+    const long units = n * ((a.H + 16 * HG - 1) / (16 * HG));
+    k<<<dim3(units, a.n_split), 256 * HG, lds, cur_stream()>>>(a);
+  });
   check_launch();
 }
 
@@ -227,10 +231,12 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   {
     const size_t lds = 32 * (qa.dimp + 8) * 2;
     by_type(y.scalar_type(), [&](auto p) {
-      auto k = latent_absorb_kernel<decltype(p)>;
-      allow_lds(k, lds);
-      k<<<dim3((rp + 63) / 64 + 1, H, (n + 31) / 32), 256, lds,
-          cur_stream()>>>(qa);
+      by_bool(all_of_8({qa.y.ld, dim, rot}), [&](auto v) {
+        auto k = latent_absorb_kernel<decltype(p), decltype(v)::value ? 8 : 1>;
+        allow_lds(k, lds);
+        k<<<dim3((rp + 127) / 128 + 1, H, (n + 31) / 32), 256, lds,
+            cur_stream()>>>(qa);
+      });
     });
     check_launch();
   }
@@ -243,38 +249,49 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   a.cu = qa.cu;
   a.list = qa.list;
   a.H = (int)H;
-  a.P = kp.size(2);
+  const int P = kp.size(2);
+  TORCH_CHECK((P & (P - 1)) == 0, "page size must be a power of two");
+  while (1 << a.p_log2 < P) ++a.p_log2;
   a.maxp = table.size(1);
   a.window = (int)window;
   a.scale = (float)scale;
-  const long units = n * ((H + 15) / 16);
+  // a workgroup a CU, two tiles of 64 keys each at least
+  const long units = n * (H > 16 ? (H + 31) / 32 : 1);
   const long seen = window > 0 ? std::min<long>(window, max_ctx) : max_ctx;
   const long tiles = (seen + 63) / 64 + 1;
-  a.n_split = (int)std::max<long>(
-      1, std::min<long>({16, 512 / std::max<long>(1, units), tiles / 2}));
-  auto pml = torch::empty({units * a.n_split, 16, 2}, fopt);
-  auto pacc = torch::empty({units * a.n_split, 16, rp}, fopt);
+  const long fill = (H > 16 ? 256 : 512) / std::max<long>(1, units);
+  a.n_split = (int)std::max<long>(1, std::min<long>({16, fill, tiles / 2}));
+  auto pml = torch::empty({n, H, a.n_split, 2}, fopt);
+  auto pacc = torch::empty({n, H, a.n_split, rp}, fopt);
+  auto olat = torch::empty({n, H, rp}, bopt);
   a.pml = pml.data_ptr<float>();
   a.pacc = pacc.data_ptr<float>();
   auto by_rot = [&](auto nd) {
     constexpr int ND = decltype(nd)::value;
-    if (ck - rp == 32) launch_decode<ND, 1>(a, units);
-    else if (ck - rp == 64) launch_decode<ND, 2>(a, units);
-    else launch_decode<ND, 4>(a, units);
+    if (ck - rp == 32) launch_decode<ND, 1>(a, n);
+    else if (ck - rp == 64) launch_decode<ND, 2>(a, n);
+    else launch_decode<ND, 4>(a, n);
   };
   if (rp == 64) by_rot(std::integral_constant<int, 1>{});
   else if (rp == 128) by_rot(std::integral_constant<int, 2>{});
   else if (rp == 256) by_rot(std::integral_constant<int, 4>{});
   else by_rot(std::integral_constant<int, 8>{});
 
-  LatentOutputArgs o{};
-  o.pml = a.pml;
-  o.pacc = a.pacc;
+  const float* sp = nullptr;
   if (sinks.has_value()) {
     CHECK_F32((*sinks));
     TORCH_CHECK(sinks->numel() == H);
-    o.sinks = sinks->data_ptr<float>();
+    sp = sinks->data_ptr<float>();
   }
+  LatentOutputArgs o{};
+  o.o = (const bf16_bits*)olat.data_ptr();
+  by_bool(a.n_split > 4, [&](auto many) {
+    latent_combine_kernel<decltype(many)::value ? 16 : 4>
+        <<<n * H, 128, 0, cur_stream()>>>(a.pml, a.pacc, sp,
+                                          (bf16_bits*)olat.data_ptr(), (int)H,
+                                          (int)rp, a.n_split);
+  });
+  check_launch();
   if (gate.has_value()) {
     TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 &&
                 gate->size(0) == out.size(0) && gate->stride(1) == 1 &&
@@ -293,9 +310,8 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   o.rp = (int)rp;
   o.vdim = (int)vdim;
   o.vp = wv.size(1);
-  o.n_split = a.n_split;
-  latent_output_kernel<<<dim3(o.vp / 64, H, (n + 15) / 16), 256,
-                         16 * (rp + 8) * 2, cur_stream()>>>(o);
+  latent_output_kernel<<<dim3(o.vp / 64, H, (n + 31) / 32), 256, 0,
+                         cur_stream()>>>(o);
   check_launch();
 }
 
@@ -354,15 +370,20 @@ void gla_step(Tensor y, Tensor a1, std::vector<long> dims,
   a.out = out.data_ptr();
   a.ldo = out.stride(0);
   if (list.numel() == 0) return;
+  // few workgroups: more waves on each state
+  const bool wide = a.H * list.numel() < 256;
   by_type(y.scalar_type(), [&](auto p) {
     by_type(out.scalar_type(), [&](auto t) {
       by_bool(a.vdim % 4 == 0, [&](auto v) {
-        constexpr int V = decltype(v)::value ? 4 : 1;
-        const size_t lds = 4 * (((3 * a.dim + 3) & ~3) + 256 * V +
-                                2 * ((a.vdim + 3) & ~3) + (size_t)a.r);
-        auto k = gla_step_kernel<decltype(p), decltype(t), V>;
-        allow_lds(k, lds);
-        k<<<dim3(a.H, list.numel()), 256, lds, cur_stream()>>>(a);
+        by_bool(wide, [&](auto w) {
+          constexpr int V = decltype(v)::value ? 4 : 1;
+          constexpr int B = decltype(w)::value ? 1024 : 256;
+          const size_t lds = 4 * (((3 * a.dim + 3) & ~3) + B * V +
+                                  2 * ((a.vdim + 3) & ~3) + (size_t)a.r);
+          auto k = gla_step_kernel<decltype(p), decltype(t), V, B>;
+          allow_lds(k, lds);
+          k<<<dim3(a.H, list.numel()), B, lds, cur_stream()>>>(a);
+        });
       });
     });
   });
@@ -380,7 +401,7 @@ static size_t prep_lds(int dp, int C, long r) {
 
 // Tokens of a chunk, 0 where the chunk form does not take these sizes.
 long gla_chunk(long dim, long vdim, long r) {
-  if (dim > 256 || vdim < 1) return 0;
+  if (dim > 256 || vdim < 1 || vdim > 512) return 0;
   const int C = chunk_of(dim);
   return prep_lds(pad_dim(dim), C, r) <= 150 * 1024 ? C : 0;
 }
@@ -396,8 +417,7 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   CHECK_F32(a1);
   TORCH_CHECK(y.dim() == 2 && a1.dim() == 2 && a1.size(0) == y.size(0));
   GlaChunkArgs a{};
-  int g_off = 0;
-  int* f[8] = {&a.q_off, &a.k_off, &a.v_off, &g_off, &a.a1_off,
+  int* f[8] = {&a.q_off, &a.k_off, &a.v_off, &a.g_off, &a.a1_off,
                &a.H, &a.dim, &a.vdim};
   for (int i = 0; i < 8; ++i) *f[i] = (int)dims[i];
   check_gla(a2, a2b, nw, state, slots, a.H, a.dim, a.vdim);
@@ -412,29 +432,28 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   auto inside = [&](int off, long n) { return off >= 0 && off + n <= a.ldy; };
   TORCH_CHECK(a.a1_off >= 0 && a.a1_off + a.r <= a.ld1 &&
               inside(a.q_off, a.H * a.dim) && inside(a.k_off, a.H * a.dim) &&
-              inside(a.v_off, a.H * a.vdim) && inside(g_off, a.H * a.vdim));
+              inside(a.v_off, a.H * a.vdim) && inside(a.g_off, a.H * a.vdim));
   TORCH_CHECK(len.numel() == chunks && ccu.numel() == list.numel() + 1 &&
               q_start.numel() == slots.numel());
   CHECK_T(out, at::kBFloat16);
   TORCH_CHECK(out.dim() == 2 && out.size(0) == N && out.size(1) >= a.H * a.vdim);
   if (chunks == 0) return;
+  a.VT = (a.vdim + 15) / 16;
   auto bopt = y.options();
-  auto fopt = bopt.dtype(at::kFloat);
-  auto qd = torch::empty({chunks, a.H, 2, C, DP}, bopt);
+  auto b = torch::empty({chunks, a.H, C, DP}, bopt.dtype(at::kFloat));
   auto kd = torch::empty({chunks, a.H, 2, C, DP}, bopt);
-  auto A = torch::empty({chunks, a.H, 2, C, C}, bopt);
-  auto dec = torch::empty({chunks, a.H, DP}, fopt);
-  auto o = torch::empty({N, a.H, a.vdim}, fopt);
+  auto S = torch::empty({chunks, a.H, a.VT, 2, DP * 16}, bopt);
   a.y = (const bf16_bits*)y.data_ptr();
   a.a1 = a1.data_ptr<float>();
   a.a2 = a2.data_ptr<float>();
   a.a2b = a2b.data_ptr<float>();
+  a.nw = nw.data_ptr<float>();
   a.state = state.data_ptr<float>();
-  a.qd = (bf16_bits*)qd.data_ptr();
+  a.b = b.data_ptr<float>();
   a.kd = (bf16_bits*)kd.data_ptr();
-  a.A = (bf16_bits*)A.data_ptr();
-  a.dec = dec.data_ptr<float>();
-  a.o = o.data_ptr<float>();
+  a.S = (bf16_bits*)S.data_ptr();
+  a.out = (bf16_bits*)out.data_ptr();
+  a.ldo = out.size(1);
   a.row0 = row0.data_ptr<int>();
   a.len = len.data_ptr<int>();
   a.ccu = ccu.data_ptr<int>();
@@ -443,6 +462,7 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   a.q_start = q_start.data_ptr<int>();
   a.qscale = (float)consts[0];
   a.inv_tau = (float)consts[1];
+  a.eps = (float)consts[2];
   auto go = [&](auto dp, auto c) {
     constexpr int D = decltype(dp)::value, CC = decltype(c)::value;
     auto prep = gla_prep_kernel<D, CC>;
@@ -451,11 +471,23 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
     prep<<<dim3(chunks, a.H), 256, l1, cur_stream()>>>(a);
     check_launch();
     auto scan = gla_scan_kernel<D, CC>;
-    const size_t l2 = 2 * (4 * CC * (D + 8) + 2 * CC * (CC + 8) + CC * 72) + 4 * D;
+    const size_t l2 = 4 * (2 * CC * (D + 8) + CC * 72 + 2 * D);
     allow_lds(scan, l2);
     scan<<<dim3((a.vdim + 63) / 64, a.H, list.numel()), 256, l2,
            cur_stream()>>>(a);
     check_launch();
+    auto fin = [&](auto nct) {
+      constexpr int N = decltype(nct)::value;
+      auto k = gla_out_kernel<D, CC, N>;
+      const size_t first = std::max(2 * CC * (D + 4), CC * (N * 128 + 8));
+      const size_t l3 = 2 * (first + 2 * CC * (D + 8) + 2 * CC * (CC + 8));
+      allow_lds(k, l3);
+      k<<<dim3(chunks, a.H), 512, l3, cur_stream()>>>(a);
+      check_launch();
+    };
+    if (a.vdim <= 128) fin(std::integral_constant<int, 1>{});
+    else if (a.vdim <= 256) fin(std::integral_constant<int, 2>{});
+    else fin(std::integral_constant<int, 4>{});
   };
   using I32 = std::integral_constant<int, 32>;
   using I64 = std::integral_constant<int, 64>;
@@ -463,15 +495,6 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   else if (DP == 64) go(I64{}, I64{});
   else if (DP == 128) go(std::integral_constant<int, 128>{}, I64{});
   else go(std::integral_constant<int, 256>{}, I32{});
-  const long waves = chunks * C * a.H;
-  by_bool(all_of_8({a.vdim, a.ldy, g_off, out.size(1)}), [&](auto v) {
-    gla_out_kernel<decltype(v)::value ? 4 : 1>
-        <<<(waves + 3) / 4, 256, 0, cur_stream()>>>(
-            a.o, a.y, a.ldy, g_off, nw.data_ptr<float>(),
-            (bf16_bits*)out.data_ptr(), out.size(1), a.row0, a.len, C,
-            (int)chunks, a.H, a.vdim, (float)consts[2]);
-  });
-  check_launch();
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {

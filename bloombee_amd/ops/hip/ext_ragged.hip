@@ -147,6 +147,7 @@ void clamped_glu(Tensor parts, long g_off, long u_off, long ff, OptTensor gb,
               out.size(1) >= ff && ff >= 1);
   GluArgs a{};
   const long N = parts.size(1);
+  a.N = N;
   a.parts = parts.data_ptr();
   a.ks = parts.size(0);
   a.ldp = parts.size(2);
@@ -173,10 +174,13 @@ void clamped_glu(Tensor parts, long g_off, long u_off, long ff, OptTensor gb,
   by_type(parts.scalar_type(), [&](auto p) {
     by_type(out.scalar_type(), [&](auto t) {
       by_bool(vec, [&](auto v) {
-        constexpr int V = decltype(v)::value ? 8 : 1;
-        clamped_glu_kernel<decltype(p), decltype(t), V>
-            <<<dim3(N, (a.ldo + 256 * V - 1) / (256 * V)), 256, 0,
-               cur_stream()>>>(a);
+        by_bool(N > 256, [&](auto many) {
+          constexpr int V = decltype(v)::value ? 8 : 1;
+          constexpr int R = decltype(many)::value ? 4 : 1;
+          clamped_glu_kernel<decltype(p), decltype(t), V, R>
+              <<<dim3((a.ldo + 256 * V - 1) / (256 * V), (N + R - 1) / R), 256,
+                 0, cur_stream()>>>(a);
+        });
       });
     });
   });
@@ -392,7 +396,7 @@ static void launch_mfma(AttnArgs& a, const Tensor& pre, const Tensor& dec,
                         long max_new, long max_ctx, const Tensor& like) {
   const int Hg = a.H / a.G;
   if (pre.numel() > 0) {
-    constexpr int QC = (DK > 128 || DV > 128) ? 1 : 2;
+    constexpr int QC = (DK > 192 || DV > 128) ? 1 : 2;
     a.list = pre.data_ptr<int>();
     const long rows = max_new * Hg;
     attn_ragged_prefill_kernel<DK, DV, QC>

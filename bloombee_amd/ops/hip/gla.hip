@@ -9,12 +9,12 @@
 //  gla_step_kernel   token by token, everything fused: decoded tokens, and any
 //                    sizes and types.
 //  gla_prep_kernel   prompts in chunks of C tokens, all chunks side by side:
-//                    cumulated log decays b, then
-//                       qd = q 2^b, kd = k 2^(b_last - b),
+//                    cumulated log decays b and kd = k 2^(b_last - b)
+//  gla_scan_kernel   chunk after chunk, a slice of value columns each: leaves
+//                    S for the chunk, then S <- 2^b_last S + kd^T v
+//  gla_out_kernel    all chunks side by side:
 //                       A[t][s] = sum_d q_t k_s 2^(b_t - b_s)   (s <= t)
-//  gla_scan_kernel   chunk after chunk, a slice of value columns each:
-//                       o = qd S + A v,   S <- 2^b_last S + kd^T v
-//  gla_out_kernel    norm and gate.
+//                       o = (q 2^b) S + A v, norm and gate
 //
 // Chunk products run on bf16 MFMAs with decayed operands, weights and states
 // split into two bf16 (the value and what its rounding lost). All exponents of
@@ -52,21 +52,21 @@ struct GlaArgs {
   float qscale, inv_tau, eps;
 };
 
-// grid (H, listed sequences). LDS: q, k, alpha (dim each), v, o (vdim each),
-// partial sums (256 * V), a1 (r).
-template <typename TP, typename T, int V>
-__global__ __launch_bounds__(256) void gla_step_kernel(GlaArgs a) {
+// grid (H, listed sequences). LDS: q, k, alpha (dim each), partial sums
+// (B * V), v, o (vdim each), a1 (r).
+template <typename TP, typename T, int V, int B>
+__global__ __launch_bounds__(B) void gla_step_kernel(GlaArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds_gla[];
-  __shared__ float red[4];
+  __shared__ float red[B / WAVE];
   const int h = blockIdx.x, s = a.list[blockIdx.y], tid = threadIdx.x;
   float* qs = lds_gla;
   float* ks = qs + a.dim;
   float* as = ks + a.dim;
   float* part = lds_gla + ((3 * a.dim + 3) & ~3);
-  float* vs = part + 256 * V;
+  float* vs = part + B * V;
   float* os = vs + ((a.vdim + 3) & ~3);
   float* a1s = os + ((a.vdim + 3) & ~3);
-  const int VQ = a.vdim / V, CW = min(VQ, 256), RG = 256 / CW;
+  const int VQ = a.vdim / V, CW = min(VQ, B), RG = B / CW;
   const int rg = tid / CW, cq = tid % CW;
   const int t0 = a.cu[s], t1 = a.cu[s + 1];
   float* S = a.state + ((long)a.slots[s] * a.H + h) * a.dim * a.vdim;
@@ -74,10 +74,10 @@ __global__ __launch_bounds__(256) void gla_step_kernel(GlaArgs a) {
     const int pos = a.tok_pos[t];
     if (pos < 0) continue;  // empty slot
     __syncthreads();
-    for (int i = tid; i < a.r; i += 256)
+    for (int i = tid; i < a.r; i += B)
       fold_parts<float, 1>(a.a1, t, a.a1_off + i, a1s + i);
     __syncthreads();
-    for (int d = tid; d < a.dim; d += 256) {
+    for (int d = tid; d < a.dim; d += B) {
       float v[1];
       const int c = h * a.dim + d;
       fold_parts<TP, 1>(a.y, t, a.q_off + c, v);
@@ -89,7 +89,7 @@ __global__ __launch_bounds__(256) void gla_step_kernel(GlaArgs a) {
       const float ls = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
       as[d] = expf(ls * a.inv_tau);
     }
-    for (int i = tid; i < a.vdim; i += 256)
+    for (int i = tid; i < a.vdim; i += B)
       fold_parts<TP, 1>(a.y, t, a.v_off + h * a.vdim + i, vs + i);
     __syncthreads();
     for (int cb = 0; cb < VQ; cb += CW) {
@@ -133,14 +133,16 @@ __global__ __launch_bounds__(256) void gla_step_kernel(GlaArgs a) {
       __syncthreads();
     }
     float ss = 0.f;
-    for (int i = tid; i < a.vdim; i += 256) ss += os[i] * os[i];
+    for (int i = tid; i < a.vdim; i += B) ss += os[i] * os[i];
     ss = wave_reduce_sum(ss);
     if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
     __syncthreads();
-    const float inv =
-        1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.vdim + a.eps);
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < B / WAVE; ++i) ss += red[i];
+    const float inv = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
     T* op = (T*)a.out + t * a.ldo + h * a.vdim;
-    for (int i = tid; i < a.vdim; i += 256) {
+    for (int i = tid; i < a.vdim; i += B) {
       float g[1];
       fold_parts<TP, 1>(a.y, t, a.g_off + h * a.vdim + i, g);
       stf(op + i, os[i] * inv * a.nw[i] * g[0] * sigmoid_f(g[0]));
@@ -153,20 +155,22 @@ struct GlaChunkArgs {
   const float* a1;          // (N, ld1), a1_off
   const float* a2;          // (r, H * dim)
   const float* a2b;
+  const float* nw;
   float* state;
-  unsigned short* qd;       // (chunks, H, 2, C, DP): high and low part
-  unsigned short* kd;
-  unsigned short* A;        // (chunks, H, 2, C, C)
-  float* dec;               // (chunks, H, DP): decay over the whole chunk
-  float* o;                 // (N, H, vdim)
+  float* b;                 // (chunks, H, C, DP): cumulated log2 decays
+  unsigned short* kd;       // (chunks, H, 2, C, DP): high and low part
+  unsigned short* S;        // (chunks, H, VT, 2, DP / 32, 64, 8): fragments of
+                            // the state before each chunk, high and low part
+  unsigned short* out;      // (N, ldo)
   const int* row0;          // (chunks,) first row
   const int* len;           // (chunks,) tokens
   const int* ccu;           // (listed + 1,) first chunk of each sequence
   const int* list;
   const int* slots;
   const int* q_start;
-  int ldy, ld1, q_off, k_off, v_off, a1_off, r, H, dim, vdim;
-  float qscale, inv_tau;
+  long ldo;
+  int ldy, ld1, q_off, k_off, v_off, g_off, a1_off, r, H, dim, vdim, VT;
+  float qscale, inv_tau, eps;
 };
 
 DEVINL void split8(const float* v, short8& hi, short8& lo) {
@@ -178,11 +182,42 @@ DEVINL void split8(const float* v, short8& hi, short8& lo) {
   }
 }
 
+// Eight channels of token t's q or k (columns off ..); zero beyond the chunk's
+// tokens and the head's channels.
+DEVINL void load_channels(const GlaChunkArgs& a, long row0, int len, int off,
+                          int h, int t, int d, float* v) {
+  if (t < len && d < a.dim) {
+    const unsigned short* p = a.y + (row0 + t) * a.ldy + off + h * a.dim + d;
+    if (d + 8 <= a.dim && ((a.ldy | (off + h * a.dim)) & 7) == 0) {
+      load_bf16x8(p, v);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = d + j < a.dim ? bf2f(p[j]) : 0.f;
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = 0.f;
+  }
+}
+
+// Eight value columns of a token as bits; zero beyond the head's.
+DEVINL short8 load_values(const GlaChunkArgs& a, long row, int h, int c, bool vec) {
+  short8 v = short8{};
+  const unsigned short* p = a.y + row * a.ldy + a.v_off + h * a.vdim + c;
+  if (vec && c + 8 <= a.vdim) {
+    v = *reinterpret_cast<const short8*>(p);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (c + j < a.vdim) v[j] = (short)p[j];
+  }
+  return v;
+}
+
 // grid (chunks, H). LDS: b (C x (DP + 4)), a1 (C x r), a2 of the head (r x DP)
 template <int DP, int C>
 __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
-  constexpr int LDB = DP + 4, NB = C / 16, NKK = DP / 32;
-  constexpr float SPAN = 80.f;  // widest safe range of exponents, log2
+  constexpr int LDB = DP + 4;
   extern __shared__ __attribute__((aligned(16))) float lds_b[];
   const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   float* a1s = lds_b + C * LDB;
@@ -209,6 +244,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
     }
   }
   __syncthreads();
+  const long base = (long)ch * a.H + h;
   if (tid < DP) {
     float s = 0.f;
 #pragma unroll 16
@@ -216,77 +252,230 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
       s += lds_b[t * LDB + tid];
       lds_b[t * LDB + tid] = s;
     }
-    a.dec[((long)ch * a.H + h) * DP + tid] = fast_exp2(s);
   }
   __syncthreads();
-
-  // eight channels of a token's q (scaled) or k; zero beyond either
-  auto load8 = [&](int off, int t, int d, float* v) {
-    if (t < len && d < a.dim) {
-      const unsigned short* p =
-          a.y + (row0 + t) * a.ldy + off + h * a.dim + d;
-      if (d + 8 <= a.dim && ((a.ldy | (off + h * a.dim)) & 7) == 0) {
-        load_bf16x8(p, v);
-      } else {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = d + j < a.dim ? bf2f(p[j]) : 0.f;
-      }
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = 0.f;
-    }
-  };
-  const long base = ((long)ch * a.H + h) * 2;
   for (int idx = tid; idx < C * DP / 8; idx += 256) {
     const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
-    float q[8], k[8];
-    load8(a.q_off, t, d, q);
-    load8(a.k_off, t, d, k);
+    float k[8], b[8];
+    load_channels(a, row0, len, a.k_off, h, t, d, k);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const float b = lds_b[t * LDB + d + j];
-      q[j] *= a.qscale * fast_exp2(b);
-      k[j] *= fast_exp2(lds_b[(C - 1) * LDB + d + j] - b);
+      b[j] = lds_b[t * LDB + d + j];
+      k[j] *= fast_exp2(lds_b[(C - 1) * LDB + d + j] - b[j]);
     }
+    stv<8>(a.b + (base * C + t) * DP + d, b);
     short8 vh, vl;
-    const long at = base * C * DP + t * DP + d;
-    split8(q, vh, vl);
-    *reinterpret_cast<short8*>(a.qd + at) = vh;
-    *reinterpret_cast<short8*>(a.qd + at + C * DP) = vl;
     split8(k, vh, vl);
+    const long at = base * 2 * C * DP + t * DP + d;
     *reinterpret_cast<short8*>(a.kd + at) = vh;
     *reinterpret_cast<short8*>(a.kd + at + C * DP) = vl;
   }
+}
 
+// grid (vdim / 64, H, listed sequences); a wave owns 16 value columns and the
+// state's whole column. The state's accumulators hold rows in the order
+//     tile 2g + n, row x*4 + y  <->  channel g*32 + x*8 + n*4 + y
+// so that a lane's registers of two tiles are eight consecutive channels: an
+// operand fragment as it is.
+template <int DP, int C>
+__global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
+  constexpr int NG = DP / 32, NC = C / 32;
+  constexpr int LDD = DP + 8, LDV = 64 + 8;
+  constexpr int PD = C * DP / 8 / 256;   // 16 B pieces a thread and plane
+  constexpr int PV = C * 64 / 8 / 256;
+  constexpr int BUF = 2 * C * LDD + C * LDV + 2 * DP;  // 16-bit elements
+  static_assert(PD >= 1 && PV >= 1, "chunk smaller than the workgroup");
+  extern __shared__ __attribute__((aligned(16))) unsigned short lds_scan[];
+  const int h = blockIdx.y, i = blockIdx.z, s = a.list[i], tid = threadIdx.x;
   const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
-  unsigned short* Ah = a.A + base * C * C;
-  for (int pair = wave; pair < NB * NB; pair += 4) {
+  const int v0 = blockIdx.x * 64, vt = blockIdx.x * 4 + wave;
+  const int col = v0 + wave * 16 + li;
+  const bool live = col < a.vdim;
+  float* S = a.state + ((long)a.slots[s] * a.H + h) * a.dim * a.vdim;
+  const bool vvec = ((a.vdim | a.ldy | a.v_off) & 7) == 0;
+
+  f32x4 acc[2 * NG];
+  const bool fresh = a.q_start[s] == 0;
+#pragma unroll
+  for (int g = 0; g < NG; ++g)
+#pragma unroll
+    for (int n = 0; n < 2; ++n)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = g * 32 + hi * 8 + n * 4 + r;
+        acc[2 * g + n][r] =
+            !fresh && live && d < a.dim ? S[(long)d * a.vdim + col] : 0.f;
+      }
+
+  short8 rk[2][PD], rv[PV];
+  float rd = 0.f;
+  auto fetch = [&](int ch) {
+    const long base = (long)ch * a.H + h;
+#pragma unroll
+    for (int p = 0; p < 2; ++p)
+#pragma unroll
+      for (int n = 0; n < PD; ++n)
+        rk[p][n] = *reinterpret_cast<const short8*>(
+            a.kd + (base * 2 + p) * C * DP + (tid + n * 256) * 8);
+    const long row0 = a.row0[ch];
+    const int len = a.len[ch];
+#pragma unroll
+    for (int n = 0; n < PV; ++n) {
+      const int idx = tid + n * 256, t = idx / 8;
+      rv[n] = short8{};
+      if (t < len) rv[n] = load_values(a, row0 + t, h, v0 + idx % 8 * 8, vvec);
+    }
+    if (tid < DP) rd = a.b[(base * C + C - 1) * DP + tid];
+  };
+  auto stage = [&](unsigned short* buf) {
+#pragma unroll
+    for (int p = 0; p < 2; ++p)
+#pragma unroll
+      for (int n = 0; n < PD; ++n) {
+        const int idx = tid + n * 256;
+        *reinterpret_cast<short8*>(buf + (p * C + idx / (DP / 8)) * LDD +
+                                   idx % (DP / 8) * 8) = rk[p][n];
+      }
+    unsigned short* vb = buf + 2 * C * LDD;
+#pragma unroll
+    for (int n = 0; n < PV; ++n) {
+      const int idx = tid + n * 256;
+      *reinterpret_cast<short8*>(vb + idx / 8 * LDV + idx % 8 * 8) = rv[n];
+    }
+    if (tid < DP) ((float*)(vb + C * LDV))[tid] = fast_exp2(rd);
+  };
+
+  const int c0 = a.ccu[i], c1 = a.ccu[i + 1];
+  if (c0 < c1) {
+    fetch(c0);
+    stage(lds_scan);
+  }
+  for (int ch = c0; ch < c1; ++ch) {
+    const unsigned short* buf = lds_scan + ((ch - c0) & 1) * BUF;
+    if (ch + 1 < c1) fetch(ch + 1);
+    // the state as it stands, for the chunk's outputs
+    if (vt < a.VT) {
+      unsigned short* sp =
+          a.S + ((((long)ch * a.H + h) * a.VT + vt) * 2 * NG) * 512 + lane * 8;
+#pragma unroll
+      for (int g = 0; g < NG; ++g) {
+        float sv[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          sv[r] = acc[2 * g][r];
+          sv[4 + r] = acc[2 * g + 1][r];
+        }
+        short8 sh, sl;
+        split8(sv, sh, sl);
+        *reinterpret_cast<short8*>(sp + g * 512) = sh;
+        *reinterpret_cast<short8*>(sp + (NG + g) * 512) = sl;
+      }
+    }
+    __syncthreads();   // buf is written; the other one is read
+    const unsigned short* vb = buf + 2 * C * LDD;
+    const float* dt = (const float*)(vb + C * LDV);
+    bf16x8 vf[NC];
+#pragma unroll
+    for (int k = 0; k < NC; ++k)
+      vf[k] = column_frag(vb, LDV, k * 32, wave * 16 + (li & 3) * 4, li, hi);
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+      for (int n = 0; n < 2; ++n) {
+        const f32x4 dv = *reinterpret_cast<const f32x4*>(dt + g * 32 + hi * 8 + n * 4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[2 * g + n][r] *= dv[r];
+#pragma unroll
+        for (int k = 0; k < NC; ++k)
+#pragma unroll
+          for (int p = 0; p < 2; ++p)
+            acc[2 * g + n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                column_frag(buf + p * C * LDD, LDD, k * 32,
+                            g * 32 + (li & 3) * 8 + n * 4, li, hi),
+                vf[k], acc[2 * g + n], 0, 0, 0);
+      }
+    if (ch + 1 < c1) stage(lds_scan + ((ch + 1 - c0) & 1) * BUF);
+  }
+  if (live) {
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+      for (int n = 0; n < 2; ++n)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int d = g * 32 + hi * 8 + n * 4 + r;
+          if (d < a.dim) S[(long)d * a.vdim + col] = acc[2 * g + n][r];
+        }
+  }
+}
+
+// grid (chunks, H), eight waves; a wave owns every eighth tile of 16 value
+// columns. Outputs are made transposed, o^T = S^T qd^T + v^T A^T: a lane holds
+// four consecutive columns of one token. LDS: b, later v; qd; A.
+template <int DP, int C, int NCT>
+__global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
+  constexpr int LDB = DP + 4, LDD = DP + 8, LDA = C + 8, NG = DP / 32;
+  constexpr int NT = C / 16, NC = C / 32, NB = C / 16, VC = NCT * 128;
+  constexpr int LDV = VC + 8;
+  constexpr int FIRST = 2 * C * LDB > C * LDV ? 2 * C * LDB : C * LDV;
+  constexpr float SPAN = 80.f;  // widest safe range of exponents, log2
+  extern __shared__ __attribute__((aligned(16))) unsigned short lds_out[];
+  __shared__ float ssum[8][C];
+  float* bs = (float*)lds_out;               // (C, LDB)
+  unsigned short* vs = lds_out;              // (C, LDV)
+  unsigned short* qs = lds_out + FIRST;      // (2, C, LDD)
+  unsigned short* as = qs + 2 * C * LDD;     // (2, C, LDA)
+  const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int lane = tid & (WAVE - 1);
+  const int li = lane & 15, hi = lane >> 4;
+  const long row0 = a.row0[ch], base = (long)ch * a.H + h;
+  const int len = a.len[ch];
+
+  for (int idx = tid; idx < C * DP / 4; idx += 512) {
+    const int t = idx / (DP / 4), d = idx % (DP / 4) * 4;
+    *reinterpret_cast<f32x4*>(bs + t * LDB + d) =
+        *reinterpret_cast<const f32x4*>(a.b + (base * C + t) * DP + d);
+  }
+  __syncthreads();
+  for (int idx = tid; idx < C * DP / 8; idx += 512) {
+    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
+    float q[8];
+    load_channels(a, row0, len, a.q_off, h, t, d, q);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) q[j] *= a.qscale * fast_exp2(bs[t * LDB + d + j]);
+    short8 vh, vl;
+    split8(q, vh, vl);
+    *reinterpret_cast<short8*>(qs + t * LDD + d) = vh;
+    *reinterpret_cast<short8*>(qs + (C + t) * LDD + d) = vl;
+  }
+  for (int pair = wave; pair < NB * NB; pair += 8) {
     const int I = pair / NB, J = pair % NB;
     f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
-    if (J <= I && J * 16 < len) {
-      const float* ref = lds_b + (I * 16 - 1) * LDB;  // row before block I
+    if (J <= I && I * 16 < len) {
+      const float* ref = bs + (I * 16 - 1) * LDB;  // row before block I
       bool near = true;
       if (J == I) {
         for (int d = lane; d < DP; d += WAVE) {
           const float r = I > 0 ? ref[d] : 0.f;
-          near = near && r - lds_b[(I * 16 + 15) * LDB + d] <= SPAN;
+          near = near && r - bs[(I * 16 + 15) * LDB + d] <= SPAN;
         }
         near = __builtin_amdgcn_ballot_w64(!near) == 0;
       }
       if (near) {
 #pragma unroll
-        for (int kk = 0; kk < NKK; ++kk) {
+        for (int kk = 0; kk < NG; ++kk) {
           const int d = kk * 32 + hi * 8, t = I * 16 + li, s = J * 16 + li;
           float q[8], k[8];
-          load8(a.q_off, t, d, q);
-          load8(a.k_off, s, d, k);
+          load_channels(a, row0, len, a.q_off, h, t, d, q);
+          load_channels(a, row0, len, a.k_off, h, s, d, k);
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
             const float r = I > 0 ? ref[d + j] : 0.f;
-            q[j] *= a.qscale * fast_exp2(lds_b[t * LDB + d + j] - r);
-            k[j] *= fast_exp2(r - lds_b[s * LDB + d + j]);
+            q[j] *= a.qscale * fast_exp2(bs[t * LDB + d + j] - r);
+            k[j] *= fast_exp2(r - bs[s * LDB + d + j]);
           }
           short8 qh, ql, kh, kl;
           split8(q, qh, ql);
@@ -310,7 +499,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
               a.y + (row0 + s) * a.ldy + a.k_off + h * a.dim;
           for (int d = 0; d < a.dim; ++d)
             sum += bf2f(qp[d]) * a.qscale * bf2f(kp[d]) *
-                   fast_exp2(lds_b[t * LDB + d] - lds_b[s * LDB + d]);
+                   fast_exp2(bs[t * LDB + d] - bs[s * LDB + d]);
           acc[r] = sum;
         }
       }
@@ -320,238 +509,107 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
       const int t = I * 16 + hi * 4 + r, s = J * 16 + li;
       const float v = s <= t ? acc[r] : 0.f;
       const unsigned short vh = cvt_bf(v);
-      Ah[t * C + s] = vh;
-      Ah[C * C + t * C + s] = cvt_bf(v - bf2f(vh));
+      as[t * LDA + s] = vh;
+      as[(C + t) * LDA + s] = cvt_bf(v - bf2f(vh));
     }
   }
-}
-
-// grid (vdim / 64, H, listed sequences); a wave owns 16 value columns and the
-// state's whole column. The state's accumulators hold rows in the order
-//     tile 2g + n, row x*4 + y  <->  channel g*32 + x*8 + n*4 + y
-// so that a lane's registers of two tiles are eight consecutive channels: the
-// B fragment of qd S.
-template <int DP, int C>
-__global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
-  constexpr int NG = DP / 32, NT = C / 16, NC = C / 32;
-  constexpr int LDD = DP + 8, LDA = C + 8, LDV = 64 + 8;
-  constexpr int PD = C * DP / 8 / 256;   // 16 B pieces a thread and plane
-  constexpr int PV = C * 64 / 8 / 256;
-  constexpr int PA = C * C / 8 >= 256 ? C * C / 8 / 256 : 1;
-  static_assert(PD >= 1 && PV >= 1, "chunk smaller than the workgroup");
-  extern __shared__ __attribute__((aligned(16))) unsigned short lds_scan[];
-  unsigned short* qt = lds_scan;             // (2, C, LDD)
-  unsigned short* kt = qt + 2 * C * LDD;     // (2, C, LDD)
-  unsigned short* at = kt + 2 * C * LDD;     // (2, C, LDA)
-  unsigned short* vt = at + 2 * C * LDA;     // (C, LDV)
-  float* dt = (float*)(vt + C * LDV);        // (DP,)
-  const int h = blockIdx.y, i = blockIdx.z, s = a.list[i], tid = threadIdx.x;
-  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
-  const int lane = tid & (WAVE - 1);
-  const int li = lane & 15, hi = lane >> 4;
-  const int v0 = blockIdx.x * 64;
-  const int col = v0 + wave * 16 + li;
-  const bool live = col < a.vdim;
-  float* S = a.state + ((long)a.slots[s] * a.H + h) * a.dim * a.vdim;
-  const bool vvec = v0 + 64 <= a.vdim && (a.vdim & 7) == 0 &&
-                    ((a.ldy | a.v_off) & 7) == 0;
-
-  f32x4 acc[2 * NG];
-  const bool fresh = a.q_start[s] == 0;
-#pragma unroll
-  for (int g = 0; g < NG; ++g)
-#pragma unroll
-    for (int n = 0; n < 2; ++n)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = g * 32 + hi * 8 + n * 4 + r;
-        acc[2 * g + n][r] =
-            !fresh && live && d < a.dim ? S[(long)d * a.vdim + col] : 0.f;
-      }
-
-  short8 rq[2][PD], rk[2][PD], ra[2][PA], rv[PV];
-  float rd = 0.f;
-  auto fetch = [&](int ch) {
-    const long base = ((long)ch * a.H + h) * 2;
-#pragma unroll
-    for (int p = 0; p < 2; ++p) {
-#pragma unroll
-      for (int n = 0; n < PD; ++n) {
-        const long at_ = (base + p) * C * DP + (tid + n * 256) * 8;
-        rq[p][n] = *reinterpret_cast<const short8*>(a.qd + at_);
-        rk[p][n] = *reinterpret_cast<const short8*>(a.kd + at_);
-      }
-#pragma unroll
-      for (int n = 0; n < PA; ++n)
-        if ((tid + n * 256) * 8 < C * C)
-          ra[p][n] = *reinterpret_cast<const short8*>(
-              a.A + (base + p) * C * C + (tid + n * 256) * 8);
-    }
-    const long row0 = a.row0[ch];
-    const int len = a.len[ch];
-#pragma unroll
-    for (int n = 0; n < PV; ++n) {
-      const int idx = tid + n * 256, t = idx / 8, c = v0 + idx % 8 * 8;
+  __syncthreads();   // b is read
+  {
+    const bool vec = ((a.vdim | a.ldy | a.v_off) & 7) == 0;
+    for (int idx = tid; idx < C * VC / 8; idx += 512) {
+      const int t = idx / (VC / 8), c = idx % (VC / 8) * 8;
       short8 v = short8{};
-      if (t < len) {
-        const unsigned short* p =
-            a.y + (row0 + t) * a.ldy + a.v_off + h * a.vdim + c;
-        if (vvec) {
-          v = *reinterpret_cast<const short8*>(p);
-        } else {
-#pragma unroll
-          for (int j = 0; j < 8; ++j)
-            if (c + j < a.vdim) v[j] = (short)p[j];
-        }
-      }
-      rv[n] = v;
+      if (t < len && c < a.vdim) v = load_values(a, row0 + t, h, c, vec);
+      *reinterpret_cast<short8*>(vs + t * LDV + c) = v;
     }
-    if (tid < DP) rd = a.dec[((long)ch * a.H + h) * DP + tid];
-  };
-  auto stage = [&]() {
-#pragma unroll
-    for (int p = 0; p < 2; ++p) {
-#pragma unroll
-      for (int n = 0; n < PD; ++n) {
-        const int idx = tid + n * 256;
-        const int to = (p * C + idx / (DP / 8)) * LDD + idx % (DP / 8) * 8;
-        *reinterpret_cast<short8*>(qt + to) = rq[p][n];
-        *reinterpret_cast<short8*>(kt + to) = rk[p][n];
-      }
-#pragma unroll
-      for (int n = 0; n < PA; ++n) {
-        const int idx = tid + n * 256;
-        if (idx * 8 < C * C)
-          *reinterpret_cast<short8*>(at + (p * C + idx / (C / 8)) * LDA +
-                                     idx % (C / 8) * 8) = ra[p][n];
-      }
-    }
-#pragma unroll
-    for (int n = 0; n < PV; ++n) {
-      const int idx = tid + n * 256;
-      *reinterpret_cast<short8*>(vt + idx / 8 * LDV + idx % 8 * 8) = rv[n];
-    }
-    if (tid < DP) dt[tid] = rd;
-  };
-  auto frag = [&](const unsigned short* tile, int ld, int row, int k) {
-    return as_bf16x8(*reinterpret_cast<const short8*>(
-        tile + (row + li) * ld + k + hi * 8));
-  };
+  }
+  __syncthreads();
 
-  const int c0 = a.ccu[i], c1 = a.ccu[i + 1];
-  if (c0 < c1) fetch(c0);
-  for (int ch = c0; ch < c1; ++ch) {
-    __syncthreads();
-    stage();
-    __syncthreads();
-    if (ch + 1 < c1) fetch(ch + 1);
-    bf16x8 vf[NC];
+  f32x4 o[NCT][NT];
 #pragma unroll
-    for (int k = 0; k < NC; ++k)
-      vf[k] = column_frag(vt, LDV, k * 32, wave * 16 + (li & 3) * 4, li, hi);
-    f32x4 o[NT];
+  for (int c = 0; c < NCT; ++c) {
 #pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      o[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < NT; ++t) o[c][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const int vt = c * 8 + wave;
+    if (vt >= a.VT) continue;
+    const unsigned short* sp = a.S + ((base * a.VT + vt) * 2 * NG) * 512 + lane * 8;
+    bf16x8 sh[NG], sl[NG];
 #pragma unroll
-      for (int k = 0; k < NC; ++k) {
+    for (int g = 0; g < NG; ++g) {
+      sh[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + g * 512));
+      sl[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + (NG + g) * 512));
+    }
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const bf16x8 vf = column_frag(vs, LDV, k * 32, vt * 16 + (li & 3) * 4, li, hi);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
         if (k * 32 > t * 16 + 15) continue;  // above the diagonal
 #pragma unroll
         for (int p = 0; p < 2; ++p)
-          o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              frag(at + p * C * LDA, LDA, t * 16, k * 32), vf[k], o[t], 0, 0, 0);
+          o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              vf, as_bf16x8(*reinterpret_cast<const short8*>(
+                      as + (p * C + t * 16 + li) * LDA + k * 32 + hi * 8)),
+              o[c][t], 0, 0, 0);
       }
     }
-#pragma unroll
-    for (int g = 0; g < NG; ++g) {
-      float sv[8];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        sv[r] = acc[2 * g][r];
-        sv[4 + r] = acc[2 * g + 1][r];
-      }
-      short8 sh, sl;
-      split8(sv, sh, sl);
-#pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        const bf16x8 qh = frag(qt, LDD, t * 16, g * 32);
-        const bf16x8 ql = frag(qt + C * LDD, LDD, t * 16, g * 32);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, as_bf16x8(sh), o[t], 0, 0, 0);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql, as_bf16x8(sh), o[t], 0, 0, 0);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, as_bf16x8(sl), o[t], 0, 0, 0);
-      }
-#pragma unroll
-      for (int n = 0; n < 2; ++n) {
-        const f32x4 dv = *reinterpret_cast<const f32x4*>(dt + g * 32 + hi * 8 + n * 4);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) acc[2 * g + n][r] *= dv[r];
-#pragma unroll
-        for (int k = 0; k < NC; ++k)
-#pragma unroll
-          for (int p = 0; p < 2; ++p)
-            acc[2 * g + n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                column_frag(kt + p * C * LDD, LDD, k * 32,
-                            g * 32 + (li & 3) * 8 + n * 4, li, hi),
-                vf[k], acc[2 * g + n], 0, 0, 0);
-      }
-    }
-    if (live) {
-      const long row0 = a.row0[ch];
-      const int len = a.len[ch];
-#pragma unroll
-      for (int t = 0; t < NT; ++t)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int tt = t * 16 + hi * 4 + r;
-          if (tt < len)
-            a.o[((row0 + tt) * a.H + h) * a.vdim + col] = o[t][r];
-        }
-    }
-  }
-  if (live) {
 #pragma unroll
     for (int g = 0; g < NG; ++g)
 #pragma unroll
-      for (int n = 0; n < 2; ++n)
+      for (int t = 0; t < NT; ++t) {
+        const bf16x8 qh = as_bf16x8(*reinterpret_cast<const short8*>(
+            qs + (t * 16 + li) * LDD + g * 32 + hi * 8));
+        const bf16x8 ql = as_bf16x8(*reinterpret_cast<const short8*>(
+            qs + (C + t * 16 + li) * LDD + g * 32 + hi * 8));
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[g], qh, o[c][t], 0, 0, 0);
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[g], ql, o[c][t], 0, 0, 0);
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[g], qh, o[c][t], 0, 0, 0);
+      }
+  }
+  // columns beyond vdim are zero: they add nothing
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < NCT; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ss += o[c][t][r] * o[c][t][r];
+    ss += __shfl_xor(ss, 16);
+    ss += __shfl_xor(ss, 32);
+    if (hi == 0) ssum[wave][t * 16 + li] = ss;
+  }
+  __syncthreads();
+  const bool vec = ((a.vdim | a.ldy | a.g_off | (int)a.ldo) & 3) == 0;
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int tt = t * 16 + li;
+    if (tt >= len) continue;
+    float ss = 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) ss += ssum[w][tt];
+    const float inv = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
+    const unsigned short* gp = a.y + (row0 + tt) * a.ldy + a.g_off + h * a.vdim;
+    unsigned short* op = a.out + (row0 + tt) * a.ldo + h * a.vdim;
+#pragma unroll
+    for (int c = 0; c < NCT; ++c) {
+      const int v0 = (c * 8 + wave) * 16 + hi * 4;
+      if (v0 >= a.vdim) continue;
+      if (vec) {
+        float g[4], w[4];
+        ldv<4>(gp + v0, g);
+        ldv<4>(a.nw + v0, w);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          w[r] *= o[c][t][r] * inv * g[r] * sigmoid_f(g[r]);
+        stv<4>(op + v0, w);
+      } else {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int d = g * 32 + hi * 8 + n * 4 + r;
-          if (d < a.dim) S[(long)d * a.vdim + col] = acc[2 * g + n][r];
+          if (v0 + r >= a.vdim) continue;
+          const float g = bf2f(gp[v0 + r]);
+          op[v0 + r] = cvt_bf(o[c][t][r] * inv * a.nw[v0 + r] * g * sigmoid_f(g));
         }
-  }
-}
-
-// grid (rows * H / 4): a wave a head. Rows of sequences not in the chunk form
-// are left alone (rows[i]: the i-th row).
-template <int V>
-__global__ __launch_bounds__(256) void gla_out_kernel(
-    const float* __restrict__ o, const unsigned short* __restrict__ y, int ldy,
-    int g_off, const float* __restrict__ nw, unsigned short* __restrict__ out,
-    long ldo, const int* __restrict__ row0, const int* __restrict__ len, int C,
-    int chunks, int H, int vdim, float eps) {
-  const long u = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
-  const int lane = threadIdx.x & (WAVE - 1);
-  const int h = u % H;
-  const long ct = u / H;
-  const int ch = ct / C, t = ct % C;
-  if (ch >= chunks || t >= len[ch]) return;
-  const long row = row0[ch] + t;
-  const float* p = o + (row * H + h) * vdim;
-  float ss = 0.f;
-  for (int i = lane * V; i < vdim; i += WAVE * V) {
-    float v[V];
-    ldv<V>(p + i, v);
-#pragma unroll
-    for (int j = 0; j < V; ++j) ss += v[j] * v[j];
-  }
-  const float inv = 1.f / sqrtf(wave_reduce_sum(ss) / (float)vdim + eps);
-  for (int i = lane * V; i < vdim; i += WAVE * V) {
-    float v[V], g[V];
-    ldv<V>(p + i, v);
-    ldv<V>(y + row * ldy + g_off + h * vdim + i, g);
-#pragma unroll
-    for (int j = 0; j < V; ++j)
-      v[j] *= inv * nw[i + j] * g[j] * sigmoid_f(g[j]);
-    stv<V>(out + row * ldo + h * vdim + i, v);
+      }
+    }
   }
 }

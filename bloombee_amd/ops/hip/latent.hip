@@ -10,11 +10,11 @@
 //  latent_absorb_kernel  queries of decoded rows, taken into the latent space:
 //                        q_lat = W_uk^T q, beside the rotated part. One head's
 //                        query then meets [c | r] itself.
-//  attn_latent_decode_kernel  decoded rows: every key tile is read once, for the
-//                        scores by rows and for the values by columns
-//                        (transposing LDS reads).
-//  latent_output_kernel  folds the splits and the sink, applies W_uv and the
-//                        sigmoid output gate.
+//  attn_latent_decode_kernel  decoded rows: every key tile is read once for up
+//                        to 32 heads, for the scores by rows and for the values
+//                        by columns (transposing LDS reads).
+//  latent_combine_kernel folds the splits and the sink.
+//  latent_output_kernel  applies W_uv and the sigmoid output gate.
 //
 // Rotary pairs are (i, i + dims/2). Angles are reduced in double, in turns.
 
@@ -143,19 +143,6 @@ struct LatentQueryArgs {
   int n_list, H, dim, rot, rdims, rp, ck, dimp, ldq;
 };
 
-// Element e of a head's rotated part for one row.
-template <typename TP>
-DEVINL float rotated(const LatentQueryArgs& a, long t, int pos, int col, int e) {
-  float v[1];
-  fold_parts<TP, 1>(a.y, t, col + e, v);
-  if (e >= a.rdims) return v[0];
-  const int half = a.rdims / 2, k = e % half;
-  float w[1], c, s;
-  fold_parts<TP, 1>(a.y, t, col + (e < half ? e + half : k), w);
-  rotation(pos, a.turns[k], c, s);
-  return e < half ? v[0] * c - w[0] * s : v[0] * c + w[0] * s;
-}
-
 // grid N: a row's queries, [dim unrotated | rot rotated | zeros] per head
 template <typename TP, typename T, int V>
 __global__ __launch_bounds__(256) void latent_rope_kernel(LatentQueryArgs a) {
@@ -170,14 +157,26 @@ __global__ __launch_bounds__(256) void latent_rope_kernel(LatentQueryArgs a) {
   const int per = a.ldq / V;
   for (int idx = tid; idx < a.H * per; idx += 256) {
     const int h = idx / per, d = (idx % per) * V;
-    const int col = h * (a.dim + a.rot);
+    const int col = h * (a.dim + a.rot), e0 = d - a.dim;
     float v[V];
     if (d + V <= a.dim) {
       fold_parts<TP, V>(a.y, t, col + d, v);
+    } else if (e0 >= 0 && e0 + V <= a.rdims && half % V == 0) {
+      // a piece inside one half: its partners are a piece, too
+      const bool first = e0 < half;
+      float w[V];
+      fold_parts<TP, V>(a.y, t, col + d, v);
+      fold_parts<TP, V>(a.y, t, col + d + (first ? half : -half), w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const int k = e0 + j - (first ? 0 : half);
+        const float c = lds_cs[k], s = lds_cs[half + k];
+        v[j] = first ? v[j] * c - w[j] * s : v[j] * c + w[j] * s;
+      }
     } else {
 #pragma unroll
       for (int j = 0; j < V; ++j) {
-        const int e = d + j - a.dim;  // may straddle the border
+        const int e = e0 + j;  // may straddle the border
         v[j] = 0.f;
         if (e >= a.rot) continue;
         float x[1], w[1];
@@ -194,9 +193,9 @@ __global__ __launch_bounds__(256) void latent_rope_kernel(LatentQueryArgs a) {
   }
 }
 
-// grid (rp / 64 + 1, H, rows / 32): 32 listed rows of one head times W_uk^T;
+// grid (rp / 128 + 1, H, rows / 32): 32 listed rows of one head times W_uk^T;
 // the last x block writes the rotated part and the zero columns.
-template <typename TP>
+template <typename TP, int V>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentQueryArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned short lds_q[];
   const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 32;
@@ -204,51 +203,76 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentQueryArgs a) {
   const int col = h * (a.dim + a.rot);
   unsigned short* out = (unsigned short*)a.q;
   if (blockIdx.x == gridDim.x - 1) {
-    const int n = a.ck - a.rp;
-    for (int idx = tid; idx < M * n; idx += 256) {
-      const int m = idx / n, e = idx % n;
+    // a pair a thread, then what does not turn
+    const int half = a.rdims / 2, rest = a.ck - a.rp - a.rdims;
+    for (int idx = tid; idx < M * half; idx += 256) {
+      const int m = idx / half, k = idx % half;
       const long row = a.cu[a.list[m0 + m]];
-      float v = 0.f;
+      float u[1], v[1], c, s;
+      fold_parts<TP, 1>(a.y, row, col + a.dim + k, u);
+      fold_parts<TP, 1>(a.y, row, col + a.dim + half + k, v);
+      rotation(max(a.tok_pos[row], 0), a.turns[k], c, s);
+      unsigned short* o = out + ((long)(m0 + m) * a.H + h) * a.ck + a.rp + k;
+      o[0] = cvt_bf(u[0] * c - v[0] * s);
+      o[half] = cvt_bf(v[0] * c + u[0] * s);
+    }
+    for (int idx = tid; idx < M * rest; idx += 256) {
+      const int m = idx / rest, e = a.rdims + idx % rest;
+      float v[1] = {0.f};
       if (e < a.rot)
-        v = rotated<TP>(a, row, max(a.tok_pos[row], 0), col + a.dim, e);
-      out[((long)(m0 + m) * a.H + h) * a.ck + a.rp + e] = cvt_bf(v);
+        fold_parts<TP, 1>(a.y, a.cu[a.list[m0 + m]], col + a.dim + e, v);
+      out[((long)(m0 + m) * a.H + h) * a.ck + a.rp + e] = cvt_bf(v[0]);
     }
     return;
   }
-  const int ldr = a.dimp + 8;
-  for (int idx = tid; idx < 32 * a.dimp; idx += 256) {
-    const int m = idx / a.dimp, d = idx % a.dimp;
-    float v[1] = {0.f};
+  const int ldr = a.dimp + 8, pieces = a.dimp / V;
+  for (int idx = tid; idx < 32 * pieces; idx += 256) {
+    const int m = idx / pieces, d = idx % pieces * V;
+    float v[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
     if (m < M && d < a.dim)
-      fold_parts<TP, 1>(a.y, a.cu[a.list[m0 + m]], col + d, v);
-    lds_q[m * ldr + d] = cvt_bf(v[0]);
+      fold_parts<TP, V>(a.y, a.cu[a.list[m0 + m]], col + d, v);
+    stv<V>(lds_q + m * ldr + d, v);
   }
   __syncthreads();
   const int wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
-  const int n0 = blockIdx.x * 64 + wave * 16;
-  if (n0 >= a.rp) return;
-  const unsigned short* w = (const unsigned short*)a.wk +
-                            ((long)h * a.rp + n0 + li) * a.dimp + hi * 8;
-  f32x4 acc[2];
-  acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < a.dimp; k += 32) {
-    const bf16x8 wf = as_bf16x8(*reinterpret_cast<const short8*>(w + k));
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
-      const bf16x8 qf = as_bf16x8(*reinterpret_cast<const short8*>(
-          lds_q + (m * 16 + li) * ldr + k + hi * 8));
-      acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf, wf, acc[m], 0, 0, 0);
+  for (int nt = 0; nt < 2; ++nt) {
+    const int n0 = blockIdx.x * 128 + nt * 64 + wave * 16;
+    if (n0 >= a.rp) return;
+    const unsigned short* w = (const unsigned short*)a.wk +
+                              ((long)h * a.rp + n0 + li) * a.dimp + hi * 8;
+    f32x4 acc[2];
+    acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < a.dimp; k0 += 128) {
+      short8 wf[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        wf[u] = k0 + u * 32 < a.dimp
+                    ? *reinterpret_cast<const short8*>(w + k0 + u * 32) : short8{};
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int k = min(k0 + u * 32, a.dimp - 32);
+#pragma unroll
+        for (int m = 0; m < 2; ++m) {
+          const bf16x8 qf = as_bf16x8(*reinterpret_cast<const short8*>(
+              lds_q + (m * 16 + li) * ldr + k + hi * 8));
+          acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              qf, as_bf16x8(wf[u]), acc[m], 0, 0, 0);
+        }
+      }
     }
+#pragma unroll
+    for (int m = 0; m < 2; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = m * 16 + hi * 4 + r;
+        if (row < M)
+          out[((long)(m0 + row) * a.H + h) * a.ck + n0 + li] = cvt_bf(acc[m][r]);
+      }
   }
-#pragma unroll
-  for (int m = 0; m < 2; ++m)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int row = m * 16 + hi * 4 + r;
-      if (row < M)
-        out[((long)(m0 + row) * a.H + h) * a.ck + n0 + li] = cvt_bf(acc[m][r]);
-    }
 }
 
 struct LatentScatterArgs {
@@ -306,9 +330,9 @@ struct LatentDecodeArgs {
   const int* tok_pos;
   const int* cu;
   const int* list;
-  float* pml;   // (units, n_split, 16, 2): max (log2 units) and sum
-  float* pacc;  // (units, n_split, 16, rp)
-  int H, P, maxp, window, n_split;
+  float* pml;   // (n_list, H, n_split, 2): max (log2 units) and sum
+  float* pacc;  // (n_list, H, n_split, rp)
+  int H, p_log2, maxp, window, n_split;
   float scale;
 };
 
@@ -336,30 +360,35 @@ DEVINL bf16x8 column_frag(const unsigned short* tile, int ld, int r0, int col,
   return as_bf16x8(v);
 }
 
-// grid (n_list * chunks of 16 heads, n_split). ck = ND * 64 + NR * 32; a wave
-// owns every fourth 16-column tile of the values.
-template <int ND, int NR>
-__global__ __launch_bounds__(256) void attn_latent_decode_kernel(LatentDecodeArgs a) {
+// grid (n_list * chunks of 16 * HG heads, n_split), four waves for each of HG
+// groups of 16 heads. ck = ND * 64 + NR * 32; a wave owns every fourth
+// 16-column tile of the values.
+template <int ND, int NR, int HG>
+__global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
+    LatentDecodeArgs a) {
   constexpr int KT = 64, RP = ND * 64, CK = RP + NR * 32, NKK = CK / 32;
   constexpr int LDK = CK + 8, LDS_S = KT + 4;
+  constexpr int LANES = 256 * HG / KT;   // threads that stage one row
+  constexpr int NP = (CK / 8 + LANES - 1) / LANES;  // 16 B pieces each
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_dec[];
   unsigned short* kt = (unsigned short*)lds_dec;
-  float* sc = (float*)(lds_dec + KT * LDK * 2);
+  const int tid = threadIdx.x;
+  const int wv = __builtin_amdgcn_readfirstlane(tid / WAVE);
+  const int wave = wv & 3, grp = wv >> 2;
+  float* sc = (float*)(lds_dec + KT * LDK * 2) + grp * 16 * LDS_S;
 
-  const int nch = (a.H + 15) / 16;
-  const int unit = blockIdx.x, i = unit / nch, h0 = unit % nch * 16;
-  const int Hl = min(16, a.H - h0);
+  const int nch = (a.H + 16 * HG - 1) / (16 * HG);
+  const int unit = blockIdx.x, i = unit / nch;
+  const int h0 = unit % nch * 16 * HG + grp * 16;
   const int s = a.list[i];
   const int pos = a.tok_pos[a.cu[s]];
-  const int tid = threadIdx.x;
-  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int* table = a.table + (long)s * a.maxp;
 
   bf16x8 qf[NKK];
   const unsigned short* qp =
-      a.q + ((long)i * a.H + h0 + min(li, Hl - 1)) * CK + hi * 8;
+      a.q + ((long)i * a.H + min(h0 + li, a.H - 1)) * CK + hi * 8;
 #pragma unroll
   for (int kk = 0; kk < NKK; ++kk)
     qf[kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
@@ -377,25 +406,29 @@ __global__ __launch_bounds__(256) void attn_latent_decode_kernel(LatentDecodeArg
   for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
   const float sc2 = a.scale * LOG2E;
 
-  short8 reg[NKK];  // this thread's 16 B pieces of the next tile
+  // a thread stages pieces piece, piece + LANES, .. of one row of the tile
+  const int srow = tid / LANES, piece = tid % LANES;
+  short8 reg[NP];
   auto fetch = [&](int t) {
+    const int key = min(t * KT + srow, pos);
+    const unsigned short* kp =
+        a.kp + (((long)table[key >> a.p_log2] << a.p_log2) +
+                (key & ((1 << a.p_log2) - 1))) * CK;
 #pragma unroll
-    for (int n = 0; n < NKK; ++n) {
-      const int idx = tid + n * 256;
-      const int key = min(t * KT + idx / (CK / 8), pos);
-      reg[n] = __builtin_nontemporal_load(reinterpret_cast<const short8*>(
-          a.kp + ((long)table[key / a.P] * a.P + key % a.P) * CK +
-          idx % (CK / 8) * 8));
+    for (int n = 0; n < NP; ++n) {
+      const int pc = piece + n * LANES;
+      if ((CK / 8) % LANES == 0 || pc < CK / 8)
+        reg[n] = *reinterpret_cast<const short8*>(kp + pc * 8);
     }
   };
   if (t_lo < t_hi) fetch(t_lo);
   for (int t = t_lo; t < t_hi; ++t) {
     __syncthreads();  // the last tile is read
 #pragma unroll
-    for (int n = 0; n < NKK; ++n) {
-      const int idx = tid + n * 256;
-      *reinterpret_cast<short8*>(kt + idx / (CK / 8) * LDK + idx % (CK / 8) * 8) =
-          reg[n];
+    for (int n = 0; n < NP; ++n) {
+      const int pc = piece + n * LANES;
+      if ((CK / 8) % LANES == 0 || pc < CK / 8)
+        *reinterpret_cast<short8*>(kt + srow * LDK + pc * 8) = reg[n];
     }
     __syncthreads();
     if (t + 1 < t_hi) fetch(t + 1);
@@ -458,8 +491,9 @@ __global__ __launch_bounds__(256) void attn_latent_decode_kernel(LatentDecodeArg
       }
     }
   }
-  if (li >= Hl) return;
-  const long u = ((long)unit * a.n_split + blockIdx.y) * 16 + li;
+  const int h = h0 + li;
+  if (h >= a.H) return;
+  const long u = ((long)i * a.H + h) * a.n_split + blockIdx.y;
   if (wave == 0 && hi == 0) {
     a.pml[u * 2] = m2;
     a.pml[u * 2 + 1] = l;
@@ -470,83 +504,98 @@ __global__ __launch_bounds__(256) void attn_latent_decode_kernel(LatentDecodeArg
         acc[n];
 }
 
+// grid n_list * H: one row's head, folded over the splits, to bf16.
+template <int NS>  // splits at most
+__global__ __launch_bounds__(128) void latent_combine_kernel(
+    const float* __restrict__ pml, const float* __restrict__ pacc,
+    const float* __restrict__ sinks, unsigned short* __restrict__ o, int H,
+    int rp, int n_split) {
+  const long u = blockIdx.x, u0 = u * n_split;
+  float w[NS];
+  float mx = sinks ? sinks[u % H] * LOG2E : NEG_BIG;
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    w[i] = i < n_split ? pml[(u0 + i) * 2] : NEG_BIG;
+    mx = fmaxf(mx, w[i]);
+  }
+  float l = sinks ? fast_exp2(sinks[u % H] * LOG2E - mx) : 0.f;
+#pragma unroll
+  for (int i = 0; i < NS; ++i) {
+    w[i] = i < n_split ? fast_exp2(w[i] - mx) : 0.f;
+    if (i < n_split) l += pml[(u0 + i) * 2 + 1] * w[i];
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  for (int d = threadIdx.x * 4; d < rp; d += 512) {
+    f32x4 v[NS];
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      v[i] = i < n_split ? *reinterpret_cast<const f32x4*>(pacc + (u0 + i) * rp + d)
+                         : (f32x4){0.f, 0.f, 0.f, 0.f};
+    float s[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[r] += v[i][r] * w[i];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s[r] *= inv;
+    stv<4>(o + u * rp + d, s);
+  }
+}
+
 struct LatentOutputArgs {
-  const float* pml;
-  const float* pacc;
-  const float* sinks;        // (H,) or null
-  const unsigned short* wv;  // (H, vp, rp): W_uv, zero padded
+  const unsigned short* o;     // (n_list, H, rp)
+  const unsigned short* wv;    // (H, vp, rp): W_uv, zero padded
   const unsigned short* gate;  // row stride ldg, or null
   unsigned short* out;         // row stride ldo
   const int* cu;
   const int* list;
   long ldg, ldo;
-  int n_list, H, rp, vdim, vp, n_split;
+  int n_list, H, rp, vdim, vp;
 };
 
-// grid (vp / 64, H, rows / 16)
+// grid (vp / 64, H, rows / 32)
 __global__ __launch_bounds__(256) void latent_output_kernel(LatentOutputArgs a) {
-  extern __shared__ __attribute__((aligned(16))) unsigned short lds_o[];
-  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 16;
-  const int M = min(16, a.n_list - m0);
-  const int nch = (a.H + 15) / 16, c = h / 16, hl = h % 16;
-  const int ldr = a.rp + 8;
-  {
-    // 16 threads a row
-    const int m = tid / 16;
-    float f = 0.f, mx = NEG_BIG;
-    const long u0 = ((long)(m0 + m) * nch + c) * a.n_split;
-    if (m < M) {
-      float l = 0.f;
-      for (int i = 0; i < a.n_split; ++i)
-        mx = fmaxf(mx, a.pml[((u0 + i) * 16 + hl) * 2]);
-      for (int i = 0; i < a.n_split; ++i)
-        l += a.pml[((u0 + i) * 16 + hl) * 2 + 1] *
-             fast_exp2(a.pml[((u0 + i) * 16 + hl) * 2] - mx);
-      f = 1.f;
-      if (a.sinks) {
-        const float s2 = a.sinks[h] * LOG2E, mn = fmaxf(mx, s2);
-        f = fast_exp2(mx - mn);
-        l = l * f + fast_exp2(s2 - mn);
-      }
-      f = l > 0.f ? f / l : 0.f;
-    }
-    for (int d = tid % 16 * 4; d < a.rp; d += 64) {
-      float o[4] = {0.f, 0.f, 0.f, 0.f};
-      if (m < M) {
-        for (int i = 0; i < a.n_split; ++i) {
-          const float w = fast_exp2(a.pml[((u0 + i) * 16 + hl) * 2] - mx);
-          const f32x4 v = *reinterpret_cast<const f32x4*>(
-              a.pacc + ((u0 + i) * 16 + hl) * a.rp + d);
-#pragma unroll
-          for (int r = 0; r < 4; ++r) o[r] += v[r] * w;
-        }
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[r] *= f;
-      }
-      stv<4>(lds_o + m * ldr + d, o);
-    }
-  }
-  __syncthreads();
+  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 32;
+  const int M = min(32, a.n_list - m0);
   const int wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int n0 = blockIdx.x * 64 + wave * 16;
   const unsigned short* w = a.wv + ((long)h * a.vp + n0 + li) * a.rp + hi * 8;
-  f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < a.rp; k += 32) {
-    const bf16x8 wf = as_bf16x8(*reinterpret_cast<const short8*>(w + k));
-    const bf16x8 of = as_bf16x8(
-        *reinterpret_cast<const short8*>(lds_o + li * ldr + k + hi * 8));
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(of, wf, acc, 0, 0, 0);
+  const unsigned short* op[2];
+#pragma unroll
+  for (int m = 0; m < 2; ++m)
+    op[m] = a.o + ((long)(m0 + min(m * 16 + li, M - 1)) * a.H + h) * a.rp + hi * 8;
+  f32x4 acc[2];
+  acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < a.rp; k0 += 256) {
+    short8 wf[8], of[2][8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int k = k0 + u * 32;
+      const bool in = k < a.rp;
+      wf[u] = in ? *reinterpret_cast<const short8*>(w + k) : short8{};
+#pragma unroll
+      for (int m = 0; m < 2; ++m)
+        of[m][u] = in ? *reinterpret_cast<const short8*>(op[m] + k) : short8{};
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+#pragma unroll
+      for (int m = 0; m < 2; ++m)
+        acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            as_bf16x8(of[m][u]), as_bf16x8(wf[u]), acc[m], 0, 0, 0);
   }
   const int d = n0 + li;
   if (d >= a.vdim) return;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int m = hi * 4 + r;
-    if (m >= M) continue;
-    const long row = a.cu[a.list[m0 + m]];
-    float v = acc[r];
-    if (a.gate) v *= sigmoid_f(bf2f(a.gate[row * a.ldg + h * a.vdim + d]));
-    a.out[row * a.ldo + h * a.vdim + d] = cvt_bf(v);
-  }
+  for (int m = 0; m < 2; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = m * 16 + hi * 4 + r;
+      if (i >= M) continue;
+      const long row = a.cu[a.list[m0 + i]];
+      float v = acc[m][r];
+      if (a.gate) v *= sigmoid_f(bf2f(a.gate[row * a.ldg + h * a.vdim + d]));
+      a.out[row * a.ldo + h * a.vdim + d] = cvt_bf(v);
+    }
 }

@@ -214,41 +214,52 @@ struct GluArgs {
   const float* gb;    // (ff,) biases, or null
   const float* ub;
   void* out;          // (N, ldo), zero beyond ff
+  long N;
   int ks, ldp, g_off, u_off, ff, ldo;
   float limit, slope;
 };
 
 // g = min(gate, limit), u = clamp(up, -limit, limit):
-// out = g * sigmoid(slope * g) * (u + 1). grid (N, chunks of 256 * V columns)
-template <typename TP, typename T, int V>
+// out = g * sigmoid(slope * g) * (u + 1). grid (chunks of 256 * V columns,
+// groups of R rows): the biases of its columns stay in a thread's registers.
+template <typename TP, typename T, int V, int R>
 __global__ __launch_bounds__(256) void clamped_glu_kernel(GluArgs a) {
-  const long t = blockIdx.x;
-  const int i = (blockIdx.y * 256 + threadIdx.x) * V;
+  const int i = (blockIdx.x * 256 + threadIdx.x) * V;
   if (i >= a.ldo) return;
-  float g[V], u[V], w[V];
+  const bool live = i < a.ff;
+  float gb[V], ub[V];
 #pragma unroll
-  for (int j = 0; j < V; ++j) g[j] = 0.f;
-  if (i < a.ff) {
-    const TP* row = (const TP*)a.parts + t * (long)a.ldp;
-    ldv<V>(row + a.g_off + i, g);
-    ldv<V>(row + a.u_off + i, u);
-    for (int s = 1; s < a.ks; ++s) {
-      ldv<V>(row + s * a.pstride + a.g_off + i, w);
+  for (int j = 0; j < V; ++j) gb[j] = ub[j] = 0.f;
+  if (live && a.gb) ldv<V>(a.gb + i, gb);
+  if (live && a.ub) ldv<V>(a.ub + i, ub);
 #pragma unroll
-      for (int j = 0; j < V; ++j) g[j] += w[j];
-      ldv<V>(row + s * a.pstride + a.u_off + i, w);
+  for (int n = 0; n < R; ++n) {
+    const long t = blockIdx.y * R + n;
+    if (R > 1 && t >= a.N) return;
+    float g[V], u[V], w[V];
 #pragma unroll
-      for (int j = 0; j < V; ++j) u[j] += w[j];
+    for (int j = 0; j < V; ++j) g[j] = 0.f;
+    if (live) {
+      const TP* row = (const TP*)a.parts + t * (long)a.ldp;
+      ldv<V>(row + a.g_off + i, g);
+      ldv<V>(row + a.u_off + i, u);
+      for (int s = 1; s < a.ks; ++s) {
+        ldv<V>(row + s * a.pstride + a.g_off + i, w);
+#pragma unroll
+        for (int j = 0; j < V; ++j) g[j] += w[j];
+        ldv<V>(row + s * a.pstride + a.u_off + i, w);
+#pragma unroll
+        for (int j = 0; j < V; ++j) u[j] += w[j];
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float gj = fminf(g[j] + gb[j], a.limit);
+        const float uj = fminf(fmaxf(u[j] + ub[j], -a.limit), a.limit);
+        g[j] = gj * sigmoid_f(a.slope * gj) * (uj + 1.f);
+      }
     }
-#pragma unroll
-    for (int j = 0; j < V; ++j) {
-      const float gj = fminf(g[j] + (a.gb ? a.gb[i + j] : 0.f), a.limit);
-      const float uj = fminf(fmaxf(u[j] + (a.ub ? a.ub[i + j] : 0.f), -a.limit),
-                             a.limit);
-      g[j] = gj * sigmoid_f(a.slope * gj) * (uj + 1.f);
-    }
+    stv<V>((T*)a.out + t * (long)a.ldo + i, g);
   }
-  stv<V>((T*)a.out + t * (long)a.ldo + i, g);
 }
 
 __global__ __launch_bounds__(256) void softcap_kernel(float* __restrict__ z,
