@@ -84,7 +84,7 @@ void latent_post(Tensor y, std::vector<long> dims, double eps, Tensor qn,
   }
   if (N == 0) return;
   const bool vec = all_of_8({a.y.ld, a.q_off, a.q_rank, a.c_off, a.rank,
-                             a.g_off, a.gn});
+                             a.g_off, a.gn, a.ldq, a.rp, a.ck});
   const dim3 grid(N, 2 + (a.gn + 2047) / 2048);
   const size_t lds = 4 * (size_t)std::max(a.q_rank, a.rank);
   by_type(y.scalar_type(), [&](auto p) {
@@ -169,7 +169,7 @@ void latent_scatter(Tensor y, Tensor ctx, Tensor valid, long dim, long rot,
   a.k = (bf16_bits*)k.data_ptr();
   a.v = (bf16_bits*)v.data_ptr();
   if (npg == 0) return;
-  by_bool(all_of_8({a.ldy, dim, a.dkp}), [&](auto vec) {
+  by_bool(all_of_8({a.ldy, dim, vdim, a.dkp, a.dvp}), [&](auto vec) {
     latent_scatter_kernel<decltype(vec)::value ? 8 : 1>
         <<<dim3(npg, a.H), 256, 0, cur_stream()>>>(a);
   });
@@ -198,15 +198,17 @@ bool latent_decode_fits(long rp, long rtp) {
 
 // Listed one-token rows: query GEMM output y -> gated attention in out.
 void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
-                   Tensor tok_pos, Tensor cu, Tensor dec, long max_ctx,
+                   Tensor tok_pos, Tensor cu, Tensor q_start, Tensor dec,
+                   long max_ctx,
                    long dim, long rot, long rdims, long vdim, double scale,
                    long window, Tensor wk, Tensor wv, OptTensor sinks,
                    OptTensor gate, Tensor out) {
   for (const Tensor& t : {kp, wk, wv}) CHECK_T(t, at::kBFloat16);
-  for (const Tensor& t : {table, cu, dec}) CHECK_I32(t);
+  for (const Tensor& t : {table, cu, q_start, dec}) CHECK_I32(t);
   TORCH_CHECK(kp.dim() == 4 && kp.size(1) == 1 && wk.dim() == 3 &&
               wv.dim() == 3 && table.dim() == 2 &&
-              cu.numel() == table.size(0) + 1);
+              cu.numel() == table.size(0) + 1 &&
+              q_start.numel() == table.size(0));
   const long H = wk.size(0), rp = wk.size(1), ck = kp.size(3);
   TORCH_CHECK(latent_decode_fits(rp, ck - rp) && rot <= ck - rp);
   TORCH_CHECK(wk.size(2) % 32 == 0 && wk.size(2) >= dim && wv.size(0) == H &&
@@ -245,8 +247,7 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   a.q = (const bf16_bits*)q.data_ptr();
   a.kp = (const bf16_bits*)kp.data_ptr();
   a.table = table.data_ptr<int>();
-  a.tok_pos = qa.tok_pos;
-  a.cu = qa.cu;
+  a.q_start = q_start.data_ptr<int>();
   a.list = qa.list;
   a.H = (int)H;
   const int P = kp.size(2);
@@ -288,8 +289,8 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   by_bool(a.n_split > 4, [&](auto many) {
     latent_combine_kernel<decltype(many)::value ? 16 : 4>
         <<<n * H, 128, 0, cur_stream()>>>(a.pml, a.pacc, sp,
-                                          (bf16_bits*)olat.data_ptr(), (int)H,
-                                          (int)rp, a.n_split);
+                                          (bf16_bits*)olat.data_ptr(), (int)n,
+                                          (int)H, (int)rp, a.n_split);
   });
   check_launch();
   if (gate.has_value()) {
@@ -310,7 +311,7 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
   o.rp = (int)rp;
   o.vdim = (int)vdim;
   o.vp = wv.size(1);
-  latent_output_kernel<<<dim3(o.vp / 64, H, (n + 31) / 32), 256, 0,
+  latent_output_kernel<<<dim3(o.vp / 64, H, (n + 15) / 16), 256, 0,
                          cur_stream()>>>(o);
   check_launch();
 }
@@ -463,31 +464,37 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   a.qscale = (float)consts[0];
   a.inv_tau = (float)consts[1];
   a.eps = (float)consts[2];
+  const bool vec = all_of_8({a.ldy, a.q_off, a.k_off, a.v_off, a.g_off, a.dim,
+                             a.vdim, a.ldo});
   auto go = [&](auto dp, auto c) {
     constexpr int D = decltype(dp)::value, CC = decltype(c)::value;
-    auto prep = gla_prep_kernel<D, CC>;
-    const size_t l1 = prep_lds(D, CC, a.r);
-    allow_lds(prep, l1);
-    prep<<<dim3(chunks, a.H), 256, l1, cur_stream()>>>(a);
-    check_launch();
-    auto scan = gla_scan_kernel<D, CC>;
-    const size_t l2 = 4 * (2 * CC * (D + 8) + CC * 72 + 2 * D);
-    allow_lds(scan, l2);
-    scan<<<dim3((a.vdim + 63) / 64, a.H, list.numel()), 256, l2,
-           cur_stream()>>>(a);
-    check_launch();
-    auto fin = [&](auto nct) {
-      constexpr int N = decltype(nct)::value;
-      auto k = gla_out_kernel<D, CC, N>;
-      const size_t first = std::max(2 * CC * (D + 4), CC * (N * 128 + 8));
-      const size_t l3 = 2 * (first + 2 * CC * (D + 8) + 2 * CC * (CC + 8));
-      allow_lds(k, l3);
-      k<<<dim3(chunks, a.H), 512, l3, cur_stream()>>>(a);
+    by_bool(vec, [&](auto v) {
+      constexpr bool VEC = decltype(v)::value;
+      auto prep = gla_prep_kernel<D, CC, VEC>;
+      const size_t l1 = prep_lds(D, CC, a.r);
+      allow_lds(prep, l1);
+      prep<<<dim3(chunks, a.H), 256, l1, cur_stream()>>>(a);
       check_launch();
-    };
-    if (a.vdim <= 128) fin(std::integral_constant<int, 1>{});
-    else if (a.vdim <= 256) fin(std::integral_constant<int, 2>{});
-    else fin(std::integral_constant<int, 4>{});
+      auto scan = gla_scan_kernel<D, CC, VEC>;
+      const size_t l2 = 4 * (2 * CC * (D + 8) + CC * 72 + 2 * D);
+      allow_lds(scan, l2);
+      scan<<<dim3((a.vdim + 63) / 64, a.H, list.numel()), 256, l2,
+             cur_stream()>>>(a);
+      check_launch();
+      auto fin = [&](auto nct) {
+        constexpr int N = decltype(nct)::value;
+        auto k = gla_out_kernel<D, CC, N, VEC>;
+        const size_t first =
+            std::max(2 * (CC + 1) * (D + 4), CC * (N * 128 + 8));
+        const size_t l3 = 2 * (first + 2 * CC * (D + 8) + 2 * CC * (CC + 8));
+        allow_lds(k, l3);
+        k<<<dim3(chunks, a.H), 512, l3, cur_stream()>>>(a);
+        check_launch();
+      };
+      if (a.vdim <= 128) fin(std::integral_constant<int, 1>{});
+      else if (a.vdim <= 256) fin(std::integral_constant<int, 2>{});
+      else fin(std::integral_constant<int, 4>{});
+    });
   };
   using I32 = std::integral_constant<int, 32>;
   using I64 = std::integral_constant<int, 64>;

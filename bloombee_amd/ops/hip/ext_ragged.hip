@@ -396,7 +396,7 @@ static void launch_mfma(AttnArgs& a, const Tensor& pre, const Tensor& dec,
                         long max_new, long max_ctx, const Tensor& like) {
   const int Hg = a.H / a.G;
   if (pre.numel() > 0) {
-    constexpr int QC = (DK > 192 || DV > 128) ? 1 : 2;
+    constexpr int QC = (DK > 128 || DV > 128) ? 1 : 2;
     a.list = pre.data_ptr<int>();
     const long rows = max_new * Hg;
     attn_ragged_prefill_kernel<DK, DV, QC>

@@ -182,40 +182,44 @@ DEVINL void split8(const float* v, short8& hi, short8& lo) {
   }
 }
 
-// Eight channels of token t's q or k (columns off ..); zero beyond the chunk's
-// tokens and the head's channels.
-DEVINL void load_channels(const GlaChunkArgs& a, long row0, int len, int off,
-                          int h, int t, int d, float* v) {
-  if (t < len && d < a.dim) {
-    const unsigned short* p = a.y + (row0 + t) * a.ldy + off + h * a.dim + d;
-    if (d + 8 <= a.dim && ((a.ldy | (off + h * a.dim)) & 7) == 0) {
-      load_bf16x8(p, v);
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = d + j < a.dim ? bf2f(p[j]) : 0.f;
-    }
+// Eight columns c.. of a head of n columns in row `row`, zero where !live and
+// beyond n. VEC: n is a multiple of 8 and rows are aligned. Addresses are
+// clamped, so that nothing branches.
+template <bool VEC>
+DEVINL short8 load_row8(const unsigned short* row, int c, int n, bool live) {
+  short8 v;
+  if constexpr (VEC) {
+    v = *reinterpret_cast<const short8*>(row + min(c, n - 8));
+    return live && c < n ? v : short8{};
   } else {
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = 0.f;
+    for (int j = 0; j < 8; ++j) v[j] = (short)row[min(c + j, n - 1)];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = live && c + j < n ? v[j] : (short)0;
+    return v;
   }
 }
 
-// Eight value columns of a token as bits; zero beyond the head's.
-DEVINL short8 load_values(const GlaChunkArgs& a, long row, int h, int c, bool vec) {
-  short8 v = short8{};
-  const unsigned short* p = a.y + row * a.ldy + a.v_off + h * a.vdim + c;
-  if (vec && c + 8 <= a.vdim) {
-    v = *reinterpret_cast<const short8*>(p);
-  } else {
+// Eight channels of token t's q or k (columns off ..).
+template <bool VEC>
+DEVINL void load_channels(const GlaChunkArgs& a, long row0, int len, int off,
+                          int h, int t, int d, float* v) {
+  const short8 u = load_row8<VEC>(
+      a.y + (row0 + min(t, len - 1)) * a.ldy + off + h * a.dim, d, a.dim, t < len);
 #pragma unroll
-    for (int j = 0; j < 8; ++j)
-      if (c + j < a.vdim) v[j] = (short)p[j];
-  }
-  return v;
+  for (int j = 0; j < 8; ++j) v[j] = bf2f((unsigned short)u[j]);
+}
+
+// Eight value columns of token t.
+template <bool VEC>
+DEVINL short8 load_values(const GlaChunkArgs& a, long row0, int len, int h, int t,
+                          int c) {
+  return load_row8<VEC>(a.y + (row0 + min(t, len - 1)) * a.ldy + a.v_off +
+                            h * a.vdim, c, a.vdim, t < len);
 }
 
 // grid (chunks, H). LDS: b (C x (DP + 4)), a1 (C x r), a2 of the head (r x DP)
-template <int DP, int C>
+template <int DP, int C, bool VEC>
 __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
   constexpr int LDB = DP + 4;
   extern __shared__ __attribute__((aligned(16))) float lds_b[];
@@ -254,10 +258,12 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
     }
   }
   __syncthreads();
-  for (int idx = tid; idx < C * DP / 8; idx += 256) {
+#pragma unroll
+  for (int n = 0; n < C * DP / 8 / 256; ++n) {
+    const int idx = tid + n * 256;
     const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
     float k[8], b[8];
-    load_channels(a, row0, len, a.k_off, h, t, d, k);
+    load_channels<VEC>(a, row0, len, a.k_off, h, t, d, k);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       b[j] = lds_b[t * LDB + d + j];
@@ -277,7 +283,7 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
 //     tile 2g + n, row x*4 + y  <->  channel g*32 + x*8 + n*4 + y
 // so that a lane's registers of two tiles are eight consecutive channels: an
 // operand fragment as it is.
-template <int DP, int C>
+template <int DP, int C, bool VEC>
 __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
   constexpr int NG = DP / 32, NC = C / 32;
   constexpr int LDD = DP + 8, LDV = 64 + 8;
@@ -294,20 +300,25 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
   const int col = v0 + wave * 16 + li;
   const bool live = col < a.vdim;
   float* S = a.state + ((long)a.slots[s] * a.H + h) * a.dim * a.vdim;
-  const bool vvec = ((a.vdim | a.ldy | a.v_off) & 7) == 0;
 
   f32x4 acc[2 * NG];
-  const bool fresh = a.q_start[s] == 0;
+  const bool kept = a.q_start[s] != 0 && live;
 #pragma unroll
-  for (int g = 0; g < NG; ++g)
+  for (int n = 0; n < 2 * NG; ++n)
 #pragma unroll
-    for (int n = 0; n < 2; ++n)
+    for (int r = 0; r < 4; ++r)
+      acc[n][r] = S[(long)min((n >> 1) * 32 + hi * 8 + (n & 1) * 4 + r, a.dim - 1) *
+                        a.vdim + min(col, a.vdim - 1)];
+  // all loads first, then the choice: else each waits behind a branch
+  __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = g * 32 + hi * 8 + n * 4 + r;
-        acc[2 * g + n][r] =
-            !fresh && live && d < a.dim ? S[(long)d * a.vdim + col] : 0.f;
-      }
+  for (int n = 0; n < 2 * NG; ++n) asm volatile("" : "+v"(acc[n]));
+#pragma unroll
+  for (int n = 0; n < 2 * NG; ++n)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (!kept || (n >> 1) * 32 + hi * 8 + (n & 1) * 4 + r >= a.dim)
+        acc[n][r] = 0.f;
 
   short8 rk[2][PD], rv[PV];
   float rd = 0.f;
@@ -323,11 +334,10 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
     const int len = a.len[ch];
 #pragma unroll
     for (int n = 0; n < PV; ++n) {
-      const int idx = tid + n * 256, t = idx / 8;
-      rv[n] = short8{};
-      if (t < len) rv[n] = load_values(a, row0 + t, h, v0 + idx % 8 * 8, vvec);
+      const int idx = tid + n * 256;
+      rv[n] = load_values<VEC>(a, row0, len, h, idx / 8, v0 + idx % 8 * 8);
     }
-    if (tid < DP) rd = a.b[(base * C + C - 1) * DP + tid];
+    rd = a.b[(base * C + C - 1) * DP + tid % DP];
   };
   auto stage = [&](unsigned short* buf) {
 #pragma unroll
@@ -414,16 +424,21 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
 // grid (chunks, H), eight waves; a wave owns every eighth tile of 16 value
 // columns. Outputs are made transposed, o^T = S^T qd^T + v^T A^T: a lane holds
 // four consecutive columns of one token. LDS: b, later v; qd; A.
-template <int DP, int C, int NCT>
+template <int DP, int C, int NCT, bool VEC>
 __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   constexpr int LDB = DP + 4, LDD = DP + 8, LDA = C + 8, NG = DP / 32;
   constexpr int NT = C / 16, NC = C / 32, NB = C / 16, VC = NCT * 128;
   constexpr int LDV = VC + 8;
-  constexpr int FIRST = 2 * C * LDB > C * LDV ? 2 * C * LDB : C * LDV;
+  constexpr int FIRST = 2 * (C + 1) * LDB > C * LDV ? 2 * (C + 1) * LDB : C * LDV;
+  constexpr int PB = C * DP / 4 / 512, PQ = C * DP / 8 / 512 > 0 ? C * DP / 8 / 512 : 1;
+  constexpr int PV = C * VC / 8 / 512;
+  // the states, too, are asked for ahead, where there are registers for them
+  constexpr bool EARLY = VEC && NCT * NG <= 8;
+  constexpr int NS = EARLY ? NCT : 1;
   constexpr float SPAN = 80.f;  // widest safe range of exponents, log2
   extern __shared__ __attribute__((aligned(16))) unsigned short lds_out[];
   __shared__ float ssum[8][C];
-  float* bs = (float*)lds_out;               // (C, LDB)
+  float* bs = (float*)lds_out + LDB;         // (C, LDB), a zero row ahead
   unsigned short* vs = lds_out;              // (C, LDV)
   unsigned short* qs = lds_out + FIRST;      // (2, C, LDD)
   unsigned short* as = qs + 2 * C * LDD;     // (2, C, LDA)
@@ -434,20 +449,56 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   const long row0 = a.row0[ch], base = (long)ch * a.H + h;
   const int len = a.len[ch];
 
-  for (int idx = tid; idx < C * DP / 4; idx += 512) {
-    const int t = idx / (DP / 4), d = idx % (DP / 4) * 4;
-    *reinterpret_cast<f32x4*>(bs + t * LDB + d) =
-        *reinterpret_cast<const f32x4*>(a.b + (base * C + t) * DP + d);
-  }
-  __syncthreads();
-  for (int idx = tid; idx < C * DP / 8; idx += 512) {
-    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
-    float q[8];
-    load_channels(a, row0, len, a.q_off, h, t, d, q);
+  // everything that comes from memory is asked for up front
+  f32x4 rb[PB];
+  float rq[PQ][8];
+  short8 rv[PV];
+  bf16x8 sh[NS][NG], sl[NS][NG];
+  auto load_state = [&](int c, bf16x8 (&u)[NG], bf16x8 (&v)[NG]) {
+    // waves beyond the last tile read that one again and drop what they make
+    const int vt = min(c * 8 + wave, a.VT - 1);
+    const unsigned short* sp = a.S + ((base * a.VT + vt) * 2 * NG) * 512 + lane * 8;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) q[j] *= a.qscale * fast_exp2(bs[t * LDB + d + j]);
+    for (int g = 0; g < NG; ++g) {
+      u[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + g * 512));
+      v[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + (NG + g) * 512));
+    }
+  };
+#pragma unroll
+  for (int n = 0; n < PB; ++n)
+    rb[n] = *reinterpret_cast<const f32x4*>(a.b + base * C * DP + (tid + n * 512) * 4);
+#pragma unroll
+  for (int n = 0; n < PQ; ++n) {
+    const int idx = min(tid + n * 512, C * DP / 8 - 1);
+    load_channels<VEC>(a, row0, len, a.q_off, h, idx / (DP / 8),
+                       idx % (DP / 8) * 8, rq[n]);
+  }
+#pragma unroll
+  for (int n = 0; n < PV; ++n) {
+    const int idx = tid + n * 512;
+    rv[n] = load_values<VEC>(a, row0, len, h, idx / (VC / 8), idx % (VC / 8) * 8);
+  }
+  if constexpr (EARLY) {
+#pragma unroll
+    for (int c = 0; c < NCT; ++c) load_state(c, sh[c], sl[c]);
+  }
+#pragma unroll
+  for (int n = 0; n < PB; ++n) {
+    const int idx = tid + n * 512;
+    *reinterpret_cast<f32x4*>(bs + idx / (DP / 4) * LDB + idx % (DP / 4) * 4) = rb[n];
+  }
+  if (tid < DP) bs[tid - LDB] = 0.f;
+  __syncthreads();
+#pragma unroll
+  for (int n = 0; n < PQ; ++n) {
+    const int idx = tid + n * 512;
+    if (idx >= C * DP / 8) continue;
+    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      rq[n][j] *= a.qscale * fast_exp2(bs[t * LDB + d + j]);
     short8 vh, vl;
-    split8(q, vh, vl);
+    split8(rq[n], vh, vl);
     *reinterpret_cast<short8*>(qs + t * LDD + d) = vh;
     *reinterpret_cast<short8*>(qs + (C + t) * LDD + d) = vl;
   }
@@ -458,28 +509,30 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
       const float* ref = bs + (I * 16 - 1) * LDB;  // row before block I
       bool near = true;
       if (J == I) {
-        for (int d = lane; d < DP; d += WAVE) {
-          const float r = I > 0 ? ref[d] : 0.f;
-          near = near && r - bs[(I * 16 + 15) * LDB + d] <= SPAN;
-        }
+        for (int d = lane; d < DP; d += WAVE)
+          near = near && ref[d] - bs[(I * 16 + 15) * LDB + d] <= SPAN;
         near = __builtin_amdgcn_ballot_w64(!near) == 0;
       }
       if (near) {
+        const int t = I * 16 + li, s = J * 16 + li;
+        float q[NG][8], k[NG][8];
 #pragma unroll
         for (int kk = 0; kk < NG; ++kk) {
-          const int d = kk * 32 + hi * 8, t = I * 16 + li, s = J * 16 + li;
-          float q[8], k[8];
-          load_channels(a, row0, len, a.q_off, h, t, d, q);
-          load_channels(a, row0, len, a.k_off, h, s, d, k);
+          load_channels<VEC>(a, row0, len, a.q_off, h, t, kk * 32 + hi * 8, q[kk]);
+          load_channels<VEC>(a, row0, len, a.k_off, h, s, kk * 32 + hi * 8, k[kk]);
+        }
+#pragma unroll
+        for (int kk = 0; kk < NG; ++kk) {
+          const int d = kk * 32 + hi * 8;
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
-            const float r = I > 0 ? ref[d + j] : 0.f;
-            q[j] *= a.qscale * fast_exp2(bs[t * LDB + d + j] - r);
-            k[j] *= fast_exp2(r - bs[s * LDB + d + j]);
+            const float r = ref[d + j];
+            q[kk][j] *= a.qscale * fast_exp2(bs[t * LDB + d + j] - r);
+            k[kk][j] *= fast_exp2(r - bs[s * LDB + d + j]);
           }
           short8 qh, ql, kh, kl;
-          split8(q, qh, ql);
-          split8(k, kh, kl);
+          split8(q[kk], qh, ql);
+          split8(k[kk], kh, kl);
           acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
               as_bf16x8(qh), as_bf16x8(kh), acc, 0, 0, 0);
           acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
@@ -514,14 +567,10 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
     }
   }
   __syncthreads();   // b is read
-  {
-    const bool vec = ((a.vdim | a.ldy | a.v_off) & 7) == 0;
-    for (int idx = tid; idx < C * VC / 8; idx += 512) {
-      const int t = idx / (VC / 8), c = idx % (VC / 8) * 8;
-      short8 v = short8{};
-      if (t < len && c < a.vdim) v = load_values(a, row0 + t, h, c, vec);
-      *reinterpret_cast<short8*>(vs + t * LDV + c) = v;
-    }
+#pragma unroll
+  for (int n = 0; n < PV; ++n) {
+    const int idx = tid + n * 512;
+    *reinterpret_cast<short8*>(vs + idx / (VC / 8) * LDV + idx % (VC / 8) * 8) = rv[n];
   }
   __syncthreads();
 
@@ -532,13 +581,8 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
     for (int t = 0; t < NT; ++t) o[c][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
     const int vt = c * 8 + wave;
     if (vt >= a.VT) continue;
-    const unsigned short* sp = a.S + ((base * a.VT + vt) * 2 * NG) * 512 + lane * 8;
-    bf16x8 sh[NG], sl[NG];
-#pragma unroll
-    for (int g = 0; g < NG; ++g) {
-      sh[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + g * 512));
-      sl[g] = as_bf16x8(*reinterpret_cast<const short8*>(sp + (NG + g) * 512));
-    }
+    const int cs = EARLY ? c : 0;
+    if constexpr (!EARLY) load_state(c, sh[0], sl[0]);
 #pragma unroll
     for (int k = 0; k < NC; ++k) {
       const bf16x8 vf = column_frag(vs, LDV, k * 32, vt * 16 + (li & 3) * 4, li, hi);
@@ -561,9 +605,9 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
             qs + (t * 16 + li) * LDD + g * 32 + hi * 8));
         const bf16x8 ql = as_bf16x8(*reinterpret_cast<const short8*>(
             qs + (C + t * 16 + li) * LDD + g * 32 + hi * 8));
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[g], qh, o[c][t], 0, 0, 0);
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[g], ql, o[c][t], 0, 0, 0);
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[g], qh, o[c][t], 0, 0, 0);
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[cs][g], qh, o[c][t], 0, 0, 0);
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[cs][g], ql, o[c][t], 0, 0, 0);
+        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[cs][g], qh, o[c][t], 0, 0, 0);
       }
   }
   // columns beyond vdim are zero: they add nothing
@@ -579,7 +623,6 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
     if (hi == 0) ssum[wave][t * 16 + li] = ss;
   }
   __syncthreads();
-  const bool vec = ((a.vdim | a.ldy | a.g_off | (int)a.ldo) & 3) == 0;
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
     const int tt = t * 16 + li;
@@ -594,7 +637,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
     for (int c = 0; c < NCT; ++c) {
       const int v0 = (c * 8 + wave) * 16 + hi * 4;
       if (v0 >= a.vdim) continue;
-      if (vec) {
+      if constexpr (VEC) {
         float g[4], w[4];
         ldv<4>(gp + v0, g);
         ldv<4>(a.nw + v0, w);

@@ -84,6 +84,23 @@ DEVINL float stage_norm(const Parts& y, long t, int off, int n, float eps,
   return 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)n + eps);
 }
 
+// o[0..cols) = x * inv * w, zero from n on; n and cols are multiples of V.
+template <typename T, int V>
+DEVINL void scale_row(T* o, const float* x, const float* w, float inv, int n,
+                      int cols) {
+  for (int i = threadIdx.x * V; i < cols; i += 256 * V) {
+    float v[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    if (i < n) {
+      ldv<V>(w + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] *= x[i + j] * inv;
+    }
+    stv<V>(o + i, v);
+  }
+}
+
 // grid (N, 2 + gate chunks of 2048): y = 0 query latent, 1 page slot, 2.. gate
 template <typename TP, typename T, int V>
 __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
@@ -94,9 +111,8 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
   if (blockIdx.y == 0) {
     const float inv = stage_norm<TP, V>(a.y, t, a.q_off, a.q_rank, a.eps,
                                         lds_sec, red);
-    T* o = (T*)a.cq + t * (long)a.ldq;
-    for (int i = tid; i < a.ldq; i += 256)
-      stf(o + i, i < a.q_rank ? lds_sec[i] * inv * a.qn[i] : 0.f);
+    scale_row<T, V>((T*)a.cq + t * (long)a.ldq, lds_sec, a.qn, inv, a.q_rank,
+                    a.ldq);
     return;
   }
   if (blockIdx.y == 1) {
@@ -106,8 +122,7 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
                                         lds_sec, red);
     const long page = a.table[(long)a.tok_seq[t] * a.maxp + pos / a.P];
     T* o = (T*)a.kp + (page * a.P + pos % a.P) * a.ck;
-    for (int i = tid; i < a.rp; i += 256)
-      stf(o + i, i < a.rank ? lds_sec[i] * inv * a.cn[i] : 0.f);
+    scale_row<T, V>(o, lds_sec, a.cn, inv, a.rank, a.rp);
     const int half = a.rdims / 2;
     for (int i = tid; i < a.ck - a.rp; i += 256) {
       float v[1] = {0.f};
@@ -284,7 +299,7 @@ struct LatentScatterArgs {
   int ldy, H, dim, rot, vdim, rp, ck, dkp, dvp, P;
 };
 
-// grid (npg, H)
+// grid (npg, H). V = 8: sizes are multiples of it.
 template <int V>
 __global__ __launch_bounds__(256) void latent_scatter_kernel(LatentScatterArgs a) {
   const long pg = blockIdx.x;
@@ -312,14 +327,34 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(LatentScatterArgs a
   }
   unsigned short* vo = a.v + (pg * a.H + h) * (long)a.dvp * a.P;
   const unsigned short* vy = y + a.H * a.dim + h * a.vdim;
-  for (int idx = tid; idx < a.dvp * (a.P / 8); idx += 256) {
-    const int d = idx % a.dvp, r0 = idx / a.dvp * 8;
-    short8 o = short8{};
-    if (d < a.vdim)
+  if constexpr (V == 8) {
+    // 8 x 8 blocks, turned in a lane's registers
+    for (int idx = tid; idx < a.dvp / 8 * (a.P / 8); idx += 256) {
+      const int d = idx % (a.dvp / 8) * 8, r0 = idx / (a.dvp / 8) * 8;
+      short8 in[8];
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        if (r0 + j < n) o[j] = (short)vy[(long)(r0 + j) * a.ldy + d];
-    *reinterpret_cast<short8*>(vo + (long)d * a.P + r0) = o;
+        in[j] = r0 + j < n && d < a.vdim
+                    ? *reinterpret_cast<const short8*>(vy + (long)(r0 + j) * a.ldy + d)
+                    : short8{};
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        short8 o;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) o[j] = in[j][e];
+        *reinterpret_cast<short8*>(vo + (long)(d + e) * a.P + r0) = o;
+      }
+    }
+  } else {
+    for (int idx = tid; idx < a.dvp * (a.P / 8); idx += 256) {
+      const int d = idx % a.dvp, r0 = idx / a.dvp * 8;
+      short8 o = short8{};
+      if (d < a.vdim)
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          if (r0 + j < n) o[j] = (short)vy[(long)(r0 + j) * a.ldy + d];
+      *reinterpret_cast<short8*>(vo + (long)d * a.P + r0) = o;
+    }
   }
 }
 
@@ -327,8 +362,7 @@ struct LatentDecodeArgs {
   const unsigned short* q;   // (n_list, H, ck)
   const unsigned short* kp;  // (np, 1, P, ck)
   const int* table;
-  const int* tok_pos;
-  const int* cu;
+  const int* q_start;        // (S,) position of a listed sequence's one token
   const int* list;
   float* pml;   // (n_list, H, n_split, 2): max (log2 units) and sum
   float* pacc;  // (n_list, H, n_split, rp)
@@ -381,39 +415,28 @@ __global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
   const int unit = blockIdx.x, i = unit / nch;
   const int h0 = unit % nch * 16 * HG + grp * 16;
   const int s = a.list[i];
-  const int pos = a.tok_pos[a.cu[s]];
+  const int pos = a.q_start[s];
   const int lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int* table = a.table + (long)s * a.maxp;
 
-  bf16x8 qf[NKK];
-  const unsigned short* qp =
-      a.q + ((long)i * a.H + min(h0 + li, a.H - 1)) * CK + hi * 8;
-#pragma unroll
-  for (int kk = 0; kk < NKK; ++kk)
-    qf[kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
-
   const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
   const int t_beg = lo / KT;
   const int t_all = pos < 0 ? 0 : pos / KT + 1 - t_beg;
-  const int per = (t_all + a.n_split - 1) / a.n_split;
-  const int t_lo = t_beg + blockIdx.y * per;
-  const int t_hi = min(t_beg + t_all, t_lo + per);
+  const int t_lo = t_beg + t_all * blockIdx.y / a.n_split;
+  const int t_hi = t_beg + t_all * (blockIdx.y + 1) / a.n_split;
 
-  float m2 = NEG_BIG, l = 0.f;
-  f32x4 acc[ND];
-#pragma unroll
-  for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  const float sc2 = a.scale * LOG2E;
-
-  // a thread stages pieces piece, piece + LANES, .. of one row of the tile
+  // a thread stages pieces piece, piece + LANES, .. of one row of the tile; the
+  // row's page is looked up a tile ahead
   const int srow = tid / LANES, piece = tid % LANES;
   short8 reg[NP];
-  auto fetch = [&](int t) {
+  auto page_of = [&](int t) {
+    return table[min(t * KT + srow, max(pos, 0)) >> a.p_log2];
+  };
+  auto fetch = [&](int t, int page) {
     const int key = min(t * KT + srow, pos);
     const unsigned short* kp =
-        a.kp + (((long)table[key >> a.p_log2] << a.p_log2) +
-                (key & ((1 << a.p_log2) - 1))) * CK;
+        a.kp + (((long)page << a.p_log2) + (key & ((1 << a.p_log2) - 1))) * CK;
 #pragma unroll
     for (int n = 0; n < NP; ++n) {
       const int pc = piece + n * LANES;
@@ -421,7 +444,29 @@ __global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
         reg[n] = *reinterpret_cast<const short8*>(kp + pc * 8);
     }
   };
-  if (t_lo < t_hi) fetch(t_lo);
+  int page = page_of(t_lo);
+  if (t_lo < t_hi) {
+    fetch(t_lo, page);
+    page = page_of(t_lo + 1);
+  }
+
+  bf16x8 qf[NKK];
+  const unsigned short* qp =
+      a.q + ((long)i * a.H + min(h0 + li, a.H - 1)) * CK + hi * 8;
+#pragma unroll
+  for (int kk = 0; kk < NKK; ++kk)
+    qf[kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
+  // the queries arrive here: else the waits for them sit in the loop and take
+  // the next tile's loads along
+#pragma unroll
+  for (int kk = 0; kk < NKK; ++kk) asm volatile("" : "+v"(qf[kk]));
+
+  float m2 = NEG_BIG, l = 0.f;
+  f32x4 acc[ND];
+#pragma unroll
+  for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  const float sc2 = a.scale * LOG2E;
+
   for (int t = t_lo; t < t_hi; ++t) {
     __syncthreads();  // the last tile is read
 #pragma unroll
@@ -431,28 +476,45 @@ __global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
         *reinterpret_cast<short8*>(kt + srow * LDK + pc * 8) = reg[n];
     }
     __syncthreads();
-    if (t + 1 < t_hi) fetch(t + 1);
-    f32x4 st = (f32x4){0.f, 0.f, 0.f, 0.f};
+    if (t + 1 < t_hi) {
+      fetch(t + 1, page);
+      page = page_of(t + 2);
+    }
+    f32x4 st[2];  // two chains
+    st[0] = st[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int kk = 0; kk < NKK; ++kk) {
       const bf16x8 kf = as_bf16x8(*reinterpret_cast<const short8*>(
           kt + (wave * 16 + li) * LDK + kk * 32 + hi * 8));
-      st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[kk], st, 0, 0, 0);
+      st[kk & 1] =
+          __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[kk], st[kk & 1], 0, 0, 0);
     }
-    *reinterpret_cast<f32x4*>(sc + li * LDS_S + wave * 16 + hi * 4) = st;
+    *reinterpret_cast<f32x4*>(sc + li * LDS_S + wave * 16 + hi * 4) =
+        st[0] + st[1];
     __syncthreads();
     // every wave takes the softmax of the whole tile
     float p[2][8];
     float rm = NEG_BIG;
 #pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(
+          sc + li * LDS_S + (q >> 1) * 32 + hi * 8 + (q & 1) * 4);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) p[q >> 1][(q & 1) * 4 + r] = v[r] * sc2;
+    }
+    if (t * KT < lo || t * KT + KT - 1 > pos) {
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const int key = t * KT + hf * 32 + hi * 8 + j;
+          if (key < lo || key > pos) p[hf][j] = NEG_BIG;
+        }
+    }
+#pragma unroll
     for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int key = t * KT + hf * 32 + hi * 8 + j;
-        const float v = sc[li * LDS_S + hf * 32 + hi * 8 + j] * sc2;
-        p[hf][j] = (key < lo || key > pos) ? NEG_BIG : v;
-        rm = fmaxf(rm, p[hf][j]);
-      }
+      for (int j = 0; j < 8; ++j) rm = fmaxf(rm, p[hf][j]);
     rm = fmaxf(rm, __shfl_xor(rm, 16));
     rm = fmaxf(rm, __shfl_xor(rm, 32));
     const float mn = fmaxf(m2, rm);  // every tile has a visible key
@@ -504,12 +566,12 @@ __global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
         acc[n];
 }
 
-// grid n_list * H: one row's head, folded over the splits, to bf16.
+// grid n_list * H: one row's head, folded over the splits, to bf16 (H, n, rp).
 template <int NS>  // splits at most
 __global__ __launch_bounds__(128) void latent_combine_kernel(
     const float* __restrict__ pml, const float* __restrict__ pacc,
-    const float* __restrict__ sinks, unsigned short* __restrict__ o, int H,
-    int rp, int n_split) {
+    const float* __restrict__ sinks, unsigned short* __restrict__ o, int n,
+    int H, int rp, int n_split) {
   const long u = blockIdx.x, u0 = u * n_split;
   float w[NS];
   float mx = sinks ? sinks[u % H] * LOG2E : NEG_BIG;
@@ -538,12 +600,12 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
       for (int r = 0; r < 4; ++r) s[r] += v[i][r] * w[i];
 #pragma unroll
     for (int r = 0; r < 4; ++r) s[r] *= inv;
-    stv<4>(o + u * rp + d, s);
+    stv<4>(o + (u % H * n + u / H) * rp + d, s);
   }
 }
 
 struct LatentOutputArgs {
-  const unsigned short* o;     // (n_list, H, rp)
+  const unsigned short* o;     // (H, n_list, rp)
   const unsigned short* wv;    // (H, vp, rp): W_uv, zero padded
   const unsigned short* gate;  // row stride ldg, or null
   unsigned short* out;         // row stride ldo
@@ -553,49 +615,45 @@ struct LatentOutputArgs {
   int n_list, H, rp, vdim, vp;
 };
 
-// grid (vp / 64, H, rows / 32)
+// grid (vp / 64, H, rows / 16)
 __global__ __launch_bounds__(256) void latent_output_kernel(LatentOutputArgs a) {
-  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 32;
-  const int M = min(32, a.n_list - m0);
+  const int tid = threadIdx.x, h = blockIdx.y, m0 = blockIdx.z * 16;
+  const int M = min(16, a.n_list - m0);
   const int wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
-  const int n0 = blockIdx.x * 64 + wave * 16;
-  const unsigned short* w = a.wv + ((long)h * a.vp + n0 + li) * a.rp + hi * 8;
-  const unsigned short* op[2];
+  const int n0 = blockIdx.x * 64 + wave * 16, d = n0 + li;
+  // what the epilogue needs is looked up while the product runs
+  long row[4];
+  float g[4];
 #pragma unroll
-  for (int m = 0; m < 2; ++m)
-    op[m] = a.o + ((long)(m0 + min(m * 16 + li, M - 1)) * a.H + h) * a.rp + hi * 8;
-  f32x4 acc[2];
-  acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int r = 0; r < 4; ++r) {
+    row[r] = a.cu[a.list[m0 + min(hi * 4 + r, M - 1)]];
+    g[r] = a.gate && d < a.vdim ? bf2f(a.gate[row[r] * a.ldg + h * a.vdim + d])
+                                : 0.f;
+  }
+  const unsigned short* w = a.wv + ((long)h * a.vp + n0 + li) * a.rp + hi * 8;
+  const unsigned short* op =
+      a.o + ((long)h * a.n_list + m0 + min(li, M - 1)) * a.rp + hi * 8;
+  f32x4 acc = (f32x4){0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < a.rp; k0 += 256) {
-    short8 wf[8], of[2][8];
+    short8 wf[8], of[8];
 #pragma unroll
     for (int u = 0; u < 8; ++u) {
       const int k = k0 + u * 32;
       const bool in = k < a.rp;
       wf[u] = in ? *reinterpret_cast<const short8*>(w + k) : short8{};
-#pragma unroll
-      for (int m = 0; m < 2; ++m)
-        of[m][u] = in ? *reinterpret_cast<const short8*>(op[m] + k) : short8{};
+      of[u] = in ? *reinterpret_cast<const short8*>(op + k) : short8{};
     }
 #pragma unroll
     for (int u = 0; u < 8; ++u)
-#pragma unroll
-      for (int m = 0; m < 2; ++m)
-        acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            as_bf16x8(of[m][u]), as_bf16x8(wf[u]), acc[m], 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(of[u]),
+                                                    as_bf16x8(wf[u]), acc, 0, 0, 0);
   }
-  const int d = n0 + li;
   if (d >= a.vdim) return;
 #pragma unroll
-  for (int m = 0; m < 2; ++m)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int i = m * 16 + hi * 4 + r;
-      if (i >= M) continue;
-      const long row = a.cu[a.list[m0 + i]];
-      float v = acc[m][r];
-      if (a.gate) v *= sigmoid_f(bf2f(a.gate[row * a.ldg + h * a.vdim + d]));
-      a.out[row * a.ldo + h * a.vdim + d] = cvt_bf(v);
-    }
+  for (int r = 0; r < 4; ++r) {
+    if (hi * 4 + r >= M) continue;
+    const float v = a.gate ? acc[r] * sigmoid_f(g[r]) : acc[r];
+    a.out[row[r] * a.ldo + h * a.vdim + d] = cvt_bf(v);
+  }
 }

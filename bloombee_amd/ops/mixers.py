@@ -203,7 +203,7 @@ def latent_attention(parts: torch.Tensor, spec: LatentSpec, w: LatentWeights,
     if batch.dec_list.numel():
         _ext().latent_decode(
             parts, turns, pages, batch.page_table, batch.tok_pos, batch.cu,
-            batch.dec_list, batch.max_ctx, s.dim, s.rot, s.rot_dims, s.vdim,
+            batch.q_start, batch.dec_list, batch.max_ctx, s.dim, s.rot, s.rot_dims, s.vdim,
             s.scale, s.window, w.uk, w.uv, w.sink, gate, out)
     if batch.pre_list.numel():
         ctx = batch.context(s.window)
