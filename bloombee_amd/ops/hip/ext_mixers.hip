@@ -181,7 +181,7 @@ static void launch_decode(LatentDecodeArgs& a, long n) {
   constexpr int CK = ND * 64 + NR * 32;
   by_bool(a.H > 16, [&](auto two) {
     constexpr int HG = decltype(two)::value ? 2 : 1;
-    constexpr size_t lds = 64 * (CK + 8) * 2 + HG * 16 * 68 * 4;
+    constexpr size_t lds = 64 * latent_tile_ld(CK) * 2 + HG * 16 * 68 * 4;
     auto k = attn_latent_decode_kernel<ND, NR, HG>;
     allow_lds(k, lds);
     const long units = n * ((a.H + 16 * HG - 1) / (16 * HG));
@@ -476,7 +476,8 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
       prep<<<dim3(chunks, a.H), 256, l1, cur_stream()>>>(a);
       check_launch();
       auto scan = gla_scan_kernel<D, CC, VEC>;
-      const size_t l2 = 4 * (2 * CC * (D + 8) + CC * 72 + 2 * D);
+      const size_t l2 =
+          4 * (2 * CC * (D == 32 ? 96 : D + 32) + CC * 72 + 2 * D);
       allow_lds(scan, l2);
       scan<<<dim3((a.vdim + 63) / 64, a.H, list.numel()), 256, l2,
              cur_stream()>>>(a);
@@ -485,7 +486,7 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
         constexpr int N = decltype(nct)::value;
         auto k = gla_out_kernel<D, CC, N, VEC>;
         const size_t first =
-            std::max(2 * (CC + 1) * (D + 4), CC * (N * 128 + 8));
+            std::max(2 * (CC + 1) * (D + 4), CC * (N * 128 + 24));
         const size_t l3 = 2 * (first + 2 * CC * (D + 8) + 2 * CC * (CC + 8));
         allow_lds(k, l3);
         k<<<dim3(chunks, a.H), 512, l3, cur_stream()>>>(a);

@@ -286,7 +286,8 @@ __global__ __launch_bounds__(256) void gla_prep_kernel(GlaChunkArgs a) {
 template <int DP, int C, bool VEC>
 __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
   constexpr int NG = DP / 32, NC = C / 32;
-  constexpr int LDD = DP + 8, LDV = 64 + 8;
+  // rows 16 banks apart (mod 64): the permuted column reads do not collide
+  constexpr int LDD = DP == 32 ? 96 : DP + 32, LDV = 64 + 8;
   constexpr int PD = C * DP / 8 / 256;   // 16 B pieces a thread and plane
   constexpr int PV = C * 64 / 8 / 256;
   constexpr int BUF = 2 * C * LDD + C * LDV + 2 * DP;  // 16-bit elements
@@ -320,6 +321,12 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
       if (!kept || (n >> 1) * 32 + hi * 8 + (n & 1) * 4 + r >= a.dim)
         acc[n][r] = 0.f;
 
+  const int c0 = a.ccu[i], c1 = a.ccu[i + 1];
+  if (c0 >= c1) return;
+  // a sequence's chunks lie one after the other
+  const long first = a.row0[c0];
+  const int total = (c1 - c0 - 1) * C + a.len[c1 - 1];
+
   short8 rk[2][PD], rv[PV];
   float rd = 0.f;
   auto fetch = [&](int ch) {
@@ -330,8 +337,8 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
       for (int n = 0; n < PD; ++n)
         rk[p][n] = *reinterpret_cast<const short8*>(
             a.kd + (base * 2 + p) * C * DP + (tid + n * 256) * 8);
-    const long row0 = a.row0[ch];
-    const int len = a.len[ch];
+    const long row0 = first + (long)(ch - c0) * C;
+    const int len = min(C, total - (ch - c0) * C);
 #pragma unroll
     for (int n = 0; n < PV; ++n) {
       const int idx = tid + n * 256;
@@ -357,14 +364,15 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
     if (tid < DP) ((float*)(vb + C * LDV))[tid] = fast_exp2(rd);
   };
 
-  const int c0 = a.ccu[i], c1 = a.ccu[i + 1];
-  if (c0 < c1) {
-    fetch(c0);
-    stage(lds_scan);
-  }
+  fetch(c0);
+  stage(lds_scan);
+  if (c0 + 1 < c1) fetch(c0 + 1);
   for (int ch = c0; ch < c1; ++ch) {
     const unsigned short* buf = lds_scan + ((ch - c0) & 1) * BUF;
-    if (ch + 1 < c1) fetch(ch + 1);
+    __syncthreads();   // buf is written, the other one is read
+    // registers hold the next chunk since an iteration ago
+    if (ch + 1 < c1) stage(lds_scan + ((ch + 1 - c0) & 1) * BUF);
+    if (ch + 2 < c1) fetch(ch + 2);
     // the state as it stands, for the chunk's outputs
     if (vt < a.VT) {
       unsigned short* sp =
@@ -383,7 +391,6 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
         *reinterpret_cast<short8*>(sp + (NG + g) * 512) = sl;
       }
     }
-    __syncthreads();   // buf is written; the other one is read
     const unsigned short* vb = buf + 2 * C * LDD;
     const float* dt = (const float*)(vb + C * LDV);
     bf16x8 vf[NC];
@@ -406,7 +413,6 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
                             g * 32 + (li & 3) * 8 + n * 4, li, hi),
                 vf[k], acc[2 * g + n], 0, 0, 0);
       }
-    if (ch + 1 < c1) stage(lds_scan + ((ch + 1 - c0) & 1) * BUF);
   }
   if (live) {
 #pragma unroll
@@ -428,7 +434,7 @@ template <int DP, int C, int NCT, bool VEC>
 __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   constexpr int LDB = DP + 4, LDD = DP + 8, LDA = C + 8, NG = DP / 32;
   constexpr int NT = C / 16, NC = C / 32, NB = C / 16, VC = NCT * 128;
-  constexpr int LDV = VC + 8;
+  constexpr int LDV = VC + 24;   // rows 12 banks apart, for column reads
   constexpr int FIRST = 2 * (C + 1) * LDB > C * LDV ? 2 * (C + 1) * LDB : C * LDV;
   constexpr int PB = C * DP / 4 / 512, PQ = C * DP / 8 / 512 > 0 ? C * DP / 8 / 512 : 1;
   constexpr int PV = C * VC / 8 / 512;
@@ -574,29 +580,34 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   }
   __syncthreads();
 
+  // v, then the states: an operand that is read serves all of the wave's tiles
   f32x4 o[NCT][NT];
 #pragma unroll
-  for (int c = 0; c < NCT; ++c) {
+  for (int c = 0; c < NCT; ++c)
 #pragma unroll
     for (int t = 0; t < NT; ++t) o[c][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const int vt = c * 8 + wave;
-    if (vt >= a.VT) continue;
-    const int cs = EARLY ? c : 0;
-    if constexpr (!EARLY) load_state(c, sh[0], sl[0]);
 #pragma unroll
-    for (int k = 0; k < NC; ++k) {
-      const bf16x8 vf = column_frag(vs, LDV, k * 32, vt * 16 + (li & 3) * 4, li, hi);
+  for (int k = 0; k < NC; ++k) {
+    bf16x8 vf[NCT];
 #pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        if (k * 32 > t * 16 + 15) continue;  // above the diagonal
+    for (int c = 0; c < NCT; ++c)
+      vf[c] = column_frag(vs, LDV, k * 32, (c * 8 + wave) * 16 + (li & 3) * 4, li, hi);
 #pragma unroll
-        for (int p = 0; p < 2; ++p)
-          o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              vf, as_bf16x8(*reinterpret_cast<const short8*>(
-                      as + (p * C + t * 16 + li) * LDA + k * 32 + hi * 8)),
-              o[c][t], 0, 0, 0);
+    for (int t = 0; t < NT; ++t) {
+      if (k * 32 > t * 16 + 15) continue;  // above the diagonal
+#pragma unroll
+      for (int p = 0; p < 2; ++p) {
+        const bf16x8 af = as_bf16x8(*reinterpret_cast<const short8*>(
+            as + (p * C + t * 16 + li) * LDA + k * 32 + hi * 8));
+#pragma unroll
+        for (int c = 0; c < NCT; ++c)
+          o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[c], af, o[c][t], 0, 0, 0);
       }
     }
+  }
+#pragma unroll
+  for (int c0 = 0; c0 < NCT; c0 += NS) {
+    if constexpr (!EARLY) load_state(c0, sh[0], sl[0]);
 #pragma unroll
     for (int g = 0; g < NG; ++g)
 #pragma unroll
@@ -605,11 +616,20 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
             qs + (t * 16 + li) * LDD + g * 32 + hi * 8));
         const bf16x8 ql = as_bf16x8(*reinterpret_cast<const short8*>(
             qs + (C + t * 16 + li) * LDD + g * 32 + hi * 8));
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[cs][g], qh, o[c][t], 0, 0, 0);
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[cs][g], ql, o[c][t], 0, 0, 0);
-        o[c][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[cs][g], qh, o[c][t], 0, 0, 0);
+#pragma unroll
+        for (int c = 0; c < NS; ++c) {
+          f32x4& r = o[c0 + c][t];
+          r = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[c][g], qh, r, 0, 0, 0);
+          r = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[c][g], ql, r, 0, 0, 0);
+          r = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[c][g], qh, r, 0, 0, 0);
+        }
       }
   }
+#pragma unroll
+  for (int c = 0; c < NCT; ++c)
+    if (c * 8 + wave >= a.VT)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) o[c][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
   // columns beyond vdim are zero: they add nothing
 #pragma unroll
   for (int t = 0; t < NT; ++t) {

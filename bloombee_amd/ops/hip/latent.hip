@@ -394,6 +394,10 @@ DEVINL bf16x8 column_frag(const unsigned short* tile, int ld, int r0, int col,
   return as_bf16x8(v);
 }
 
+// Row stride of a key tile, in elements: rows and columns are read without
+// bank conflicts.
+constexpr int latent_tile_ld(int ck) { return ck + (ck / 2 % 64 < 32 ? 24 : 8); }
+
 // grid (n_list * chunks of 16 * HG heads, n_split), four waves for each of HG
 // groups of 16 heads. ck = ND * 64 + NR * 32; a wave owns every fourth
 // 16-column tile of the values.
@@ -401,7 +405,7 @@ template <int ND, int NR, int HG>
 __global__ __launch_bounds__(256 * HG, 3 - HG) void attn_latent_decode_kernel(
     LatentDecodeArgs a) {
   constexpr int KT = 64, RP = ND * 64, CK = RP + NR * 32, NKK = CK / 32;
-  constexpr int LDK = CK + 8, LDS_S = KT + 4;
+  constexpr int LDK = latent_tile_ld(CK), LDS_S = KT + 4;
   constexpr int LANES = 256 * HG / KT;   // threads that stage one row
   constexpr int NP = (CK / 8 + LANES - 1) / LANES;  // 16 B pieces each
   extern __shared__ __attribute__((aligned(16))) unsigned char lds_dec[];
