@@ -42,6 +42,9 @@ def main():
                     help="cuda:0 / cpu (default: cuda if available)")
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--attn-cache-tokens", type=int, default=1 << 18)
+    ap.add_argument("--attn-cache-sequences", type=int, default=None,
+                    help="sequences live at a time, for models with recurrent "
+                         "layers (their state slots; BBAMD_KV_MAX_SEQS)")
     ap.add_argument("--update-period", type=float, default=30.0)
     ap.add_argument("--checkpoint-dir", default=None,
                     help="per-block .npy weight dir (random init if absent)")
@@ -123,6 +126,7 @@ def main():
         max_batch_size=args.max_batch_size,
         announce_host=args.announce_host,
         announce_port=args.announce_port,
+        kv_max_seqs=args.attn_cache_sequences,
     )
     server.run()
 

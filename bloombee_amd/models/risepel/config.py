@@ -62,7 +62,8 @@ RISEPEL_PRESETS = {
         _latent(32, 128, 64, 128, 512, 1536, 1024, ff=14336, kv_from=0)]),
     "risepel-tiny": _preset(192, 320, [
         _gla(3, 32, 48, ff=256), _latent(6, 32, 16, 48, 80, 96, 24),
-        _gla(3, 32, 48), _latent(6, 32, 16, 48, 80, 96, 33, ff=256, kv_from=1)]),
+        _latent(6, 32, 16, 48, 80, 96, 40),
+        _latent(4, 32, 16, 48, 80, 96, 33, ff=256, kv_from=2)]),
 }
 
 

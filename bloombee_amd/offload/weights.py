@@ -223,8 +223,8 @@ class OffloadedBlockStack:
         return hidden
 
     # passthroughs
-    def make_kv(self, max_tokens: int):
-        return self.stack.make_kv(max_tokens)
+    def make_kv(self, max_tokens: int, max_seqs: Optional[int] = None):
+        return self.stack.make_kv(max_tokens, max_seqs)
 
     @property
     def blocks(self):

@@ -39,7 +39,8 @@ class StackBackend:
                  kv_max_tokens: int = 1 << 18,
                  checkpoint_dir: Optional[str] = None,
                  offload_policy=None,
-                 max_batch_size: int = 2048):
+                 max_batch_size: int = 2048,
+                 kv_max_seqs: Optional[int] = None):
         self.config = config
         self.start, self.end = start, end
         self.device = torch.device(device)
@@ -56,7 +57,8 @@ class StackBackend:
             _ops.set_attn_sparsity(offload_policy.attn_sparsity)
         self.compress_swap = bool(offload_policy is not None
                                   and offload_policy.compress_cache)
-        self.kv_pool: PagedKVCache = self.stack.make_kv(kv_max_tokens)
+        self.kv_pool: PagedKVCache = self.stack.make_kv(kv_max_tokens,
+                                                       kv_max_seqs)
         self.is_last_block = (end == config.num_hidden_layers)
         self.pruner = None
         if self.is_last_block:

@@ -18,7 +18,8 @@ def _free_port():
         return s.getsockname()[1]
 
 
-MODELS = {"llama-tiny": 1000, "mubasun-tiny": 320}   # name -> vocab
+MODELS = {"llama-tiny": 1000, "mubasun-tiny": 320,
+          "risepel-tiny": 320}   # name -> vocab
 
 
 def _worker(rank, world, q, port, model):
