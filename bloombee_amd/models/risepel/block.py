@@ -1,7 +1,7 @@
 """Risepel decoder block on the ragged-batch ops.
 
 Norms come after the sums: x <- norm1(alpha x + mixer(x)), then
-x <- norm2(alpha x + ff(x)). The sublayers read x itself, so a layer hands the
+x <- norm2(alpha x + ff(x)). Nothing is normed ahead of a sublayer: a layer hands the
 next one its rows in the activation type (Carried) and owes it nothing.
 
 Latent attention, one GEMM for everything that reads x:

@@ -142,7 +142,7 @@ class RisepelConfig(ModelConfig):
 
     @property
     def norm_offset(self) -> float:
-        """Layer and final norm weights are stored around zero."""
+        """Layer and final norms scale by one plus their stored weight."""
         return 1.0
 
     @property

@@ -1,5 +1,5 @@
 """Client side of the Risepel family: embeddings without positions, a final
-norm whose weight is stored around zero, capped logits
+norm that scales by one plus its stored weight, capped logits
 (models/ragged_head.py)."""
 from __future__ import annotations
 
