@@ -15,7 +15,9 @@ logger = get_logger(__name__)
 class RemoteGenerationMixin:
     """Requires: self.transformer (with .remote embedding/norm API below) and
     self.lm_head. The host model implements:
-        embed(input_ids) -> hidden
+        embed(input_ids, start_pos) -> hidden; if transformer.uses_previous,
+            embed(input_ids, start_pos, last): last is the token each row was
+            fed before, None at the start
         final_norm(hidden) -> hidden
         lm_head(hidden) -> logits
         remote (RemoteSequential)
@@ -43,8 +45,7 @@ class RemoteGenerationMixin:
         out_tokens = [input_ids]
         try:
             fresh = session.position == 0
-            hidden = self.embed(input_ids,
-                                session.position + (pre if fresh else 0))
+            hidden = self._embed_next(input_ids, session, pre if fresh else 0)
             if pe is not None and fresh:
                 p = pe.detach().to(hidden.dtype).unsqueeze(0).expand(B, -1, -1)
                 hidden = torch.cat([p, hidden], dim=1)
@@ -55,7 +56,7 @@ class RemoteGenerationMixin:
                                   top_p, generator)
             out_tokens.append(next_tok.view(B, 1))
             for _ in range(max_new_tokens - 1):
-                hidden = self.embed(next_tok.view(B, 1), session.position)
+                hidden = self._embed_next(next_tok.view(B, 1), session)
                 hidden = session.step(hidden)
                 logits = self.lm_head(self.final_norm(hidden[:, -1:]))[:, -1]
                 next_tok = self._pick(logits, do_sample, temperature, top_k,
@@ -65,6 +66,16 @@ class RemoteGenerationMixin:
             if own_session:
                 session.close()
         return torch.cat(out_tokens, dim=1)
+
+    def _embed_next(self, ids: torch.Tensor, session,
+                    offset: int = 0) -> torch.Tensor:
+        """Embeds the tokens a session is fed next."""
+        pos = session.position + offset
+        if not getattr(getattr(self, "transformer", None), "uses_previous", False):
+            return self.embed(ids, pos)
+        hidden = self.embed(ids, pos, session.last_ids)
+        session.last_ids = ids[:, -1]
+        return hidden
 
     @staticmethod
     def _pick(logits: torch.Tensor, do_sample: bool, temperature: float,

@@ -147,6 +147,8 @@ class InferenceSession:
         self.batch_size: Optional[int] = None
         self.spans: List[_SpanSession] = []
         self.position = 0           # committed tokens across the chain
+        # (B,) last token the client embedded, None at the start
+        self.last_ids: Optional[torch.Tensor] = None
         self.step_count = 0
         # (pos, span0 input, deep prompts or None)
         self.history: List[Tuple[int, torch.Tensor, Optional[torch.Tensor]]] = []

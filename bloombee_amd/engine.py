@@ -252,15 +252,26 @@ class LocalEngine:
         return F.linear(y, self.lm_head_w)
 
     def _embed(self, input_ids: torch.Tensor,
-               start: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """(B, T) ids; start (B,): position of each row's first token (learned
-        positions only, default 0)."""
+               start: Optional[torch.Tensor] = None,
+               kv: Optional[SessionHandle] = None) -> torch.Tensor:
+        """(B, T) ids; start (B,): position of each row's first token (families
+        that embed positions only, default 0); kv: the session they continue
+        (families that embed pairs of tokens only)."""
         if self.head is not None:
             B, T = input_ids.shape
+            input_ids = input_ids.to(self.device)
+            prev = None
+            if self.head.uses_previous:
+                if kv is None:
+                    raise NotImplementedError(
+                        f"{self.config.model_type}: embeds tokens with the ones "
+                        f"before them, which this step does not follow")
+                prev = ragged.previous_ids(input_ids, kv.previous(self.device))
+                kv.last_ids = input_ids[:, -1].clone()
             pos = torch.arange(T, dtype=torch.int32, device=self.device)
             pos = (pos.expand(B, T) if start is None
                    else start.view(B, 1).int() + pos)
-            return self.head.embed(input_ids.to(self.device), pos)
+            return self.head.embed(input_ids, pos, prev)
         h = F.embedding(input_ids.to(self.device), self.embed)
         if self.embed_scale != 1.0:
             h = h * self.embed_scale
@@ -305,10 +316,18 @@ class LocalEngine:
             h.extend(len(toks))
         if self.stack.token_batched:
             batch = session_batch([(h, len(t)) for h, t, _ in entries])
-            ids = torch.tensor([t for _, toks, _ in entries for t in toks],
-                               dtype=torch.int32).to(self.device)
+            ids = [t for _, toks, _ in entries for t in toks]
+            prev = None
+            if self.head.uses_previous:
+                prev = [t for h, toks, _ in entries
+                        for t in [int(h.previous("cpu")), *toks[:-1]]]
+            both = torch.tensor([ids] if prev is None else [ids, prev],
+                                dtype=torch.int32).to(self.device)
             hidden = self.stack.forward_batch(
-                self.head.embed(ids, batch.tok_pos), batch)
+                self.head.embed(both[0], batch.tok_pos,
+                                None if prev is None else both[1]), batch)
+            for h, toks, _ in entries:
+                h.last_ids = [toks[-1]]
         else:
             outs = []
             for h, toks, _ in entries:
@@ -357,7 +376,7 @@ class LocalEngine:
         start = torch.tensor([s.l_spec for s in kv.seqs], dtype=torch.int32,
                              device=self.device)
         kv.extend(T)
-        hidden = self._embed(input_ids, start)
+        hidden = self._embed(input_ids, start, kv)
         hidden = self.stack.forward_inference(hidden, kv, start)
         return self.logits_for(hidden[:, -1]).argmax(-1)
 
@@ -367,7 +386,7 @@ class LocalEngine:
         start = torch.tensor([s.l_spec for s in kv.seqs], dtype=torch.int32,
                              device=self.device)
         kv.extend(1)
-        hidden = self._embed(input_ids.view(-1, 1), start)
+        hidden = self._embed(input_ids.view(-1, 1), start, kv)
         hidden = self.stack.forward_inference(hidden, kv, start)
         return self.logits_for(hidden[:, -1]).argmax(-1)
 
@@ -535,7 +554,8 @@ class _DecodeGraph:
 
     def _body(self) -> torch.Tensor:
         eng, b = self.engine, self.slots.batch
-        x = eng.stack.forward_batch(eng.head.embed(self.slots.ids, b.tok_pos), b)
+        x = eng.stack.forward_batch(
+            eng.head.embed(self.slots.ids, b.tok_pos, self.slots.prev), b)
         return eng.logits_for(x)
 
     def run(self, entries) -> torch.Tensor:
@@ -543,8 +563,12 @@ class _DecodeGraph:
         for h, _ in entries:
             h.extend(1)
         seqs = [h.seqs[0] for h, _ in entries]
+        prev = ([int(h.previous("cpu")) for h, _ in entries]
+                if self.engine.head.uses_previous else None)
         self.slots.fill([t for _, t in entries], [s.l_spec - 1 for s in seqs],
-                        [s.pages for s in seqs], [s.slot for s in seqs])
+                        [s.pages for s in seqs], [s.slot for s in seqs], prev)
+        for h, t in entries:
+            h.last_ids = [t]
         n = len(entries)
         if self.graph is None and self.calls < self.WARMUP:
             self.calls += 1

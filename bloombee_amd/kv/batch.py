@@ -220,22 +220,24 @@ class DecodeSlots:
         dev = cache.device
         self.B = B
         self.max_pages = (max_len + cache.page_size - 1) // cache.page_size
-        n = 3 * B + B * self.max_pages
+        n = 4 * B + B * self.max_pages
         self._dev = torch.zeros(n, dtype=torch.int32, device=dev)
         self.ids = self._dev[:B]
         pos = self._dev[B:2 * B]
         slots = self._dev[2 * B:3 * B]
+        self.prev = self._dev[3 * B:4 * B]   # token before each, -1 = none
         idx = torch.arange(B, dtype=torch.int32, device=dev)
         self.batch = TokenBatch(
             cache, tok_seq=idx, tok_pos=pos,
             cu=torch.arange(B + 1, dtype=torch.int32, device=dev),
-            q_start=pos, page_table=self._dev[3 * B:].view(B, self.max_pages),
+            q_start=pos, page_table=self._dev[4 * B:].view(B, self.max_pages),
             pre_list=idx[:0], dec_list=idx, max_new=1,
             max_ctx=self.max_pages * cache.page_size, slots=slots)
 
     def fill(self, tokens: Sequence[int], positions: Sequence[int],
              pages: Sequence[Sequence[int]],
-             slots: Optional[Sequence[int]] = None) -> None:
+             slots: Optional[Sequence[int]] = None,
+             prev: Optional[Sequence[int]] = None) -> None:
         B, n = self.B, len(tokens)
         host = torch.zeros(self._dev.numel(), dtype=torch.int32,
                            pin_memory=self._dev.is_cuda)
@@ -245,7 +247,9 @@ class DecodeSlots:
         buf[B:B + n] = positions
         if slots is not None:
             buf[2 * B:2 * B + n] = slots
-        table = buf[3 * B:].reshape(B, self.max_pages)
+        if prev is not None:
+            buf[3 * B:3 * B + n] = prev
+        table = buf[4 * B:].reshape(B, self.max_pages)
         for i, pg in enumerate(pages):
             table[i, :len(pg)] = pg
         self._dev.copy_(host, non_blocking=True)

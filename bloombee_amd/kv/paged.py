@@ -81,7 +81,8 @@ class PagedKVCache:
         list). `shares[l]` = j makes layer l read layer j's planes (cross-layer
         KV sharing): it owns no storage, and copies skip it.
         `state_shapes[l]` gives layer l a recurrent state of that shape (f32)
-        for each of `max_seqs` sequences. A session holds a state slot per
+        for each of `max_seqs` sequences; {name: shape} gives it several
+        tensors. A session holds a state slot per
         sequence for as long as it lives, host-offloaded or not: the state is
         small and does not grow. A sequence that starts at position 0 starts
         from a zero state, so slots are not cleared when they change hands.
@@ -130,10 +131,16 @@ class PagedKVCache:
         self.own_layers = [l for l in range(num_layers)
                            if self.shares[l] is None
                            and self.layout[l] != "none"]
-        self.states = [
-            None if shape is None else torch.zeros(
-                max_seqs, *shape, device=self.device, dtype=torch.float32)
-            for shape in as_list(state_shapes)]
+
+        def make_state(shape):
+            if shape is None:
+                return None
+            if isinstance(shape, dict):
+                return {n: make_state(s) for n, s in shape.items()}
+            return torch.zeros(max_seqs, *shape, device=self.device,
+                               dtype=torch.float32)
+
+        self.states = [make_state(s) for s in as_list(state_shapes)]
         self.has_state = any(t is not None for t in self.states)
         self.max_seqs = max_seqs
         self._free_slots: List[int] = list(range(max_seqs - 1, -1, -1))
@@ -173,8 +180,8 @@ class PagedKVCache:
         d = self.v_head_dim_per_layer[layer]
         return v.view(self.n_pages, hkv, d, self.page_size)
 
-    def state(self, layer: int) -> torch.Tensor:
-        """Recurrent states of a layer, (max_seqs, *shape) f32."""
+    def state(self, layer: int):
+        """Recurrent states of a layer, (max_seqs, *shape) f32 each."""
         return self.states[layer]
 
     # -- admission --------------------------------------------------------
@@ -299,6 +306,10 @@ class SessionHandle:
         self.seqs = [_SeqState(slot=n) for n in slots or [-1] * batch_size]
         self._slots = None if not cache.has_state else torch.tensor(
             [s.slot for s in self.seqs], dtype=torch.int32).to(cache.device)
+        # token that each sequence was last fed, -1 = none yet: a list or a (B,)
+        # tensor, None = not known (tokens were taken back). Kept by whoever
+        # embeds, for embeddings that look at the token before.
+        self.last_ids = [-1] * batch_size
         self._max_pages = (max_length + cache.page_size - 1) // cache.page_size
         self._page_table = torch.zeros(
             batch_size, self._max_pages, device=cache.device, dtype=torch.int32
@@ -416,6 +427,8 @@ class SessionHandle:
         """Drop tokens above l_acc and free orphaned pages."""
         P = self.cache.page_size
         freed: List[int] = []
+        if any(s.l_spec > s.l_acc for s in self.seqs):
+            self._forget_last()
         for s in self.seqs:
             s.l_spec = s.l_acc
             keep = (s.l_acc + P - 1) // P
@@ -841,6 +854,16 @@ class SessionHandle:
         for s, n in zip(self.seqs, new_lengths):
             s.l_acc = n
         self.rollback()
+
+    def _forget_last(self) -> None:
+        fresh = all(s.l_acc == 0 for s in self.seqs)
+        self.last_ids = [-1] * self.batch_size if fresh else None
+
+    def previous(self, device) -> torch.Tensor:
+        """(B,) int32: the token each sequence was last fed."""
+        if self.last_ids is None:
+            raise PagedKVError("the last tokens of this session are not known")
+        return torch.as_tensor(self.last_ids, dtype=torch.int32).to(device)
 
     # -- kernel-facing views ----------------------------------------------
     def page_table(self) -> torch.Tensor:

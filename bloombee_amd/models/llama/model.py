@@ -159,8 +159,8 @@ class DistributedLlamaForCausalLM(RemoteGenerationMixin, torch.nn.Module):
     def remote(self) -> RemoteSequential:
         return self.transformer.remote
 
-    def embed(self, input_ids, start_pos: int = 0):
-        return self.transformer.embed(input_ids, start_pos)
+    def embed(self, input_ids, start_pos: int = 0, *last):
+        return self.transformer.embed(input_ids, start_pos, *last)
 
     def final_norm(self, hidden):
         return self.transformer.final_norm(hidden)

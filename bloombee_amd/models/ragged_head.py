@@ -4,8 +4,10 @@ LocalEngine, the pipeline and the swarm client, and the distributed model
 classes over it.
 
 What differs between families are properties of the config: `learned_positions`
-(a table "pos" is added to the embedding), `norm_groups`, `norm_offset` (norm
-weights are stored as their distance from it), `logit_softcap` (0 = none).
+(a table "pos" is added to the embedding), `sinusoidal_positions`, `bigram` (a
+table "bigram" of hashed token pairs is added: buckets, mul_prev, mul_cur),
+`norm_groups`, `norm_offset` (norm weights are stored as their distance from it),
+`scalar_norm` (one norm weight for all coordinates), `logit_softcap` (0 = none).
 """
 from __future__ import annotations
 
@@ -19,7 +21,7 @@ from bloombee_amd.models.base import ModelConfig
 from bloombee_amd.models.llama.model import (DistributedLlamaForCausalLM,
                                              DistributedLlamaModel)
 from bloombee_amd.ops import ragged
-from bloombee_amd.ops.ragged import pad_k, round_up
+from bloombee_amd.ops.ragged import PairTable, pad_k, round_up
 
 
 class RaggedHead(torch.nn.Module):
@@ -42,6 +44,15 @@ class RaggedHead(torch.nn.Module):
         self.embed_w = p(V, W)
         self.pos_w = (p(config.max_position_embeddings, W)
                       if getattr(config, "learned_positions", False) else None)
+        pair = getattr(config, "bigram", None)
+        self.pair_w = p(pair["buckets"] + 1, W) if pair else None
+        self.pairs = (PairTable(self.pair_w, pair["mul_prev"], pair["mul_cur"])
+                      if pair else None)
+        self.turns = None
+        if getattr(config, "sinusoidal_positions", False):
+            self.turns = torch.nn.Parameter(
+                ragged.sinusoid_turns(W).to(device), requires_grad=False)
+        self.scalar_norm = getattr(config, "scalar_norm", False)
         self.norm_w = p(W, dtype=torch.float32)
         self.head_w = p(round_up(V, 64), pad_k(W))   # zero padding
         if checkpoint_dir is not None:
@@ -52,29 +63,44 @@ class RaggedHead(torch.nn.Module):
             draw = {"embed": (V, W), "head": (V, W)}
             if self.pos_w is not None:
                 draw["pos"] = tuple(self.pos_w.shape)
+            if self.pair_w is not None:
+                draw["bigram"] = tuple(self.pair_w.shape)
             ts = {n: torch.randn(s, generator=gen).mul_(0.02)
                   for n, s in draw.items()}
-            ts["final.norm"] = torch.full((W,), 1.0 - self.norm_offset)
+            ts["final.norm"] = torch.full(() if self.scalar_norm else (W,),
+                                          1.0 - self.norm_offset)
             self.load_tensors(ts.__getitem__)
 
     @torch.no_grad()
     def load_tensors(self, get) -> None:
         W, V = self.config.hidden_size, self.config.vocab_size
         for name, w in (("embed", self.embed_w), ("pos", self.pos_w),
-                        ("final.norm", self.norm_w),
+                        ("bigram", self.pair_w), ("final.norm", self.norm_w),
                         ("head", self.head_w[:V, :W])):
             if w is None:
                 continue
             t = get(name)
-            if t.shape != w.shape:
+            one = name == "final.norm" and self.scalar_norm
+            if t.shape != (() if one else w.shape):
                 raise ValueError(f"{name}: shape {tuple(t.shape)}, expected "
-                                 f"{tuple(w.shape)}")
+                                 f"{() if one else tuple(w.shape)}")
             w.copy_(t)
         self.norm_w.add_(self.norm_offset)
 
-    def embed(self, ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
-        """ids, positions of one shape -> (..., W) f32."""
-        return ragged.embed_rows(ids, positions, self.embed_w, self.pos_w)
+    @property
+    def uses_previous(self) -> bool:
+        """embed() needs the token before each."""
+        return self.pairs is not None
+
+    def embed(self, ids: torch.Tensor, positions: torch.Tensor,
+              prev: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """ids, positions of one shape -> (..., W) f32; prev: the token before
+        each, -1 = none (only if uses_previous)."""
+        if self.uses_previous and prev is None:
+            raise ValueError("this family embeds tokens with the ones before "
+                             "them: they are missing")
+        return ragged.embed_rows(ids, positions, self.embed_w, self.pos_w, prev,
+                                 self.pairs, self.turns)
 
     def final_norm(self, hidden: torch.Tensor) -> torch.Tensor:
         W = self.config.hidden_size
@@ -133,11 +159,22 @@ class DistributedRaggedModel(DistributedLlamaModel):
                     torch.zeros(config.num_hidden_layers, pre_seq_len,
                                 config.hidden_size, device=device))
 
-    def embed(self, input_ids: torch.Tensor, start_pos: int = 0) -> torch.Tensor:
+    @property
+    def uses_previous(self) -> bool:
+        return self.head.uses_previous
+
+    def embed(self, input_ids: torch.Tensor, start_pos: int = 0,
+              last: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """last (B,): the token before each row's first, None = there is none."""
         B, T = input_ids.shape
+        ids = input_ids.to(self.device_)
         pos = torch.arange(start_pos, start_pos + T, dtype=torch.int32,
                            device=self.device_).expand(B, T)
-        return self.head.embed(input_ids.to(self.device_), pos)
+        prev = None
+        if self.uses_previous:
+            prev = ragged.previous_ids(
+                ids, torch.full((B,), -1) if last is None else last)
+        return self.head.embed(ids, pos, prev)
 
     def final_norm(self, hidden: torch.Tensor) -> torch.Tensor:
         if hidden.requires_grad:

@@ -9,24 +9,11 @@
 #include "latent.hip"
 #include "gla.hip"
 
-static Parts as_parts(const Tensor& t) {
-  check_act(t);
-  TORCH_CHECK(t.dim() == 3 && t.is_contiguous());
-  return Parts{t.data_ptr(), t.size(1) * t.size(2), (int)t.size(0),
-               (int)t.size(2)};
-}
-
 static void check_turns(const OptTensor& t, long rdims) {
   TORCH_CHECK(rdims % 2 == 0 && t.has_value() && t->is_cuda() &&
                   t->is_contiguous() && t->scalar_type() == at::kDouble &&
                   t->numel() == rdims / 2,
               "rotary frequencies: one double per pair");
-}
-
-static bool all_of_8(std::initializer_list<long> v) {
-  for (long x : v)
-    if (x % 8) return false;
-  return true;
 }
 
 // dims: [q_off, c_off, g_off, q_rank, rank, rot, rdims, rp, gate columns,

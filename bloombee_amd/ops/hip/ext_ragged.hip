@@ -12,26 +12,51 @@
 #include "moe_routed.hip"
 #include "gemm_skinny.hip"
 
-Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table) {
+// pair: [buckets, mul_prev, mul_cur] with prev and pair_table
+Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table,
+                  OptTensor prev, OptTensor pair_table, std::vector<long> pair,
+                  OptTensor turns) {
   CHECK_I32(ids);
   CHECK_I32(pos);
   check_act(table);
   TORCH_CHECK(table.is_contiguous() && table.dim() == 2 &&
               ids.numel() == pos.numel());
+  EmbedArgs a{};
+  const long N = ids.numel();
+  a.W = table.size(1);
+  a.vocab = table.size(0);
+  a.ids = ids.data_ptr<int>();
+  a.pos = pos.data_ptr<int>();
+  a.table = table.data_ptr();
   if (pos_table.has_value()) {
     CHECK_T((*pos_table), table.scalar_type());
-    TORCH_CHECK(pos_table->dim() == 2 && table.size(1) == pos_table->size(1));
+    TORCH_CHECK(pos_table->dim() == 2 && a.W == pos_table->size(1));
+    a.pos_table = pos_table->data_ptr();
+    a.max_pos = pos_table->size(0);
   }
-  const long N = ids.numel();
-  auto x = torch::empty({N, table.size(1)}, table.options().dtype(at::kFloat));
+  if (pair_table.has_value()) {
+    CHECK_T((*pair_table), table.scalar_type());
+    TORCH_CHECK(prev.has_value(), "rows of token pairs need the previous tokens");
+    CHECK_I32((*prev));
+    TORCH_CHECK(pair.size() == 3 && pair[0] >= 1 && pair[1] >= 0 && pair[2] >= 0 &&
+                pair_table->dim() == 2 && pair_table->size(0) == pair[0] + 1 &&
+                pair_table->size(1) == a.W && prev->numel() == N);
+    a.pair_table = pair_table->data_ptr();
+    a.prev = prev->data_ptr<int>();
+    a.buckets = pair[0];
+    a.mul_prev = pair[1];
+    a.mul_cur = pair[2];
+  }
+  if (turns.has_value()) {
+    CHECK_T((*turns), at::kDouble);
+    TORCH_CHECK(turns->numel() == (a.W + 1) / 2);
+    a.turns = turns->data_ptr<double>();
+  }
+  auto x = torch::empty({N, a.W}, table.options().dtype(at::kFloat));
   if (N == 0) return x;
+  a.x = x.data_ptr<float>();
   by_type(table.scalar_type(), [&](auto t) {
-    using T = decltype(t);
-    embed_rows_kernel<T><<<N, 256, 0, cur_stream()>>>(
-        ids.data_ptr<int>(), pos.data_ptr<int>(), (const T*)table.data_ptr(),
-        pos_table.has_value() ? (const T*)pos_table->data_ptr() : nullptr,
-        x.data_ptr<float>(), (int)table.size(1), (int)table.size(0),
-        pos_table.has_value() ? (int)pos_table->size(0) : 0);
+    embed_rows_kernel<decltype(t)><<<N, 256, 0, cur_stream()>>>(a);
   });
   check_launch();
   return x;
@@ -44,7 +69,7 @@ Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table) {
 void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
                    OptTensor idw, OptTensor hprev, OptTensor nw, long groups,
                    double eps, OptTensor h, double alpha, OptTensor bias,
-                   bool post) {
+                   bool post, OptTensor bw) {
   CHECK_F32(x);
   TORCH_CHECK(x.dim() == 2);
   const long N = x.size(0);
@@ -62,6 +87,11 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
     TORCH_CHECK(parts.has_value() && bias->numel() == W);
     a.bias = bias->data_ptr<float>();
   }
+  if (bw.has_value()) {
+    CHECK_F32((*bw));
+    TORCH_CHECK(bw->numel() == W && (parts.has_value() || routed.has_value()));
+    a.bw = bw->data_ptr<float>();
+  }
   bool vec = W % 4 == 0;
   at::ScalarType tp = at::kFloat, ta = at::kFloat;
   if (parts.has_value()) {
@@ -76,7 +106,7 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
     vec = vec && a.ldp % 4 == 0;
   }
   if (routed.has_value()) {
-    TORCH_CHECK(parts.has_value() && ids.has_value());
+    TORCH_CHECK(ids.has_value());
     check_act(*routed);
     CHECK_I32((*ids));
     TORCH_CHECK(routed->is_contiguous() && routed->dim() == 3 &&
@@ -201,6 +231,38 @@ void softcap(Tensor z, double cap) {
 // input GEMM -> q, K/V pages, gate, activation, routing
 // ---------------------------------------------------------------------------
 
+static void set_logits(RouteArgs& r, const Tensor& rparts, long N) {
+  CHECK_F32(rparts);
+  TORCH_CHECK(rparts.dim() == 3 && rparts.size(1) == N);
+  r.parts = rparts.data_ptr<float>();
+  r.ks = rparts.size(0);
+  r.ld = rparts.size(2);
+  r.stride = N * (long)r.ld;
+}
+
+static void set_routing(RouteArgs& r, long N, const OptTensor& corr, Tensor ids,
+                        Tensor wts, const OptTensor& idw) {
+  const int n = r.E + r.NI;
+  TORCH_CHECK(n <= MAX_ROUTED && r.top >= 1 && r.top <= n);
+  TORCH_CHECK(r.off >= 0 && r.off + n <= r.ld);
+  CHECK_I32(ids);
+  CHECK_F32(wts);
+  TORCH_CHECK(ids.numel() == N * r.top && wts.numel() == N * r.top);
+  r.ids = ids.data_ptr<int>();
+  r.wts = wts.data_ptr<float>();
+  if (corr.has_value()) {
+    CHECK_F32((*corr));
+    TORCH_CHECK(corr->numel() == n);
+    r.corr = corr->data_ptr<float>();
+  }
+  TORCH_CHECK(r.NI == 0 || idw.has_value());
+  if (idw.has_value()) {
+    CHECK_F32((*idw));
+    TORCH_CHECK(idw->numel() == N);
+    r.idw = idw->data_ptr<float>();
+  }
+}
+
 // dims: [q,k,v,g,u,u2,r,sg offsets, H, G, dim, vdim, has_kv, act, ff, act_col,
 //        E, NI, top]; consts: [eps, xp, xq, rscale]
 void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
@@ -219,13 +281,13 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
   a.ldp = parts.size(2);
   a.pstride = N * (long)a.ldp;
   int* f[19] = {&a.q_off, &a.k_off, &a.v_off, &a.g_off, &a.u_off, &a.u2_off,
-                &a.r_off, &a.sg_off, &a.H, &a.G, &a.dim, &a.vdim, &a.has_kv,
-                &a.act, &a.ff, &a.act_col, &a.E, &a.NI, &a.top};
+                &a.rt.off, &a.sg_off, &a.H, &a.G, &a.dim, &a.vdim, &a.has_kv,
+                &a.act, &a.ff, &a.act_col, &a.rt.E, &a.rt.NI, &a.rt.top};
   for (int i = 0; i < 19; ++i) *f[i] = (int)dims[i];
   a.eps = (float)consts[0];
   a.xp = (float)consts[1];
   a.xq = (float)consts[2];
-  a.rscale = (float)consts[3];
+  a.rt.scale = (float)consts[3];
   const auto ta = q.scalar_type();
   for (const Tensor& t : {q, a2, kp, vp})
     TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == ta,
@@ -279,31 +341,16 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
     a.act_col = HV;
     a.ff = 0;
   }
-  if (a.E + a.NI > 0 || a.act == 2) {
+  const int routed = a.rt.E + a.rt.NI;
+  if (routed > 0 || a.act == 2) {
     TORCH_CHECK(rparts.has_value());
-    CHECK_F32((*rparts));
-    TORCH_CHECK(rparts->dim() == 3 && rparts->size(1) == N);
-    a.rparts = rparts->data_ptr<float>();
-    a.rks = rparts->size(0);
-    a.ldr = rparts->size(2);
-    a.rstride = N * (long)a.ldr;
-    TORCH_CHECK(a.act != 2 || (a.sg_off >= 0 && a.sg_off < a.ldr));
+    set_logits(a.rt, *rparts, N);
+    TORCH_CHECK(a.act != 2 || (a.sg_off >= 0 && a.sg_off < a.rt.ld));
   }
-  if (a.E + a.NI > 0) {
-    TORCH_CHECK(a.E + a.NI <= MAX_ROUTED && a.top >= 1 && a.top <= a.E + a.NI);
-    TORCH_CHECK(a.r_off >= 0 && a.r_off + a.E + a.NI <= a.ldr);
+  if (routed > 0) {
     TORCH_CHECK(corr.has_value() && ids.has_value() && wts.has_value() &&
                 idw.has_value());
-    CHECK_F32((*corr));
-    CHECK_I32((*ids));
-    CHECK_F32((*wts));
-    CHECK_F32((*idw));
-    TORCH_CHECK(corr->numel() == a.E + a.NI && ids->numel() == N * a.top &&
-                wts->numel() == N * a.top && idw->numel() == N);
-    a.corr = corr->data_ptr<float>();
-    a.ids = ids->data_ptr<int>();
-    a.wts = wts->data_ptr<float>();
-    a.idw = idw->data_ptr<float>();
+    set_routing(a.rt, N, corr, *ids, *wts, idw);
   }
   if (N == 0) return;
   bool vec = true;
@@ -321,6 +368,130 @@ void proj_post(Tensor parts, OptTensor rparts, std::vector<long> dims,
                                   decltype(v)::value ? 8 : 1>;
         allow_lds(k, lds);
         k<<<grid, POST_BLOCK, lds, cur_stream()>>>(a);
+      });
+    });
+  });
+  check_launch();
+}
+
+// dims: [q,k,v offsets, H, G, dim, vdim]; consts: [eps, temperature's
+// coefficient and step]
+void head_post(Tensor parts, std::vector<long> dims, std::vector<double> consts,
+               OptTensor qb, OptTensor kb, OptTensor vb, Tensor qn, Tensor kn,
+               Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
+               Tensor tok_pos) {
+  TORCH_CHECK(dims.size() == 7 && consts.size() == 3);
+  HeadPostArgs a{};
+  a.y = as_parts(parts);
+  const long N = parts.size(1);
+  int* f[7] = {&a.q_off, &a.k_off, &a.v_off, &a.H, &a.G, &a.dim, &a.vdim};
+  for (int i = 0; i < 7; ++i) *f[i] = (int)dims[i];
+  a.eps = (float)consts[0];
+  a.temp_coef = (float)consts[1];
+  a.temp_every = consts[2];
+  TORCH_CHECK(a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.dim >= 1 &&
+              a.vdim >= 1 && a.temp_every > 0);
+  auto inside = [&](int off, int n) { return off >= 0 && off + n <= a.y.ld; };
+  TORCH_CHECK(inside(a.q_off, a.H * a.dim) && inside(a.k_off, a.G * a.dim) &&
+              inside(a.v_off, a.G * a.vdim));
+  const OptTensor* bs[3] = {&qb, &kb, &vb};
+  const float** bp[3] = {&a.qb, &a.kb, &a.vb};
+  const int bn[3] = {a.H * a.dim, a.G * a.dim, a.G * a.vdim};
+  for (int i = 0; i < 3; ++i)
+    if (bs[i]->has_value()) {
+      CHECK_F32((**bs[i]));
+      TORCH_CHECK((*bs[i])->numel() == bn[i]);
+      *bp[i] = (*bs[i])->data_ptr<float>();
+    }
+  CHECK_F32(qn);
+  CHECK_F32(kn);
+  TORCH_CHECK(qn.numel() == a.dim && kn.numel() == a.dim);
+  a.qn = qn.data_ptr<float>();
+  a.kn = kn.data_ptr<float>();
+  check_act(q);
+  const auto ta = q.scalar_type();
+  for (const Tensor& t : {q, kp, vp})
+    TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == ta,
+                "q and the pages share one element type");
+  a.dkp = q.size(2);
+  TORCH_CHECK(q.dim() == 3 && q.size(0) == N && q.size(1) == a.H &&
+              a.dkp >= a.dim);
+  TORCH_CHECK(kp.dim() == 4 && vp.dim() == 4 && kp.size(1) == a.G &&
+              vp.size(1) == a.G && kp.size(3) == a.dkp &&
+              vp.size(3) == kp.size(2) && vp.size(2) >= a.vdim &&
+              vp.size(0) == kp.size(0));
+  a.q = q.data_ptr();
+  a.kp = kp.data_ptr();
+  a.vp = vp.data_ptr();
+  a.P = kp.size(2);
+  a.dvp = vp.size(2);
+  CHECK_I32(table);
+  CHECK_I32(tok_seq);
+  CHECK_I32(tok_pos);
+  TORCH_CHECK(tok_seq.numel() == N && tok_pos.numel() == N && table.dim() == 2);
+  a.table = table.data_ptr<int>();
+  a.maxp = table.size(1);
+  a.tok_seq = tok_seq.data_ptr<int>();
+  a.tok_pos = tok_pos.data_ptr<int>();
+  if (N == 0) return;
+  bool vec = true;
+  for (int v : {a.y.ld, a.q_off, a.k_off, a.dim, a.dkp}) vec = vec && v % 4 == 0;
+  const size_t lds = 4 * 4 * ((size_t)(a.dim + 7) & ~7);
+  by_type(parts.scalar_type(), [&](auto p) {
+    by_type(ta, [&](auto t) {
+      by_bool(vec, [&](auto v) {
+        auto k = head_post_kernel<decltype(p), decltype(t),
+                                  decltype(v)::value ? 4 : 1>;
+        allow_lds(k, lds);
+        k<<<dim3(N, (a.H + 2 * a.G + 3) / 4), 256, lds, cur_stream()>>>(a);
+      });
+    });
+  });
+  check_launch();
+}
+
+// dims: [act, gate or up, up, ff, router offset, E, NI, top, sigmoid scores]
+void ff_post(OptTensor parts, OptTensor rparts, std::vector<long> dims,
+             double rscale, OptTensor corr, Tensor out, OptTensor ids,
+             OptTensor wts, OptTensor idw) {
+  TORCH_CHECK(dims.size() == 9);
+  FfPostArgs a{};
+  int* f[9] = {&a.act, &a.u_off, &a.u2_off, &a.ff, &a.rt.off,
+               &a.rt.E, &a.rt.NI, &a.rt.top, &a.rt.sigmoid};
+  for (int i = 0; i < 9; ++i) *f[i] = (int)dims[i];
+  check_act(out);
+  TORCH_CHECK(out.dim() == 2 && out.is_contiguous());
+  const long N = out.size(0);
+  a.out = out.data_ptr();
+  a.ldo = out.size(1);
+  TORCH_CHECK(a.act >= 0 && a.act <= 2 && a.ff >= 0 && a.ff <= a.ldo);
+  auto tp = at::kFloat;
+  if (a.act) {
+    TORCH_CHECK(parts.has_value());
+    a.y = as_parts(*parts);
+    tp = parts->scalar_type();
+    auto inside = [&](int off) { return off >= 0 && off + a.ff <= a.y.ld; };
+    TORCH_CHECK(parts->size(1) == N && inside(a.u_off) &&
+                (a.act != 1 || inside(a.u2_off)));
+  } else {
+    a.ff = 0;
+  }
+  if (a.rt.E + a.rt.NI > 0) {
+    TORCH_CHECK(rparts.has_value() && ids.has_value() && wts.has_value());
+    a.rt.scale = (float)rscale;
+    set_logits(a.rt, *rparts, N);
+    set_routing(a.rt, N, corr, *ids, *wts, idw);
+  }
+  if (N == 0) return;
+  bool vec = a.ldo % 8 == 0 && a.ff % 8 == 0;
+  if (a.act)
+    for (int v : {a.y.ld, a.u_off, a.u2_off}) vec = vec && (v < 0 || v % 8 == 0);
+  const dim3 grid(N, 1 + (a.ldo + POST_CHUNK - 1) / POST_CHUNK);
+  by_type(tp, [&](auto p) {
+    by_type(out.scalar_type(), [&](auto t) {
+      by_bool(vec, [&](auto v) {
+        ff_post_kernel<decltype(p), decltype(t), decltype(v)::value ? 8 : 1>
+            <<<grid, POST_BLOCK, 0, cur_stream()>>>(a);
       });
     });
   });
@@ -535,22 +706,24 @@ void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
 // routed experts
 // ---------------------------------------------------------------------------
 
-// h (N, K), gate_up (E, 2, F, K), down (E, Wp, F), ids/wts (N, top)
-// -> y (N, top, Wp); rows of skipped choices are not written.
-Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
-                   Tensor wts) {
+// h (N, K), up (E, planes, F, K), down (E, Wp, F), ids/wts (N, top)
+// -> y (N, top, Wp); rows of skipped choices are not written. Two planes:
+// silu(gate) * up, one: relu(up)^2. win: the weight multiplies the expert's
+// input, else its output.
+Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
+                   bool win) {
   check_act(h);
   const auto ta = h.scalar_type();
-  for (const Tensor& t : {h, gate_up, down})
+  for (const Tensor& t : {h, up, down})
     TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == ta);
   CHECK_I32(ids);
   CHECK_F32(wts);
-  TORCH_CHECK(h.dim() == 2 && gate_up.dim() == 4 && down.dim() == 3 &&
-              ids.dim() == 2 && gate_up.size(1) == 2);
+  TORCH_CHECK(h.dim() == 2 && up.dim() == 4 && down.dim() == 3 &&
+              ids.dim() == 2 && (up.size(1) == 1 || up.size(1) == 2));
   const int N = h.size(0), K = h.size(1);
-  const int E = gate_up.size(0), F = gate_up.size(2), Wp = down.size(1);
+  const int E = up.size(0), F = up.size(2), Wp = down.size(1);
   const int top = ids.size(1), S = N * top;
-  TORCH_CHECK(ids.size(0) == N && wts.numel() == S && gate_up.size(3) == K &&
+  TORCH_CHECK(ids.size(0) == N && wts.numel() == S && up.size(3) == K &&
               down.size(0) == E && down.size(2) == F && E >= 1 &&
               E <= MOE_MAX_E && top >= 1);
   TORCH_CHECK(K % 64 == 0 && F % 64 == 0 && Wp % 64 == 0,
@@ -560,22 +733,30 @@ Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
   auto act = torch::empty({S, F}, h.options());
   const int* idp = ids.data_ptr<int>();
   const float* wp = wts.data_ptr<float>();
+  const float* w1 = win ? wp : nullptr;
+  const float* w2 = win ? nullptr : wp;
   auto st = cur_stream();
+  auto by_planes = [&](auto f) {
+    if (up.size(1) == 2) f(std::integral_constant<int, 2>{});
+    else f(std::integral_constant<int, 1>{});
+  };
 
   if (ta == at::kBFloat16 && N <= 32) {
     const bf16_bits* hp = (const bf16_bits*)h.data_ptr();
     bf16_bits* actp = (bf16_bits*)act.data_ptr();
     by_bool(K % 256 == 0, [&](auto full) {
-      moe_skinny_kernel<true, decltype(full)::value>
-          <<<dim3(F / 64, E), 256, 0, st>>>(
-              hp, (const bf16_bits*)gate_up.data_ptr(), idp, wp, actp, S, top,
-              F, K, K, F);
+      by_planes([&](auto np) {
+        moe_skinny_kernel<decltype(np)::value, decltype(full)::value>
+            <<<dim3(F / 64, E), 256, 0, st>>>(
+                hp, (const bf16_bits*)up.data_ptr(), idp, w1, actp, S, top, F,
+                K, K, F);
+      });
     });
     check_launch();
     by_bool(F % 256 == 0, [&](auto full) {
-      moe_skinny_kernel<false, decltype(full)::value>
+      moe_skinny_kernel<0, decltype(full)::value>
           <<<dim3(Wp / 64, E), 256, 0, st>>>(
-              actp, (const bf16_bits*)down.data_ptr(), idp, wp,
+              actp, (const bf16_bits*)down.data_ptr(), idp, w2,
               (bf16_bits*)y.data_ptr(), S, top, Wp, F, F, Wp);
     });
     check_launch();
@@ -594,27 +775,33 @@ Tensor moe_experts(Tensor h, Tensor gate_up, Tensor down, Tensor ids,
   moe_sort_kernel<<<1, 1024, 0, st>>>(idp, offp, sp, tp, S, E, BM, max_tiles);
   check_launch();
   if (ta == at::kFloat) {
-    moe_simple_kernel<true><<<dim3(F / 64, max_tiles), 256, 0, st>>>(
-        h.data_ptr<float>(), gate_up.data_ptr<float>(), offp, sp, tp, wp,
-        act.data_ptr<float>(), top, F, K, K, F);
+    by_planes([&](auto np) {
+      moe_simple_kernel<decltype(np)::value>
+          <<<dim3(F / 64, max_tiles), 256, 0, st>>>(
+              h.data_ptr<float>(), up.data_ptr<float>(), offp, sp, tp, w1,
+              act.data_ptr<float>(), top, F, K, K, F);
+    });
     check_launch();
-    moe_simple_kernel<false><<<dim3(Wp / 64, max_tiles), 256, 0, st>>>(
-        act.data_ptr<float>(), down.data_ptr<float>(), offp, sp, tp, wp,
+    moe_simple_kernel<0><<<dim3(Wp / 64, max_tiles), 256, 0, st>>>(
+        act.data_ptr<float>(), down.data_ptr<float>(), offp, sp, tp, w2,
         y.data_ptr<float>(), top, Wp, F, F, Wp);
     check_launch();
     return y;
   }
   auto tile = [&](auto bm) {
     constexpr int B = decltype(bm)::value;
-    const int nu = (F + 127) / 128, nd = (Wp + 255) / 256;
-    moe_tile_kernel<B, true><<<nu * max_tiles, 256, 0, st>>>(
-        (const bf16_bits*)h.data_ptr(), (const bf16_bits*)gate_up.data_ptr(),
-        offp, sp, tp, wp, (bf16_bits*)act.data_ptr(), max_tiles, nu, top, F, K,
-        K, F);
+    const int per = up.size(1) == 2 ? 128 : 256;
+    const int nu = (F + per - 1) / per, nd = (Wp + 255) / 256;
+    by_planes([&](auto np) {
+      moe_tile_kernel<B, decltype(np)::value><<<nu * max_tiles, 256, 0, st>>>(
+          (const bf16_bits*)h.data_ptr(), (const bf16_bits*)up.data_ptr(), offp,
+          sp, tp, w1, (bf16_bits*)act.data_ptr(), max_tiles, nu, top, F, K, K,
+          F);
+    });
     check_launch();
-    moe_tile_kernel<B, false><<<nd * max_tiles, 256, 0, st>>>(
+    moe_tile_kernel<B, 0><<<nd * max_tiles, 256, 0, st>>>(
         (const bf16_bits*)act.data_ptr(), (const bf16_bits*)down.data_ptr(),
-        offp, sp, tp, wp, (bf16_bits*)y.data_ptr(), max_tiles, nd, top, Wp, F,
+        offp, sp, tp, w2, (bf16_bits*)y.data_ptr(), max_tiles, nd, top, Wp, F,
         F, Wp);
     check_launch();
   };
@@ -629,6 +816,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("clamped_glu", &clamped_glu);
   m.def("softcap", &softcap);
   m.def("proj_post", &proj_post);
+  m.def("head_post", &head_post);
+  m.def("ff_post", &ff_post);
   m.def("router_gemm", &router_gemm);
   m.def("gemm_parts", &gemm_parts);
   m.def("attn_ragged", &attn_ragged);

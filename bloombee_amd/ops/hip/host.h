@@ -5,6 +5,8 @@
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
 
+#include "rows.hip"
+
 using torch::Tensor;
 using OptTensor = c10::optional<Tensor>;
 typedef unsigned short bf16_bits;
@@ -53,4 +55,17 @@ static void allow_lds(K kernel, size_t bytes) {
                     hipFuncAttributeMaxDynamicSharedMemorySize,
                     (int)bytes) == hipSuccess,
                 "cannot reserve ", bytes, " bytes of LDS");
+}
+
+static inline Parts as_parts(const Tensor& t) {
+  check_act(t);
+  TORCH_CHECK(t.dim() == 3 && t.is_contiguous());
+  return Parts{t.data_ptr(), t.size(1) * t.size(2), (int)t.size(0),
+               (int)t.size(2)};
+}
+
+static inline bool all_of_8(std::initializer_list<long> v) {
+  for (long x : v)
+    if (x % 8) return false;
+  return true;
 }

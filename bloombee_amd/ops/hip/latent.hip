@@ -22,32 +22,6 @@
 #include "common.h"
 #include "rows.hip"
 
-// A GEMM output that may lie in split-K partials.
-struct Parts {
-  const void* p;  // (ks, N, ld)
-  long stride;    // elements between splits
-  int ks, ld;
-};
-
-template <typename TP, int V>
-DEVINL void fold_parts(const Parts& a, long t, int c, float* o) {
-  const TP* row = (const TP*)a.p + t * (long)a.ld + c;
-  ldv<V>(row, o);
-  for (int s = 1; s < a.ks; ++s) {
-    float u[V];
-    ldv<V>(row + s * a.stride, u);
-#pragma unroll
-    for (int j = 0; j < V; ++j) o[j] += u[j];
-  }
-}
-
-// turns: frequency / 2 pi
-DEVINL void rotation(int pos, double turns, float& c, float& s) {
-  double r = (double)pos * turns;
-  r -= rint(r);
-  sincospif(2.f * (float)r, &s, &c);
-}
-
 struct LatentPostArgs {
   Parts y;              // [query latent | c | r | gate] columns
   const float* qn;      // (q_rank,)

@@ -3,11 +3,19 @@
 //   act[.]  = silu(W_gate[e] h) * (W_up[e] h)          one fused launch
 //   y[slot] = wts[slot] * (W_down[e] act)              one launch
 //
+// or act = relu(W_up[e] h)^2, and the weight may multiply h instead: by then
+// it has passed through the linear map, so the first launch's epilogue applies
+// it ahead of the activation.
+//
 // ids[slot] < 0 marks a choice without weights (an identity expert, which the
 // residual fold adds by itself): it is skipped everywhere.
 //
-// gate_up (E, 2, F, K): row f of plane 0 is the gate of activation f, of plane
-// 1 its up projection. down (E, N, F). K, F and N are padded to 64.
+// First weights (E, planes, F, K): of two planes, row f of plane 0 is the gate of
+// activation f, of plane 1 its up projection; a single plane is the up projection
+// of relu^2. down (E, N, F). K, F and N are padded to 64.
+//
+// Kernels take UP, the planes of the first product, 0 for the second, and wts,
+// the weights to apply or null.
 //
 //  * moe_skinny_kernel — up to 32 tokens: streams each chosen expert's weights
 //    once; a workgroup finds its expert's slots by scanning the ids itself, so
@@ -86,15 +94,20 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(
 // skinny: grid (N / 64, E), at most 32 tokens
 // ---------------------------------------------------------------------------
 
-// UP: A row = slot / top (the token), out row = slot, silu(gate) * up.
-// else: A row = slot, out row = slot, times wts[slot].
-template <bool UP, bool FULL>  // FULL: K % 256 == 0
+DEVINL float relu_sq(float z) {
+  const float r = fmaxf(z, 0.f);
+  return r * r;
+}
+
+// UP: A row = slot / top (the token), out row = slot, activation.
+// else: A row = slot, out row = slot.
+template <int UP, bool FULL>  // FULL: K % 256 == 0
 __global__ __launch_bounds__(256) void moe_skinny_kernel(
     const unsigned short* __restrict__ A, const unsigned short* __restrict__ W,
     const int* __restrict__ ids, const float* __restrict__ wts,
     unsigned short* __restrict__ C, int S, int top, int N, int K, int lda,
     int ldc) {
-  constexpr int NW = UP ? 2 : 1, U = 4, KSTEP = 256, RS = KSTEP + 8;
+  constexpr int NW = UP ? UP : 1, U = 4, KSTEP = 256, RS = KSTEP + 8;
   __shared__ __attribute__((aligned(16))) unsigned short at[32 * RS];
   __shared__ int slots[32];
   __shared__ int n_slots;
@@ -211,11 +224,10 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
       const int m = t * 16 + hi * 4 + r;
       if (m >= cnt) continue;
       const int sl = slots[m];
-      float v = acc[0][t][r];
-      if constexpr (UP)
-        v = v * sigmoid_f(v) * acc[1][t][r];
-      else
-        v *= wts[sl];
+      const float w = wts ? wts[sl] : 1.f;
+      float v = acc[0][t][r] * w;
+      if constexpr (UP == 2) v = v * sigmoid_f(v) * (acc[NW - 1][t][r] * w);
+      if constexpr (UP == 1) v = relu_sq(v);
       C[(long)sl * ldc + n0 + li] = f2bf(v);
     }
 }
@@ -232,13 +244,13 @@ DEVINL void copy16_to_lds(const unsigned short* g, unsigned char* l) {
 }
 
 // UP: A row = sorted slot / top, out row = sorted position, N = activations
-//     (128 per tile: 128 gate rows and 128 up rows of W).
+//     (two planes: 128 per tile, 128 gate rows and 128 up rows of W; one: 256).
 // else: A row = sorted position, out row = slot, 256 columns per tile.
 //
 // A BM x 256 tile per workgroup; each of the four waves holds all BM rows of
 // 64 columns, so a W fragment read from LDS feeds BM / 16 MFMAs. LDS rows are
 // 64 B (32 of K) in four 16 B pieces, piece c of row r at c ^ (r / 4 % 4).
-template <int BM, bool UP>
+template <int BM, int UP>
 __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
     const unsigned short* __restrict__ A, const unsigned short* __restrict__ W,
     const int* __restrict__ off, const int* __restrict__ sorted,
@@ -262,7 +274,7 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
   const int e = tiles[2 * rt];
   const int p0 = tiles[2 * rt + 1];
   const int cnt = min(BM, off[e + 1] - p0);
-  const int n0 = nt * (UP ? HN : BN);
+  const int n0 = nt * (UP == 2 ? HN : BN);
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
   const int lane = threadIdx.x & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
@@ -281,8 +293,8 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
     const int ch = (i * 4 + wave) * 64 + lane;
     const int r = ch / 4, c = (ch % 4) ^ ((r >> 2) & 3);
     const long wrow =
-        UP ? ((long)e * 2 + r / HN) * N + min(n0 + r % HN, N - 1)
-           : (long)e * N + min(n0 + r, N - 1);
+        UP == 2 ? ((long)e * 2 + r / HN) * N + min(n0 + r % HN, N - 1)
+                : (long)e * N + min(n0 + r, N - 1);
     bp[i] = W + wrow * K + c * 8;
   }
   auto issue = [&](int k, int buf) {
@@ -293,11 +305,11 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
     for (int i = 0; i < BI; ++i)
       copy16_to_lds(bp[i] + k, lds[buf] + BM * RB + (i * 4 + wave) * 1024);
   };
-  // W rows of this wave's four column tiles: UP pairs gate and up columns
+  // W rows of this wave's four column tiles: two planes pair gate and up columns
   int brow[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n)
-    brow[n] = (UP ? (n >> 1) * HN + wave * 32 + (n & 1) * 16
+    brow[n] = (UP == 2 ? (n >> 1) * HN + wave * 32 + (n & 1) * 16
                   : wave * 64 + n * 16) + li;
 
   f32x4 acc[MT][NT];
@@ -335,7 +347,9 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
   for (int m = 0; m < MT; ++m) {
     const int r = m * 16 + li;
     if (r >= cnt) continue;
-    if constexpr (UP) {
+    const int sl = sorted[p0 + r];
+    const float w = wts ? wts[sl] : 1.f;
+    if constexpr (UP == 2) {
 #pragma unroll
       for (int n = 0; n < 2; ++n) {
         const int col = n0 + wave * 32 + n * 16 + hi * 4;
@@ -343,22 +357,23 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
         float v[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          const float z = acc[m][n][j];
-          v[j] = z * sigmoid_f(z) * acc[m][n + 2][j];
+          const float z = acc[m][n][j] * w;
+          v[j] = z * sigmoid_f(z) * (acc[m][n + 2][j] * w);
         }
         stv<4>(C + (long)(p0 + r) * ldc + col, v);
       }
     } else {
-      const int sl = sorted[p0 + r];
-      const float w = wts[sl];
 #pragma unroll
       for (int n = 0; n < NT; ++n) {
         const int col = n0 + wave * 64 + n * 16 + hi * 4;
         if (col >= N) continue;
         float v[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = acc[m][n][j] * w;
-        stv<4>(C + (long)sl * ldc + col, v);
+        for (int j = 0; j < 4; ++j) {
+          v[j] = acc[m][n][j] * w;
+          if constexpr (UP == 1) v[j] = relu_sq(v[j]);
+        }
+        stv<4>(C + (long)(UP ? p0 + r : sl) * ldc + col, v);
       }
     }
   }
@@ -368,13 +383,13 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
 // plain f32: 64 x 64 tiles, same row tiles (BM = 64)
 // ---------------------------------------------------------------------------
 
-template <bool UP>
+template <int UP>
 __global__ __launch_bounds__(256) void moe_simple_kernel(
     const float* __restrict__ A, const float* __restrict__ W,
     const int* __restrict__ off, const int* __restrict__ sorted,
     const int* __restrict__ tiles, const float* __restrict__ wts,
     float* __restrict__ C, int top, int N, int K, int lda, int ldc) {
-  constexpr int NW = UP ? 2 : 1, BK = 16;
+  constexpr int NW = UP ? UP : 1, BK = 16;
   __shared__ float al[BK][64 + 4], wl[NW][BK][64 + 4];
   const int e = tiles[2 * blockIdx.y];
   if (e < 0) return;
@@ -406,12 +421,12 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(
     const int r = ty * 4 + i;
     if (r >= cnt) continue;
     const int sl = sorted[p0 + r];
+    const float w = wts ? wts[sl] : 1.f;
     for (int j = 0; j < 4; ++j) {
-      float v = acc[0][i][j];
-      if constexpr (UP)
-        C[(long)(p0 + r) * ldc + n0 + tx * 4 + j] = v * sigmoid_f(v) * acc[NW - 1][i][j];
-      else
-        C[(long)sl * ldc + n0 + tx * 4 + j] = v * wts[sl];
+      float v = acc[0][i][j] * w;
+      if constexpr (UP == 2) v = v * sigmoid_f(v) * (acc[NW - 1][i][j] * w);
+      if constexpr (UP == 1) v = relu_sq(v);
+      C[(long)(UP ? p0 + r : sl) * ldc + n0 + tx * 4 + j] = v;
     }
   }
 }

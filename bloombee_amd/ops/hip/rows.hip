@@ -4,11 +4,16 @@
 //     partials of its output GEMM, routed expert rows, identity-expert
 //     weights) into the 32-bit residual and emits the next layer's grouped
 //     RMS norm, in one pass per row. For norms after the sum the residual is
-//     scaled first and the normed row takes its place.
+//     scaled first and the normed row takes its place; for norms around a
+//     sublayer what is pending is normed before it is added.
 // proj_post_kernel — everything between the fused input GEMM and attention:
 //     folds split-K partials, RMS-norms q and k over the whole projection,
 //     writes K/V into the pages, hands on the output gate, applies the
 //     feed-forward activation and routes the token to its experts.
+// head_post_kernel — the same step for projections with biases, a norm per head
+//     and a query temperature, without feed-forward.
+// ff_post_kernel — feed-forward activation and routing of layers whose
+//     feed-forward has an input of its own.
 // clamped_glu_kernel — bias, clamps, gate and product of a gated feed-forward.
 // softcap_kernel — cap * tanh(z / cap), in place.
 // router_gemm_kernel — f32 router logits where the input GEMM emits bf16.
@@ -87,6 +92,32 @@ DEVINL void stv(float* p, const float* v) {
   }
 }
 
+// A GEMM's output as ks partial sums (N, ld).
+struct Parts {
+  const void* p;  // (ks, N, ld)
+  long stride;    // elements between splits
+  int ks, ld;
+};
+
+template <typename TP, int V>
+DEVINL void fold_parts(const Parts& a, long t, int c, float* o) {
+  const TP* row = (const TP*)a.p + t * (long)a.ld + c;
+  ldv<V>(row, o);
+  for (int s = 1; s < a.ks; ++s) {
+    float u[V];
+    ldv<V>(row + s * a.stride, u);
+#pragma unroll
+    for (int j = 0; j < V; ++j) o[j] += u[j];
+  }
+}
+
+// turns: frequency / 2 pi
+DEVINL void rotation(int pos, double turns, float& c, float& s) {
+  double r = (double)pos * turns;
+  r -= rint(r);
+  sincospif(2.f * (float)r, &s, &c);
+}
+
 DEVINL float sigmoid_f(float z) {
   return __builtin_amdgcn_rcpf(1.f + fast_exp2(-z * LOG2E));
 }
@@ -112,6 +143,7 @@ struct ResidualArgs {
   const float* idw;    // (N,) weight of the layer's own input, or null
   const void* hprev;   // (N, ldhp) that input
   const float* bias;   // (W,) of the pending GEMM, or null
+  const float* bw;     // (W,) norm weight of what is pending; null = no norm
   const float* nw;     // (W,) norm weight; null = fold only
   void* h;             // (N, ldh) normed row, zero beyond W
   int W, ks, ldp, top, ldr, ldhp, ldh, groups;
@@ -119,7 +151,7 @@ struct ResidualArgs {
   float eps, alpha;    // alpha scales x before the sum
 };
 
-// LDS: W floats (the row) + groups * subs partial sums.
+// LDS: W floats (the row) + at least 32 and groups * subs partial sums.
 template <typename TP, typename T, int V, int BLOCK>
 __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
   extern __shared__ float lds_row[];
@@ -132,51 +164,95 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
   const T* hp = (const T*)a.hprev + t * (long)a.ldhp;
   const float iw = a.idw ? a.idw[t] : 0.f;
 
-  for (int i = threadIdx.x * V; i < W; i += BLOCK * V) {
-    float v[V], u[V];
-    ldv<V>(xr + i, v);
-#pragma unroll
-    for (int j = 0; j < V; ++j) v[j] *= a.alpha;
+  // what is pending at columns i..
+  auto owed = [&](int i, float* d) {
+    float u[V];
     if (a.parts) {
-      float d[V];
       ldv<V>(pr + i, d);
       for (int s = 1; s < a.ks; ++s) {
         ldv<V>(pr + s * a.pstride + i, u);
 #pragma unroll
         for (int j = 0; j < V; ++j) d[j] += u[j];
       }
-      if (a.routed) {
-        for (int k = 0; k < a.top; ++k) {
-          if (a.ids[t * a.top + k] < 0) continue;
-          ldv<V>(rr + (long)k * a.ldr + i, u);
+    } else {
 #pragma unroll
-          for (int j = 0; j < V; ++j) d[j] += u[j];
-        }
-      }
-      if (iw != 0.f) {
-        ldv<V>(hp + i, u);
-#pragma unroll
-        for (int j = 0; j < V; ++j) d[j] += iw * u[j];
-      }
-      if (a.bias) {
-        ldv<V>(a.bias + i, u);
+      for (int j = 0; j < V; ++j) d[j] = 0.f;
+    }
+    if (a.routed) {
+      for (int k = 0; k < a.top; ++k) {
+        if (a.ids[t * a.top + k] < 0) continue;
+        ldv<V>(rr + (long)k * a.ldr + i, u);
 #pragma unroll
         for (int j = 0; j < V; ++j) d[j] += u[j];
       }
+    }
+    if (iw != 0.f) {
+      ldv<V>(hp + i, u);
 #pragma unroll
-      for (int j = 0; j < V; ++j) v[j] += d[j];
+      for (int j = 0; j < V; ++j) d[j] += iw * u[j];
+    }
+    if (a.bias) {
+      ldv<V>(a.bias + i, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) d[j] += u[j];
+    }
+  };
+  constexpr int NWAVE = BLOCK / WAVE;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const bool some = a.parts || a.routed;
+  if (a.bw && some) {
+    float ss = 0.f;
+    for (int i = threadIdx.x * V; i < W; i += BLOCK * V) {
+      float d[V];
+      owed(i, d);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        lds_row[i + j] = d[j];
+        ss += d[j] * d[j];
+      }
+    }
+    ss = wave_reduce_sum(ss);
+    if (lane == 0) stat[wave] = ss;
+    __syncthreads();
+    ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NWAVE; ++k) ss += stat[k];
+    const float inv = 1.f / sqrtf(ss / (float)W + a.eps);
+    __syncthreads();   // stat is written again below
+    // a thread reads back what it wrote
+    for (int i = threadIdx.x * V; i < W; i += BLOCK * V) {
+      float v[V], w[V];
+      ldv<V>(xr + i, v);
+      ldv<V>(a.bw + i, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        v[j] = v[j] * a.alpha + lds_row[i + j] * inv * w[j];
+        lds_row[i + j] = v[j];
+      }
       if (!a.post) stv<V>(xr + i, v);
     }
+  } else {
+    for (int i = threadIdx.x * V; i < W; i += BLOCK * V) {
+      float v[V];
+      ldv<V>(xr + i, v);
 #pragma unroll
-    for (int j = 0; j < V; ++j) lds_row[i + j] = v[j];
+      for (int j = 0; j < V; ++j) v[j] *= a.alpha;
+      if (some) {
+        float d[V];
+        owed(i, d);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[j] += d[j];
+        if (!a.post) stv<V>(xr + i, v);
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) lds_row[i + j] = v[j];
+    }
   }
   if (!a.nw) return;
   __syncthreads();
 
   // sums of squares: every unit (a group, or an even share of one where
   // there are fewer groups than waves) belongs to one wave
-  constexpr int NWAVE = BLOCK / WAVE;
-  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   const int gs = W / a.groups;
   const int subs = a.groups >= NWAVE ? 1 : NWAVE / a.groups;
   for (int un = wave; un < a.groups * subs; un += NWAVE) {
@@ -268,32 +344,138 @@ __global__ __launch_bounds__(256) void softcap_kernel(float* __restrict__ z,
     z[i] = cap * tanhf(z[i] / cap);
 }
 
-// x[n] = table[ids[n]] (+ pos_table[pos[n]]) in f32; indices are clamped.
+struct EmbedArgs {
+  const int* ids;
+  const int* pos;
+  const int* prev;      // token before each, < 0 = none; with pair_table only
+  const void* table;    // (vocab, W)
+  const void* pos_table;   // (max_pos, W) or null: learned positions
+  const void* pair_table;  // (buckets + 1, W) or null: rows of token pairs
+  const double* turns;     // ((W + 1) / 2,) or null: sines and cosines
+  float* x;                // (N, W)
+  long buckets, mul_prev, mul_cur;
+  int W, vocab, max_pos;
+};
+
+// x[n] = table[ids[n]] (+ pos_table[pos[n]]) (+ pair_table[row of the pair])
+// (+ sin at 2i, cos at 2i + 1 of pos[n] * frequency i) in f32; indices are
+// clamped. A token without a predecessor takes the pair table's last row.
 template <typename T>
-__global__ __launch_bounds__(256) void embed_rows_kernel(
-    const int* __restrict__ ids, const int* __restrict__ pos,
-    const T* __restrict__ table, const T* __restrict__ pos_table,
-    float* __restrict__ x, int W, int vocab, int max_pos) {
+__global__ __launch_bounds__(256) void embed_rows_kernel(EmbedArgs a) {
   const long n = blockIdx.x;
-  const T* a = table + (long)min(max(ids[n], 0), vocab - 1) * W;
-  if (!pos_table) {
-    for (int i = threadIdx.x; i < W; i += 256) x[n * W + i] = ldf(a + i);
-    return;
+  const int W = a.W, id = min(max(a.ids[n], 0), a.vocab - 1);
+  const T* e = (const T*)a.table + (long)id * W;
+  const T *p = nullptr, *q = nullptr;
+  if (a.pos_table)
+    p = (const T*)a.pos_table + (long)min(max(a.pos[n], 0), a.max_pos - 1) * W;
+  if (a.pair_table) {
+    const int b = a.prev[n];
+    const long r = b < 0 ? a.buckets
+                         : (min(b, a.vocab - 1) * a.mul_prev + id * a.mul_cur) %
+                               a.buckets;
+    q = (const T*)a.pair_table + r * W;
   }
-  const T* b = pos_table + (long)min(max(pos[n], 0), max_pos - 1) * W;
-  for (int i = threadIdx.x; i < W; i += 256) x[n * W + i] = ldf(a + i) + ldf(b + i);
+  for (int i = threadIdx.x; i < W; i += 256) {
+    float v = ldf(e + i);
+    if (p) v += ldf(p + i);
+    if (q) v += ldf(q + i);
+    if (a.turns) {
+      float c, s;
+      rotation(max(a.pos[n], 0), a.turns[i / 2], c, s);
+      v += i & 1 ? c : s;
+    }
+    a.x[n * W + i] = v;
+  }
 }
 
 // ---------------------------------------------------------------------------
 
+static constexpr int MAX_ROUTED = 1024;  // router outputs
+
+struct RouteArgs {
+  const float* parts;   // (ks, N, ld) router logits, f32
+  long stride;
+  const float* corr;    // (E + NI,) added to the scores for the choice only,
+                        // or null
+  int* ids;             // (N, top)
+  float* wts;           // (N, top)
+  float* idw;           // (N,) or null
+  int ks, ld, off, E, NI, top;
+  int sigmoid;          // scores: sigmoid of each logit, else softmax
+  float scale;
+};
+
+DEVINL float router_logit(const RouteArgs& a, long t, int c) {
+  const float* r = a.parts + t * a.ld + c;
+  float v = r[0];
+  for (int s = 1; s < a.ks; ++s) v += r[s * a.stride];
+  return v;
+}
+
+// Chooses token t's experts; one wave. LDS: s and ch, MAX_ROUTED each.
+DEVINL void route_row(const RouteArgs& a, long t, float* s, float* ch) {
+  const int n = a.E + a.NI, lane = threadIdx.x & (WAVE - 1);
+  float inv = 1.f;
+  if (a.sigmoid) {
+    for (int i = lane; i < n; i += WAVE)
+      s[i] = 1.f / (1.f + expf(-router_logit(a, t, a.off + i)));
+  } else {
+    float mx = NEG_BIG;
+    for (int i = lane; i < n; i += WAVE) {
+      const float z = router_logit(a, t, a.off + i);
+      s[i] = z;
+      mx = fmaxf(mx, z);
+    }
+    mx = wave_reduce_max(mx);
+    float sum = 0.f;
+    for (int i = lane; i < n; i += WAVE) {
+      s[i] = expf(s[i] - mx);
+      sum += s[i];
+    }
+    inv = 1.f / wave_reduce_sum(sum);
+  }
+  for (int i = lane; i < n; i += WAVE) {
+    s[i] *= inv;
+    ch[i] = s[i] + (a.corr ? a.corr[i] : 0.f);
+  }
+  // every lane reads and writes its own columns only
+  float idw = 0.f;
+  for (int k = 0; k < a.top; ++k) {
+    float best = -__builtin_inff();
+    int at = n;
+    for (int i = lane; i < n; i += WAVE)
+      if (ch[i] > best || at == n) { best = ch[i]; at = i; }
+#pragma unroll
+    for (int m = 1; m < WAVE; m <<= 1) {
+      const float ob = __shfl_xor(best, m);
+      const int oa = __shfl_xor(at, m);
+      if (oa < n && (at == n || ob > best || (ob == best && oa < at))) {
+        best = ob;
+        at = oa;
+      }
+    }
+    // the owning lane holds the score; broadcast it
+    float w = 0.f;
+    if ((at & (WAVE - 1)) == lane) {
+      w = s[at] * a.scale;
+      ch[at] = -__builtin_inff();
+    }
+    w = __shfl(w, at & (WAVE - 1));
+    if (at >= a.E) idw += w;
+    if (lane == 0) {
+      a.ids[t * a.top + k] = at < a.E ? at : -1;
+      a.wts[t * a.top + k] = w;
+    }
+  }
+  if (lane == 0 && a.idw) a.idw[t] = idw;
+}
+
 struct PostArgs {
   const void* parts;    // (ks, N, ldp) input GEMM output
   long pstride;
-  const float* rparts;  // (rks, N, ldr) router logits, f32
-  long rstride;
+  RouteArgs rt;         // router, and the shared expert's gate at rt column sg_off
   const float* qn;      // (H*dim,) q norm weight
   const float* kn;      // (G*dim,)
-  const float* corr;    // (E + NI,) added to the scores for the choice only
   void* q;              // (N, H, dkp)
   void* gate;           // (N, H*vdim) or null: the reader takes it from parts
   void* a2;             // (N, lda2): [attention | activation | zeros]
@@ -302,23 +484,17 @@ struct PostArgs {
   const int* table;     // (S, maxp)
   const int* tok_seq;
   const int* tok_pos;
-  int* ids;             // (N, top)
-  float* wts;           // (N, top)
-  float* idw;           // (N,)
-  int ks, ldp, rks, ldr;
-  int q_off, k_off, v_off, g_off, u_off, u2_off, r_off, sg_off;
+  int ks, ldp;
+  int q_off, k_off, v_off, g_off, u_off, u2_off, sg_off;
   int H, G, dim, vdim, dkp, dvp, P, maxp;
   int has_kv;
   int act;              // 0 none, 1 xIELU, 2 silu(gate) * up
   int ff, act_col, lda2;
-  int E, NI, top;
-  float eps, xp, xq, rscale;
+  float eps, xp, xq;
 };
 
 static constexpr int POST_BLOCK = 256;
 static constexpr int POST_CHUNK = 2048;  // elementwise columns per workgroup
-static constexpr int MAX_ROUTED = 1024;  // router outputs
-
 template <typename TP, int V>
 DEVINL void fold(const PostArgs& a, const TP* row, int c, float* o) {
   ldv<V>(row + c, o);
@@ -328,13 +504,6 @@ DEVINL void fold(const PostArgs& a, const TP* row, int c, float* o) {
 #pragma unroll
     for (int j = 0; j < V; ++j) o[j] += u[j];
   }
-}
-
-DEVINL float router_logit(const PostArgs& a, long t, int c) {
-  const float* r = a.rparts + t * a.ldr + c;
-  float v = r[0];
-  for (int s = 1; s < a.rks; ++s) v += r[s * a.rstride];
-  return v;
 }
 
 // One projection section of n columns into LDS; returns 1 / rms over all n.
@@ -411,58 +580,8 @@ __global__ __launch_bounds__(POST_BLOCK) void proj_post_kernel(PostArgs a) {
     return;
   }
   if (role == 2) {
-    const int n = a.E + a.NI;
-    if (n == 0 || threadIdx.x >= WAVE) return;
-    float* s = lds_sec;                // scores
-    float* ch = lds_sec + MAX_ROUTED;  // choice scores
-    const int lane = threadIdx.x;
-    float mx = NEG_BIG;
-    for (int i = lane; i < n; i += WAVE) {
-      const float z = router_logit(a, t, a.r_off + i);
-      s[i] = z;
-      mx = fmaxf(mx, z);
-    }
-    mx = wave_reduce_max(mx);
-    float sum = 0.f;
-    for (int i = lane; i < n; i += WAVE) {
-      s[i] = expf(s[i] - mx);
-      sum += s[i];
-    }
-    const float inv = 1.f / wave_reduce_sum(sum);
-    for (int i = lane; i < n; i += WAVE) {
-      s[i] *= inv;
-      ch[i] = s[i] + a.corr[i];
-    }
-    // every lane reads and writes its own columns only
-    float idw = 0.f;
-    for (int k = 0; k < a.top; ++k) {
-      float best = -__builtin_inff();
-      int at = n;
-      for (int i = lane; i < n; i += WAVE)
-        if (ch[i] > best || at == n) { best = ch[i]; at = i; }
-#pragma unroll
-      for (int m = 1; m < WAVE; m <<= 1) {
-        const float ob = __shfl_xor(best, m);
-        const int oa = __shfl_xor(at, m);
-        if (oa < n && (at == n || ob > best || (ob == best && oa < at))) {
-          best = ob;
-          at = oa;
-        }
-      }
-      // the owning lane holds the score; broadcast it
-      float w = 0.f;
-      if ((at & (WAVE - 1)) == lane) {
-        w = s[at] * a.rscale;
-        ch[at] = -__builtin_inff();
-      }
-      w = __shfl(w, at & (WAVE - 1));
-      if (at >= a.E) idw += w;
-      if (lane == 0) {
-        a.ids[t * a.top + k] = at < a.E ? at : -1;
-        a.wts[t * a.top + k] = w;
-      }
-    }
-    if (lane == 0) a.idw[t] = idw;
+    if (a.rt.E + a.rt.NI > 0 && threadIdx.x < WAVE)
+      route_row(a.rt, t, lds_sec, lds_sec + MAX_ROUTED);
     return;
   }
 
@@ -473,7 +592,7 @@ __global__ __launch_bounds__(POST_BLOCK) void proj_post_kernel(PostArgs a) {
   const int base = (role - 3) * POST_CHUNK;
   const int end = min(base + POST_CHUNK, total);
   float sg = 1.f;
-  if (a.act == 2) sg = sigmoid_f(router_logit(a, t, a.sg_off));
+  if (a.act == 2) sg = sigmoid_f(router_logit(a.rt, t, a.sg_off));
   for (int i = base + threadIdx.x * V; i < end; i += POST_BLOCK * V) {
     float v[V];
     if (i < gn) {
@@ -501,6 +620,139 @@ __global__ __launch_bounds__(POST_BLOCK) void proj_post_kernel(PostArgs a) {
       }
     }
     stv<V>((T*)a.a2 + t * (long)a.lda2 + c, v);
+  }
+}
+
+// ---------------------------------------------------------------------------
+
+struct HeadPostArgs {
+  Parts y;              // q, k, v columns
+  const float* qb;      // biases (H*dim,), (G*dim,), (G*vdim,), or null
+  const float* kb;
+  const float* vb;
+  const float* qn;      // (dim,) norm weights, shared by the heads
+  const float* kn;
+  void* q;              // (N, H, dkp)
+  void* kp;             // (np, G, P, dkp)
+  void* vp;             // (np, G, dvp, P)
+  const int* table;     // (S, maxp)
+  const int* tok_seq;
+  const int* tok_pos;
+  int q_off, k_off, v_off, H, G, dim, vdim, dkp, dvp, P, maxp;
+  float eps;
+  float temp_coef;      // query temperature 1 + coef ln(floor((pos+1)/every)+1)
+  double temp_every;
+};
+
+// grid (N, (H + 2 G) / 4), a wave a head: q heads, k heads, v heads. LDS: four
+// heads of dim.
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(256) void head_post_kernel(HeadPostArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds_head[];
+  const long t = blockIdx.x;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int unit = blockIdx.y * 4 + wave;
+  if (unit >= a.H + 2 * a.G) return;
+  const int pos = a.tok_pos[t];
+  const bool is_q = unit < a.H;
+  if (!is_q && pos < 0) return;   // an empty slot writes no K/V
+  long page = 0;
+  int slot = 0;
+  if (!is_q) {
+    page = a.table[(long)a.tok_seq[t] * a.maxp + pos / a.P];
+    slot = pos % a.P;
+  }
+  if (unit >= a.H + a.G) {
+    const int g = unit - a.H - a.G;
+    T* vp = (T*)a.vp + ((page * a.G + g) * a.dvp) * (long)a.P + slot;
+    for (int d = lane; d < a.dvp; d += WAVE) {
+      float v[1] = {0.f};
+      if (d < a.vdim) {
+        fold_parts<TP, 1>(a.y, t, a.v_off + g * a.vdim + d, v);
+        if (a.vb) v[0] += a.vb[g * a.vdim + d];
+      }
+      stf(vp + (long)d * a.P, v[0]);
+    }
+    return;
+  }
+  const int h = is_q ? unit : unit - a.H;
+  const float* bias = is_q ? a.qb : a.kb;
+  const float* nw = is_q ? a.qn : a.kn;
+  float* row = lds_head + wave * ((a.dim + 7) & ~7);
+  float ss = 0.f;
+  for (int i = lane * V; i < a.dim; i += WAVE * V) {
+    float v[V], b[V];
+    fold_parts<TP, V>(a.y, t, (is_q ? a.q_off : a.k_off) + h * a.dim + i, v);
+    if (bias) {
+      ldv<V>(bias + h * a.dim + i, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] += b[j];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      row[i + j] = v[j];
+      ss += v[j] * v[j];
+    }
+  }
+  float f = 1.f / sqrtf(wave_reduce_sum(ss) / (float)a.dim + a.eps);
+  if (is_q && a.temp_coef != 0.f)
+    f *= 1.f + a.temp_coef *
+                   logf((float)(floor((double)(max(pos, 0) + 1) / a.temp_every) + 1.0));
+  T* o = is_q ? (T*)a.q + (t * a.H + h) * (long)a.dkp
+              : (T*)a.kp + ((page * a.G + h) * a.P + slot) * (long)a.dkp;
+  // a lane reads back what it wrote
+  for (int i = lane * V; i < a.dkp; i += WAVE * V) {
+    float v[V], w[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    if (i < a.dim) {
+      ldv<V>(nw + i, w);
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = row[i + j] * f * w[j];
+    }
+    stv<V>(o + i, v);
+  }
+}
+
+struct FfPostArgs {
+  Parts y;              // feed-forward columns, or null
+  RouteArgs rt;         // E = 0: no router
+  void* out;            // (N, ldo), zero beyond ff
+  int act;              // 1 silu(gate) * up, 2 relu(up)^2
+  int u_off, u2_off, ff, ldo;  // act 1: gate, up; act 2: up
+};
+
+// grid (N, 1 + chunks): y = 0 router, 1.. elementwise.
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(POST_BLOCK) void ff_post_kernel(FfPostArgs a) {
+  __shared__ float lds_rt[2 * MAX_ROUTED];
+  const long t = blockIdx.x;
+  if (blockIdx.y == 0) {
+    if (a.rt.E + a.rt.NI > 0 && threadIdx.x < WAVE)
+      route_row(a.rt, t, lds_rt, lds_rt + MAX_ROUTED);
+    return;
+  }
+  const int base = (blockIdx.y - 1) * POST_CHUNK;
+  const int end = min(base + POST_CHUNK, a.ldo);
+  for (int i = base + threadIdx.x * V; i < end; i += POST_BLOCK * V) {
+    float v[V], u[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] = 0.f;
+    if (i < a.ff) {
+      fold_parts<TP, V>(a.y, t, a.u_off + i, v);
+      if (a.act == 1) {
+        fold_parts<TP, V>(a.y, t, a.u2_off + i, u);
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[j] = v[j] * sigmoid_f(v[j]) * u[j];
+      } else {
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          const float r = fmaxf(v[j], 0.f);
+          v[j] = r * r;
+        }
+      }
+    }
+    stv<V>((T*)a.out + t * (long)a.ldo + i, v);
   }
 }
 

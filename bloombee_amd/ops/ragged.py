@@ -12,7 +12,10 @@ token):
   linear_parts   [attention | activation] @ [W_o | W_down]^T, left Pending
 
 Layers with a norm after every sum use sum_norm instead, and clamped_glu for
-their feed-forward; other mixers are in ops/mixers.py.
+their feed-forward. Layers with a norm around every sublayer leave sums Pending
+with the norm they pass first; where attention and feed-forward have inputs of
+their own, head_post and ff_post take proj_post's place. Other mixers are in
+ops/mixers.py and ops/recurrent.py.
 
 Device tensors run the _hip_ragged extension and fail loudly without it; CPU
 tensors run the forms in ops/reference.py. Activations are bf16 or f32; the
@@ -73,20 +76,23 @@ def pad_k(k: int) -> int:
 class Routing:
     ids: torch.Tensor   # (N, top) int32, -1 = identity expert
     wts: torch.Tensor   # (N, top) f32
-    idw: torch.Tensor   # (N,) f32: summed weight of identity experts
+    idw: Optional[torch.Tensor]   # (N,) f32: summed weight of identity experts
 
 
 @dataclass
 class Pending:
     """What a layer still owes the residual: the output GEMM's partials and,
-    for routed layers, the experts' rows and the layer's own input."""
-    parts: torch.Tensor                      # (ks, N, >= W)
+    for routed layers, the experts' rows and the layer's own input; with norm,
+    all of it is RMS-normed with these weights first."""
+    parts: Optional[torch.Tensor]            # (ks, N, >= W)
     routed: Optional[torch.Tensor] = None    # (N, top, >= W)
     routing: Optional[Routing] = None
     h: Optional[torch.Tensor] = None         # (N, >= W)
+    norm: Optional[torch.Tensor] = None      # (W,) f32
+    eps: float = 0.0                         # of that norm
 
     def settle(self, x: torch.Tensor) -> None:
-        residual_norm(x, self)
+        residual_norm(x, self, eps=self.eps)
 
 
 @dataclass
@@ -105,25 +111,30 @@ def residual_norm(x: torch.Tensor, pending: Optional[Pending],
                   dtype: torch.dtype = torch.bfloat16,
                   ) -> Optional[torch.Tensor]:
     """x (N, W) f32 += pending, in place; returns norm(x) as (N, cols) in
-    dtype with zero columns beyond W, or None without a weight."""
+    dtype with zero columns beyond W, or None without a weight. eps is that of
+    the pending sum's own norm, too, if it has one."""
     N, W = x.shape
     p = pending
     rt = p.routing if p is not None else None
+    idw = rt.idw if rt is not None else None
     if x.is_cuda:
         h = (torch.empty(N, cols or W, dtype=dtype, device=x.device)
              if weight is not None else None)
         _ext().residual_norm(
             x, p.parts if p else None,
             p.routed if p and p.routed is not None else None,
-            rt.ids if rt else None, rt.idw if rt else None,
-            p.h if rt else None, weight, groups, eps, h, 1.0, None, False)
+            rt.ids if rt else None, idw, p.h if idw is not None else None,
+            weight, groups, eps, h, 1.0, None, False, p.norm if p else None)
         return h
     if p is not None:
-        d = p.parts.float().sum(0)[:, :W]
-        if rt is not None:
-            if p.routed is not None:
-                d = d + p.routed.float().sum(1)[:, :W]
-            d = d + rt.idw[:, None] * p.h[:, :W].float()
+        d = (p.parts.float().sum(0)[:, :W] if p.parts is not None
+             else torch.zeros_like(x))
+        if p.routed is not None:
+            d = d + p.routed.float().sum(1)[:, :W]
+        if idw is not None:
+            d = d + idw[:, None] * p.h[:, :W].float()
+        if p.norm is not None:
+            d = ref.grouped_rms_norm(d, p.norm, 1, eps)
         x += d
     if weight is None:
         return None
@@ -141,7 +152,7 @@ def sum_norm(x: torch.Tensor, parts: torch.Tensor,
     if x.is_cuda:
         h = torch.empty(N, cols, dtype=dtype, device=x.device)
         _ext().residual_norm(x, parts, None, None, None, None, weight, 1, eps,
-                             h, alpha, bias, True)
+                             h, alpha, bias, True, None)
         return h
     y = alpha * x + parts.float().sum(0)[:, :W]
     if bias is not None:
@@ -182,19 +193,63 @@ def softcap_(z: torch.Tensor, cap: float) -> torch.Tensor:
     return z.div_(cap).tanh_().mul_(cap)
 
 
+def sinusoid_turns(width: int) -> torch.Tensor:
+    """Frequencies 10000^(-2 i / width) over 2 pi of a sinusoidal position
+    vector, sine at entry 2 i and cosine at 2 i + 1; float64."""
+    i = torch.arange((width + 1) // 2, dtype=torch.float64)
+    base = torch.tensor(10000.0, dtype=torch.float64)
+    return torch.pow(base, -2.0 * i / width) / (2 * torch.pi)
+
+
+@dataclass
+class PairTable:
+    """Embedding of token pairs: row (previous * mul_prev + token * mul_cur)
+    mod buckets, the last row where there is no previous token."""
+    table: torch.Tensor   # (buckets + 1, W)
+    mul_prev: int
+    mul_cur: int
+
+    @property
+    def buckets(self) -> int:
+        return self.table.shape[0] - 1
+
+    def rows(self, ids: torch.Tensor, prev: torch.Tensor) -> torch.Tensor:
+        r = (prev.long() * self.mul_prev + ids.long() * self.mul_cur) \
+            % self.buckets
+        return torch.where(prev < 0, self.buckets, r)
+
+
+def previous_ids(ids: torch.Tensor, last: torch.Tensor) -> torch.Tensor:
+    """The token before each of ids (B, T); last (B,): the one before a row's
+    first, -1 = none."""
+    last = last.to(device=ids.device, dtype=ids.dtype).view(-1, 1)
+    return torch.cat([last, ids[:, :-1]], 1)
+
+
 def embed_rows(ids: torch.Tensor, positions: torch.Tensor,
                table: torch.Tensor, pos_table: Optional[torch.Tensor],
-               ) -> torch.Tensor:
-    """table[ids] (+ pos_table[positions]) in f32, (..., W)."""
+               prev: Optional[torch.Tensor] = None,
+               pairs: Optional[PairTable] = None,
+               turns: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """table[ids] (+ pos_table[positions]) (+ the row of each token and its
+    predecessor) (+ sinusoidal positions) in f32, (..., W)."""
     if table.is_cuda:
-        x = _ext().embed_rows(ids.reshape(-1).int(),
-                              positions.reshape(-1).int(), table, pos_table)
+        x = _ext().embed_rows(
+            ids.reshape(-1).int(), positions.reshape(-1).int(), table, pos_table,
+            prev.reshape(-1).int() if pairs is not None else None,
+            pairs.table if pairs is not None else None,
+            [pairs.buckets, pairs.mul_prev, pairs.mul_cur]
+            if pairs is not None else [], turns)
         return x.view(*ids.shape, -1)
-    if pos_table is None:
-        return F.embedding(ids.long(), table).float()
+    x = F.embedding(ids.long(), table).float()
     pos = positions.long().clamp(min=0)
-    return (F.embedding(ids.long(), table).float()
-            + F.embedding(pos, pos_table).float())
+    if pos_table is not None:
+        x = x + F.embedding(pos, pos_table).float()
+    if pairs is not None:
+        x = x + F.embedding(pairs.rows(ids, prev), pairs.table).float()
+    if turns is not None:
+        x = x + ref.sinusoid(pos, turns, table.shape[1])
+    return x
 
 
 def linear_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -256,9 +311,10 @@ class ProjSpec:
         return self.experts + self.identity > 0
 
 
-def input_projection(h: torch.Tensor, w: torch.Tensor, spec: ProjSpec,
+def input_projection(h: torch.Tensor, w: torch.Tensor, spec,
                      ) -> Tuple[torch.Tensor, Optional[torch.Tensor], int]:
-    """(parts, router parts, first router column in them)."""
+    """(parts, router parts, first router column in them). The router's columns
+    spec.router_off .. + router_n, the last ones, are computed in f32."""
     r = spec.router_off
     if r < 0:
         return linear_parts(h, w), None, 0
@@ -344,14 +400,119 @@ def proj_post(parts: torch.Tensor, rparts: Optional[torch.Tensor], r0: int,
     return q, gate, a2, rt
 
 
-def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
-                rt: Routing) -> torch.Tensor:
+@dataclass
+class HeadSpec:
+    """A q, k, v projection with biases and a norm per head, and the columns of
+    its sections. temp_coef, temp_every: queries are multiplied by
+    1 + coef * ln(floor((position + 1) / every) + 1)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    eps: float
+    q_off: int = 0
+    k_off: int = 0
+    v_off: int = 0
+    temp_coef: float = 0.0
+    temp_every: float = 1.0
+    router_off: int = -1
+
+
+def head_post(parts: torch.Tensor, spec: HeadSpec, biases, q_norm: torch.Tensor,
+              k_norm: torch.Tensor, batch, k_pages: torch.Tensor,
+              v_pages: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """Normed queries (N, H, stored dim); keys and values go to the pages.
+    biases: of q, k and v, each (columns,) f32 or None; q_norm, k_norm (dim,)."""
+    s = spec
+    _, N, _ = parts.shape
+    H, G, D, V = s.heads, s.kv_heads, s.dim, s.vdim
+    dkp = k_pages.shape[3]
+    if parts.is_cuda:
+        q = torch.empty(N, H, dkp, dtype=dtype, device=parts.device)
+        _ext().head_post(
+            parts, [s.q_off, s.k_off, s.v_off, H, G, D, V],
+            [s.eps, s.temp_coef, s.temp_every], *biases, q_norm, k_norm, q,
+            k_pages, v_pages, batch.page_table, batch.tok_seq, batch.tok_pos)
+        return q
+    y = parts.float().sum(0)
+
+    def heads(off, n, d, bias):
+        t = y[:, off:off + n * d]
+        return (t if bias is None else t + bias).reshape(N, n, d)
+
+    q = ref.grouped_rms_norm(heads(s.q_off, H, D, biases[0]), q_norm, 1, s.eps)
+    q = q * ref.query_temperature(batch.tok_pos, s.temp_coef,
+                                  s.temp_every).view(N, 1, 1)
+    k = ref.grouped_rms_norm(heads(s.k_off, G, D, biases[1]), k_norm, 1, s.eps)
+    v = heads(s.v_off, G, V, biases[2])
+    P = k_pages.shape[2]
+    live = (batch.tok_pos >= 0).nonzero()[:, 0]
+    pos = batch.tok_pos[live].long()
+    page = batch.page_table[batch.tok_seq[live].long(), pos // P].long()
+    k_pages[page, :, pos % P, :D] = k[live].to(dtype)
+    v_pages[page, :, :V, pos % P] = v[live].to(dtype)
+    return F.pad(q, (0, dkp - D)).to(dtype)
+
+
+@dataclass
+class FfSpec:
+    """A feed-forward's input projection: dense columns (one activation), then
+    the router's, which start a 64-row block."""
+    act: int = 0             # 0 none, 1 silu(gate) * up, 2 relu(up)^2
+    ff: int = 0
+    gate_off: int = -1
+    up_off: int = -1
+    cols: int = 0            # inner size of the output projection
+    router_off: int = -1
+    router_n: int = 0
+    top: int = 0
+    sigmoid: bool = False    # scores: sigmoid, else softmax
+    scale: float = 1.0
+
+
+def ff_post(parts: Optional[torch.Tensor], rparts: Optional[torch.Tensor],
+            r0: int, spec: FfSpec, correction: Optional[torch.Tensor], n: int,
+            device, dtype: torch.dtype):
+    """Activations (N, cols), zero beyond ff, and Routing or None."""
+    s, E = spec, spec.router_n
+    if parts is not None and parts.is_cuda or rparts is not None and rparts.is_cuda:
+        out = torch.empty(n, s.cols, dtype=dtype, device=device)
+        rt = None
+        if E:
+            rt = Routing(
+                torch.empty(n, s.top, dtype=torch.int32, device=device),
+                torch.empty(n, s.top, dtype=torch.float32, device=device), None)
+        first = s.gate_off if s.act == 1 else s.up_off
+        _ext().ff_post(
+            parts if s.act else None, rparts if E else None,
+            [s.act, first, s.up_off, s.ff, r0, E, 0, s.top, int(s.sigmoid)],
+            s.scale, correction, out, rt.ids if rt else None,
+            rt.wts if rt else None, None)
+        return out, rt
+    out = torch.zeros(n, s.cols, dtype=dtype)
+    if s.act:
+        y = parts.float().sum(0)
+        u = y[:, s.up_off:s.up_off + s.ff]
+        a = (F.silu(y[:, s.gate_off:s.gate_off + s.ff]) * u if s.act == 1
+             else torch.relu(u) ** 2)
+        out[:, :s.ff] = a.to(dtype)
+    rt = None
+    if E:
+        ids, wts, _ = ref.route_topk(rparts.sum(0)[:, r0:r0 + E], correction, E,
+                                     s.top, s.scale, s.sigmoid)
+        rt = Routing(ids, wts, None)
+    return out, rt
+
+
+def moe_experts(h: torch.Tensor, up: torch.Tensor, down: torch.Tensor,
+                rt: Routing, weight_input: bool = False) -> torch.Tensor:
     """(N, top, W) weighted outputs of the chosen experts; the rows of
-    identity choices are not defined. gate_up (E, 2, F, K), down (E, W, F),
-    K, F and W padded to 64."""
+    identity choices are not defined. up (E, 2, F, K): silu(gate) * up, or
+    (E, 1, F, K): relu(up)^2; down (E, W, F); K, F and W padded to 64. The
+    weight multiplies an expert's output, or its input."""
     if h.is_cuda:
-        return _ext().moe_experts(h, gate_up, down, rt.ids, rt.wts)
-    return ref.moe_experts(h, gate_up, down, rt.ids, rt.wts)
+        return _ext().moe_experts(h, up, down, rt.ids, rt.wts, weight_input)
+    return ref.moe_experts(h, up, down, rt.ids, rt.wts, weight_input)
 
 
 def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor,

@@ -462,14 +462,16 @@ def xielu(z: torch.Tensor, pos: float, neg: float) -> torch.Tensor:
 
 
 def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
-               top: int, scale: float):
-    """Softmax scores; the choice adds `correction`, the weights do not and
+               top: int, scale: float, sigmoid: bool = False):
+    """Softmax (or sigmoid) scores; the choice adds `correction`, the weights do not and
     are not renormalized. Outputs from `experts` on are identity experts.
     Returns ids (N, top) int32 with -1 for identity choices, weights (N, top)
     and the identity experts' summed weight (N,)."""
-    s = torch.softmax(logits.float(), dim=-1)
+    s = (torch.sigmoid(logits.float()) if sigmoid
+         else torch.softmax(logits.float(), dim=-1))
+    choice = s if correction is None else s + correction.float()
     # stable sort: the lowest index wins a tie
-    ids = torch.sort(s + correction.float(), dim=-1, descending=True,
+    ids = torch.sort(choice, dim=-1, descending=True,
                      stable=True).indices[:, :top]
     w = torch.gather(s, 1, ids) * scale
     ident = ids >= experts
@@ -518,21 +520,45 @@ def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
     return out.to(q.dtype)
 
 
-def moe_experts(h, gate_up, down, ids, wts) -> torch.Tensor:
-    """y (N, top, W): wts * down(silu(gate h) * up h) of every chosen expert;
-    rows of skipped choices (id < 0) are zero."""
+def moe_experts(h, up, down, ids, wts, weight_input: bool = False,
+                ) -> torch.Tensor:
+    """y (N, top, W): wts * down(act) of every chosen expert, or down of the
+    activation of wts * h; act = silu(gate h) * up h with two planes (E, 2, F, K)
+    of first weights, relu(up h)^2 with one. Rows of skipped choices (id < 0)
+    are zero."""
     N, top = ids.shape
     y = torch.zeros(N, top, down.shape[1], dtype=torch.float32, device=h.device)
-    for e in range(gate_up.shape[0]):
+    for e in range(up.shape[0]):
         t, k = (ids == e).nonzero(as_tuple=True)
         if t.numel() == 0:
             continue
-        x = h[t].float()
-        g = x @ gate_up[e, 0].float().t()
-        u = x @ gate_up[e, 1].float().t()
-        a = (g * torch.sigmoid(g) * u).to(h.dtype).float()
-        y[t, k] = (a @ down[e].float().t()) * wts[t, k, None]
+        x, w = h[t].float(), wts[t, k, None]
+        if weight_input:
+            x, w = x * w, 1.0
+        z = x @ up[e, -1].float().t()
+        if up.shape[1] == 2:
+            z = F.silu(x @ up[e, 0].float().t()) * z
+        else:
+            z = torch.relu(z) ** 2
+        y[t, k] = (z.to(h.dtype).float() @ down[e].float().t()) * w
     return y.to(h.dtype)
+
+
+def sinusoid(positions: torch.Tensor, turns: torch.Tensor,
+             width: int) -> torch.Tensor:
+    """(..., width) f32: sine of position * frequency i at entry 2 i, cosine at
+    2 i + 1; turns: frequencies / 2 pi in float64."""
+    r = positions.double()[..., None] * turns
+    ang = (r - r.round()) * (2 * math.pi)
+    y = torch.stack([torch.sin(ang), torch.cos(ang)], -1).flatten(-2)
+    return y[..., :width].float()
+
+
+def query_temperature(positions: torch.Tensor, coef: float,
+                      every: float) -> torch.Tensor:
+    """1 + coef * ln(floor((position + 1) / every) + 1), fp32."""
+    steps = torch.floor((positions.double().clamp(min=0) + 1) / every)
+    return (1 + coef * torch.log1p(steps)).float()
 
 
 def clamped_glu(gate, up, gate_b, up_b, limit: float, slope: float):
@@ -573,3 +599,59 @@ def gla_scan(q, k, v, alpha, state):
                  + k[t].unsqueeze(-1) * v[t].unsqueeze(-2))
         out.append((state * q[t].unsqueeze(-1)).sum(-2))
     return torch.stack(out), state
+
+
+def mlstm_gates(z: torch.Tensor, bias: torch.Tensor, cap: float):
+    """Log gates (N, H) of a matrix memory from z (N, 2 H), input gates first:
+    i = cap tanh(z / cap), f = log sigmoid(cap tanh(z / cap)), fp32."""
+    z = cap * torch.tanh((z.float() + bias) / cap)
+    i, f = z.chunk(2, -1)
+    return i, F.logsigmoid(f)
+
+
+def mlstm_scan(q, k, v, i, f, S, n, m):
+    """Matrix memory of one sequence, token by token: q, k (T, H, D), v
+    (T, H, V), log gates i, f (T, H), state S (H, D, V), n (H, D), running
+    maximum m (H,) -> o (T, H, V), new state."""
+    out = []
+    for t in range(q.shape[0]):
+        new = torch.maximum(f[t] + m, i[t])
+        keep, add = torch.exp(f[t] + m - new), torch.exp(i[t] - new)
+        ki = k[t] * add.unsqueeze(-1)
+        S = keep[:, None, None] * S + ki.unsqueeze(-1) * v[t].unsqueeze(-2)
+        n = keep[:, None] * n + ki
+        m = new
+        den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+        out.append((S * q[t].unsqueeze(-1)).sum(-2) / den.unsqueeze(-1))
+    return torch.stack(out), (S, n, m)
+
+
+def causal_conv(x: torch.Tensor, past: torch.Tensor, taps: torch.Tensor,
+                bias: torch.Tensor) -> torch.Tensor:
+    """Per-channel convolution of x (..., T, C) after past (..., K - 1, C), taps
+    (K, C) with the current token's last."""
+    K, T = taps.shape[0], x.shape[-2]
+    full = torch.cat([past, x], -2)
+    return bias + sum(taps[j] * full[..., j:j + T, :] for j in range(K))
+
+
+def rglru_inputs(u, gates_w, gates_b, decay):
+    """What enters a gated linear recurrent unit, from u (..., C): log a and
+    sqrt(1 - a^2) * i * u, with r and i the sigmoids of a block-diagonal product,
+    gates_w (B, 2, C / B, C / B) [out, in], gates_b (2, C), log a = decay * r."""
+    B, _, D, _ = gates_w.shape
+    ub = u.float().reshape(-1, B, D).transpose(0, 1)
+    z = [torch.matmul(ub, gates_w[:, g].float().transpose(1, 2).contiguous())
+         .transpose(0, 1).reshape(u.shape) + gates_b[g] for g in range(2)]
+    log_a = decay * torch.sigmoid(z[0])
+    x = torch.sqrt(-torch.expm1(2 * log_a)) * torch.sigmoid(z[1]) * u.float()
+    return log_a, x
+
+
+def rglru_scan(log_a, x, S):
+    """S <- exp(log_a) S + x token by token: (T, C) -> states (T, C), last."""
+    out = []
+    for t in range(x.shape[0]):
+        S = torch.exp(log_a[t]) * S + x[t]
+        out.append(S)
+    return torch.stack(out), S

@@ -27,6 +27,7 @@ from bloombee_amd.engine import BlockStack
 from bloombee_amd.kv.paged import PagedKVCache
 from bloombee_amd.kv.views import SessionView
 from bloombee_amd.models.base import ModelConfig, get_family, resolve_config
+from bloombee_amd.ops.ragged import previous_ids
 from bloombee_amd.utils.logging import get_logger
 
 logger = get_logger(__name__)
@@ -130,6 +131,11 @@ class PipelineStage:
             head_cls = get_family(cfg.model_type).head_cls
             if head_cls is not None:
                 self.head = head_cls(cfg, device=self.device, seed=seed)
+        # last token fed to every sequence, for heads that embed pairs
+        self._last_ids: Optional[torch.Tensor] = None
+        if self.head is not None and self.head.uses_previous:
+            self._last_ids = torch.full((global_batch,), -1, dtype=torch.long,
+                                        device=self.device)
         if self.is_client and self.head is None:
             self.embed = (torch.randn(cfg.vocab_size, cfg.hidden_size, generator=gen)
                           .mul_(0.02).to(dt).to(self.device))
@@ -165,7 +171,11 @@ class PipelineStage:
             return F.embedding(ids, self.embed)
         pos = torch.arange(ids.shape[1], dtype=torch.int32, device=self.device)
         pos = pos.expand(*ids.shape) if start is None else start.view(-1, 1) + pos
-        return self.head.embed(ids, pos)
+        if self._last_ids is None:
+            return self.head.embed(ids, pos)
+        x = self.head.embed(ids, pos, previous_ids(ids, self._last_ids))
+        self._last_ids.copy_(ids[:, -1])
+        return x
 
     def _run_local(self, hidden: torch.Tensor, view, start_pos: torch.Tensor):
         return self.stack.forward_inference(hidden, view, start_pos)
