@@ -249,7 +249,7 @@ def random_weights(cfg, seed=0):
 
     def put(name, *shape, std=None, mean=0.0):
         std = std if std is not None else shape[-1] ** -0.5
-        w[name] = (mean + std * torch.randn(*shape, generator=g)).bfloat16().float()
+        w[name] = (mean + std * torch.randn(shape, generator=g)).bfloat16().float()
 
     put("embed", V, W, std=1.0)
     put("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, W, std=1.0)
