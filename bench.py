@@ -200,7 +200,11 @@ LAYER_PAIRS = [("mubasun-8b-4l", "llama-3-8b"),
                ("mubasun-64e-4l", None),
                ("risepel-8b-latent-4l", "mubasun-8b-4l"),
                ("risepel-8b-gla-4l", "mubasun-8b-4l"),
-               ("risepel-8b-4l", "llama-3-8b")]
+               ("risepel-8b-4l", "llama-3-8b"),
+               ("vumedra-8b-attn-4l", "llama-3-8b"),
+               ("vumedra-8b-mlstm-4l", "risepel-8b-gla-4l"),
+               ("vumedra-8b-rglru-4l", "risepel-8b-gla-4l"),
+               ("vumedra-8x7b-4l", "mubasun-8x7b-4l")]
 LAYERS = 4
 
 
@@ -307,8 +311,8 @@ def main():
                     help="pipeline = raw RCCL pipeline stages (flagship); "
                          "swarm = the full decentralized serving stack "
                          "(DHT + sessions + handler) over the same device plane; "
-                         "layers = mubasun and risepel layers beside the "
-                         "closest family's")
+                         "layers = mubasun, risepel and vumedra layers "
+                         "beside the closest family's")
     ap.add_argument("--pair", default=None,
                     help="layers mode: only pairs whose model name contains this")
     args = ap.parse_args()

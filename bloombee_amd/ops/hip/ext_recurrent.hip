@@ -291,8 +291,8 @@ void rglru_step(Tensor y, std::vector<long> dims, std::vector<Tensor> w, Tensor 
   a.n_list = list.numel();
   if (a.n_list == 0) return;
   by_type(y.scalar_type(), [&](auto p) {
-    rglru_gates_kernel<decltype(p), true>
-        <<<dim3(a.B * (a.Cp / 64), (a.n_list + 63) / 64), 256, 0,
+    rglru_step_kernel<decltype(p)>
+        <<<dim3(a.B * (a.Cp / 16), (a.n_list + 15) / 16), 64, 0,
            cur_stream()>>>(a);
   });
   check_launch();
@@ -325,11 +325,10 @@ void rglru_chunks(Tensor y, std::vector<long> dims, std::vector<Tensor> w,
   a.L = L.data_ptr<float>();
   a.S0 = S0.data_ptr<float>();
   const bool vec = all_of_8({a.y.ld, a.y_off, a.W, a.ldo});
+  rglru_gates_kernel<<<dim3(a.B * (a.Cp / 64), chunks), 256, 0, cur_stream()>>>(a);
+  check_launch();
   by_type(y.scalar_type(), [&](auto p) {
     using TP = decltype(p);
-    rglru_gates_kernel<TP, false>
-        <<<dim3(a.B * (a.Cp / 64), chunks), 256, 0, cur_stream()>>>(a);
-    check_launch();
     rglru_carry_kernel<TP>
         <<<dim3((a.W + 63) / 64, a.n_list), 64, 0, cur_stream()>>>(a);
     check_launch();

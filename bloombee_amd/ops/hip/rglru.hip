@@ -8,10 +8,11 @@
 // taps - 1 inputs, 32-bit. A sequence whose portion starts at position 0 starts
 // from zero, whatever its slot holds.
 //
-//  rglru_conv_kernel   u of all rows; reads the inputs' state, writes none.
-//  rglru_gates_kernel  both gates as one MFMA product per block of channels. In
-//                      its epilogue either the recurrence of single tokens up to
-//                      the output, or, for portions in chunks of 64 tokens, the
+//  rglru_conv_kernel   u of all rows; the inputs' state of single tokens moves on
+//                      here, that of portions with the kernel that ends them.
+//  rglru_step_kernel   single tokens: both gates as one MFMA product per block of
+//                      channels, the recurrence and the output.
+//  rglru_gates_kernel  portions in chunks of 64 tokens: both gates, and the
 //                      chunk's own recurrence from zero: h and the cumulated
 //                      log a, 32-bit.
 //  rglru_carry_kernel  S from chunk to chunk, and the states.
@@ -85,10 +86,12 @@ DEVINL void lru_step(float zr, float zi, float u, float decay, float& la, float&
   x = sqrtf(-expm1f(2.f * la)) * i * u;
 }
 
-// Channel c's last K - 1 inputs after the n tokens of sequence s; one thread a
-// channel, ascending, so that an entry is read before it is overwritten.
+// Channel c's last K - 1 inputs after the n tokens of sequence s, unless the
+// convolution kernel kept them (n = 1); one thread a channel, ascending, so that
+// an entry is read before it is overwritten.
 template <typename TP>
 DEVINL void lru_keep_inputs(const LruArgs& a, int s, int n, int c) {
+  if (n == 1) return;
   const int start = a.q_start[s];
   const long t0 = a.cu[s];
   float* st = a.conv + (long)a.slots[s] * (a.K - 1) * a.W + c;
@@ -101,7 +104,8 @@ DEVINL void lru_keep_inputs(const LruArgs& a, int s, int n, int c) {
   }
 }
 
-// grid (channels / (256 V), N)
+// grid (channels / (256 V), N). Where the row is all that its sequence brings,
+// the thread is also the only reader of the kept inputs and moves them on.
 template <typename TP, typename T, int V>
 __global__ __launch_bounds__(256) void rglru_conv_kernel(LruArgs a) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * V;
@@ -110,40 +114,101 @@ __global__ __launch_bounds__(256) void rglru_conv_kernel(LruArgs a) {
   const int pos = a.tok_pos[t];
   if (pos < 0) return;
   const int s = a.tok_seq[t], start = a.q_start[s];
-  const float* st = a.conv + (long)a.slots[s] * (a.K - 1) * a.W + c;
-  float o[V], x[V], w[V];
+  const bool one = a.cu[s + 1] - a.cu[s] == 1;
+  float* st = a.conv + (long)a.slots[s] * (a.K - 1) * a.W + c;
+  float o[V], x[V], w[V], held[V];
   ldv<V>(a.cb + c, o);
-  for (int j = 0; j < a.K && j <= pos; ++j) {
+  int j = 0;
+  for (; j < a.K && j <= pos; ++j) {
+    const long e = a.K - 1 + pos - j - start;   // the input's entry, if kept
     if (pos - j >= start) lru_input<TP, V>(a, t - j, c, x);
-    else ldv<V>(st + (long)(a.K - 1 + pos - j - start) * a.W, x);
+    else ldv<V>(st + e * a.W, x);
+    if (one && j > 0) stv<V>(st + e * a.W, held);
     ldv<V>(a.taps + (long)(a.K - 1 - j) * a.W + c, w);
 #pragma unroll
-    for (int k = 0; k < V; ++k) o[k] += w[k] * x[k];
+    for (int k = 0; k < V; ++k) {
+      o[k] += w[k] * x[k];
+      held[k] = x[k];
+    }
   }
+  if (one && j < a.K) stv<V>(st + (long)(a.K - 1 - j) * a.W, held);
   T* u = (T*)a.u + t * a.B * a.Cp;
   stv<V>(u + c / a.Cb * a.Cp + c % a.Cb, o);
 }
 
-// grid (B * Cp / 64, tiles of 64 rows): a wave holds both gates of 16 channels.
-// STEP: tile rows are the listed one-token rows; else those of a chunk.
-template <typename TP, bool STEP>
+// Single tokens: gates, recurrence and output. grid (B * Cp / 16, rows / 16), a
+// wave: both gates of 16 channels and up to 16 listed rows.
+template <typename TP>
+__global__ __launch_bounds__(64) void rglru_step_kernel(LruArgs a) {
+  const int lane = threadIdx.x, li = lane & 15, hi = lane >> 4;
+  const int tiles = a.Cp / 16, b = blockIdx.x / tiles;
+  const int n0 = blockIdx.x % tiles * 16;
+  const int m0 = blockIdx.y * 16, cnt = min(16, a.n_list - m0);
+  const long ldu = (long)a.B * a.Cp;
+  const unsigned short* u = (const unsigned short*)a.u + (long)b * a.Cp;
+  const unsigned short* xr =
+      u + (long)a.cu[a.list[m0 + min(li, cnt - 1)]] * ldu + hi * 8;
+  const unsigned short* wr[2];
+#pragma unroll
+  for (int g = 0; g < 2; ++g)
+    wr[g] = (const unsigned short*)a.gw +
+            (((long)b * 2 + g) * a.Cp + n0 + li) * a.Cp + hi * 8;
+
+  // what the epilogue needs is asked for ahead of the product
+  const int cl = n0 + li, c = b * a.Cb + min(cl, a.Cb - 1);
+  const float br = a.gb[c], bi = a.gb[a.W + c], dec = a.decay[c], yb = a.yb[c];
+  long t[4];
+  int pos[4];
+  float S[4], uv[4], y[4];
+  float* sp[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int s = a.list[m0 + min(hi * 4 + r, cnt - 1)];
+    t[r] = a.cu[s];
+    sp[r] = a.S + (long)a.slots[s] * a.W + c;
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    pos[r] = a.tok_pos[t[r]];
+    S[r] = *sp[r];
+    uv[r] = bf2f(u[t[r] * ldu + min(cl, a.Cb - 1)]);
+    fold_parts<TP, 1>(a.y, t[r], a.y_off + c, y + r);
+  }
+
+  f32x4 acc[2];
+  acc[0] = acc[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+  for (int k = 0; k < a.Cp; k += 32) {
+    const bf16x8 x = as_bf16x8(*reinterpret_cast<const short8*>(xr + k));
+#pragma unroll
+    for (int g = 0; g < 2; ++g)
+      acc[g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          x, as_bf16x8(*reinterpret_cast<const short8*>(wr[g] + k)), acc[g], 0, 0, 0);
+  }
+  if (cl >= a.Cb) return;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    if (hi * 4 + r >= cnt || pos[r] < 0) continue;   // none, or an empty slot
+    float la, x;
+    lru_step(acc[0][r] + br, acc[1][r] + bi, uv[r], dec, la, x);
+    x += pos[r] > 0 ? S[r] * expf(la) : 0.f;
+    *sp[r] = x;
+    ((unsigned short*)a.out)[t[r] * a.ldo + c] = cvt_bf(x * gelu_tanh_f(y[r] + yb));
+  }
+}
+
+// grid (B * Cp / 64, chunks): a wave holds both gates of 16 channels.
 __global__ __launch_bounds__(256) void rglru_gates_kernel(LruArgs a) {
   constexpr int LDU = LRU_KC + 8, LDC = 65;
   __shared__ __attribute__((aligned(16))) unsigned char
       lds[64 * LDU * 2 > 2 * 64 * LDC * 4 ? 64 * LDU * 2 : 2 * 64 * LDC * 4];
-  __shared__ int rows[64];
   unsigned short* us = (unsigned short*)lds;
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int li = lane & 15, hi = lane >> 4;
   const int tiles = a.Cp / 64, b = blockIdx.x / tiles;
   const int n0 = blockIdx.x % tiles * 64;     // first channel in the block
-  const int cnt = STEP ? min(64, a.n_list - (int)blockIdx.y * 64)
-                       : a.len[blockIdx.y];
-  if (tid < 64) {
-    const int i = min(tid, cnt - 1);
-    rows[tid] = STEP ? a.cu[a.list[blockIdx.y * 64 + i]] : a.row0[blockIdx.y] + i;
-  }
-  __syncthreads();
+  const int cnt = a.len[blockIdx.y];
+  const long row0 = a.row0[blockIdx.y];
   const int mt = (cnt + 15) / 16;
   const unsigned short* gw = (const unsigned short*)a.gw;
   const unsigned short* wr[2];
@@ -164,7 +229,7 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(LruArgs a) {
     for (int i = tid; i < mt * 16 * pc; i += 256) {
       const int r = i / pc, c = i % pc * 8;
       *reinterpret_cast<short8*>(us + r * LDU + c) =
-          *reinterpret_cast<const short8*>(u + rows[r] * ldu + k0 + c);
+          *reinterpret_cast<const short8*>(u + (row0 + min(r, cnt - 1)) * ldu + k0 + c);
     }
     __syncthreads();
 #pragma unroll 4
@@ -188,73 +253,49 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(LruArgs a) {
   }
 
   const int cl = n0 + wave * 16 + li;           // channel in the block
-  const bool live = cl < a.Cb;
   const int c = b * a.Cb + min(cl, a.Cb - 1);
   const float br = a.gb[c], bi = a.gb[a.W + c], dec = a.decay[c];
-  if constexpr (STEP) {
-    if (!live) return;
+  float* hs = (float*)lds;          // (64, LDC): state from zero
+  float* ls = hs + 64 * LDC;        // cumulated log a
 #pragma unroll
-    for (int m = 0; m < 4; ++m)
+  for (int m = 0; m < 4; ++m)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int at = m * 16 + hi * 4 + r;
-        if (at >= cnt) continue;
-        const long t = rows[at];
-        const int pos = a.tok_pos[t];
-        if (pos < 0) continue;   // empty slot
-        const int s = a.list[blockIdx.y * 64 + at];
-        float la, x;
-        lru_step(acc[0][m][r] + br, acc[1][m][r] + bi, bf2f(u[t * ldu + cl]), dec,
-                 la, x);
-        float* sp = a.S + (long)a.slots[s] * a.W + c;
-        const float S = (pos > 0 ? *sp * expf(la) : 0.f) + x;
-        *sp = S;
-        ((unsigned short*)a.out)[t * a.ldo + c] = cvt_bf(S * lru_branch<TP>(a, t, c));
-        lru_keep_inputs<TP>(a, s, 1, c);
-      }
-  } else {
-    float* hs = (float*)lds;          // (64, LDC): state from zero
-    float* ls = hs + 64 * LDC;        // cumulated log a
-#pragma unroll
-    for (int m = 0; m < 4; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int at = m * 16 + hi * 4 + r;
-        float la = 0.f, x = 0.f;
-        if (at < cnt)
-          lru_step(acc[0][m][r] + br, acc[1][m][r] + bi,
-                   bf2f(u[rows[at] * ldu + cl]), dec, la, x);
-        hs[at * LDC + wave * 16 + li] = x;
-        ls[at * LDC + wave * 16 + li] = la;
-      }
-    __syncthreads();
-    // a thread takes 16 tokens of a channel, then adds what came before them
-    const int cc = tid & 63, t0 = tid / 64 * 16;
-    float S = 0.f, L = 0.f;
-#pragma unroll
-    for (int t = t0; t < t0 + 16; ++t) {
-      const float la = ls[t * LDC + cc];
-      S = S * expf(la) + hs[t * LDC + cc];
-      L += la;
-      hs[t * LDC + cc] = S;
-      ls[t * LDC + cc] = L;
+    for (int r = 0; r < 4; ++r) {
+      const int at = m * 16 + hi * 4 + r;
+      float la = 0.f, x = 0.f;
+      if (at < cnt)
+        lru_step(acc[0][m][r] + br, acc[1][m][r] + bi,
+                 bf2f(u[(row0 + at) * ldu + cl]), dec, la, x);
+      hs[at * LDC + wave * 16 + li] = x;
+      ls[at * LDC + wave * 16 + li] = la;
     }
-    __syncthreads();
-    S = L = 0.f;
-    for (int t = 15; t < t0; t += 16) {
-      const float l = ls[t * LDC + cc];
-      S = S * expf(l) + hs[t * LDC + cc];
-      L += l;
-    }
-    if (n0 + cc >= a.Cb) return;
-    const long o = (long)a.row0[blockIdx.y] * a.W + b * a.Cb + n0 + cc;
+  __syncthreads();
+  // a thread takes 16 tokens of a channel, then adds what came before them
+  const int cc = tid & 63, t0 = tid / 64 * 16;
+  float S = 0.f, L = 0.f;
 #pragma unroll
-    for (int t = t0; t < t0 + 16; ++t) {
-      if (t >= cnt) break;
-      const float l = ls[t * LDC + cc];
-      a.h[o + (long)t * a.W] = hs[t * LDC + cc] + S * expf(l);
-      a.L[o + (long)t * a.W] = l + L;
-    }
+  for (int t = t0; t < t0 + 16; ++t) {
+    const float la = ls[t * LDC + cc];
+    S = S * expf(la) + hs[t * LDC + cc];
+    L += la;
+    hs[t * LDC + cc] = S;
+    ls[t * LDC + cc] = L;
+  }
+  __syncthreads();
+  S = L = 0.f;
+  for (int t = 15; t < t0; t += 16) {
+    const float l = ls[t * LDC + cc];
+    S = S * expf(l) + hs[t * LDC + cc];
+    L += l;
+  }
+  if (n0 + cc >= a.Cb) return;
+  const long o = row0 * a.W + b * a.Cb + n0 + cc;
+#pragma unroll
+  for (int t = t0; t < t0 + 16; ++t) {
+    if (t >= cnt) break;
+    const float l = ls[t * LDC + cc];
+    a.h[o + (long)t * a.W] = hs[t * LDC + cc] + S * expf(l);
+    a.L[o + (long)t * a.W] = l + L;
   }
 }
 
