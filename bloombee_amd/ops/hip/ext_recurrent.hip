@@ -319,10 +319,10 @@ void rglru_chunks(Tensor y, std::vector<long> dims, std::vector<Tensor> w,
   a.ccu = ccu.data_ptr<int>();
   auto fopt = u.options().dtype(at::kFloat);
   auto h = torch::empty({a.N, a.W}, fopt);
-  auto L = torch::empty({a.N, a.W}, fopt);
+  auto F = torch::empty({a.N, a.W}, fopt);
   auto S0 = torch::empty({chunks, a.W}, fopt);
   a.h = h.data_ptr<float>();
-  a.L = L.data_ptr<float>();
+  a.F = F.data_ptr<float>();
   a.S0 = S0.data_ptr<float>();
   const bool vec = all_of_8({a.y.ld, a.y_off, a.W, a.ldo});
   rglru_gates_kernel<<<dim3(a.B * (a.Cp / 64), chunks), 256, 0, cur_stream()>>>(a);

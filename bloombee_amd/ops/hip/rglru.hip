@@ -13,10 +13,10 @@
 //  rglru_step_kernel   single tokens: both gates as one MFMA product per block of
 //                      channels, the recurrence and the output.
 //  rglru_gates_kernel  portions in chunks of 64 tokens: both gates, and the
-//                      chunk's own recurrence from zero: h and the cumulated
-//                      log a, 32-bit.
+//                      chunk's own recurrence from zero: h and the product F
+//                      of the factors a since the chunk's start, 32-bit.
 //  rglru_carry_kernel  S from chunk to chunk, and the states.
-//  rglru_out_kernel    (h + e^(cumulated log a) S) gelu(y), all rows side by side.
+//  rglru_out_kernel    (h + F S) gelu(y), all rows side by side.
 //  rglru_seq_kernel    token by token from finished gate products: 32-bit runs.
 
 #pragma once
@@ -40,7 +40,7 @@ struct LruArgs {
   void* u;             // (N, B * Cp): block b's channels from b * Cp on
   const float* z;      // seq: (B, N, 2 * Cb) gate products
   float* h;            // (N, W) chunk form
-  float* L;            // (N, W)
+  float* F;            // (N, W)
   float* S0;           // (chunks, W): S before each chunk
   void* out;           // (N, ldo), W columns
   const int* slots;
@@ -79,11 +79,28 @@ DEVINL float lru_branch(const LruArgs& a, long t, int c) {
   return gelu_tanh_f(v[0] + a.yb[c]);
 }
 
-// Gate logits -> log a and what enters the state.
-DEVINL void lru_step(float zr, float zi, float u, float decay, float& la, float& x) {
-  const float r = 1.f / (1.f + expf(-zr)), i = 1.f / (1.f + expf(-zi));
-  la = decay * r;
-  x = sqrtf(-expm1f(2.f * la)) * i * u;
+// 1 - e^z for z <= 0. Near zero the series, where the difference would cancel.
+DEVINL float one_minus_exp(float z) {
+  const float far = 1.f - fast_expf(z);
+  const float t = 1.f + z * (1.f / 5) * (1.f + z * (1.f / 6) * (1.f + z * (1.f / 7)));
+  const float near =
+      -z * (1.f + z * (1.f / 2) * (1.f + z * (1.f / 3) * (1.f + z * (1.f / 4) * t)));
+  return z > -0.5f ? near : far;
+}
+
+// Gate logits -> the state's factor and what enters it. FAST: the hardware's
+// exponential and reciprocal, an ulp or two each.
+template <bool FAST>
+DEVINL void lru_step(float zr, float zi, float u, float decay, float& f, float& x) {
+  if constexpr (FAST) {
+    const float la = decay * sigmoid_f(zr);
+    f = fast_expf(la);
+    x = __builtin_amdgcn_sqrtf(one_minus_exp(2.f * la)) * sigmoid_f(zi) * u;
+  } else {
+    const float la = decay / (1.f + expf(-zr));
+    f = expf(la);
+    x = sqrtf(-expm1f(2.f * la)) / (1.f + expf(-zi)) * u;
+  }
 }
 
 // Channel c's last K - 1 inputs after the n tokens of sequence s, unless the
@@ -189,9 +206,9 @@ __global__ __launch_bounds__(64) void rglru_step_kernel(LruArgs a) {
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     if (hi * 4 + r >= cnt || pos[r] < 0) continue;   // none, or an empty slot
-    float la, x;
-    lru_step(acc[0][r] + br, acc[1][r] + bi, uv[r], dec, la, x);
-    x += pos[r] > 0 ? S[r] * expf(la) : 0.f;
+    float f, x;
+    lru_step<true>(acc[0][r] + br, acc[1][r] + bi, uv[r], dec, f, x);
+    x += pos[r] > 0 ? S[r] * f : 0.f;
     *sp[r] = x;
     ((unsigned short*)a.out)[t[r] * a.ldo + c] = cvt_bf(x * gelu_tanh_f(y[r] + yb));
   }
@@ -256,46 +273,49 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(LruArgs a) {
   const int c = b * a.Cb + min(cl, a.Cb - 1);
   const float br = a.gb[c], bi = a.gb[a.W + c], dec = a.decay[c];
   float* hs = (float*)lds;          // (64, LDC): state from zero
-  float* ls = hs + 64 * LDC;        // cumulated log a
+  float* fs = hs + 64 * LDC;        // factors, then their products
 #pragma unroll
   for (int m = 0; m < 4; ++m)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int at = m * 16 + hi * 4 + r;
-      float la = 0.f, x = 0.f;
+      float f = 1.f, x = 0.f;
       if (at < cnt)
-        lru_step(acc[0][m][r] + br, acc[1][m][r] + bi,
-                 bf2f(u[(row0 + at) * ldu + cl]), dec, la, x);
+        lru_step<true>(acc[0][m][r] + br, acc[1][m][r] + bi,
+                       bf2f(u[(row0 + at) * ldu + cl]), dec, f, x);
       hs[at * LDC + wave * 16 + li] = x;
-      ls[at * LDC + wave * 16 + li] = la;
+      fs[at * LDC + wave * 16 + li] = f;
     }
   __syncthreads();
   // a thread takes 16 tokens of a channel, then adds what came before them
   const int cc = tid & 63, t0 = tid / 64 * 16;
-  float S = 0.f, L = 0.f;
+  float S[16], F[16];
 #pragma unroll
-  for (int t = t0; t < t0 + 16; ++t) {
-    const float la = ls[t * LDC + cc];
-    S = S * expf(la) + hs[t * LDC + cc];
-    L += la;
-    hs[t * LDC + cc] = S;
-    ls[t * LDC + cc] = L;
+  for (int t = 0; t < 16; ++t) {
+    S[t] = hs[(t0 + t) * LDC + cc];
+    F[t] = fs[(t0 + t) * LDC + cc];
   }
+#pragma unroll
+  for (int t = 1; t < 16; ++t) {
+    S[t] += S[t - 1] * F[t];
+    F[t] *= F[t - 1];
+  }
+  hs[(t0 + 15) * LDC + cc] = S[15];
+  fs[(t0 + 15) * LDC + cc] = F[15];
   __syncthreads();
-  S = L = 0.f;
+  float S0 = 0.f, F0 = 1.f;
   for (int t = 15; t < t0; t += 16) {
-    const float l = ls[t * LDC + cc];
-    S = S * expf(l) + hs[t * LDC + cc];
-    L += l;
+    const float f = fs[t * LDC + cc];
+    S0 = S0 * f + hs[t * LDC + cc];
+    F0 *= f;
   }
   if (n0 + cc >= a.Cb) return;
   const long o = row0 * a.W + b * a.Cb + n0 + cc;
 #pragma unroll
-  for (int t = t0; t < t0 + 16; ++t) {
-    if (t >= cnt) break;
-    const float l = ls[t * LDC + cc];
-    a.h[o + (long)t * a.W] = hs[t * LDC + cc] + S * expf(l);
-    a.L[o + (long)t * a.W] = l + L;
+  for (int t = 0; t < 16; ++t) {
+    if (t0 + t >= cnt) break;
+    a.h[o + (long)(t0 + t) * a.W] = S[t] + S0 * F[t];
+    a.F[o + (long)(t0 + t) * a.W] = F[t] * F0;
   }
 }
 
@@ -310,19 +330,19 @@ __global__ __launch_bounds__(64) void rglru_carry_kernel(LruArgs a) {
   const int c0 = a.ccu[blockIdx.y], c1 = a.ccu[blockIdx.y + 1];
   constexpr int U = 8;   // chunks whose loads are in flight together
   for (int k = c0; k < c1; k += U) {
-    float h[U], l[U];
+    float h[U], f[U];
 #pragma unroll
     for (int j = 0; j < U; ++j) {
       const int ch = min(k + j, c1 - 1);
       const long at = ((long)a.row0[ch] + a.len[ch] - 1) * a.W + c;
       h[j] = a.h[at];
-      l[j] = a.L[at];
+      f[j] = a.F[at];
     }
 #pragma unroll
     for (int j = 0; j < U; ++j) {
       if (k + j >= c1) break;
       a.S0[(long)(k + j) * a.W + c] = S;
-      S = h[j] + S * expf(l[j]);
+      S = h[j] + S * f[j];
     }
   }
   *sp = S;
@@ -341,13 +361,13 @@ __global__ __launch_bounds__(256) void rglru_out_kernel(LruArgs a) {
 #pragma unroll 4
   for (int i = blockIdx.y * 16; i < end; ++i) {
     const long t = a.row0[ch] + i;
-    float h[V], l[V], y[V];
+    float h[V], f[V], y[V];
     ldv<V>(a.h + t * a.W + c, h);
-    ldv<V>(a.L + t * a.W + c, l);
+    ldv<V>(a.F + t * a.W + c, f);
     fold_parts<TP, V>(a.y, t, a.y_off + c, y);
 #pragma unroll
     for (int j = 0; j < V; ++j)
-      h[j] = (h[j] + fast_expf(l[j]) * S[j]) * gelu_tanh_f(y[j] + yb[j]);
+      h[j] = (h[j] + f[j] * S[j]) * gelu_tanh_f(y[j] + yb[j]);
     stv<V>((T*)a.out + t * a.ldo + c, h);
   }
 }
@@ -366,10 +386,11 @@ __global__ __launch_bounds__(64) void rglru_seq_kernel(LruArgs a) {
   const float br = a.gb[c], bi = a.gb[a.W + c], dec = a.decay[c];
   for (long t = t0; t < t1; ++t) {
     const float* z = a.z + ((long)b * a.N + t) * 2 * a.Cb + cl;
-    float la, x;
-    lru_step(z[0] + br, z[a.Cb] + bi,
-             ldf((const T*)a.u + t * a.B * a.Cp + (long)b * a.Cp + cl), dec, la, x);
-    S = S * expf(la) + x;
+    float f, x;
+    lru_step<false>(z[0] + br, z[a.Cb] + bi,
+                    ldf((const T*)a.u + t * a.B * a.Cp + (long)b * a.Cp + cl), dec,
+                    f, x);
+    S = S * f + x;
     stf((T*)a.out + t * a.ldo + c, S * lru_branch<TP>(a, t, c));
   }
   *sp = S;
