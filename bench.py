@@ -204,7 +204,11 @@ LAYER_PAIRS = [("mubasun-8b-4l", "llama-3-8b"),
                ("vumedra-8b-attn-4l", "llama-3-8b"),
                ("vumedra-8b-mlstm-4l", "risepel-8b-gla-4l"),
                ("vumedra-8b-rglru-4l", "risepel-8b-gla-4l"),
-               ("vumedra-8x7b-4l", "mubasun-8x7b-4l")]
+               ("vumedra-8x7b-4l", "mubasun-8x7b-4l"),
+               ("zatusun-8b-latent-4l", "risepel-8b-latent-mixer-4l"),
+               ("zatusun-8b-diff-4l", "vumedra-8b-attn-mixer-4l"),
+               ("zatusun-8b-hgrn2-4l", "risepel-8b-gla-mixer-4l"),
+               ("zatusun-8x7b-4l", "mubasun-8x7b-4l")]
 LAYERS = 4
 
 
@@ -219,7 +223,7 @@ def _layer_numbers(model: str, args) -> dict:
     dev = args.device or ("cuda:0" if torch.cuda.is_available() else "cpu")
     on_gpu = dev.startswith("cuda")
     stack = BlockStack(cfg, 0, LAYERS, device=dev, seed=0)
-    W = cfg.hidden_size
+    W = cfg.hidden_columns
     gen = torch.Generator().manual_seed(1)
     sync = torch.cuda.synchronize if on_gpu else (lambda: None)
     out = {}

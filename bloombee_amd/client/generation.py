@@ -47,7 +47,7 @@ class RemoteGenerationMixin:
             fresh = session.position == 0
             hidden = self._embed_next(input_ids, session, pre if fresh else 0)
             if pe is not None and fresh:
-                p = pe.detach().to(hidden.dtype).unsqueeze(0).expand(B, -1, -1)
+                p = self.transformer.prompt_hidden(hidden).detach()
                 hidden = torch.cat([p, hidden], dim=1)
             hidden = session.step(
                 hidden, prompts=dp.detach() if dp is not None else None)

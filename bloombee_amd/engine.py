@@ -47,9 +47,15 @@ class BlockStack(torch.nn.Module):
         # blocks that run whole ragged steps (kv/batch.py)
         self.token_batched = self.rope is None
         self.blocks = torch.nn.ModuleList()
+        owners: Dict[int, torch.nn.Module] = {}   # of weights, by first layer
         for i in range(start, end):
             blk = block_cls(config, layer_index=i, rope=self.rope).to(device)
-            blk.init_random(seed=seed * 10_000 + i)
+            j = config.weights_of(i)
+            if j in owners:
+                blk.share_weights(owners[j])
+            else:
+                blk.init_random(seed=seed * 10_000 + j)
+                owners[j] = blk
             blk.layer_index = i - start  # KV page index local to this stack's pool
             self.blocks.append(blk)
         # chain blocks so each one's down-proj epilogue can leave row
@@ -115,15 +121,15 @@ class BlockStack(torch.nn.Module):
             if tree_mask is not None or position_ids is not None:
                 raise NotImplementedError(
                     f"{self.config.model_type}: no tree-structured steps")
-            B, T, W = hidden.shape
-            x = hidden.reshape(B * T, W).to(torch.float32, copy=True)
+            B, T, C = hidden.shape
+            x = hidden.reshape(B * T, C).to(torch.float32, copy=True)
             hook = None
             if n_over > 0:
                 def hook(i):
-                    x.view(B, T, W)[:, :n_over] += \
-                        deep_prompts[i, sp0:sp0 + n_over].to(x.dtype)
+                    dp = deep_prompts[i, sp0:sp0 + n_over].to(x.dtype)
+                    x.view(B, T, C)[:, :n_over, :dp.shape[-1]] += dp
             self.forward_batch(x, lockstep_batch(kv, start_pos, B, T), hook)
-            return x.view(B, T, W)
+            return x.view(B, T, C)
         for i, blk in enumerate(self.blocks):
             if n_over > 0:
                 dp = deep_prompts[i, sp0:sp0 + n_over].to(hidden.dtype)
@@ -136,11 +142,12 @@ class BlockStack(torch.nn.Module):
         return hidden
 
     @torch.no_grad()
-    def forward_batch(self, x: torch.Tensor, batch: TokenBatch,
+    def forward_batch(self, hidden: torch.Tensor, batch: TokenBatch,
                       before_block=None) -> torch.Tensor:
-        """One ragged step: x (N, W) f32 through all blocks, in place. A block
-        may leave something to the next one (its sum, for that one's norm to
-        fold in); before_block(i) needs the sum, so it forces the fold."""
+        """One ragged step: hidden (N, columns) f32 through all blocks, in place.
+        A block may leave something to the next one (its sum, for that one's norm
+        to fold in); before_block(i) needs the sum, so it forces the fold."""
+        x = batch.split_hidden(hidden, self.config.hidden_size)
         left = None
         for i, blk in enumerate(self.blocks):
             if before_block is not None:
@@ -150,7 +157,7 @@ class BlockStack(torch.nn.Module):
                 before_block(i)
             left = blk.forward_tokens(x, left, batch)
         left.settle(x)
-        return x
+        return hidden
 
     def forward_train(self, hidden: torch.Tensor, start_pos: int = 0,
                       deep_prompts: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -159,6 +166,7 @@ class BlockStack(torch.nn.Module):
             if pre > 0 and hidden.shape[1] >= pre:
                 # functional (not in-place) so prompt grads flow in backward
                 dp = deep_prompts[i].to(hidden.dtype).unsqueeze(0)
+                dp = F.pad(dp, (0, hidden.shape[-1] - dp.shape[-1]))
                 hidden = torch.cat([hidden[:, :pre] + dp, hidden[:, pre:]], 1)
             hidden = blk.forward_train(hidden, start_pos)
         return hidden

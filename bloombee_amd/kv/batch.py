@@ -57,6 +57,8 @@ class TokenBatch:
     max_new: int               # longest portion
     max_ctx: int               # longest context after this step (upper bound)
     slots: Optional[torch.Tensor] = None   # (S,) int32: recurrent state rows
+    # (N, W) f32: the embedding output, for layers that read it again
+    embedded: Optional[torch.Tensor] = None
     # host copies of starts, counts and page lists, where a step has portions
     host: Optional[Tuple[Sequence[int], Sequence[int],
                          Sequence[Sequence[int]]]] = None
@@ -105,6 +107,13 @@ class TokenBatch:
                 [np.asarray(v, dtype=np.int32) for v in (row0, length, cu)],
                 self.cache.device))
         return self._cut[key]
+
+    def split_hidden(self, hidden: torch.Tensor, width: int) -> torch.Tensor:
+        """The residual among the columns of hidden states (N, columns), as a
+        view; what travels behind it is kept for the layers that read it."""
+        if hidden.shape[1] > width:
+            self.embedded = hidden[:, width:]
+        return hidden[:, :width]
 
     @property
     def n_tokens(self) -> int:

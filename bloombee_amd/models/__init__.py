@@ -16,3 +16,4 @@ import bloombee_amd.models.gemma4  # noqa: F401,E402
 import bloombee_amd.models.mubasun  # noqa: F401,E402
 import bloombee_amd.models.risepel  # noqa: F401,E402
 import bloombee_amd.models.vumedra  # noqa: F401,E402
+import bloombee_amd.models.zatusun  # noqa: F401,E402

@@ -60,6 +60,16 @@ class ModelConfig:
         """Type of the hidden states between blocks and on the wire."""
         return self.dtype
 
+    @property
+    def hidden_columns(self) -> int:
+        """Their width: the residual's, and what travels behind it."""
+        return self.hidden_size
+
+    def weights_of(self, layer: int) -> int:
+        """The first layer with the same weights (itself, unless layers run
+        several times)."""
+        return layer
+
     @classmethod
     def from_dict(cls, d: dict) -> "ModelConfig":
         d = dict(d)

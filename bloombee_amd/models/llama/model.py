@@ -85,6 +85,11 @@ class DistributedLlamaModel(torch.nn.Module):
     def final_norm(self, hidden: torch.Tensor) -> torch.Tensor:
         return ops.rms_norm(hidden, self.norm_w, self.config.rms_norm_eps)
 
+    def prompt_hidden(self, like: torch.Tensor) -> torch.Tensor:
+        """The trained prompt as hidden states ahead of `like` (B, T, columns)."""
+        return self.prompt_embeds.to(like.dtype).unsqueeze(0).expand(
+            like.shape[0], -1, -1)
+
     def trainable_parameters(self):
         """The client-side fine-tune state (ref ptune.py: everything the
         swarm trains lives on the client — shallow + deep prompts; server
@@ -100,9 +105,7 @@ class DistributedLlamaModel(torch.nn.Module):
         """Training-path full forward (no KV): returns final hidden states."""
         h = self.embed(input_ids, self.pre_seq_len)
         if self.prompt_embeds is not None:
-            B = h.shape[0]
-            p = self.prompt_embeds.to(h.dtype).unsqueeze(0).expand(B, -1, -1)
-            h = torch.cat([p, h], dim=1)
+            h = torch.cat([self.prompt_hidden(h), h], dim=1)
         h = self.remote(h, prompts=self.deep_prompts)
         return self.final_norm(h)
 

@@ -3,8 +3,10 @@ embeddings, final norm and vocabulary projection as one module, shared by
 LocalEngine, the pipeline and the swarm client, and the distributed model
 classes over it.
 
-What differs between families are properties of the config: `learned_positions`
-(a table "pos" is added to the embedding), `sinusoidal_positions`, `bigram` (a
+What differs between families are properties of the config: `embedding_scale`
+(of the token's row), `learned_positions` (a table "pos" is added to the
+embedding), `hidden_columns` (a multiple of the width: the embedding output
+travels behind the residual), `sinusoidal_positions`, `bigram` (a
 table "bigram" of hashed token pairs is added: buckets, mul_prev, mul_cur),
 `norm_groups`, `norm_offset` (norm weights are stored as their distance from it),
 `scalar_norm` (one norm weight for all coordinates), `logit_softcap` (0 = none).
@@ -34,6 +36,8 @@ class RaggedHead(torch.nn.Module):
         self.groups = getattr(config, "norm_groups", 1)
         self.norm_offset = getattr(config, "norm_offset", 0.0)
         self.softcap = getattr(config, "logit_softcap", 0.0)
+        self.embed_scale = getattr(config, "embedding_scale", 1.0)
+        self.copies = config.hidden_columns // config.hidden_size
         W, V, dt = config.hidden_size, config.vocab_size, config.dtype
 
         def p(*shape, dtype=dt):
@@ -94,17 +98,18 @@ class RaggedHead(torch.nn.Module):
 
     def embed(self, ids: torch.Tensor, positions: torch.Tensor,
               prev: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """ids, positions of one shape -> (..., W) f32; prev: the token before
+        """ids, positions of one shape -> (..., columns) f32; prev: the token before
         each, -1 = none (only if uses_previous)."""
         if self.uses_previous and prev is None:
             raise ValueError("this family embeds tokens with the ones before "
                              "them: they are missing")
         return ragged.embed_rows(ids, positions, self.embed_w, self.pos_w, prev,
-                                 self.pairs, self.turns)
+                                 self.pairs, self.turns, self.embed_scale,
+                                 self.copies)
 
     def final_norm(self, hidden: torch.Tensor) -> torch.Tensor:
         W = self.config.hidden_size
-        x = hidden.reshape(-1, W).float().contiguous()
+        x = hidden.reshape(-1, hidden.shape[-1]).float()[:, :W]
         h = ragged.residual_norm(x, None, self.norm_w, self.groups,
                                  self.config.rms_norm_eps, self.head_w.shape[1],
                                  self.head_w.dtype)
@@ -121,6 +126,7 @@ class RaggedHead(torch.nn.Module):
     # differentiable forms (fine-tuning)
     def train_norm(self, hidden: torch.Tensor) -> torch.Tensor:
         from bloombee_amd.ops.reference import grouped_rms_norm
+        hidden = hidden[..., :self.config.hidden_size]
         y = grouped_rms_norm(hidden, self.norm_w, self.groups,
                              self.config.rms_norm_eps).to(self.head_w.dtype)
         return F.pad(y, (0, self.head_w.shape[1] - y.shape[-1]))
@@ -162,6 +168,10 @@ class DistributedRaggedModel(DistributedLlamaModel):
     @property
     def uses_previous(self) -> bool:
         return self.head.uses_previous
+
+    def prompt_hidden(self, like: torch.Tensor) -> torch.Tensor:
+        p = super().prompt_hidden(like)
+        return torch.cat([p] * self.head.copies, -1)
 
     def embed(self, input_ids: torch.Tensor, start_pos: int = 0,
               last: Optional[torch.Tensor] = None) -> torch.Tensor:

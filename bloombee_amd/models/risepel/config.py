@@ -55,6 +55,11 @@ RISEPEL_PRESETS = {
     # the same with 16 recurrent heads of 128 keys and 256 values
     "risepel-8b-gla-4l": _preset(4096, 32000, [
         _gla(16, 128, 256, ff=14336) for _ in range(4)]),
+    # the mixers of both without feed-forward
+    "risepel-8b-latent-mixer-4l": _preset(4096, 32000, [
+        _latent(32, 128, 64, 128, 512, 1536, 0) for _ in range(4)]),
+    "risepel-8b-gla-mixer-4l": _preset(4096, 32000, [
+        _gla(16, 128, 256) for _ in range(4)]),
     # both kinds, a shared latent
     "risepel-8b-4l": _preset(4096, 32000, [
         _latent(32, 128, 64, 128, 512, 1536, 1024, ff=14336),

@@ -57,6 +57,9 @@ VUMEDRA_PRESETS = {
     # layers of llama-3-8b's width, heads and feed-forward
     "vumedra-8b-attn-4l": _preset(4096, 32000, [
         _attention(32, 8, 128, 128, _dense(14336)) for _ in range(4)], 65521),
+    # the same without feed-forward
+    "vumedra-8b-attn-mixer-4l": _preset(4096, 32000, [
+        _attention(32, 8, 128, 128, None) for _ in range(4)], 65521),
     # 16 memory heads of 128 keys and 256 values
     "vumedra-8b-mlstm-4l": _preset(4096, 32000, [
         _mlstm(16, 128, 256, _dense(14336)) for _ in range(4)], 65521),

@@ -23,6 +23,7 @@ from typing import Dict, List, Optional
 
 import numpy as np
 import torch
+import torch.nn.functional as F
 
 from bloombee_amd import ops
 from bloombee_amd.engine import BlockStack
@@ -103,6 +104,11 @@ class OffloadedBlockStack:
         self._host: Dict[int, Dict[str, _HostParam]] = {}
 
         if self.resident < n:
+            # blocks that share their weights stream them one by one
+            for blk in stack.blocks[self.resident:]:
+                for name, p in list(blk.named_parameters(recurse=False)):
+                    setattr(blk, name, torch.nn.Parameter(
+                        p.data, requires_grad=p.requires_grad))
             # host copies + free the device params of offloaded blocks
             ndisk = int(round((n - self.resident)
                               * policy.weight_disk_percent / 100.0))
@@ -197,7 +203,8 @@ class OffloadedBlockStack:
                     if self._arena_owner[nxt % 2] != nxt:
                         self._fill(nxt, nxt % 2)
             if n_over > 0:
-                hidden[:, :n_over] += deep_prompts[i, sp0:sp0 + n_over].to(hidden.dtype)
+                dp = deep_prompts[i, sp0:sp0 + n_over].to(hidden.dtype)
+                hidden[:, :n_over, :dp.shape[-1]] += dp
             if tree_mask is not None:
                 hidden = blk.forward_inference(hidden, kv, start_pos,
                                                position_ids, tree_mask=tree_mask)
@@ -218,6 +225,7 @@ class OffloadedBlockStack:
                 self._ensure(i)
             if pre > 0 and hidden.shape[1] >= pre:
                 dp = deep_prompts[i].to(hidden.dtype).unsqueeze(0)
+                dp = F.pad(dp, (0, hidden.shape[-1] - dp.shape[-1]))
                 hidden = torch.cat([hidden[:, :pre] + dp, hidden[:, pre:]], 1)
             hidden = blk.forward_train(hidden, start_pos)
         return hidden

@@ -1,9 +1,10 @@
 // Paged attention over ragged batches: rows of many sequences, each with its
-// own position, with a sliding window, a linear distance bias
+// own position, with a sliding window, chunks (a row sees its own stretch of
+// positions, counted from the sequence's start), a linear distance bias
 // (score - slope_h * (i - j)), separate key and value sizes, grouped key/value
 // heads, a sink (one more score per head, unscaled and without a value) and a
 // sigmoid output gate in the epilogue. Every one of these is a parameter;
-// window 0, null slopes, null sinks and a null gate switch them off.
+// window 0, chunk 0, null slopes, null sinks and a null gate switch them off.
 //
 // Two MFMA kernels and one plain kernel:
 //  * attn_ragged_prefill_kernel: sequences that bring two tokens or more. The
@@ -14,7 +15,8 @@
 //    and split over waves and workgroups.
 //  * attn_ragged_simple_kernel: one wave per (row, head), f32 arithmetic on
 //    any element type and any head size. Without value pages the values are
-//    the first vdim elements of the keys.
+//    the first vdim elements of the keys. Keys may hold several maps side by
+//    side, of which query heads take turns.
 //
 // Both MFMA kernels compute S^T = K Q^T and O^T = V^T P^T. The rows of a
 // 32-key tile are handed to the two score MFMAs in the order
@@ -47,12 +49,16 @@ struct AttnArgs {
   float* pml;           // decode splits: (units, 16, 2) max and sum
   float* pacc;          // (units, 16, dvp)
   long ldg, ldo;
-  int H, G, dim, vdim, dkp, dvp, P, maxp, window, n_split;
+  int H, G, dim, vdim, dkp, dvp, P, maxp, window, chunk, n_split;
+  int maps;             // of a key (plain kernel): its rows are maps * dkp long
   float scale;
 };
 
-DEVINL int first_key(int pos, int window) {
-  return window > 0 ? max(0, pos - window + 1) : 0;
+// First position that a row sees.
+DEVINL int first_key(const AttnArgs& a, int pos) {
+  int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  if (a.chunk > 0) lo = max(lo, pos - max(pos, 0) % a.chunk);
+  return lo;
 }
 
 // Takes a sink (log2 units) into a row's softmax: returns the factor of its
@@ -133,7 +139,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefil
   const unsigned short* vpool = (const unsigned short*)a.vp;
 
   // this lane's rows (columns of S^T): token, head, position
-  int tok[QC], head[QC], qpos[QC];
+  int tok[QC], head[QC], qpos[QC], sees[QC];
   float sl2[QC];
   bf16x8 qf[QC][NKK];
 #pragma unroll
@@ -142,6 +148,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefil
     tok[c] = r / Hg;
     head[c] = g * Hg + r % Hg;
     qpos[c] = qs + tok[c];
+    sees[c] = qpos[c] - first_key(a, qpos[c]) + 1;
     sl2[c] = a.slopes ? a.slopes[head[c]] * LOG2E : 0.f;
     const unsigned short* qp = (const unsigned short*)a.q +
         ((long)(t0 + tok[c]) * a.H + head[c]) * DK + hi * 8;
@@ -150,17 +157,16 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefil
       qf[c][kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
   }
   const float sc2 = a.scale * LOG2E;
-  const int wlim = a.window > 0 ? a.window : 0x7fffffff;
 
   // visible keys of the workgroup and of this wave
   const int last = min(base + 64 * QC, R) - 1;
   const int kend = qs + last / Hg + 1;
-  const int kbeg = first_key(qs + base / Hg, a.window) & ~31;
+  const int kbeg = first_key(a, qs + base / Hg) & ~31;
   const int wr0 = min(base + wave * QC * 16, R - 1);
   const int wr1 = min(base + (wave + 1) * QC * 16, R) - 1;
-  const int wlo = first_key(qs + wr0 / Hg, a.window);   // any row sees >= wlo
+  const int wlo = first_key(a, qs + wr0 / Hg);   // any row sees >= wlo
   const int whi = qs + max(wr0, wr1) / Hg;              // any row sees <= whi
-  const int flo = first_key(qs + max(wr0, wr1) / Hg, a.window);  // all rows do
+  const int flo = first_key(a, qs + max(wr0, wr1) / Hg);  // all rows do
   const int fhi = qs + wr0 / Hg;
 
   float m2[QC], l[QC];
@@ -262,7 +268,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_prefil
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
             const int dist = d0[c] - (hf * 32 + j);
-            if (dist < 0 || dist >= wlim) p[c][hf][j] = NEG_BIG;
+            if (dist < 0 || dist >= sees[c]) p[c][hf][j] = NEG_BIG;
           }
     }
 #pragma unroll
@@ -369,7 +375,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_ragged_decode
     qf[kk] = as_bf16x8(*reinterpret_cast<const short8*>(qp + kk * 32));
 
   // tiles of the visible range, this split's share, this wave's every fourth
-  const int lo = first_key(pos, a.window);
+  const int lo = first_key(a, pos);
   const int t_beg = lo / 32;
   const int t_all = pos < 0 ? 0 : pos / 32 + 1 - t_beg;
   const int per = (t_all + a.n_split - 1) / a.n_split;
@@ -568,7 +574,7 @@ __global__ __launch_bounds__(256) void attn_ragged_combine_kernel(AttnArgs a) {
 
 static constexpr int SIMPLE_MAXD = 1024;
 
-template <typename T>
+template <typename T, typename TO>
 __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
   __shared__ float q_lds[SIMPLE_MAXD];
   __shared__ float p_lds[64];
@@ -580,6 +586,7 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
   const T* kpool = (const T*)a.kp;
   const T* vpool = a.vp ? (const T*)a.vp : kpool;
   const long vstep = a.vp ? a.P : 1;  // between a value's elements
+  const long ldk = (long)a.maps * a.dkp, map0 = h % a.maps * a.dkp;
   for (int d = lane; d < a.dim; d += 64)
     q_lds[d] = ldf((const T*)a.q + ((long)row * a.H + h) * a.dkp + d);
   __syncthreads();
@@ -588,17 +595,17 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
   float acc[SIMPLE_MAXD / 64];
 #pragma unroll
   for (int i = 0; i < SIMPLE_MAXD / 64; ++i) acc[i] = 0.f;
-  for (int kb = first_key(pos, a.window); kb <= pos; kb += 64) {
+  for (int kb = first_key(a, pos); kb <= pos; kb += 64) {
     const int key = kb + lane;
     float sc = NEG_BIG;
     if (key <= pos) {
       const long pg = (long)table[key / a.P] * a.G + g;
-      const T* kr = kpool + (pg * a.P + key % a.P) * a.dkp;
+      const T* kr = kpool + (pg * a.P + key % a.P) * ldk + map0;
       float dot = 0.f;
       for (int d = 0; d < a.dim; ++d) dot += q_lds[d] * ldf(kr + d);
       sc = dot * a.scale - slope * (float)(pos - key);
       v_lds[lane] = a.vp ? pg * a.dvp * a.P + key % a.P
-                         : (pg * a.P + key % a.P) * a.dkp;
+                         : (pg * a.P + key % a.P) * ldk;
     }
     const float mn = fmaxf(m, wave_reduce_max(sc));
     const float corr = expf(m - mn);
@@ -632,6 +639,6 @@ __global__ __launch_bounds__(64) void attn_ragged_simple_kernel(AttnArgs a) {
     float o = acc[i] * inv;
     if (a.gate)
       o *= sigmoid_f(ldf((const T*)a.gate + row * a.ldg + h * a.vdim + d));
-    stf((T*)a.out + row * a.ldo + h * a.vdim + d, o);
+    stf((TO*)a.out + row * a.ldo + h * a.vdim + d, o);
   }
 }

@@ -8,6 +8,7 @@
 #include "rows.hip"
 #include "latent.hip"
 #include "gla.hip"
+#include "gla_host.h"
 
 static void check_turns(const OptTensor& t, long rdims) {
   TORCH_CHECK(rdims % 2 == 0 && t.has_value() && t->is_cuda() &&
@@ -18,7 +19,7 @@ static void check_turns(const OptTensor& t, long rdims) {
 
 // dims: [q_off, c_off, g_off, q_rank, rank, rot, rdims, rp, gate columns,
 //        has_kv]
-void latent_post(Tensor y, std::vector<long> dims, double eps, Tensor qn,
+void latent_post(Tensor y, std::vector<long> dims, double eps, double amp, Tensor qn,
                  OptTensor cn, OptTensor turns, Tensor cq, OptTensor gate,
                  Tensor kp, Tensor table, Tensor tok_seq, Tensor tok_pos) {
   TORCH_CHECK(dims.size() == 10);
@@ -29,6 +30,7 @@ void latent_post(Tensor y, std::vector<long> dims, double eps, Tensor qn,
                 &a.rdims, &a.rp, &a.gn, &a.has_kv};
   for (int i = 0; i < 10; ++i) *f[i] = (int)dims[i];
   a.eps = (float)eps;
+  a.amp = (float)amp;
   check_act(cq);
   const auto ta = cq.scalar_type();
   CHECK_F32(qn);
@@ -89,7 +91,7 @@ void latent_post(Tensor y, std::vector<long> dims, double eps, Tensor qn,
 
 static LatentQueryArgs query_args(const Tensor& y, const OptTensor& turns,
                                   const Tensor& tok_pos, long dim, long rot,
-                                  long rdims, long H) {
+                                  long rdims, double amp, long H) {
   LatentQueryArgs a{};
   a.y = as_parts(y);
   CHECK_I32(tok_pos);
@@ -102,16 +104,17 @@ static LatentQueryArgs query_args(const Tensor& y, const OptTensor& turns,
   a.dim = (int)dim;
   a.rot = (int)rot;
   a.rdims = (int)rdims;
+  a.amp = (float)amp;
   return a;
 }
 
 // q (N, H, ld) from the query GEMM
 void latent_rope(Tensor y, OptTensor turns, Tensor tok_pos, long dim, long rot,
-                 long rdims, Tensor q) {
+                 long rdims, double amp, Tensor q) {
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(0) == y.size(1) &&
               q.size(2) >= dim + rot);
   check_act(q);
-  auto a = query_args(y, turns, tok_pos, dim, rot, rdims, q.size(1));
+  auto a = query_args(y, turns, tok_pos, dim, rot, rdims, amp, q.size(1));
   a.q = q.data_ptr();
   a.ldq = q.size(2);
   if (q.size(0) == 0) return;
@@ -186,8 +189,8 @@ bool latent_decode_fits(long rp, long rtp) {
 // Listed one-token rows: query GEMM output y -> gated attention in out.
 void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
                    Tensor tok_pos, Tensor cu, Tensor q_start, Tensor dec,
-                   long max_ctx,
-                   long dim, long rot, long rdims, long vdim, double scale,
+                   long max_ctx, long dim, long rot, long rdims, double amp,
+                   long vdim, double scale,
                    long window, Tensor wk, Tensor wv, OptTensor sinks,
                    OptTensor gate, Tensor out) {
   for (const Tensor& t : {kp, wk, wv}) CHECK_T(t, at::kBFloat16);
@@ -205,7 +208,7 @@ void latent_decode(Tensor y, OptTensor turns, Tensor kp, Tensor table,
               out.size(1) >= H * vdim);
   const long n = dec.numel();
   if (n == 0) return;
-  auto qa = query_args(y, turns, tok_pos, dim, rot, rdims, H);
+  auto qa = query_args(y, turns, tok_pos, dim, rot, rdims, amp, H);
   auto bopt = kp.options();
   auto fopt = bopt.dtype(at::kFloat);
   auto q = torch::empty({n, H, ck}, bopt);
@@ -378,15 +381,6 @@ void gla_step(Tensor y, Tensor a1, std::vector<long> dims,
   check_launch();
 }
 
-static int pad_dim(long dim) {
-  return dim <= 32 ? 32 : dim <= 64 ? 64 : dim <= 128 ? 128 : 256;
-}
-static int chunk_of(long dim) { return dim <= 128 ? 64 : 32; }
-
-static size_t prep_lds(int dp, int C, long r) {
-  return 4 * ((size_t)C * (dp + 4) + (C + dp) * r);
-}
-
 // Tokens of a chunk, 0 where the chunk form does not take these sizes.
 long gla_chunk(long dim, long vdim, long r) {
   if (dim > 256 || vdim < 1 || vdim > 512) return 0;
@@ -453,43 +447,7 @@ void gla_chunks(Tensor y, Tensor a1, std::vector<long> dims,
   a.eps = (float)consts[2];
   const bool vec = all_of_8({a.ldy, a.q_off, a.k_off, a.v_off, a.g_off, a.dim,
                              a.vdim, a.ldo});
-  auto go = [&](auto dp, auto c) {
-    constexpr int D = decltype(dp)::value, CC = decltype(c)::value;
-    by_bool(vec, [&](auto v) {
-      constexpr bool VEC = decltype(v)::value;
-      auto prep = gla_prep_kernel<D, CC, VEC>;
-      const size_t l1 = prep_lds(D, CC, a.r);
-      allow_lds(prep, l1);
-      prep<<<dim3(chunks, a.H), 256, l1, cur_stream()>>>(a);
-      check_launch();
-      auto scan = gla_scan_kernel<D, CC, VEC>;
-      const size_t l2 =
-          4 * (2 * CC * (D == 32 ? 96 : D + 32) + CC * 72 + 2 * D);
-      allow_lds(scan, l2);
-      scan<<<dim3((a.vdim + 63) / 64, a.H, list.numel()), 256, l2,
-             cur_stream()>>>(a);
-      check_launch();
-      auto fin = [&](auto nct) {
-        constexpr int N = decltype(nct)::value;
-        auto k = gla_out_kernel<D, CC, N, VEC>;
-        const size_t first =
-            std::max(2 * (CC + 1) * (D + 4), CC * (N * 128 + 24));
-        const size_t l3 = 2 * (first + 2 * CC * (D + 8) + 2 * CC * (CC + 8));
-        allow_lds(k, l3);
-        k<<<dim3(chunks, a.H), 512, l3, cur_stream()>>>(a);
-        check_launch();
-      };
-      if (a.vdim <= 128) fin(std::integral_constant<int, 1>{});
-      else if (a.vdim <= 256) fin(std::integral_constant<int, 2>{});
-      else fin(std::integral_constant<int, 4>{});
-    });
-  };
-  using I32 = std::integral_constant<int, 32>;
-  using I64 = std::integral_constant<int, 64>;
-  if (DP == 32) go(I32{}, I64{});
-  else if (DP == 64) go(I64{}, I64{});
-  else if (DP == 128) go(std::integral_constant<int, 128>{}, I64{});
-  else go(std::integral_constant<int, 256>{}, I32{});
+  launch_chunks<false>(a, chunks, list.numel(), vec);
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {

@@ -15,7 +15,7 @@
 // pair: [buckets, mul_prev, mul_cur] with prev and pair_table
 Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table,
                   OptTensor prev, OptTensor pair_table, std::vector<long> pair,
-                  OptTensor turns) {
+                  OptTensor turns, double scale, long copies) {
   CHECK_I32(ids);
   CHECK_I32(pos);
   check_act(table);
@@ -52,7 +52,10 @@ Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table,
     TORCH_CHECK(turns->numel() == (a.W + 1) / 2);
     a.turns = turns->data_ptr<double>();
   }
-  auto x = torch::empty({N, a.W}, table.options().dtype(at::kFloat));
+  TORCH_CHECK(copies >= 1);
+  a.scale = (float)scale;
+  a.copies = (int)copies;
+  auto x = torch::empty({N, copies * a.W}, table.options().dtype(at::kFloat));
   if (N == 0) return x;
   a.x = x.data_ptr<float>();
   by_type(table.scalar_type(), [&](auto t) {
@@ -69,13 +72,19 @@ Tensor embed_rows(Tensor ids, Tensor pos, Tensor table, OptTensor pos_table,
 void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
                    OptTensor idw, OptTensor hprev, OptTensor nw, long groups,
                    double eps, OptTensor h, double alpha, OptTensor bias,
-                   bool post, OptTensor bw) {
-  CHECK_F32(x);
-  TORCH_CHECK(x.dim() == 2);
+                   bool post, OptTensor bw, OptTensor other) {
+  // rows may lie apart (columns of a wider matrix)
+  auto rows_f32 = [](const Tensor& t) {
+    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.scalar_type() == at::kFloat &&
+                    (t.stride(1) == 1 || t.size(1) == 1) && t.stride(0) >= t.size(1),
+                "f32 rows on the device");
+  };
+  rows_f32(x);
   const long N = x.size(0);
   const int W = x.size(1);
   ResidualArgs a{};
   a.x = x.data_ptr<float>();
+  a.ldx = x.stride(0);
   a.W = W;
   a.eps = (float)eps;
   a.groups = (int)groups;
@@ -92,7 +101,10 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
     TORCH_CHECK(bw->numel() == W && (parts.has_value() || routed.has_value()));
     a.bw = bw->data_ptr<float>();
   }
-  bool vec = W % 4 == 0;
+  auto aligned = [](const Tensor& t) {
+    return t.stride(0) % 4 == 0 && (size_t)t.data_ptr() % 16 == 0;
+  };
+  bool vec = W % 4 == 0 && aligned(x);
   at::ScalarType tp = at::kFloat, ta = at::kFloat;
   if (parts.has_value()) {
     check_act(*parts);
@@ -145,6 +157,21 @@ void residual_norm(Tensor x, OptTensor parts, OptTensor routed, OptTensor ids,
     a.h = h->data_ptr();
     a.ldh = h->size(1);
     vec = vec && a.ldh % 4 == 0;
+  }
+  if (other.has_value()) {
+    rows_f32(*other);
+    TORCH_CHECK(!nw.has_value() && h.has_value() && other->size(0) == N &&
+                other->size(1) == W);
+    check_act(*h);
+    TORCH_CHECK(h->is_contiguous() && h->size(0) == N && h->size(1) >= 2 * W);
+    TORCH_CHECK(!(routed.has_value() || idw.has_value()) ||
+                h->scalar_type() == ta, "one activation type per call");
+    ta = h->scalar_type();
+    a.other = other->data_ptr<float>();
+    a.ldx2 = other->stride(0);
+    a.h = h->data_ptr();
+    a.ldh = h->size(1);
+    vec = vec && a.ldh % 4 == 0 && aligned(*other);
   }
   if (N == 0) return;
   const size_t lds = 4 * (((W + 3) & ~3) + (size_t)a.groups + 32);
@@ -450,15 +477,80 @@ void head_post(Tensor parts, std::vector<long> dims, std::vector<double> consts,
   check_launch();
 }
 
-// dims: [act, gate or up, up, ff, router offset, E, NI, top, sigmoid scores]
+// dims: [q,k,v offsets, H, G, maps, dim, vdim, rotated dimensions]
+void rope_post(Tensor parts, std::vector<long> dims, double amp, Tensor turns,
+               Tensor q, Tensor kp, Tensor vp, Tensor table, Tensor tok_seq,
+               Tensor tok_pos) {
+  TORCH_CHECK(dims.size() == 9);
+  RopePostArgs a{};
+  a.y = as_parts(parts);
+  const long N = parts.size(1);
+  int* f[9] = {&a.q_off, &a.k_off, &a.v_off, &a.H, &a.G, &a.M, &a.dim, &a.vdim,
+               &a.rdims};
+  for (int i = 0; i < 9; ++i) *f[i] = (int)dims[i];
+  a.amp = (float)amp;
+  TORCH_CHECK(a.H >= 1 && a.G >= 1 && a.H % a.G == 0 && a.M >= 1 && a.dim >= 1 &&
+              a.vdim >= 1 && a.rdims >= 2 && a.rdims % 2 == 0 && a.rdims <= a.dim);
+  auto inside = [&](int off, int n) { return off >= 0 && off + n <= a.y.ld; };
+  TORCH_CHECK(inside(a.q_off, a.H * a.M * a.dim) &&
+              inside(a.k_off, a.G * a.M * a.dim) && inside(a.v_off, a.G * a.vdim));
+  CHECK_T(turns, at::kDouble);
+  TORCH_CHECK(turns.numel() == a.rdims / 2);
+  a.turns = turns.data_ptr<double>();
+  check_act(q);
+  const auto ta = q.scalar_type();
+  for (const Tensor& t : {q, kp, vp})
+    TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == ta,
+                "q and the pages share one element type");
+  TORCH_CHECK(q.dim() == 4 && q.size(0) == N && q.size(1) == a.H &&
+              q.size(2) == a.M && q.size(3) >= a.dim);
+  a.dk = q.size(3);
+  TORCH_CHECK(kp.dim() == 4 && vp.dim() == 4 && kp.size(1) == a.G &&
+              vp.size(1) == a.G && kp.size(3) == (long)a.M * a.dk &&
+              vp.size(3) == kp.size(2) && vp.size(2) >= a.vdim &&
+              vp.size(0) == kp.size(0));
+  a.q = q.data_ptr();
+  a.kp = kp.data_ptr();
+  a.vp = vp.data_ptr();
+  a.P = kp.size(2);
+  a.dvp = vp.size(2);
+  CHECK_I32(table);
+  CHECK_I32(tok_seq);
+  CHECK_I32(tok_pos);
+  TORCH_CHECK(tok_seq.numel() == N && tok_pos.numel() == N && table.dim() == 2);
+  a.table = table.data_ptr<int>();
+  a.maxp = table.size(1);
+  a.tok_seq = tok_seq.data_ptr<int>();
+  a.tok_pos = tok_pos.data_ptr<int>();
+  if (N == 0) return;
+  bool vec = true;
+  for (int v : {a.y.ld, a.q_off, a.k_off, a.v_off, a.dim, a.vdim, a.dk, a.dvp})
+    vec = vec && v % 8 == 0;
+  // few rows: more workgroups on each
+  const int units = (a.H + a.G) * a.M + a.G;
+  a.per = N >= 256 ? units : 8;
+  const size_t lds = 4 * (size_t)a.rdims;
+  by_type(parts.scalar_type(), [&](auto p) {
+    by_type(ta, [&](auto t) {
+      by_bool(vec, [&](auto v) {
+        rope_post_kernel<decltype(p), decltype(t), decltype(v)::value ? 8 : 1>
+            <<<dim3(N, (units + a.per - 1) / a.per), 256, lds, cur_stream()>>>(a);
+      });
+    });
+  });
+  check_launch();
+}
+
+// dims: [act, gate or up, up, ff, router offset, E, NI, top, sigmoid scores,
+//        renormalize]
 void ff_post(OptTensor parts, OptTensor rparts, std::vector<long> dims,
              double rscale, OptTensor corr, Tensor out, OptTensor ids,
              OptTensor wts, OptTensor idw) {
-  TORCH_CHECK(dims.size() == 9);
+  TORCH_CHECK(dims.size() == 10);
   FfPostArgs a{};
-  int* f[9] = {&a.act, &a.u_off, &a.u2_off, &a.ff, &a.rt.off,
-               &a.rt.E, &a.rt.NI, &a.rt.top, &a.rt.sigmoid};
-  for (int i = 0; i < 9; ++i) *f[i] = (int)dims[i];
+  int* f[10] = {&a.act, &a.u_off, &a.u2_off, &a.ff, &a.rt.off, &a.rt.E,
+                &a.rt.NI, &a.rt.top, &a.rt.sigmoid, &a.rt.renorm};
+  for (int i = 0; i < 10; ++i) *f[i] = (int)dims[i];
   check_act(out);
   TORCH_CHECK(out.dim() == 2 && out.is_contiguous());
   const long N = out.size(0);
@@ -581,8 +673,7 @@ static void launch_mfma(AttnArgs& a, const Tensor& pre, const Tensor& dec,
     const long units = dec.numel() * a.G * nch;
     // tiles a sequence can see, and enough workgroups to fill the chip with
     // at least two tiles for each wave of them
-    const long seen = a.window > 0 ? std::min<long>(a.window, max_ctx) : max_ctx;
-    const long tiles = (seen + 31) / 32 + 1;
+    const long tiles = (seen_keys(a, max_ctx) + 31) / 32 + 1;
     a.n_split = (int)std::max<long>(
         1, std::min<long>({32, 512 / std::max<long>(1, units), tiles / 8}));
     Tensor pml, pacc;
@@ -606,8 +697,8 @@ static void launch_mfma(AttnArgs& a, const Tensor& pre, const Tensor& dec,
 void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
                  Tensor tok_seq, Tensor tok_pos, Tensor cu, Tensor q_start,
                  Tensor pre, Tensor dec, long max_new, long max_ctx, long dim,
-                 long vdim, double scale, long window, OptTensor slopes,
-                 OptTensor sinks, OptTensor gate, Tensor out) {
+                 long vdim, double scale, long window, long chunk,
+                 OptTensor slopes, OptTensor sinks, OptTensor gate, Tensor out) {
   check_act(q);
   const auto ta = q.scalar_type();
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous());
@@ -669,6 +760,8 @@ void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
   a.out = out.data_ptr();
   a.ldo = out.stride(0);
   a.window = (int)window;
+  a.chunk = (int)chunk;
+  a.maps = 1;
   a.scale = (float)scale;
   a.n_split = 1;
 
@@ -696,7 +789,7 @@ void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
   TORCH_CHECK(dim <= SIMPLE_MAXD && vdim <= SIMPLE_MAXD,
               "head size above ", SIMPLE_MAXD);
   by_type(ta, [&](auto t) {
-    attn_ragged_simple_kernel<decltype(t)>
+    attn_ragged_simple_kernel<decltype(t), decltype(t)>
         <<<dim3(N, a.H), 64, 0, cur_stream()>>>(a);
   });
   check_launch();
@@ -708,10 +801,11 @@ void attn_ragged(Tensor q, Tensor kp, OptTensor vp, Tensor table,
 
 // h (N, K), up (E, planes, F, K), down (E, Wp, F), ids/wts (N, top)
 // -> y (N, top, Wp); rows of skipped choices are not written. Two planes:
-// silu(gate) * up, one: relu(up)^2. win: the weight multiplies the expert's
-// input, else its output.
+// gated activation (limit, slope, shift), one: relu(up)^2. win: the weight
+// multiplies the expert's input, else its output.
 Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
-                   bool win) {
+                   bool win, double limit, double slope, double shift) {
+  const GluConst glu{(float)limit, (float)slope, (float)shift};
   check_act(h);
   const auto ta = h.scalar_type();
   for (const Tensor& t : {h, up, down})
@@ -749,7 +843,7 @@ Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
         moe_skinny_kernel<decltype(np)::value, decltype(full)::value>
             <<<dim3(F / 64, E), 256, 0, st>>>(
                 hp, (const bf16_bits*)up.data_ptr(), idp, w1, actp, S, top, F,
-                K, K, F);
+                K, K, F, glu);
       });
     });
     check_launch();
@@ -757,7 +851,7 @@ Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
       moe_skinny_kernel<0, decltype(full)::value>
           <<<dim3(Wp / 64, E), 256, 0, st>>>(
               actp, (const bf16_bits*)down.data_ptr(), idp, w2,
-              (bf16_bits*)y.data_ptr(), S, top, Wp, F, F, Wp);
+              (bf16_bits*)y.data_ptr(), S, top, Wp, F, F, Wp, glu);
     });
     check_launch();
     return y;
@@ -779,12 +873,12 @@ Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
       moe_simple_kernel<decltype(np)::value>
           <<<dim3(F / 64, max_tiles), 256, 0, st>>>(
               h.data_ptr<float>(), up.data_ptr<float>(), offp, sp, tp, w1,
-              act.data_ptr<float>(), top, F, K, K, F);
+              act.data_ptr<float>(), top, F, K, K, F, glu);
     });
     check_launch();
     moe_simple_kernel<0><<<dim3(Wp / 64, max_tiles), 256, 0, st>>>(
         act.data_ptr<float>(), down.data_ptr<float>(), offp, sp, tp, w2,
-        y.data_ptr<float>(), top, Wp, F, F, Wp);
+        y.data_ptr<float>(), top, Wp, F, F, Wp, glu);
     check_launch();
     return y;
   }
@@ -796,13 +890,13 @@ Tensor moe_experts(Tensor h, Tensor up, Tensor down, Tensor ids, Tensor wts,
       moe_tile_kernel<B, decltype(np)::value><<<nu * max_tiles, 256, 0, st>>>(
           (const bf16_bits*)h.data_ptr(), (const bf16_bits*)up.data_ptr(), offp,
           sp, tp, w1, (bf16_bits*)act.data_ptr(), max_tiles, nu, top, F, K, K,
-          F);
+          F, glu);
     });
     check_launch();
     moe_tile_kernel<B, 0><<<nd * max_tiles, 256, 0, st>>>(
         (const bf16_bits*)act.data_ptr(), (const bf16_bits*)down.data_ptr(),
         offp, sp, tp, w2, (bf16_bits*)y.data_ptr(), max_tiles, nd, top, Wp, F,
-        F, Wp);
+        F, Wp, glu);
     check_launch();
   };
   if (BM == 128) tile(std::integral_constant<int, 128>{});
@@ -817,6 +911,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("softcap", &softcap);
   m.def("proj_post", &proj_post);
   m.def("head_post", &head_post);
+  m.def("rope_post", &rope_post);
   m.def("ff_post", &ff_post);
   m.def("router_gemm", &router_gemm);
   m.def("gemm_parts", &gemm_parts);

@@ -6,6 +6,10 @@
 // portion starts at position 0 starts from a zero state, whatever its slot
 // holds.
 //
+// The same with a forget gate that also decides what is written (HGRN2; WRITES in
+// the kernels): alpha = lower + (1 - lower) sigmoid(z + b) and k = 1 - alpha, z a
+// projection in f32 like q, which passes through silu; no output gate.
+//
 //  gla_step_kernel   token by token, everything fused: decoded tokens, and any
 //                    sizes and types.
 //  gla_prep_kernel   prompts in chunks of C tokens, all chunks side by side:
@@ -15,6 +19,7 @@
 //  gla_out_kernel    all chunks side by side:
 //                       A[t][s] = sum_d q_t k_s 2^(b_t - b_s)   (s <= t)
 //                       o = (q 2^b) S + A v, norm and gate
+//  hgrn_prep_kernel  gla_prep_kernel for gates that write
 //
 // Chunk products run on bf16 MFMAs with decayed operands, weights and states
 // split into two bf16 (the value and what its rounding lost). All exponents of
@@ -35,11 +40,24 @@ DEVINL float log2_sigmoid(float z) {
   return fminf(z, 0.f) * LOG2E - l;
 }
 
+// A forget gate in (lower, 1) and what it leaves room for, 1 - gate.
+DEVINL float forget_room(float lower, float z) {
+  return (1.f - lower) * sigmoid_f(-z);
+}
+
+// log2 of the gate, accurate where it is nearly one. A gate below 2^-64 forgets
+// all there is.
+DEVINL float log2_forget(float lower, float z, float room) {
+  if (room < 0.01f) return -(room + 0.5f * room * room + room * room * room * (1.f / 3)) * LOG2E;
+  return __builtin_amdgcn_logf(fmaxf(lower + (1.f - lower) * sigmoid_f(z), 5.4e-20f));
+}
+
 struct GlaArgs {
-  Parts y;            // q, k, v, g columns
-  Parts a1;           // f32; a1_off: first column
+  Parts y;            // q, k, v, g columns; WRITES: q, v
+  Parts a1;           // f32; a1_off: first column; WRITES: z
   const float* a2;    // (r, H * dim)
   const float* a2b;   // (H * dim,)
+  const float* lower; // (H * dim,), WRITES
   const float* nw;    // (vdim,)
   float* state;       // (slots, H, dim, vdim)
   void* out;          // row stride ldo, H * vdim columns
@@ -54,7 +72,7 @@ struct GlaArgs {
 
 // grid (H, listed sequences). LDS: q, k, alpha (dim each), partial sums
 // (B * V), v, o (vdim each), a1 (r).
-template <typename TP, typename T, int V, int B>
+template <typename TP, typename T, int V, int B, bool WRITES = false>
 __global__ __launch_bounds__(B) void gla_step_kernel(GlaArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds_gla[];
   __shared__ float red[B / WAVE];
@@ -74,13 +92,25 @@ __global__ __launch_bounds__(B) void gla_step_kernel(GlaArgs a) {
     const int pos = a.tok_pos[t];
     if (pos < 0) continue;  // empty slot
     __syncthreads();
-    for (int i = tid; i < a.r; i += B)
-      fold_parts<float, 1>(a.a1, t, a.a1_off + i, a1s + i);
-    __syncthreads();
+    if constexpr (!WRITES) {
+      for (int i = tid; i < a.r; i += B)
+        fold_parts<float, 1>(a.a1, t, a.a1_off + i, a1s + i);
+      __syncthreads();
+    }
     for (int d = tid; d < a.dim; d += B) {
       float v[1];
       const int c = h * a.dim + d;
       fold_parts<TP, 1>(a.y, t, a.q_off + c, v);
+      if constexpr (WRITES) {
+        float z[1];
+        fold_parts<float, 1>(a.a1, t, a.a1_off + c, z);
+        z[0] += a.a2b[c];
+        const float lo = a.lower[c];
+        qs[d] = v[0] / (1.f + expf(-v[0]));
+        ks[d] = (1.f - lo) / (1.f + expf(z[0]));
+        as[d] = lo + (1.f - lo) / (1.f + expf(-z[0]));
+        continue;
+      }
       qs[d] = v[0] * a.qscale;
       fold_parts<TP, 1>(a.y, t, a.k_off + c, v);
       ks[d] = v[0];
@@ -143,18 +173,23 @@ __global__ __launch_bounds__(B) void gla_step_kernel(GlaArgs a) {
     const float inv = 1.f / sqrtf(ss / (float)a.vdim + a.eps);
     T* op = (T*)a.out + t * a.ldo + h * a.vdim;
     for (int i = tid; i < a.vdim; i += B) {
-      float g[1];
-      fold_parts<TP, 1>(a.y, t, a.g_off + h * a.vdim + i, g);
-      stf(op + i, os[i] * inv * a.nw[i] * g[0] * sigmoid_f(g[0]));
+      float v = os[i] * inv * a.nw[i];
+      if constexpr (!WRITES) {
+        float g[1];
+        fold_parts<TP, 1>(a.y, t, a.g_off + h * a.vdim + i, g);
+        v *= g[0] * sigmoid_f(g[0]);
+      }
+      stf(op + i, v);
     }
   }
 }
 
 struct GlaChunkArgs {
   const unsigned short* y;  // (N, ldy) bf16
-  const float* a1;          // (N, ld1), a1_off
+  const float* a1;          // (N, ld1), a1_off; WRITES: z
   const float* a2;          // (r, H * dim)
   const float* a2b;
+  const float* lower;       // (H * dim,), WRITES
   const float* nw;
   float* state;
   float* b;                 // (chunks, H, C, DP): cumulated log2 decays
@@ -216,6 +251,94 @@ DEVINL short8 load_values(const GlaChunkArgs& a, long row0, int len, int h, int 
                           int c) {
   return load_row8<VEC>(a.y + (row0 + min(t, len - 1)) * a.ldy + a.v_off +
                             h * a.vdim, c, a.vdim, t < len);
+}
+
+// Gates that write: the room eight channels of token t leave, zero where !live
+// and beyond the head; l2 gets their log2.
+template <bool VEC>
+DEVINL void load_gates(const GlaChunkArgs& a, long row0, int len, int h, int t,
+                       int d, float* room, float* l2) {
+  const float* z = a.a1 + (row0 + min(t, len - 1)) * a.ld1 + a.a1_off + h * a.dim;
+  const float* zb = a.a2b + h * a.dim;
+  const float* lo = a.lower + h * a.dim;
+  float zv[8], bv[8], lv[8];
+  if constexpr (VEC) {
+    const int c = min(d, a.dim - 8);
+    ldv<8>(z + c, zv);
+    ldv<8>(zb + c, bv);
+    ldv<8>(lo + c, lv);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int c = min(d + j, a.dim - 1);
+      zv[j] = z[c];
+      bv[j] = zb[c];
+      lv[j] = lo[c];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const bool in = t < len && d + j < a.dim;
+    const float r = forget_room(lv[j], zv[j] + bv[j]);
+    room[j] = in ? r : 0.f;
+    if (l2) l2[j] = in ? log2_forget(lv[j], zv[j] + bv[j], r) : 0.f;
+  }
+}
+
+// Eight channels of token t's silu(q).
+template <bool VEC>
+DEVINL void load_silu(const GlaChunkArgs& a, long row0, int len, int h, int t,
+                      int d, float* v) {
+  load_channels<VEC>(a, row0, len, a.q_off, h, t, d, v);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] *= sigmoid_f(v[j]);
+}
+
+// grid (chunks, H). LDS: b (C x (DP + 4))
+template <int DP, int C, bool VEC>
+__global__ __launch_bounds__(256) void hgrn_prep_kernel(GlaChunkArgs a) {
+  constexpr int LDB = DP + 4, PN = C * DP / 8 / 256;
+  extern __shared__ __attribute__((aligned(16))) float lds_b[];
+  const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+  const long row0 = a.row0[ch];
+  const int len = a.len[ch];
+  float k[PN][8];
+#pragma unroll
+  for (int n = 0; n < PN; ++n) {
+    const int idx = tid + n * 256;
+    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
+    float l2[8];
+    load_gates<VEC>(a, row0, len, h, t, d, k[n], l2);
+    stv<8>(lds_b + t * LDB + d, l2);
+  }
+  __syncthreads();
+  const long base = (long)ch * a.H + h;
+  if (tid < DP) {
+    float s = 0.f;
+#pragma unroll 16
+    for (int t = 0; t < C; ++t) {
+      s += lds_b[t * LDB + tid];
+      lds_b[t * LDB + tid] = s;
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int n = 0; n < PN; ++n) {
+    const int idx = tid + n * 256;
+    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
+    float b[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      b[j] = lds_b[t * LDB + d + j];
+      k[n][j] *= fast_exp2(lds_b[(C - 1) * LDB + d + j] - b[j]);
+    }
+    stv<8>(a.b + (base * C + t) * DP + d, b);
+    short8 vh, vl;
+    split8(k[n], vh, vl);
+    const long at = base * 2 * C * DP + t * DP + d;
+    *reinterpret_cast<short8*>(a.kd + at) = vh;
+    *reinterpret_cast<short8*>(a.kd + at + C * DP) = vl;
+  }
 }
 
 // grid (chunks, H). LDS: b (C x (DP + 4)), a1 (C x r), a2 of the head (r x DP)
@@ -429,13 +552,15 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(GlaChunkArgs a) {
 
 // grid (chunks, H), eight waves; a wave owns every eighth tile of 16 value
 // columns. Outputs are made transposed, o^T = S^T qd^T + v^T A^T: a lane holds
-// four consecutive columns of one token. LDS: b, later v; qd; A.
-template <int DP, int C, int NCT, bool VEC>
+// four consecutive columns of one token. LDS: b, later v; qd; A. WRITES: beside b
+// silu(q) and k, which the blocks of A read several times.
+template <int DP, int C, int NCT, bool VEC, bool WRITES = false>
 __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   constexpr int LDB = DP + 4, LDD = DP + 8, LDA = C + 8, NG = DP / 32;
   constexpr int NT = C / 16, NC = C / 32, NB = C / 16, VC = NCT * 128;
   constexpr int LDV = VC + 24;   // rows 12 banks apart, for column reads
-  constexpr int FIRST = 2 * (C + 1) * LDB > C * LDV ? 2 * (C + 1) * LDB : C * LDV;
+  constexpr int BQK = 2 * (C + 1) * LDB + (WRITES ? 4 * C * LDB : 0);
+  constexpr int FIRST = BQK > C * LDV ? BQK : C * LDV;
   constexpr int PB = C * DP / 4 / 512, PQ = C * DP / 8 / 512 > 0 ? C * DP / 8 / 512 : 1;
   constexpr int PV = C * VC / 8 / 512;
   // the states, too, are asked for ahead, where there are registers for them
@@ -448,6 +573,8 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
   unsigned short* vs = lds_out;              // (C, LDV)
   unsigned short* qs = lds_out + FIRST;      // (2, C, LDD)
   unsigned short* as = qs + 2 * C * LDD;     // (2, C, LDA)
+  float* q32 = bs + C * LDB;                 // (C, LDB), WRITES
+  float* k32 = q32 + C * LDB;                // (C, LDB), WRITES
   const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int lane = tid & (WAVE - 1);
@@ -476,8 +603,16 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
 #pragma unroll
   for (int n = 0; n < PQ; ++n) {
     const int idx = min(tid + n * 512, C * DP / 8 - 1);
-    load_channels<VEC>(a, row0, len, a.q_off, h, idx / (DP / 8),
-                       idx % (DP / 8) * 8, rq[n]);
+    const int t = idx / (DP / 8), d = idx % (DP / 8) * 8;
+    if constexpr (WRITES) {
+      float k[8];
+      load_silu<VEC>(a, row0, len, h, t, d, rq[n]);
+      load_gates<VEC>(a, row0, len, h, t, d, k, nullptr);
+      stv<8>(q32 + t * LDB + d, rq[n]);
+      stv<8>(k32 + t * LDB + d, k);
+    } else {
+      load_channels<VEC>(a, row0, len, a.q_off, h, t, d, rq[n]);
+    }
   }
 #pragma unroll
   for (int n = 0; n < PV; ++n) {
@@ -524,8 +659,13 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
         float q[NG][8], k[NG][8];
 #pragma unroll
         for (int kk = 0; kk < NG; ++kk) {
-          load_channels<VEC>(a, row0, len, a.q_off, h, t, kk * 32 + hi * 8, q[kk]);
-          load_channels<VEC>(a, row0, len, a.k_off, h, s, kk * 32 + hi * 8, k[kk]);
+          if constexpr (WRITES) {
+            ldv<8>(q32 + t * LDB + kk * 32 + hi * 8, q[kk]);
+            ldv<8>(k32 + s * LDB + kk * 32 + hi * 8, k[kk]);
+          } else {
+            load_channels<VEC>(a, row0, len, a.q_off, h, t, kk * 32 + hi * 8, q[kk]);
+            load_channels<VEC>(a, row0, len, a.k_off, h, s, kk * 32 + hi * 8, k[kk]);
+          }
         }
 #pragma unroll
         for (int kk = 0; kk < NG; ++kk) {
@@ -552,6 +692,13 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
           const int t = I * 16 + hi * 4 + r, s = J * 16 + li;
           if (s > t || t >= len) continue;
           float sum = 0.f;
+          if constexpr (WRITES) {
+            for (int d = 0; d < a.dim; ++d)
+              sum += q32[t * LDB + d] * k32[s * LDB + d] *
+                     fast_exp2(bs[t * LDB + d] - bs[s * LDB + d]);
+            acc[r] = sum;
+            continue;
+          }
           const unsigned short* qp =
               a.y + (row0 + t) * a.ldy + a.q_off + h * a.dim;
           const unsigned short* kp =
@@ -659,18 +806,24 @@ __global__ __launch_bounds__(512) void gla_out_kernel(GlaChunkArgs a) {
       if (v0 >= a.vdim) continue;
       if constexpr (VEC) {
         float g[4], w[4];
-        ldv<4>(gp + v0, g);
+        if constexpr (!WRITES) ldv<4>(gp + v0, g);
         ldv<4>(a.nw + v0, w);
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          w[r] *= o[c][t][r] * inv * g[r] * sigmoid_f(g[r]);
+        for (int r = 0; r < 4; ++r) {
+          w[r] *= o[c][t][r] * inv;
+          if constexpr (!WRITES) w[r] *= g[r] * sigmoid_f(g[r]);
+        }
         stv<4>(op + v0, w);
       } else {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           if (v0 + r >= a.vdim) continue;
-          const float g = bf2f(gp[v0 + r]);
-          op[v0 + r] = cvt_bf(o[c][t][r] * inv * a.nw[v0 + r] * g * sigmoid_f(g));
+          float w = o[c][t][r] * inv * a.nw[v0 + r];
+          if constexpr (!WRITES) {
+            const float g = bf2f(gp[v0 + r]);
+            w *= g * sigmoid_f(g);
+          }
+          op[v0 + r] = cvt_bf(w);
         }
       }
     }

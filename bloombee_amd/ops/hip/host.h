@@ -64,6 +64,15 @@ static inline Parts as_parts(const Tensor& t) {
                (int)t.size(2)};
 }
 
+// Keys a row sees at most.
+template <typename Args>
+static long seen_keys(const Args& a, long max_ctx) {
+  long n = max_ctx;
+  if (a.window > 0) n = std::min<long>(n, a.window);
+  if (a.chunk > 0) n = std::min<long>(n, a.chunk);
+  return n;
+}
+
 static inline bool all_of_8(std::initializer_list<long> v) {
   for (long x : v)
     if (x % 8) return false;

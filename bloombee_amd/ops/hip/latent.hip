@@ -35,7 +35,7 @@ struct LatentPostArgs {
   const int* tok_pos;
   int q_off, c_off, g_off, q_rank, rank, rot, rdims, rp, ck, ldq, gn, P, maxp;
   int has_kv;
-  float eps;
+  float eps, amp;       // amp: factor of cosine and sine
 };
 
 // Section of n columns into LDS; returns 1 / rms.
@@ -106,6 +106,8 @@ __global__ __launch_bounds__(256) void latent_post_kernel(LatentPostArgs a) {
         float w[1], c, s;
         fold_parts<TP, 1>(a.y, t, a.c_off + a.rank + (i < half ? i + half : k), w);
         rotation(pos, a.turns[k], c, s);
+        c *= a.amp;
+        s *= a.amp;
         v[0] = i < half ? v[0] * c - w[0] * s : v[0] * c + w[0] * s;
       }
       stf(o + a.rp + i, v[0]);
@@ -130,6 +132,7 @@ struct LatentQueryArgs {
   const void* wk;       // (H, rp, dimp): W_uk^T, zero padded
   void* q;              // rope: (N, H, ldq); absorb: (n_list, H, ck)
   int n_list, H, dim, rot, rdims, rp, ck, dimp, ldq;
+  float amp;            // factor of cosine and sine
 };
 
 // grid N: a row's queries, [dim unrotated | rot rotated | zeros] per head
@@ -139,45 +142,20 @@ __global__ __launch_bounds__(256) void latent_rope_kernel(LatentQueryArgs a) {
   const long t = blockIdx.x;
   const int tid = threadIdx.x, half = a.rdims / 2;
   const int pos = max(a.tok_pos[t], 0);
-  for (int k = tid; k < half; k += 256)
-    rotation(pos, a.turns[k], lds_cs[k], lds_cs[half + k]);
+  for (int k = tid; k < half; k += 256) {
+    float c, s;
+    rotation(pos, a.turns[k], c, s);
+    lds_cs[k] = c * a.amp;
+    lds_cs[half + k] = s * a.amp;
+  }
   __syncthreads();
   T* q = (T*)a.q + t * (long)a.H * a.ldq;
   const int per = a.ldq / V;
   for (int idx = tid; idx < a.H * per; idx += 256) {
     const int h = idx / per, d = (idx % per) * V;
-    const int col = h * (a.dim + a.rot), e0 = d - a.dim;
     float v[V];
-    if (d + V <= a.dim) {
-      fold_parts<TP, V>(a.y, t, col + d, v);
-    } else if (e0 >= 0 && e0 + V <= a.rdims && half % V == 0) {
-      // a piece inside one half: its partners are a piece, too
-      const bool first = e0 < half;
-      float w[V];
-      fold_parts<TP, V>(a.y, t, col + d, v);
-      fold_parts<TP, V>(a.y, t, col + d + (first ? half : -half), w);
-#pragma unroll
-      for (int j = 0; j < V; ++j) {
-        const int k = e0 + j - (first ? 0 : half);
-        const float c = lds_cs[k], s = lds_cs[half + k];
-        v[j] = first ? v[j] * c - w[j] * s : v[j] * c + w[j] * s;
-      }
-    } else {
-#pragma unroll
-      for (int j = 0; j < V; ++j) {
-        const int e = e0 + j;  // may straddle the border
-        v[j] = 0.f;
-        if (e >= a.rot) continue;
-        float x[1], w[1];
-        fold_parts<TP, 1>(a.y, t, col + d + j, x);
-        v[j] = x[0];
-        if (e < 0 || e >= a.rdims) continue;
-        const int k = e % half;
-        fold_parts<TP, 1>(a.y, t, col + a.dim + (e < half ? e + half : k), w);
-        const float c = lds_cs[k], s = lds_cs[half + k];
-        v[j] = e < half ? x[0] * c - w[0] * s : x[0] * c + w[0] * s;
-      }
-    }
+    turned_piece<TP, V>(a.y, t, h * (a.dim + a.rot), d, a.dim + a.rot, a.dim,
+                        a.rdims, lds_cs, v);
     stv<V>(q + (long)h * a.ldq + d, v);
   }
 }
@@ -201,6 +179,8 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentQueryArgs a) {
       fold_parts<TP, 1>(a.y, row, col + a.dim + k, u);
       fold_parts<TP, 1>(a.y, row, col + a.dim + half + k, v);
       rotation(max(a.tok_pos[row], 0), a.turns[k], c, s);
+      c *= a.amp;
+      s *= a.amp;
       unsigned short* o = out + ((long)(m0 + m) * a.H + h) * a.ck + a.rp + k;
       o[0] = cvt_bf(u[0] * c - v[0] * s);
       o[half] = cvt_bf(v[0] * c + u[0] * s);

@@ -1,9 +1,11 @@
 // Routed experts over (token, choice) slots: slot = token * top + choice.
 //
-//   act[.]  = silu(W_gate[e] h) * (W_up[e] h)          one fused launch
+//   act[.]  = glu(W_gate[e] h, W_up[e] h)              one fused launch
 //   y[slot] = wts[slot] * (W_down[e] act)              one launch
 //
-// or act = relu(W_up[e] h)^2, and the weight may multiply h instead: by then
+// with glu(g, u) = g sigmoid(slope g) (u + shift) after g = min(g, limit) and
+// u = clamp(u, -limit, limit): silu(g) * u for an infinite limit, slope 1 and
+// shift 0; or act = relu(W_up[e] h)^2, and the weight may multiply h instead: by then
 // it has passed through the linear map, so the first launch's epilogue applies
 // it ahead of the activation.
 //
@@ -29,6 +31,16 @@
 #include "rows.hip"
 
 static constexpr int MOE_MAX_E = 1024;
+
+struct GluConst {
+  float limit, slope, shift;
+};
+
+DEVINL float gated(const GluConst& c, float g, float u) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit) + c.shift;
+  return g * sigmoid_f(c.slope * g) * u;
+}
 
 // XCD-aware order: consecutive tiles, which share operand rows, on one XCD.
 DEVINL int xcd_order(int id, int n) {
@@ -106,7 +118,7 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
     const unsigned short* __restrict__ A, const unsigned short* __restrict__ W,
     const int* __restrict__ ids, const float* __restrict__ wts,
     unsigned short* __restrict__ C, int S, int top, int N, int K, int lda,
-    int ldc) {
+    int ldc, GluConst glu) {
   constexpr int NW = UP ? UP : 1, U = 4, KSTEP = 256, RS = KSTEP + 8;
   __shared__ __attribute__((aligned(16))) unsigned short at[32 * RS];
   __shared__ int slots[32];
@@ -226,7 +238,7 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
       const int sl = slots[m];
       const float w = wts ? wts[sl] : 1.f;
       float v = acc[0][t][r] * w;
-      if constexpr (UP == 2) v = v * sigmoid_f(v) * (acc[NW - 1][t][r] * w);
+      if constexpr (UP == 2) v = gated(glu, v, acc[NW - 1][t][r] * w);
       if constexpr (UP == 1) v = relu_sq(v);
       C[(long)sl * ldc + n0 + li] = f2bf(v);
     }
@@ -256,7 +268,7 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
     const int* __restrict__ off, const int* __restrict__ sorted,
     const int* __restrict__ tiles, const float* __restrict__ wts,
     unsigned short* __restrict__ C, int max_tiles, int ntn, int top, int N,
-    int K, int lda, int ldc) {
+    int K, int lda, int ldc, GluConst glu) {
   constexpr int BK = 32, RB = BK * 2, BN = 256, HN = BN / 2;
   constexpr int AI = BM * 4 / 256, BI = BN * 4 / 256;  // 16 B pieces per thread
   constexpr int MT = BM / 16, NT = 4;
@@ -356,10 +368,8 @@ __global__ __launch_bounds__(256, BM > 64 ? 2 : 3) void moe_tile_kernel(
         if (col >= N) continue;
         float v[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const float z = acc[m][n][j] * w;
-          v[j] = z * sigmoid_f(z) * (acc[m][n + 2][j] * w);
-        }
+        for (int j = 0; j < 4; ++j)
+          v[j] = gated(glu, acc[m][n][j] * w, acc[m][n + 2][j] * w);
         stv<4>(C + (long)(p0 + r) * ldc + col, v);
       }
     } else {
@@ -388,7 +398,8 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(
     const float* __restrict__ A, const float* __restrict__ W,
     const int* __restrict__ off, const int* __restrict__ sorted,
     const int* __restrict__ tiles, const float* __restrict__ wts,
-    float* __restrict__ C, int top, int N, int K, int lda, int ldc) {
+    float* __restrict__ C, int top, int N, int K, int lda, int ldc,
+    GluConst glu) {
   constexpr int NW = UP ? UP : 1, BK = 16;
   __shared__ float al[BK][64 + 4], wl[NW][BK][64 + 4];
   const int e = tiles[2 * blockIdx.y];
@@ -424,7 +435,7 @@ __global__ __launch_bounds__(256) void moe_simple_kernel(
     const float w = wts ? wts[sl] : 1.f;
     for (int j = 0; j < 4; ++j) {
       float v = acc[0][i][j] * w;
-      if constexpr (UP == 2) v = v * sigmoid_f(v) * (acc[NW - 1][i][j] * w);
+      if constexpr (UP == 2) v = gated(glu, v, acc[NW - 1][i][j] * w);
       if constexpr (UP == 1) v = relu_sq(v);
       C[(long)(UP ? p0 + r : sl) * ldc + n0 + tx * 4 + j] = v;
     }

@@ -5,13 +5,16 @@
 //     weights) into the 32-bit residual and emits the next layer's grouped
 //     RMS norm, in one pass per row. For norms after the sum the residual is
 //     scaled first and the normed row takes its place; for norms around a
-//     sublayer what is pending is normed before it is added.
+//     sublayer what is pending is normed before it is added. Without a norm it
+//     can hand on the sum as it is, beside the row of another matrix.
 // proj_post_kernel — everything between the fused input GEMM and attention:
 //     folds split-K partials, RMS-norms q and k over the whole projection,
 //     writes K/V into the pages, hands on the output gate, applies the
 //     feed-forward activation and routes the token to its experts.
 // head_post_kernel — the same step for projections with biases, a norm per head
 //     and a query temperature, without feed-forward.
+// rope_post_kernel — the same step for projections with rotary positions and one
+//     or several queries and keys per head.
 // ff_post_kernel — feed-forward activation and routing of layers whose
 //     feed-forward has an input of its own.
 // clamped_glu_kernel — bias, clamps, gate and product of a gated feed-forward.
@@ -118,6 +121,47 @@ DEVINL void rotation(int pos, double turns, float& c, float& s) {
   sincospif(2.f * (float)r, &s, &c);
 }
 
+// V consecutive elements d.. of a vector of `size` elements at column col of row
+// t, those from r0 on to r0 + rdims turned, element r0 + k with r0 + rdims / 2 + k;
+// zero from size on. cs: cosines of the pairs, then sines.
+template <typename TP, int V>
+DEVINL void turned_piece(const Parts& y, long t, int col, int d, int size, int r0,
+                         int rdims, const float* cs, float* v) {
+  const int half = rdims / 2, e0 = d - r0;
+  if (d + V <= size && (e0 + V <= 0 || e0 >= rdims)) {
+    fold_parts<TP, V>(y, t, col + d, v);
+    return;
+  }
+  if (e0 >= 0 && e0 + V <= rdims && half % V == 0) {
+    // a piece inside one half: its partners are a piece, too
+    const bool first = e0 < half;
+    float w[V];
+    fold_parts<TP, V>(y, t, col + d, v);
+    fold_parts<TP, V>(y, t, col + d + (first ? half : -half), w);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      const int k = e0 + j - (first ? 0 : half);
+      const float c = cs[k], s = cs[half + k];
+      v[j] = first ? v[j] * c - w[j] * s : v[j] * c + w[j] * s;
+    }
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    const int e = e0 + j;  // may straddle the border
+    v[j] = 0.f;
+    if (d + j >= size) continue;
+    float x[1], w[1];
+    fold_parts<TP, 1>(y, t, col + d + j, x);
+    v[j] = x[0];
+    if (e < 0 || e >= rdims) continue;
+    const int k = e % half;
+    fold_parts<TP, 1>(y, t, col + r0 + (e < half ? e + half : k), w);
+    const float c = cs[k], s = cs[half + k];
+    v[j] = e < half ? x[0] * c - w[0] * s : x[0] * c + w[0] * s;
+  }
+}
+
 DEVINL float sigmoid_f(float z) {
   return __builtin_amdgcn_rcpf(1.f + fast_exp2(-z * LOG2E));
 }
@@ -135,7 +179,7 @@ DEVINL float exp_minus_1_minus(float z) {
 // ---------------------------------------------------------------------------
 
 struct ResidualArgs {
-  float* x;            // (N, W) f32 residual, updated in place
+  float* x;            // (N, W) f32 residual, row stride ldx, updated in place
   const void* parts;   // (ks, N, ldp) pending GEMM output, or null
   long pstride;        // elements between splits
   const void* routed;  // (N, top, ldr) weighted expert outputs, or null
@@ -145,7 +189,9 @@ struct ResidualArgs {
   const float* bias;   // (W,) of the pending GEMM, or null
   const float* bw;     // (W,) norm weight of what is pending; null = no norm
   const float* nw;     // (W,) norm weight; null = fold only
+  const float* other;  // (N, W) f32, row stride ldx2: without nw, h is [x | other]
   void* h;             // (N, ldh) normed row, zero beyond W
+  long ldx, ldx2;
   int W, ks, ldp, top, ldr, ldhp, ldh, groups;
   int post;            // the normed row becomes the residual
   float eps, alpha;    // alpha scales x before the sum
@@ -158,7 +204,7 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
   float* stat = lds_row + ((a.W + 3) & ~3);
   const long t = blockIdx.x;
   const int W = a.W;
-  float* xr = a.x + t * W;
+  float* xr = a.x + t * a.ldx;
   const TP* pr = (const TP*)a.parts + t * a.ldp;
   const T* rr = (const T*)a.routed + t * (long)a.top * a.ldr;
   const T* hp = (const T*)a.hprev + t * (long)a.ldhp;
@@ -248,7 +294,25 @@ __global__ __launch_bounds__(BLOCK) void residual_norm_kernel(ResidualArgs a) {
       for (int j = 0; j < V; ++j) lds_row[i + j] = v[j];
     }
   }
-  if (!a.nw) return;
+  if (!a.nw) {
+    if (!a.other) return;
+    T* hr = (T*)a.h + t * (long)a.ldh;
+    const float* xo = a.other + t * a.ldx2;
+    // a thread reads back what it wrote
+    for (int i = threadIdx.x * V; i < a.ldh; i += BLOCK * V) {
+      float v[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = 0.f;
+      if (i < W) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) v[j] = lds_row[i + j];
+      } else if (i < 2 * W) {
+        ldv<V>(xo + i - W, v);
+      }
+      stv<V>(hr + i, v);
+    }
+    return;
+  }
   __syncthreads();
 
   // sums of squares: every unit (a group, or an even share of one where
@@ -352,12 +416,13 @@ struct EmbedArgs {
   const void* pos_table;   // (max_pos, W) or null: learned positions
   const void* pair_table;  // (buckets + 1, W) or null: rows of token pairs
   const double* turns;     // ((W + 1) / 2,) or null: sines and cosines
-  float* x;                // (N, W)
+  float* x;                // (N, copies * W)
   long buckets, mul_prev, mul_cur;
-  int W, vocab, max_pos;
+  int W, vocab, max_pos, copies;
+  float scale;
 };
 
-// x[n] = table[ids[n]] (+ pos_table[pos[n]]) (+ pair_table[row of the pair])
+// x[n] = scale * table[ids[n]] (+ pos_table[pos[n]]) (+ pair_table[row of the pair])
 // (+ sin at 2i, cos at 2i + 1 of pos[n] * frequency i) in f32; indices are
 // clamped. A token without a predecessor takes the pair table's last row.
 template <typename T>
@@ -376,7 +441,7 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(EmbedArgs a) {
     q = (const T*)a.pair_table + r * W;
   }
   for (int i = threadIdx.x; i < W; i += 256) {
-    float v = ldf(e + i);
+    float v = ldf(e + i) * a.scale;
     if (p) v += ldf(p + i);
     if (q) v += ldf(q + i);
     if (a.turns) {
@@ -384,7 +449,7 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(EmbedArgs a) {
       rotation(max(a.pos[n], 0), a.turns[i / 2], c, s);
       v += i & 1 ? c : s;
     }
-    a.x[n * W + i] = v;
+    for (int c = 0; c < a.copies; ++c) a.x[(n * a.copies + c) * W + i] = v;
   }
 }
 
@@ -402,6 +467,7 @@ struct RouteArgs {
   float* idw;           // (N,) or null
   int ks, ld, off, E, NI, top;
   int sigmoid;          // scores: sigmoid of each logit, else softmax
+  int renorm;           // the chosen scores are divided by their sum
   float scale;
 };
 
@@ -439,7 +505,7 @@ DEVINL void route_row(const RouteArgs& a, long t, float* s, float* ch) {
     ch[i] = s[i] + (a.corr ? a.corr[i] : 0.f);
   }
   // every lane reads and writes its own columns only
-  float idw = 0.f;
+  float idw = 0.f, total = 0.f, mine = 0.f;
   for (int k = 0; k < a.top; ++k) {
     float best = -__builtin_inff();
     int at = n;
@@ -462,10 +528,19 @@ DEVINL void route_row(const RouteArgs& a, long t, float* s, float* ch) {
     }
     w = __shfl(w, at & (WAVE - 1));
     if (at >= a.E) idw += w;
+    total += w;
+    if (lane == k) mine = w;
     if (lane == 0) {
       a.ids[t * a.top + k] = at < a.E ? at : -1;
-      a.wts[t * a.top + k] = w;
+      if (!a.renorm || k >= WAVE) a.wts[t * a.top + k] = w;
     }
+  }
+  if (a.renorm) {
+    const float f = a.scale / total;
+    idw *= f;
+    if (lane < a.top) a.wts[t * a.top + lane] = mine * f;
+    if (lane == 0)
+      for (int k = WAVE; k < a.top; ++k) a.wts[t * a.top + k] *= f;
   }
   if (lane == 0 && a.idw) a.idw[t] = idw;
 }
@@ -711,6 +786,77 @@ __global__ __launch_bounds__(256) void head_post_kernel(HeadPostArgs a) {
       for (int j = 0; j < V; ++j) v[j] = row[i + j] * f * w[j];
     }
     stv<V>(o + i, v);
+  }
+}
+
+struct RopePostArgs {
+  Parts y;              // q, k, v columns
+  const double* turns;  // (rdims / 2,)
+  void* q;              // (N, H, M, dk)
+  void* kp;             // (np, G, P, M * dk)
+  void* vp;             // (np, G, dvp, P)
+  const int* table;     // (S, maxp)
+  const int* tok_seq;
+  const int* tok_pos;
+  int q_off, k_off, v_off, H, G, M, dim, vdim, rdims, dk, dvp, P, maxp;
+  int per;              // units of a workgroup
+  float amp;            // factor of cosine and sine
+};
+
+// grid (N, units / per); units are the H M queries, G M keys and G values of a
+// row. LDS: cosine and sine of every pair.
+template <typename TP, typename T, int V>
+__global__ __launch_bounds__(256) void rope_post_kernel(RopePostArgs a) {
+  extern __shared__ float lds_cs[];
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, half = a.rdims / 2, pos = a.tok_pos[t];
+  for (int k = tid; k < half; k += 256) {
+    float c, s;
+    rotation(max(pos, 0), a.turns[k], c, s);
+    lds_cs[k] = c * a.amp;
+    lds_cs[half + k] = s * a.amp;
+  }
+  __syncthreads();
+  const int nq = a.H * a.M, nk = a.G * a.M;
+  const int u0 = blockIdx.y * a.per, u1 = min(u0 + a.per, nq + nk + a.G);
+  long page = 0;
+  int slot = 0;
+  if (pos >= 0) {
+    page = a.table[(long)a.tok_seq[t] * a.maxp + pos / a.P];
+    slot = pos % a.P;
+  }
+  const int pieces = max(a.dk, a.dvp) / V;
+  for (int idx = tid; idx < (u1 - u0) * pieces; idx += 256) {
+    const int u = u0 + idx / pieces, d = idx % pieces * V;
+    if (u >= nq && pos < 0) break;   // an empty slot writes no K/V
+    float v[V];
+    if (u >= nq + nk) {
+      if (d >= a.dvp) continue;
+      const int g = u - nq - nk;
+#pragma unroll
+      for (int j = 0; j < V; ++j) v[j] = 0.f;
+      if (d + V <= a.vdim) {
+        fold_parts<TP, V>(a.y, t, a.v_off + g * a.vdim + d, v);
+      } else {
+#pragma unroll
+        for (int j = 0; j < V; ++j)
+          if (d + j < a.vdim)
+            fold_parts<TP, 1>(a.y, t, a.v_off + g * a.vdim + d + j, v + j);
+      }
+      T* vp = (T*)a.vp + ((page * a.G + g) * a.dvp + d) * (long)a.P + slot;
+#pragma unroll
+      for (int j = 0; j < V; ++j) stf(vp + j * a.P, v[j]);
+      continue;
+    }
+    if (d >= a.dk) continue;
+    const bool is_q = u < nq;
+    const int i = is_q ? u : u - nq;
+    turned_piece<TP, V>(a.y, t, (is_q ? a.q_off : a.k_off) + i * a.dim, d, a.dim, 0,
+                        a.rdims, lds_cs, v);
+    T* o = is_q ? (T*)a.q + (t * nq + i) * a.dk
+                : (T*)a.kp + ((page * a.G + i / a.M) * a.P + slot) * (long)(a.M * a.dk) +
+                      i % a.M * a.dk;
+    stv<V>(o + d, v);
   }
 }
 

@@ -1,17 +1,20 @@
 """Token mixers over ragged batches beside plain attention (ops/ragged.py):
-latent attention and gated linear attention.
+latent attention, differential attention, gated linear attention, and gated linear
+attention whose forget gate also decides what is written.
 
-Both take the output of a layer's fused input GEMM (parts, as linear_parts
-returns it) and give the gated mixer output, the input of the layer's output
-GEMM. Single tokens and portions of prompts of one step take different kernels
-and fill different rows of one result.
+They take the output of a layer's fused input GEMM (parts, as linear_parts
+returns it) and give the mixer output, the input of the layer's output GEMM.
+Single tokens and portions of prompts of one step take different kernels and fill
+different rows of one result.
 
-Device tensors run the _hip_mixers and _hip_ragged extensions and fail loudly
-without them; CPU tensors run the forms in ops/reference.py.
+Device tensors run the _hip_mixers, _hip_differential, _hip_hgrn and _hip_ragged
+extensions and fail loudly without them; CPU tensors run the forms in
+ops/reference.py.
 """
 from __future__ import annotations
 
 import importlib
+import math
 from dataclasses import dataclass
 from typing import Optional, Tuple
 
@@ -20,28 +23,75 @@ import torch.nn.functional as F
 
 from bloombee_amd.ops import ragged
 from bloombee_amd.ops import reference as ref
-from bloombee_amd.ops.ragged import pad_head, round_up
+from bloombee_amd.ops.ragged import RopeSpec, pad_head, round_up
 
-_hip_mixers = None   # loaded by the first device call
+_loaded = {}   # extension modules, by the first device call of each
 
 
-def _ext():
-    global _hip_mixers
-    if _hip_mixers is None:
+def _ext(name: str = "_hip_mixers"):
+    if name not in _loaded:
         try:
-            _hip_mixers = importlib.import_module("bloombee_amd.ops._hip_mixers")
+            _loaded[name] = importlib.import_module(f"bloombee_amd.ops.{name}")
         except ImportError as e:
             raise RuntimeError(
-                "the _hip_mixers extension is not built but a tensor is on "
+                f"the {name} extension is not built but a tensor is on "
                 "GPU. Run `python setup.py hip` (PYTORCH_ROCM_ARCH=gfx950). "
                 f"Import error was: {e}") from e
-    return _hip_mixers
+    return _loaded[name]
 
 
 def _mixed(out_cols: int, used: int, n: int, dtype, device) -> torch.Tensor:
     """Result of a mixer: kernels write `used` columns, the rest is zero."""
     make = torch.empty if out_cols == used else torch.zeros
     return make(n, out_cols, dtype=dtype, device=device)
+
+
+# ---------------------------------------------------------------------------
+# rotations
+# ---------------------------------------------------------------------------
+
+def _frequencies(base: float, dims: int) -> torch.Tensor:
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    return torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
+
+
+def rotary_turns(base: float, dims: int) -> torch.Tensor:
+    """Frequencies base^(-2 i / dims) over 2 pi, float64: turns per position."""
+    return _frequencies(base, dims) / (2 * torch.pi)
+
+
+def banded_turns(base: float, dims: int, factor: float, low: float, high: float,
+                 original: float) -> torch.Tensor:
+    """rotary_turns stretched by wavelength (reference.banded_frequencies)."""
+    return ref.banded_frequencies(_frequencies(base, dims), factor, low, high,
+                                  original) / (2 * torch.pi)
+
+
+def yarn_turns(base: float, dims: int, factor: float, original: float,
+               fast: float, slow: float) -> Tuple[torch.Tensor, float]:
+    """rotary_turns stretched pair by pair (YaRN): pairs that turn more than
+    `fast` times over the original context keep their frequency, those that turn
+    less than `slow` times have it divided by factor, a linear ramp between. Also
+    the factor of cosine and sine that goes with it."""
+    def pair(turns: float) -> float:
+        return (dims * math.log(original / (2 * math.pi * turns))
+                / (2 * math.log(base)))
+
+    lo = max(math.floor(pair(fast)), 0)
+    hi = min(math.ceil(pair(slow)), dims - 1)
+    f = _frequencies(base, dims)
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    f = f / factor * ramp + f * (1 - ramp)
+    return f / (2 * torch.pi), 0.1 * math.log(factor) + 1
+
+
+def half_order(dims: int, size: int) -> torch.Tensor:
+    """The kernels turn element i with element i + dims / 2. Rows of a projection
+    whose elements 2 i and 2 i + 1 turn together, taken in this order, do the same
+    as they are: a score does not notice an order that queries and keys share."""
+    i = torch.arange(size)
+    return torch.cat([i[0:dims:2], i[1:dims:2], i[dims:]])
 
 
 # ---------------------------------------------------------------------------
@@ -84,6 +134,7 @@ class LatentSpec:
     g_off: int = 0
     out_cols: int = 0   # inner size of the output projection
     q_cols: int = 0     # inner size of the query projection
+    amp: float = 1.0    # factor of cosine and sine
 
     @property
     def has_kv(self) -> bool:
@@ -104,13 +155,6 @@ class LatentSpec:
         """The MFMA kernels take these sizes."""
         return (self.rank <= LATENT_SIZES[-1] and self.rot <= ROTATED_SIZES[-1]
                 and self.dim + self.rot <= 256 and self.vdim <= 256)
-
-
-def rotary_turns(base: float, dims: int) -> torch.Tensor:
-    """Frequencies base^(-2 i / dims) over 2 pi, float64: turns per position."""
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    return torch.pow(torch.tensor(base, dtype=torch.float64),
-                     -2.0 * i / dims) / (2 * torch.pi)
 
 
 @dataclass
@@ -137,7 +181,7 @@ def latent_post(parts: torch.Tensor, spec: LatentSpec, q_norm: torch.Tensor,
                 else torch.empty(N, gn, dtype=dtype, device=dev))
         _ext().latent_post(
             parts, [s.q_off, s.c_off, s.g_off, s.q_rank, s.rank, s.rot,
-                    s.rot_dims, s.rp, gn, int(s.has_kv)], s.eps, q_norm,
+                    s.rot_dims, s.rp, gn, int(s.has_kv)], s.eps, s.amp, q_norm,
             c_norm, turns, cq, None if in_place else gate, pages,
             batch.page_table, batch.tok_seq, batch.tok_pos)
         return cq, gate
@@ -146,7 +190,7 @@ def latent_post(parts: torch.Tensor, spec: LatentSpec, q_norm: torch.Tensor,
     if s.has_kv:
         c = ref.grouped_rms_norm(y[:, s.c_off:s.c_off + s.rank], c_norm, 1, s.eps)
         at = s.c_off + s.rank
-        r = ref.rotate_half(y[:, at:at + s.rot], batch.tok_pos, turns)
+        r = ref.rotate_half(y[:, at:at + s.rot], batch.tok_pos, turns, s.amp)
         P = pages.shape[2]
         live = (batch.tok_pos >= 0).nonzero()[:, 0]
         pos = batch.tok_pos[live].long()
@@ -166,11 +210,11 @@ def _absorbed(parts: torch.Tensor, spec: LatentSpec, w: LatentWeights,
     if parts.is_cuda:
         q = torch.empty(N, H, s.dim + s.rot, dtype=dtype, device=parts.device)
         _ext().latent_rope(parts, turns, batch.tok_pos, s.dim, s.rot,
-                           s.rot_dims, q)
+                           s.rot_dims, s.amp, q)
     else:
         y = parts.float().sum(0)[:, :H * (s.dim + s.rot)].view(N, H, -1)
         q = torch.cat([y[..., :s.dim], ref.rotate_half(
-            y[..., s.dim:], batch.tok_pos, turns)], -1).to(dtype)
+            y[..., s.dim:], batch.tok_pos, turns, s.amp)], -1).to(dtype)
     qn = q[..., :s.dim].transpose(0, 1).contiguous()
     lat = torch.bmm(qn, w.uk[:, :, :s.dim].transpose(1, 2).contiguous())
     ql = torch.zeros(N, H, s.ck, dtype=dtype, device=q.device)
@@ -203,8 +247,8 @@ def latent_attention(parts: torch.Tensor, spec: LatentSpec, w: LatentWeights,
     if batch.dec_list.numel():
         _ext().latent_decode(
             parts, turns, pages, batch.page_table, batch.tok_pos, batch.cu,
-            batch.q_start, batch.dec_list, batch.max_ctx, s.dim, s.rot, s.rot_dims, s.vdim,
-            s.scale, s.window, w.uk, w.uv, w.sink, gate, out)
+            batch.q_start, batch.dec_list, batch.max_ctx, s.dim, s.rot, s.rot_dims,
+            s.amp, s.vdim, s.scale, s.window, w.uk, w.uv, w.sink, gate, out)
     if batch.pre_list.numel():
         ctx = batch.context(s.window)
         n, P = ctx.pages.numel(), pages.shape[2]
@@ -217,10 +261,53 @@ def latent_attention(parts: torch.Tensor, spec: LatentSpec, w: LatentWeights,
                               k, v)
         q = torch.empty(N, H, dk, dtype=dtype, device=out.device)
         _ext().latent_rope(parts, turns, batch.tok_pos, s.dim, s.rot,
-                           s.rot_dims, q)
+                           s.rot_dims, s.amp, q)
         ragged.attn_ragged(q, k, v, batch, out, s.dim + s.rot, s.vdim, s.scale,
                            s.window, gate=gate, sinks=w.sink, table=ctx.table,
                            portions_only=True)
+    return out
+
+
+# ---------------------------------------------------------------------------
+# differential attention
+# ---------------------------------------------------------------------------
+
+@dataclass
+class DiffSpec:
+    """Two attentions per head over the same values and how they combine:
+    rms(a1 - lam a2) factor, the norm over the head's values and without a
+    weight. A key's two maps lie one after the other in its page slot."""
+    rope: RopeSpec
+    scale: float
+    lam: float
+    factor: float
+    eps: float
+    window: int = 0       # 0 = none
+    chunk: int = 0
+    out_cols: int = 0     # inner size of the output projection
+
+
+def differential_attention(parts: torch.Tensor, spec: DiffSpec,
+                           turns: torch.Tensor, batch, k_pages: torch.Tensor,
+                           v_pages: torch.Tensor,
+                           dtype: torch.dtype) -> torch.Tensor:
+    """(N, out_cols) from the input GEMM's parts; keys and values go to the
+    pages."""
+    s, r = spec, spec.rope
+    N = parts.shape[1]
+    q = ragged.rope_post(parts, r, turns, batch, k_pages, v_pages, dtype)
+    used = r.heads * r.vdim
+    out = _mixed(s.out_cols, used, N, dtype, parts.device)
+    if parts.is_cuda:
+        _ext("_hip_differential").attn_differential(
+            q, k_pages, v_pages, batch.page_table, batch.tok_seq, batch.tok_pos,
+            batch.cu, batch.q_start, batch.pre_list, batch.dec_list, batch.max_new,
+            batch.max_ctx, r.dim, r.vdim, s.scale, s.window, s.chunk, s.lam,
+            s.factor, s.eps, out)
+        return out
+    out[:, :used] = ref.attn_differential(q, k_pages, v_pages, batch, r.dim,
+                                          r.vdim, s.scale, s.lam, s.factor, s.eps,
+                                          s.window, s.chunk)
     return out
 
 
@@ -286,7 +373,16 @@ def gla_mix(parts: torch.Tensor, aparts: torch.Tensor, a0: int, spec: GlaSpec,
     r = a2.shape[0]
     alpha = ref.channel_decays(aparts.sum(0)[:, a0:a0 + r], a2, a2_b,
                                s.tau).view(N, H, s.dim)
-    o = torch.zeros(N, H, s.vdim)
+    o = _scan_sequences(q, k, v, alpha, state, batch)
+    o = ref.grouped_rms_norm(o, norm, 1, s.eps).reshape(N, H * s.vdim)
+    g = y[:, s.g_off:s.g_off + H * s.vdim]
+    out[:, :H * s.vdim] = (o * F.silu(g)).to(dtype)
+    return out
+
+
+def _scan_sequences(q, k, v, alpha, state, batch) -> torch.Tensor:
+    """reference.gla_scan of every sequence of a step, states in place."""
+    o = torch.zeros(*q.shape[:2], v.shape[-1])
     for i, (a, b) in enumerate(zip(batch.cu[:-1].tolist(), batch.cu[1:].tolist())):
         if int(batch.tok_pos[a]) < 0:
             continue
@@ -294,7 +390,67 @@ def gla_mix(parts: torch.Tensor, aparts: torch.Tensor, a0: int, spec: GlaSpec,
         S = state[slot] if int(batch.q_start[i]) > 0 else \
             torch.zeros_like(state[slot])
         o[a:b], state[slot] = ref.gla_scan(q[a:b], k[a:b], v[a:b], alpha[a:b], S)
-    o = ref.grouped_rms_norm(o, norm, 1, s.eps).reshape(N, H * s.vdim)
-    g = y[:, s.g_off:s.g_off + H * s.vdim]
-    out[:, :H * s.vdim] = (o * F.silu(g)).to(dtype)
+    return o
+
+
+# ---------------------------------------------------------------------------
+# gated linear attention that writes what it forgets (HGRN2)
+# ---------------------------------------------------------------------------
+
+@dataclass
+class HgrnSpec:
+    """Sizes of the layer and the columns of its input projection. The forget
+    gate's logits are last and computed in f32 (input_projection's router
+    section)."""
+    heads: int
+    dim: int
+    vdim: int
+    eps: float
+    q_off: int = 0
+    v_off: int = 0
+    router_off: int = -1
+    router_n: int = 0     # heads * dim
+    out_cols: int = 0
+
+
+def hgrn_mix(parts: torch.Tensor, fparts: torch.Tensor, f0: int, spec: HgrnSpec,
+             f_b: torch.Tensor, lower: torch.Tensor, norm: torch.Tensor,
+             state: torch.Tensor, batch, dtype: torch.dtype) -> torch.Tensor:
+    """(N, out_cols) of a step, states updated in place. Per head
+    S <- diag(f) S + (1 - f) v^T, o = S^T silu(q), normed over vdim, with
+    f = lower + (1 - lower) sigmoid(z + f_b). fparts (splits, N, >= f0 + heads *
+    dim) f32: z from column f0 on; f_b, lower (heads * dim,) f32."""
+    s = spec
+    N, H, n = parts.shape[1], s.heads, s.heads * s.dim
+    out = _mixed(s.out_cols, H * s.vdim, N, dtype, parts.device)
+    dims = [s.q_off, s.v_off, f0, H, s.dim, s.vdim]
+    if parts.is_cuda:
+        ext = _ext("_hip_hgrn")
+        steps = [batch.dec_list]
+        if batch.pre_list.numel():
+            C = ext.hgrn_chunk(s.dim, s.vdim) if dtype == torch.bfloat16 else 0
+            if C:
+                ch = batch.chunks(C)
+                y = (parts[0] if parts.shape[0] == 1 and parts.dtype == dtype
+                     else parts.sum(0).to(dtype))
+                z = fparts[0] if fparts.shape[0] == 1 else fparts.sum(0)
+                ext.hgrn_chunks(y, z, dims, s.eps, f_b, lower, norm, state,
+                                batch.slots, batch.q_start, batch.pre_list,
+                                ch.row0, ch.len, ch.cu, out)
+            else:
+                steps.append(batch.pre_list)
+        for seqs in steps:
+            if seqs.numel():
+                ext.hgrn_step(parts, fparts, dims, s.eps, f_b, lower, norm,
+                              state, batch.slots, batch.tok_pos, batch.cu, seqs,
+                              out)
+        return out
+    y = parts.float().sum(0)
+    f, k = ref.forget_gates(fparts.sum(0)[:, f0:f0 + n], f_b, lower)
+    head = lambda t: t.reshape(N, H, -1)
+    o = _scan_sequences(head(F.silu(y[:, s.q_off:s.q_off + n])), head(k),
+                        head(y[:, s.v_off:s.v_off + H * s.vdim]), head(f), state,
+                        batch)
+    o = ref.grouped_rms_norm(o, norm, 1, s.eps)
+    out[:, :H * s.vdim] = o.reshape(N, H * s.vdim).to(dtype)
     return out

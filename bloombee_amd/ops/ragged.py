@@ -14,8 +14,10 @@ token):
 Layers with a norm after every sum use sum_norm instead, and clamped_glu for
 their feed-forward. Layers with a norm around every sublayer leave sums Pending
 with the norm they pass first; where attention and feed-forward have inputs of
-their own, head_post and ff_post take proj_post's place. Other mixers are in
-ops/mixers.py and ops/recurrent.py.
+their own, head_post (norms per head) or rope_post (rotations) and ff_post take
+proj_post's place. join_rows lets a product read the residual beside other rows
+and put its result in the residual's place. Other mixers are in ops/mixers.py and
+ops/recurrent.py.
 
 Device tensors run the _hip_ragged extension and fail loudly without it; CPU
 tensors run the forms in ops/reference.py. Activations are bf16 or f32; the
@@ -38,6 +40,7 @@ _hip_ragged = None   # loaded by the first device call
 # padded to the next one with zeros
 HEAD_SIZES = (32, 64, 128, 256)
 SKINNY_ROWS = 32   # up to here a GEMM is a weight stream (split-K kernel)
+ROUTER_COLS = 1024   # beyond, the vendor GEMM makes 32-bit columns, too
 
 
 def _ext():
@@ -83,13 +86,16 @@ class Routing:
 class Pending:
     """What a layer still owes the residual: the output GEMM's partials and,
     for routed layers, the experts' rows and the layer's own input; with norm,
-    all of it is RMS-normed with these weights first."""
+    all of it is RMS-normed with these weights first. The residual is scaled by
+    keep before it is added: 0 puts the sum in its place."""
     parts: Optional[torch.Tensor]            # (ks, N, >= W)
     routed: Optional[torch.Tensor] = None    # (N, top, >= W)
     routing: Optional[Routing] = None
     h: Optional[torch.Tensor] = None         # (N, >= W)
     norm: Optional[torch.Tensor] = None      # (W,) f32
     eps: float = 0.0                         # of that norm
+    bias: Optional[torch.Tensor] = None      # (W,) f32, added to parts
+    keep: float = 1.0
 
     def settle(self, x: torch.Tensor) -> None:
         residual_norm(x, self, eps=self.eps)
@@ -110,9 +116,9 @@ def residual_norm(x: torch.Tensor, pending: Optional[Pending],
                   eps: float = 1e-5, cols: int = 0,
                   dtype: torch.dtype = torch.bfloat16,
                   ) -> Optional[torch.Tensor]:
-    """x (N, W) f32 += pending, in place; returns norm(x) as (N, cols) in
-    dtype with zero columns beyond W, or None without a weight. eps is that of
-    the pending sum's own norm, too, if it has one."""
+    """x (N, W) f32 += pending, in place (rows may lie apart); returns norm(x) as
+    (N, cols) in dtype with zero columns beyond W, or None without a weight. eps
+    is that of the pending sum's own norm, too, if it has one."""
     N, W = x.shape
     p = pending
     rt = p.routing if p is not None else None
@@ -124,22 +130,46 @@ def residual_norm(x: torch.Tensor, pending: Optional[Pending],
             x, p.parts if p else None,
             p.routed if p and p.routed is not None else None,
             rt.ids if rt else None, idw, p.h if idw is not None else None,
-            weight, groups, eps, h, 1.0, None, False, p.norm if p else None)
+            weight, groups, eps, h, p.keep if p else 1.0, p.bias if p else None,
+            False, p.norm if p else None, None)
         return h
     if p is not None:
         d = (p.parts.float().sum(0)[:, :W] if p.parts is not None
              else torch.zeros_like(x))
+        if p.bias is not None:
+            d = d + p.bias
         if p.routed is not None:
             d = d + p.routed.float().sum(1)[:, :W]
         if idw is not None:
             d = d + idw[:, None] * p.h[:, :W].float()
         if p.norm is not None:
             d = ref.grouped_rms_norm(d, p.norm, 1, eps)
-        x += d
+        x.mul_(p.keep).add_(d)
     if weight is None:
         return None
     y = ref.grouped_rms_norm(x, weight, groups, eps).to(dtype)
     return F.pad(y, (0, (cols or W) - W))
+
+
+def join_rows(x: torch.Tensor, pending: Optional[Pending],
+              other: torch.Tensor, cols: int, dtype: torch.dtype) -> torch.Tensor:
+    """x (N, W) f32 += pending, in place; returns [x | other] as (N, cols) in
+    dtype with zero columns beyond 2 W. other (N, W) f32; the rows of both may lie
+    apart."""
+    p = pending
+    if x.is_cuda:
+        rt = p.routing if p is not None else None
+        idw = rt.idw if rt is not None else None
+        h = torch.empty(x.shape[0], cols, dtype=dtype, device=x.device)
+        _ext().residual_norm(
+            x, p.parts if p else None, p.routed if p else None,
+            rt.ids if rt else None, idw, p.h if idw is not None else None, None,
+            1, p.eps if p else 0.0, h, p.keep if p else 1.0,
+            p.bias if p else None, False, p.norm if p else None, other)
+        return h
+    if p is not None:
+        p.settle(x)
+    return input_rows(torch.cat([x, other], 1), cols, dtype)
 
 
 def sum_norm(x: torch.Tensor, parts: torch.Tensor,
@@ -152,7 +182,7 @@ def sum_norm(x: torch.Tensor, parts: torch.Tensor,
     if x.is_cuda:
         h = torch.empty(N, cols, dtype=dtype, device=x.device)
         _ext().residual_norm(x, parts, None, None, None, None, weight, 1, eps,
-                             h, alpha, bias, True, None)
+                             h, alpha, bias, True, None, None)
         return h
     y = alpha * x + parts.float().sum(0)[:, :W]
     if bias is not None:
@@ -230,18 +260,20 @@ def embed_rows(ids: torch.Tensor, positions: torch.Tensor,
                table: torch.Tensor, pos_table: Optional[torch.Tensor],
                prev: Optional[torch.Tensor] = None,
                pairs: Optional[PairTable] = None,
-               turns: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """table[ids] (+ pos_table[positions]) (+ the row of each token and its
-    predecessor) (+ sinusoidal positions) in f32, (..., W)."""
+               turns: Optional[torch.Tensor] = None, scale: float = 1.0,
+               copies: int = 1) -> torch.Tensor:
+    """scale * table[ids] (+ pos_table[positions]) (+ the row of each token and
+    its predecessor) (+ sinusoidal positions) in f32, `copies` times side by side:
+    (..., copies * W)."""
     if table.is_cuda:
         x = _ext().embed_rows(
             ids.reshape(-1).int(), positions.reshape(-1).int(), table, pos_table,
             prev.reshape(-1).int() if pairs is not None else None,
             pairs.table if pairs is not None else None,
             [pairs.buckets, pairs.mul_prev, pairs.mul_cur]
-            if pairs is not None else [], turns)
+            if pairs is not None else [], turns, scale, copies)
         return x.view(*ids.shape, -1)
-    x = F.embedding(ids.long(), table).float()
+    x = F.embedding(ids.long(), table).float() * scale
     pos = positions.long().clamp(min=0)
     if pos_table is not None:
         x = x + F.embedding(pos, pos_table).float()
@@ -249,7 +281,7 @@ def embed_rows(ids: torch.Tensor, positions: torch.Tensor,
         x = x + F.embedding(pairs.rows(ids, prev), pairs.table).float()
     if turns is not None:
         x = x + ref.sinusoid(pos, turns, table.shape[1])
-    return x
+    return x if copies == 1 else torch.cat([x] * copies, -1)
 
 
 def linear_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -259,6 +291,14 @@ def linear_parts(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     if (x.is_cuda and x.dtype == torch.bfloat16 and x.shape[0] <= SKINNY_ROWS):
         return _ext().gemm_parts(x, w, 0)
     return F.linear(x, w).unsqueeze(0)
+
+
+def linear_sums(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """linear_parts with 32-bit sums for any number of rows: for what takes the
+    residual's place."""
+    if x.is_cuda and x.dtype == torch.bfloat16 and x.shape[0] > SKINNY_ROWS:
+        return torch.mm(x, w.t(), out_dtype=torch.float32).unsqueeze(0)
+    return linear_parts(x, w)
 
 
 def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
@@ -311,6 +351,16 @@ class ProjSpec:
         return self.experts + self.identity > 0
 
 
+def router_logits(h: torch.Tensor, w: torch.Tensor, n: int) -> torch.Tensor:
+    """h (N, K) @ the first n rows of w (rows, K)^T in f32: (splits, N, >= n)."""
+    if not h.is_cuda:
+        return F.linear(h.float(), w[:n].float()).unsqueeze(0)
+    if h.dtype == torch.bfloat16 and h.shape[0] > SKINNY_ROWS:
+        return (linear_sums(h, w[:n]) if n > ROUTER_COLS
+                else _ext().router_gemm(h, w[:n]))
+    return linear_parts(h, w)      # f32 either way
+
+
 def input_projection(h: torch.Tensor, w: torch.Tensor, spec,
                      ) -> Tuple[torch.Tensor, Optional[torch.Tensor], int]:
     """(parts, router parts, first router column in them). The router's columns
@@ -318,13 +368,9 @@ def input_projection(h: torch.Tensor, w: torch.Tensor, spec,
     r = spec.router_off
     if r < 0:
         return linear_parts(h, w), None, 0
-    if h.is_cuda and h.dtype == torch.bfloat16 and h.shape[0] > SKINNY_ROWS:
+    if not h.is_cuda or (h.dtype == torch.bfloat16 and h.shape[0] > SKINNY_ROWS):
         return (F.linear(h, w[:r]).unsqueeze(0),
-                _ext().router_gemm(h, w[r:r + spec.router_n]), 0)
-    if not h.is_cuda:
-        return (F.linear(h, w[:r]).unsqueeze(0),
-                F.linear(h.float(), w[r:r + spec.router_n].float()).unsqueeze(0),
-                0)
+                router_logits(h, w[r:], spec.router_n), 0)
     parts = linear_parts(h, w)      # f32 either way
     return parts, parts, r
 
@@ -455,6 +501,61 @@ def head_post(parts: torch.Tensor, spec: HeadSpec, biases, q_norm: torch.Tensor,
 
 
 @dataclass
+class RopeSpec:
+    """A q, k, v projection whose queries and keys turn: every head has `maps`
+    queries (and keys) of dim elements, of each of which the first rot_dims are
+    rotated, element i with element i + rot_dims / 2."""
+    heads: int
+    kv_heads: int
+    maps: int
+    dim: int
+    vdim: int
+    rot_dims: int
+    q_off: int = 0
+    k_off: int = 0
+    v_off: int = 0
+    amp: float = 1.0      # factor of cosine and sine
+
+    @property
+    def dk(self) -> int:
+        """Stored size of one query or key."""
+        return pad_head(self.dim)
+
+
+def rope_post(parts: torch.Tensor, spec: RopeSpec, turns: torch.Tensor, batch,
+              k_pages: torch.Tensor, v_pages: torch.Tensor,
+              dtype: torch.dtype) -> torch.Tensor:
+    """Rotated queries (N, H, maps, dk); keys, the maps of a head one after the
+    other, and values go to the pages. turns (rot_dims / 2,) f64."""
+    s = spec
+    _, N, _ = parts.shape
+    H, G, M, D, V = s.heads, s.kv_heads, s.maps, s.dim, s.vdim
+    if parts.is_cuda:
+        q = torch.empty(N, H, M, s.dk, dtype=dtype, device=parts.device)
+        _ext().rope_post(
+            parts, [s.q_off, s.k_off, s.v_off, H, G, M, D, V, s.rot_dims], s.amp,
+            turns, q, k_pages, v_pages, batch.page_table, batch.tok_seq,
+            batch.tok_pos)
+        return q
+    y = parts.float().sum(0)
+
+    def heads(off, n):
+        t = y[:, off:off + n * M * D].reshape(N, n, M, D)
+        return F.pad(ref.rotate_half(t, batch.tok_pos, turns, s.amp),
+                     (0, s.dk - D)).to(dtype)
+
+    k = heads(s.k_off, G).view(N, G, M * s.dk)
+    v = y[:, s.v_off:s.v_off + G * V].reshape(N, G, V).to(dtype)
+    P = k_pages.shape[2]
+    live = (batch.tok_pos >= 0).nonzero()[:, 0]
+    pos = batch.tok_pos[live].long()
+    page = batch.page_table[batch.tok_seq[live].long(), pos // P].long()
+    k_pages[page, :, pos % P] = k[live]
+    v_pages[page, :, :V, pos % P] = v[live]
+    return heads(s.q_off, H)
+
+
+@dataclass
 class FfSpec:
     """A feed-forward's input projection: dense columns (one activation), then
     the router's, which start a 64-row block."""
@@ -467,6 +568,7 @@ class FfSpec:
     router_n: int = 0
     top: int = 0
     sigmoid: bool = False    # scores: sigmoid, else softmax
+    renorm: bool = False     # the chosen weights sum to scale
     scale: float = 1.0
 
 
@@ -485,7 +587,8 @@ def ff_post(parts: Optional[torch.Tensor], rparts: Optional[torch.Tensor],
         first = s.gate_off if s.act == 1 else s.up_off
         _ext().ff_post(
             parts if s.act else None, rparts if E else None,
-            [s.act, first, s.up_off, s.ff, r0, E, 0, s.top, int(s.sigmoid)],
+            [s.act, first, s.up_off, s.ff, r0, E, 0, s.top, int(s.sigmoid),
+             int(s.renorm)],
             s.scale, correction, out, rt.ids if rt else None,
             rt.wts if rt else None, None)
         return out, rt
@@ -499,20 +602,43 @@ def ff_post(parts: Optional[torch.Tensor], rparts: Optional[torch.Tensor],
     rt = None
     if E:
         ids, wts, _ = ref.route_topk(rparts.sum(0)[:, r0:r0 + E], correction, E,
-                                     s.top, s.scale, s.sigmoid)
+                                     s.top, s.scale, s.sigmoid, s.renorm)
         rt = Routing(ids, wts, None)
     return out, rt
 
 
+def route(h: torch.Tensor, w: torch.Tensor, spec: FfSpec) -> Routing:
+    """Experts of feed-forwards without dense columns: w (rows, K), the router's
+    rows first."""
+    return ff_post(None, router_logits(h, w, spec.router_n), 0, spec, None,
+                   h.shape[0], h.device, h.dtype)[1]
+
+
+@dataclass
+class GluSpec:
+    """Activation of gated experts: g sigmoid(slope g) (u + shift) with
+    g = min(gate, limit) and u = clamp(up, -limit, limit). silu(gate) * up as it
+    stands."""
+    limit: float = float("inf")
+    slope: float = 1.0
+    shift: float = 0.0
+
+
+SILU = GluSpec()
+
+
 def moe_experts(h: torch.Tensor, up: torch.Tensor, down: torch.Tensor,
-                rt: Routing, weight_input: bool = False) -> torch.Tensor:
+                rt: Routing, weight_input: bool = False,
+                act: GluSpec = SILU) -> torch.Tensor:
     """(N, top, W) weighted outputs of the chosen experts; the rows of
-    identity choices are not defined. up (E, 2, F, K): silu(gate) * up, or
-    (E, 1, F, K): relu(up)^2; down (E, W, F); K, F and W padded to 64. The
+    identity choices are not defined. up (E, 2, F, K): the gated activation act,
+    or (E, 1, F, K): relu(up)^2; down (E, W, F); K, F and W padded to 64. The
     weight multiplies an expert's output, or its input."""
+    consts = (act.limit, act.slope, act.shift)
     if h.is_cuda:
-        return _ext().moe_experts(h, up, down, rt.ids, rt.wts, weight_input)
-    return ref.moe_experts(h, up, down, rt.ids, rt.wts, weight_input)
+        return _ext().moe_experts(h, up, down, rt.ids, rt.wts, weight_input,
+                                  *consts)
+    return ref.moe_experts(h, up, down, rt.ids, rt.wts, weight_input, *consts)
 
 
 def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor,
@@ -522,9 +648,10 @@ def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor,
                 gate: Optional[torch.Tensor] = None,
                 sinks: Optional[torch.Tensor] = None,
                 table: Optional[torch.Tensor] = None,
-                portions_only: bool = False) -> None:
+                portions_only: bool = False, chunk: int = 0) -> None:
     """Attention of a ragged batch into out[:, :H*vdim] (see
-    reference.attn_ragged). Without v_pages the values are the first vdim
+    reference.attn_ragged): a window of the last keys, or a chunk of the positions
+    counted from the sequence's start (0 = none). Without v_pages the values are the first vdim
     elements of the keys. table: page table of pages that are not the
     cache's; portions_only leaves the rows of single tokens alone (where the
     sizes are those of the tiled kernels)."""
@@ -534,8 +661,8 @@ def attn_ragged(q: torch.Tensor, k_pages: torch.Tensor,
         _ext().attn_ragged(
             q, k_pages, v_pages, table, batch.tok_seq, batch.tok_pos, batch.cu,
             batch.q_start, batch.pre_list, dec, batch.max_new, batch.max_ctx,
-            dim, vdim, scale, window, slopes, sinks, gate, out)
+            dim, vdim, scale, window, chunk, slopes, sinks, gate, out)
         return
     n = q.shape[1] * vdim
     out[:, :n] = ref.attn_ragged(q, k_pages, v_pages, batch, dim, vdim, scale,
-                                 window, slopes, gate, sinks)
+                                 window, slopes, gate, sinks, chunk)

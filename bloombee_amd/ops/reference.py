@@ -75,6 +75,18 @@ def layer_norm(
 # RoPE
 # ---------------------------------------------------------------------------
 
+def banded_frequencies(inv_freq: torch.Tensor, factor: float, low: float,
+                       high: float, original: float) -> torch.Tensor:
+    """Rotary frequencies stretched to longer contexts by wavelength (llama-3
+    style): kept where the wavelength is below original / high, divided by factor
+    where it is above original / low, blended between."""
+    wavelen = 2 * math.pi / inv_freq
+    smooth = (original / wavelen - low) / (high - low)
+    out = (1 - smooth) * inv_freq / factor + smooth * inv_freq
+    out = torch.where(wavelen > original / low, inv_freq / factor, out)
+    return torch.where(wavelen < original / high, inv_freq, out)
+
+
 def rope_cos_sin(
     head_dim: int, max_pos: int, theta: float = 10000.0, device=None, dtype=torch.float32,
     scaling: Optional[dict] = None,
@@ -87,17 +99,10 @@ def rope_cos_sin(
     """
     inv_freq = 1.0 / (theta ** (torch.arange(0, head_dim, 2, dtype=torch.float64) / head_dim))
     if scaling is not None and scaling.get("rope_type", scaling.get("type")) == "llama3":
-        factor = scaling["factor"]
-        low = scaling["low_freq_factor"]
-        high = scaling["high_freq_factor"]
-        orig = scaling["original_max_position_embeddings"]
-        wavelen = 2 * math.pi / inv_freq
-        ratio = orig / wavelen
-        smooth = ((ratio - low) / (high - low)).clamp(0.0, 1.0)
-        scaled = inv_freq / factor
-        smoothed = (1 - smooth) * scaled + smooth * inv_freq
-        inv_freq = torch.where(wavelen > 2 * math.pi * orig / low, scaled, smoothed)
-        inv_freq = torch.where(wavelen < 2 * math.pi * orig / high, 1.0 * inv_freq, inv_freq)
+        inv_freq = banded_frequencies(
+            inv_freq, scaling["factor"], scaling["low_freq_factor"],
+            scaling["high_freq_factor"],
+            scaling["original_max_position_embeddings"])
     t = torch.arange(max_pos, dtype=torch.float64)
     freqs = torch.outer(t, inv_freq)
     cos = freqs.cos().to(dtype)
@@ -462,9 +467,12 @@ def xielu(z: torch.Tensor, pos: float, neg: float) -> torch.Tensor:
 
 
 def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
-               top: int, scale: float, sigmoid: bool = False):
+               top: int, scale: float, sigmoid: bool = False,
+               renorm: bool = False):
     """Softmax (or sigmoid) scores; the choice adds `correction`, the weights do not and
-    are not renormalized. Outputs from `experts` on are identity experts.
+    are not renormalized, unless renorm: then a token's weights sum to scale
+    (with softmax scores: a softmax over the chosen logits). Outputs from
+    `experts` on are identity experts.
     Returns ids (N, top) int32 with -1 for identity choices, weights (N, top)
     and the identity experts' summed weight (N,)."""
     s = (torch.sigmoid(logits.float()) if sigmoid
@@ -473,7 +481,10 @@ def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
     # stable sort: the lowest index wins a tie
     ids = torch.sort(choice, dim=-1, descending=True,
                      stable=True).indices[:, :top]
-    w = torch.gather(s, 1, ids) * scale
+    w = torch.gather(s, 1, ids)
+    if renorm:
+        w = w / w.sum(-1, keepdim=True)
+    w = w * scale
     ident = ids >= experts
     idw = (w * ident).sum(-1)
     return torch.where(ident, -1, ids).int(), w, idw
@@ -481,9 +492,10 @@ def route_topk(logits: torch.Tensor, correction: torch.Tensor, experts: int,
 
 def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
                 window: int = 0, slopes=None, gate=None,
-                sinks=None) -> torch.Tensor:
+                sinks=None, chunk: int = 0) -> torch.Tensor:
     """Paged attention of a ragged batch: q (N, H, >= dim) -> (N, H * vdim).
-    Row n sees positions j of its own sequence with 0 <= pos - j (< window);
+    Row n sees positions j of its own sequence with 0 <= pos - j (< window),
+    with chunk only those of its own stretch of that many positions;
     score = q.k * scale - slope_h * (pos - j); sinks_h is one more score that
     has no value; out *= sigmoid(gate). Without v_pages the values are the
     first vdim elements of the keys."""
@@ -508,6 +520,8 @@ def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
         seen = dist >= 0
         if window > 0:
             seen &= dist < window
+        if chunk > 0:
+            seen &= dist <= pos.view(-1, 1) % chunk
         sc = sc.masked_fill(~seen, float("-inf"))
         if sinks is not None:
             sc = torch.cat([sc, sinks.float().view(-1, 1, 1).expand(
@@ -520,12 +534,30 @@ def attn_ragged(q, k_pages, v_pages, batch, dim: int, vdim: int, scale: float,
     return out.to(q.dtype)
 
 
+def attn_differential(q, k_pages, v_pages, batch, dim: int, vdim: int,
+                      scale: float, lam: float, factor: float, eps: float,
+                      window: int = 0, chunk: int = 0) -> torch.Tensor:
+    """Two attentions per head over the same values: q (N, H, 2, stored dim),
+    keys (np, G, P, 2 * stored dim); (a1 - lam * a2), RMS-normed per head, times
+    factor: (N, H * vdim)."""
+    N, H, _, dp = q.shape
+    a = [attn_ragged(q[:, :, m].float(), k_pages[..., m * dp:(m + 1) * dp],
+                     v_pages, batch, dim, vdim, scale, window, chunk=chunk)
+         for m in range(2)]
+    o = (a[0] - lam * a[1]).view(N, H, vdim)
+    one = torch.ones(vdim, device=q.device)
+    return (grouped_rms_norm(o, one, 1, eps) * factor).reshape(N, H * vdim).to(
+        q.dtype)
+
+
 def moe_experts(h, up, down, ids, wts, weight_input: bool = False,
-                ) -> torch.Tensor:
+                limit: float = math.inf, slope: float = 1.0,
+                shift: float = 0.0) -> torch.Tensor:
     """y (N, top, W): wts * down(act) of every chosen expert, or down of the
-    activation of wts * h; act = silu(gate h) * up h with two planes (E, 2, F, K)
-    of first weights, relu(up h)^2 with one. Rows of skipped choices (id < 0)
-    are zero."""
+    activation of wts * h; act = g sigmoid(slope g) (u + shift) with
+    g = min(gate h, limit), u = clamp(up h, -limit, limit) with two planes
+    (E, 2, F, K) of first weights, relu(up h)^2 with one. Rows of skipped
+    choices (id < 0) are zero."""
     N, top = ids.shape
     y = torch.zeros(N, top, down.shape[1], dtype=torch.float32, device=h.device)
     for e in range(up.shape[0]):
@@ -537,7 +569,8 @@ def moe_experts(h, up, down, ids, wts, weight_input: bool = False,
             x, w = x * w, 1.0
         z = x @ up[e, -1].float().t()
         if up.shape[1] == 2:
-            z = F.silu(x @ up[e, 0].float().t()) * z
+            g = (x @ up[e, 0].float().t()).clamp(max=limit)
+            z = g * torch.sigmoid(slope * g) * (z.clamp(-limit, limit) + shift)
         else:
             z = torch.relu(z) ** 2
         y[t, k] = (z.to(h.dtype).float() @ down[e].float().t()) * w
@@ -571,15 +604,17 @@ def clamped_glu(gate, up, gate_b, up_b, limit: float, slope: float):
 
 
 def rotate_half(x: torch.Tensor, positions: torch.Tensor,
-                turns: torch.Tensor) -> torch.Tensor:
+                turns: torch.Tensor, amp: float = 1.0) -> torch.Tensor:
     """Rotary positions on the first 2 * len(turns) elements of the last axis,
     element i with element i + len(turns). x (N, ..., D), positions (N,);
-    turns: frequencies / 2 pi in float64, angles are reduced in float64."""
+    turns: frequencies / 2 pi in float64, angles are reduced in float64; amp
+    multiplies cosine and sine."""
     half = turns.numel()
     r = positions.double().clamp(min=0)[:, None] * turns
     ang = ((r - r.round()) * (2 * math.pi)).reshape(
         r.shape[0], *[1] * (x.dim() - 2), half)
-    c, s = torch.cos(ang).to(x.dtype), torch.sin(ang).to(x.dtype)
+    c = (amp * torch.cos(ang)).to(x.dtype)
+    s = (amp * torch.sin(ang)).to(x.dtype)
     u, v = x[..., :half], x[..., half:2 * half]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
 
@@ -588,6 +623,13 @@ def channel_decays(a1, a2, a2_b, tau: float) -> torch.Tensor:
     """sigmoid(a1 @ a2 + b)^(1 / tau), fp32. a2 (r, channels)."""
     z = a1.float() @ a2.float() + a2_b.float()
     return torch.exp(F.logsigmoid(z) / tau)
+
+
+def forget_gates(z, bias, lower):
+    """f = lower + (1 - lower) sigmoid(z + bias) and 1 - f, fp32."""
+    z = z.float() + bias
+    return (lower + (1 - lower) * torch.sigmoid(z),
+            (1 - lower) * torch.sigmoid(-z))
 
 
 def gla_scan(q, k, v, alpha, state):

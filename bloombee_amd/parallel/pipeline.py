@@ -149,7 +149,7 @@ class PipelineStage:
         self.prev_rank = ((self.pp_stage - 1) % self.pp_world) * tp
         self.is_leader = self.tp_rank == 0
         # persistent recv buffers per micro-batch
-        self._recv_buf = [torch.empty(self.mb, 1, cfg.hidden_size, dtype=cfg.hidden_dtype,
+        self._recv_buf = [torch.empty(self.mb, 1, cfg.hidden_columns, dtype=cfg.hidden_dtype,
                                       device=self.device) for _ in range(self.M)]
         # hipGraph decode capture (single-rank fast path): the whole decode
         # step — embed, 32 blocks, LM head, argmax, position bump — replays as
@@ -243,7 +243,7 @@ class PipelineStage:
             if self.is_client:
                 hid = self._embed(ids.view(B, 1), start_all)
             else:
-                hid = torch.empty(B, 1, cfg.hidden_size, dtype=cfg.hidden_dtype,
+                hid = torch.empty(B, 1, cfg.hidden_columns, dtype=cfg.hidden_dtype,
                                   device=self.device)
             if self.tp > 1:
                 dist.broadcast(hid, src=0, group=self.tp_group)
@@ -295,7 +295,7 @@ class PipelineStage:
         B = self.global_batch
         assert self.kv.seqs[0].l_spec == 0, "CP prefill is one-shot"
         assert T % self.tp == 0, "prompt length must divide by cp degree"
-        hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
+        hid = torch.empty(B, T, cfg.hidden_columns, dtype=cfg.hidden_dtype,
                           device=self.device)
         if self.pp_stage == 0:
             if self.is_client:
@@ -344,13 +344,13 @@ class PipelineStage:
         self.kv.extend(T)
         views = self._views()
         pending = []
-        bufs = [torch.empty(mb, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
+        bufs = [torch.empty(mb, T, cfg.hidden_columns, dtype=cfg.hidden_dtype,
                             device=self.device) for _ in range(M)]
         if self.pp_stage == 0:
             if self.is_client:
                 hid = self._embed(ids, start_all)
             else:
-                hid = torch.empty(B, T, cfg.hidden_size, dtype=cfg.hidden_dtype,
+                hid = torch.empty(B, T, cfg.hidden_columns, dtype=cfg.hidden_dtype,
                                   device=self.device)
             if self.tp > 1:
                 dist.broadcast(hid, src=0, group=self.tp_group)

@@ -39,8 +39,10 @@ class NativeCheckpoint:
         """From the file's header, no data is read."""
         return tuple(self._file.get_slice(name).get_shape())
 
-    def layer(self, index: int):
-        return lambda name: self._file.get_tensor(f"l{index}.{name}")
+    def layer(self, index: int, model_tensors=()):
+        """get() for one layer's tensors; model_tensors are named without it."""
+        return lambda name: self.get(name if name in model_tensors
+                                     else f"l{index}.{name}")
 
 
 def is_native(path: str) -> bool:
@@ -110,7 +112,9 @@ def load_block_weights(block: torch.nn.Module, ckpt_dir: str, index: int) -> int
     Supports the fused qkv/gate_up layout directly and falls back to
     concatenating the reference's split q/k/v and gate/up files."""
     if hasattr(block, "load_tensors"):
-        return block.load_tensors(NativeCheckpoint(ckpt_dir).layer(index))
+        return block.load_tensors(NativeCheckpoint(ckpt_dir).layer(
+            getattr(block, "checkpoint_index", index),
+            getattr(block, "model_tensors", ())))
     d = Path(ckpt_dir)
     loaded = 0
     for pname, stem in _BLOCK_PARAM_MAP.items():

@@ -35,7 +35,7 @@ def measure_compute_rps(config: ModelConfig, device: str = "cpu",
     stack = BlockStack(config, 0, 1, device=device, seed=0)
     kv = stack.make_kv(max(4096, batch * (n_tokens * (n_steps + 2) + 8)))
     h = kv.allocate(batch, n_tokens * (n_steps + 2) + 8)
-    hidden = torch.randn(batch, n_tokens, config.hidden_size).to(
+    hidden = torch.randn(batch, n_tokens, config.hidden_columns).to(
         config.dtype).to(device)
     pos = 0
     # warmup

@@ -19,10 +19,13 @@ HIP_DIR = ROOT / "bloombee_amd" / "ops" / "hip"
 OPS_DIR = ROOT / "bloombee_amd" / "ops"
 # module -> source. _hip_ragged holds what all ragged-batch models need,
 # _hip_mixers latent attention and gated linear attention, _hip_recurrent the
-# matrix memory and the gated linear recurrent unit.
+# matrix memory and the gated linear recurrent unit, _hip_differential differential
+# attention, _hip_hgrn gated linear attention that writes what it forgets.
 MODULES = {"_hip_ops": "ext.hip", "_hip_ragged": "ext_ragged.hip",
            "_hip_mixers": "ext_mixers.hip",
-           "_hip_recurrent": "ext_recurrent.hip"}
+           "_hip_recurrent": "ext_recurrent.hip",
+           "_hip_differential": "ext_differential.hip",
+           "_hip_hgrn": "ext_hgrn.hip"}
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 

@@ -19,7 +19,7 @@ def _free_port():
 
 
 MODELS = {"llama-tiny": 1000, "mubasun-tiny": 320,
-          "risepel-tiny": 320, "vumedra-tiny": 320}   # name -> vocab
+          "risepel-tiny": 320, "vumedra-tiny": 320, "zatusun-tiny": 320}   # name -> vocab
 
 
 def _worker(rank, world, q, port, model):
