@@ -125,15 +125,13 @@ class ZatusunBlock(torch.nn.Module):
                                    round_up(self.Fe, 64), dtype=dt)
         if self.enters is not None:
             self.loop_w = p(round_up(W, 64), pad_k(2 * W), dtype=dt)
-            self.step = p(W)     # of this pass
+            self.steps = p(int(config.loop["times"]), W)
 
     # -- weights ----------------------------------------------------------
     def share_weights(self, other: "ZatusunBlock") -> None:
-        """Use the weights of another run of the same layer; what belongs to the
-        pass stays."""
+        """Use the weights of another run of the same layer."""
         for name, w in other.named_parameters():
-            if name != "step":
-                setattr(self, name, w)
+            setattr(self, name, w)
         self.spec = other.spec
 
     def tensor_shapes(self) -> Dict[str, Tuple[int, ...]]:
@@ -159,7 +157,7 @@ class ZatusunBlock(torch.nn.Module):
                 out[f"mlp.e{e}.down"] = (W, self.Fe)
         if self.enters is not None:
             out["loop.in"] = (W, 2 * W)
-            out["loop.step"] = (int(self.config.loop["times"]), W)
+            out["loop.step"] = tuple(self.steps.shape)
         return out
 
     @torch.no_grad()
@@ -222,7 +220,7 @@ class ZatusunBlock(torch.nn.Module):
                     take(f"mlp.e{e}.down"))
         if self.enters is not None:
             self.loop_w[:W, :2 * W].copy_(take("loop.in"))
-            self.step.copy_(take("loop.step")[self.enters])
+            self.steps.copy_(take("loop.step"))
         return len(shapes)
 
     @torch.no_grad()
@@ -278,7 +276,7 @@ class ZatusunBlock(torch.nn.Module):
             rows = ragged.join_rows(x, pending, batch.embedded,
                                     self.loop_w.shape[1], dt)
             pending = Pending(ragged.linear_sums(rows, self.loop_w),
-                              bias=self.step, keep=0.0)
+                              bias=self.steps[self.enters], keep=0.0)
         h = ragged.residual_norm(x, pending, self.norm1_w, 1, eps, self.K, dt)
         left = Pending(ragged.linear_parts(self._mix(h, batch), self.out_w))
         if self.mlp is None:
@@ -398,7 +396,8 @@ class ZatusunBlock(torch.nn.Module):
         hidden = hidden.float()
         x = hidden[..., :W]
         if self.enters is not None:
-            x = F.linear(hidden.to(dt), self.loop_w[:W, :2 * W]).float() + self.step
+            x = (F.linear(hidden.to(dt), self.loop_w[:W, :2 * W]).float()
+                 + self.steps[self.enters])
         x = x + self._train_mixer(rms(x, self.norm1_w), start_pos).float()
         if self.mlp is not None:
             x = x + self._train_ff(rms(x, self.norm2_w))

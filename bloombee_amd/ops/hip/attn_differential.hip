@@ -23,6 +23,7 @@
 
 struct DiffArgs : AttnArgs {
   float lam, factor, eps;
+  int p_log2;           // of the page size
 };
 
 // Four consecutive output columns of one row.
@@ -41,27 +42,36 @@ DEVINL void store_diff4(const DiffArgs& a, long row, int h, int d, const float* 
 // prefill: grid (row tiles of the longest portion, G, sequences)
 // ---------------------------------------------------------------------------
 
-template <int DK, int DV>  // DK: one map
-__global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_kernel(
+// A K/V tile of 64 keys in LDS, filled by loads that bypass the registers: 16 B
+// pieces, piece c of row r at c ^ swizzle(r), so that eight rows read at one piece
+// lie in different banks.
+template <int DK, int DV>
+struct DiffTile {
+  static constexpr int KT = 64, RC = DK / 4;      // pieces of a key row, two maps
+  static constexpr int KB = KT * RC * 16;         // bytes
+  static constexpr int VB = DV * KT * 2;
+  static constexpr int BYTES = KB + VB;
+  static constexpr int KSW = RC >= 16 ? 15 : 7;
+};
+
+// NW waves of 16 rows; tiles are double-buffered.
+template <int DK, int DV, int NW>  // DK: one map
+__global__ __launch_bounds__(NW * 64, NW / 4) void attn_diff_prefill_kernel(
     DiffArgs a) {
-  constexpr int KT = 64;                 // keys per tile
-  constexpr int KROW = 2 * DK * 2 + 16;  // bytes
-  constexpr int VROW = KT * 2 + 16;
-  constexpr int NKK = DK / 32, ND = DV / 16, KC = 2 * DK / 8;
-  constexpr int KCH = KT * KC / 256;     // 16 B pieces per thread
-  constexpr int VCH = DV * (KT / 8) / 256;
-  static_assert(KCH >= 1 && VCH >= 1, "tile smaller than the workgroup");
-  __shared__ __attribute__((aligned(16))) unsigned char
-      lds[KT * KROW + DV * VROW];
-  unsigned char* k_lds = lds;
-  unsigned char* v_lds = lds + KT * KROW;
+  using Tile = DiffTile<DK, DV>;
+  constexpr int KT = Tile::KT, RC = Tile::RC, KB = Tile::KB;
+  constexpr int NKK = DK / 32, ND = DV / 16;
+  constexpr int KI = KB / 1024, VI = Tile::VB / 1024;  // loads of a wave's width
+  constexpr int KN = (KI + NW - 1) / NW, VN = (VI + NW - 1) / NW;
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds_tiles[];
 
   const int s = a.list[blockIdx.z];
   const int g = blockIdx.y;
   const int Hg = a.H / a.G;
   const int t0 = a.cu[s], T = a.cu[s + 1] - t0, qs = a.q_start[s];
   const int R = T * Hg;
-  const int base = blockIdx.x * 64;
+  // late rows see the most keys: they go first
+  const int base = (int)(gridDim.x - 1 - blockIdx.x) * (16 * NW);
   if (base >= R) return;
   const int tid = threadIdx.x;
   const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
@@ -70,6 +80,7 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
   const int* table = a.table + (long)s * a.maxp;
   const unsigned short* kpool = (const unsigned short*)a.kp;
   const unsigned short* vpool = (const unsigned short*)a.vp;
+  const int plog = a.p_log2, pmask = (1 << plog) - 1;
 
   // this lane's row (column of S^T): token, head, position
   const int r = min(base + wave * 16 + li, R - 1);
@@ -87,7 +98,7 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
   const float sc2 = a.scale * LOG2E;
 
   // visible keys of the workgroup and of this wave
-  const int last = min(base + 64, R) - 1;
+  const int last = min(base + 16 * NW, R) - 1;
   const int kend = qs + last / Hg + 1;
   const int kbeg = first_key(a, qs + base / Hg) & ~31;
   const int wr0 = min(base + wave * 16, R - 1);
@@ -96,6 +107,47 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
   const int whi = qs + wr1 / Hg;                 // any row sees <= whi
   const int flo = first_key(a, qs + wr1 / Hg);   // all rows do
   const int fhi = qs + wr0 / Hg;
+
+  // where this lane's pieces come from: LDS row r of the keys is MFMA row order,
+  // n * 16 + x * 4 + y  <->  key x * 8 + n * 4 + y  (of 32)
+  int kkey[KN], kcol[KN], vblk[VN], vrow[VN];
+#pragma unroll
+  for (int i = 0; i < KN; ++i) {
+    const int at = min(wave + i * NW, KI - 1) * 64 + lane;
+    const int row = at / RC, q = row & 31;
+    kcol[i] = ((at % RC) ^ (row & Tile::KSW)) * 8;
+    kkey[i] = (row & 32) + ((q >> 2) & 3) * 8 + (q >> 4) * 4 + (q & 3);
+  }
+#pragma unroll
+  for (int i = 0; i < VN; ++i) {
+    const int at = min(wave + i * NW, VI - 1) * 64 + lane;
+    vrow[i] = at / 8;
+    vblk[i] = (at % 8) ^ (vrow[i] & 7);
+  }
+  // lanes 0..7: the pages of a tile's eight blocks of eight keys
+  auto pages_of = [&](int kb) {
+    return table[min(kb + (lane & 7) * 8, kend - 1) >> plog];
+  };
+  auto issue = [&](int kb, int pages, unsigned char* buf) {
+#pragma unroll
+    for (int i = 0; i < KN; ++i) {
+      if (KI % NW && wave + i * NW >= KI) break;
+      const int pos = min(kb + kkey[i], kend - 1);
+      const long page = __shfl(pages, kkey[i] >> 3);
+      copy16_to_lds(kpool + (((page * a.G + g) << plog) + (pos & pmask)) * (2 * DK) +
+                        kcol[i],
+                    buf + (wave + i * NW) * 1024);
+    }
+#pragma unroll
+    for (int i = 0; i < VN; ++i) {
+      if (VI % NW && wave + i * NW >= VI) break;
+      const int pos = min(kb + vblk[i] * 8, (kend - 1) & ~7);
+      const long page = __shfl(pages, vblk[i]);
+      copy16_to_lds(vpool + (((page * a.G + g) * DV + vrow[i]) << plog) +
+                        (pos & pmask),
+                    buf + KB + (wave + i * NW) * 1024);
+    }
+  };
 
   float m2[2], l[2];
   f32x4 acc[2][ND];
@@ -107,55 +159,10 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
     for (int n = 0; n < ND; ++n) acc[m][n] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
 
-  short8 kreg[KCH], vreg[VCH];
-  auto fetch = [&](int kb) {
-#pragma unroll
-    for (int i = 0; i < KCH; ++i) {
-      const int idx = tid + i * 256;
-      const int pos = kb + idx / KC, d8 = (idx % KC) * 8;
-      kreg[i] = short8{};
-      if (pos < kend)
-        kreg[i] = *reinterpret_cast<const short8*>(
-            kpool +
-            (((long)table[pos / a.P] * a.G + g) * a.P + pos % a.P) * (2 * DK) + d8);
-    }
-#pragma unroll
-    for (int i = 0; i < VCH; ++i) {
-      const int idx = tid + i * 256;
-      const int d = idx / (KT / 8), pos = kb + (idx % (KT / 8)) * 8;
-      vreg[i] = short8{};
-      if (pos < kend)
-        vreg[i] = *reinterpret_cast<const short8*>(
-            vpool + (((long)table[pos / a.P] * a.G + g) * DV + d) * a.P + pos % a.P);
-    }
-  };
-  auto stage = [&]() {
-#pragma unroll
-    for (int i = 0; i < KCH; ++i) {
-      const int idx = tid + i * 256;
-      const int key = idx / KC, c8 = idx % KC;
-      const int k = key & 31;  // LDS row = MFMA n * 16 + row
-      const int row = (key & 32) + ((k >> 2) & 1) * 16 + (k >> 3) * 4 + (k & 3);
-      *reinterpret_cast<short8*>(k_lds + row * KROW + c8 * 16) = kreg[i];
-    }
-#pragma unroll
-    for (int i = 0; i < VCH; ++i) {
-      const int idx = tid + i * 256;
-      *reinterpret_cast<short8*>(v_lds + (idx / (KT / 8)) * VROW +
-                                 (idx % (KT / 8)) * 16) = vreg[i];
-    }
-  };
-
-  fetch(kbeg);
-  for (int kb = kbeg; kb < kend; kb += KT) {
-    __syncthreads();
-    stage();
-    __syncthreads();
-    if (kb + KT < kend) fetch(kb + KT);
-    if (kb > whi || kb + KT <= wlo) continue;  // nothing here for this wave
+  auto compute = [&](int kb, const unsigned char* kt) {
+    const unsigned char* vt = kt + KB;
     const bool inside = kb >= flo && kb + KT - 1 <= fhi;
     const int d0 = qpos - kb - hi * 8;
-
     float p[2][2][8];
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf)
@@ -163,13 +170,14 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
       for (int n = 0; n < 2; ++n) {
         f32x4 st[2];
         st[0] = st[1] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        const unsigned char* row = kt + (hf * 32 + n * 16 + li) * RC * 16;
 #pragma unroll
         for (int kk = 0; kk < NKK; ++kk)
 #pragma unroll
           for (int m = 0; m < 2; ++m) {
+            const int c = m * (DK / 8) + kk * 4 + hi;
             const bf16x8 kf = as_bf16x8(*reinterpret_cast<const short8*>(
-                k_lds + (hf * 32 + n * 16 + li) * KROW + m * DK * 2 + hi * 16 +
-                kk * 64));
+                row + (c ^ (li & Tile::KSW)) * 16));
             st[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m][kk], st[m],
                                                             0, 0, 0);
           }
@@ -227,16 +235,33 @@ __global__ __launch_bounds__(256, DK + DV > 192 ? 1 : 2) void attn_diff_prefill_
 #pragma unroll
       for (int n = 0; n < ND; ++n) {
         const bf16x8 vf = as_bf16x8(*reinterpret_cast<const short8*>(
-            v_lds + (n * 16 + li) * VROW + hf * 64 + hi * 16));
+            vt + (n * 16 + li) * 128 + ((hf * 4 + hi) ^ (li & 7)) * 16));
 #pragma unroll
-        for (int m = 0; m < 2; ++m) {
+        for (int m = 0; m < 2; ++m)
           acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[m],
                                                               acc[m][n], 0, 0, 0);
+#pragma unroll
+        for (int m = 0; m < 2; ++m)
           acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[m],
                                                               acc[m][n], 0, 0, 0);
-        }
       }
     }
+  };
+
+  // page numbers are looked up a tile ahead of the loads that need them
+  int pages = pages_of(kbeg);
+  issue(kbeg, pages, lds_tiles);
+  pages = pages_of(kbeg + KT);
+  __syncthreads();
+  int buf = 0;
+  for (int kb = kbeg; kb < kend; kb += KT) {
+    if (kb + KT < kend) {
+      issue(kb + KT, pages, lds_tiles + (buf ^ 1) * Tile::BYTES);
+      pages = pages_of(kb + 2 * KT);
+    }
+    if (kb <= whi && kb + KT > wlo) compute(kb, lds_tiles + buf * Tile::BYTES);
+    __syncthreads();
+    buf ^= 1;
   }
 
   // a row's values are spread over the four lanes of its column; those beyond
@@ -319,30 +344,31 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_diff_decode_k
 #pragma unroll
   for (int n = 0; n < ND; ++n) acc[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
 
-  auto load_k = [&](bf16x8 (&kf)[2][NKK], int tile) {
+  // page numbers of a tile: this lane's block of eight keys, then of values
+  const int plog = a.p_log2, pmask = (1 << plog) - 1;
+  auto pages_of = [&](int tile, int (&pg)[2]) {
+    pg[0] = table[min(tile * 32 + (li >> 2) * 8, max(pos, 0)) >> plog];
+    pg[1] = table[min(tile * 32 + hi * 8, max(pos, 0)) >> plog];
+  };
+  auto load = [&](bf16x8 (&kf)[2][NKK], bf16x8 (&vf)[ND], int tile,
+                  const int (&pg)[2]) {
+    const unsigned short* kr = kpool + (((long)pg[0] * a.G + g) << plog) * DK + hi * 8;
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
       const int key = min(tile * 32 + (li >> 2) * 8 + n * 4 + (li & 3), pos);
-      const unsigned short* kr = kpool +
-          (((long)table[key / a.P] * a.G + g) * a.P + key % a.P) * DK + hi * 8;
 #pragma unroll
       for (int kk = 0; kk < NKK; ++kk)
         kf[n][kk] = as_bf16x8(__builtin_nontemporal_load(
-            reinterpret_cast<const short8*>(kr + kk * 32)));
+            reinterpret_cast<const short8*>(kr + (key & pmask) * DK + kk * 32)));
     }
-  };
-  auto load_v = [&](bf16x8 (&vf)[ND], int tile) {
-    const int vpos = tile * 32 + hi * 8;
-    const bool live = vpos <= pos;
-    const long vrow = live ? ((long)table[vpos / a.P] * a.G + g) * DV : 0;
+    // values beyond the last key weigh nothing
+    const int vpos = min(tile * 32 + hi * 8, pos & ~7);
+    const unsigned short* vr = vpool +
+        ((((long)pg[1] * a.G + g) * DV + li) << plog) + (vpos & pmask);
 #pragma unroll
-    for (int n = 0; n < ND; ++n) {
-      vf[n] = as_bf16x8(short8{});
-      if (live)
-        vf[n] = as_bf16x8(__builtin_nontemporal_load(
-            reinterpret_cast<const short8*>(
-                vpool + (vrow + n * 16 + li) * a.P + vpos % a.P)));
-    }
+    for (int n = 0; n < ND; ++n)
+      vf[n] = as_bf16x8(__builtin_nontemporal_load(
+          reinterpret_cast<const short8*>(vr + ((long)n << (plog + 4)))));
   };
   auto compute = [&](const bf16x8 (&kf)[2][NKK], const bf16x8 (&vf)[ND],
                      int tile) {
@@ -391,25 +417,22 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_diff_decode_k
     }
   };
 
-  // two named buffers: the next tile's loads fly behind this one's compute
+  // two named buffers: the next tile's loads fly behind this one's compute, and
+  // page numbers are looked up a tile ahead of them
   bf16x8 k0[2][NKK], v0[ND], k1[2][NKK], v1[ND];
+  int pg[2];
   int t = t_lo + wave;
-  if (t < t_hi) {
-    load_k(k0, t);
-    load_v(v0, t);
-  }
+  pages_of(t, pg);
+  if (t < t_hi) load(k0, v0, t, pg);
+  pages_of(t + 4, pg);
   for (; t < t_hi; t += 8) {
-    if (t + 4 < t_hi) {
-      load_k(k1, t + 4);
-      load_v(v1, t + 4);
-    }
+    if (t + 4 < t_hi) load(k1, v1, t + 4, pg);
+    pages_of(t + 8, pg);
     __builtin_amdgcn_sched_barrier(0);
     compute(k0, v0, t);
     if (t + 4 >= t_hi) break;
-    if (t + 8 < t_hi) {
-      load_k(k0, t + 8);
-      load_v(v0, t + 8);
-    }
+    if (t + 8 < t_hi) load(k0, v0, t + 8, pg);
+    pages_of(t + 12, pg);
     __builtin_amdgcn_sched_barrier(0);
     compute(k1, v1, t + 4);
   }
@@ -478,43 +501,51 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void attn_diff_decode_k
   }
 }
 
-// grid = units; 32 threads a head
+// grid = units; 32 threads a head, of which each looks after one split at first
 __global__ __launch_bounds__(256) void attn_diff_combine_kernel(DiffArgs a) {
   constexpr int NP = 2;  // pieces of four columns a thread, dvp <= 256
   const int Hg = a.H / a.G;
   const int nch = (Hg + 7) / 8;
   const int unit = blockIdx.x;
   const int h0 = (unit % nch) * 8;
-  const int col = threadIdx.x / 32, d0 = (threadIdx.x % 32) * 4;
+  const int col = threadIdx.x / 32, part = threadIdx.x % 32, d0 = part * 4;
   if (h0 + col >= Hg) return;   // whole groups of 32 lanes
   const int row = a.cu[a.list[unit / (a.G * nch)]];
   const long u0 = (long)unit * a.n_split * 16 + col;
-  float o[2][NP][4];
+  float w[2];   // weight of this thread's split
 #pragma unroll
   for (int m = 0; m < 2; ++m) {
-    const long um = u0 + m * 8;
-    float mx = NEG_BIG, l = 0.f;
-    for (int i = 0; i < a.n_split; ++i)
-      mx = fmaxf(mx, a.pml[(um + i * 16) * 2]);
-    for (int i = 0; i < a.n_split; ++i)
-      l += a.pml[(um + i * 16) * 2 + 1] * fast_exp2(a.pml[(um + i * 16) * 2] - mx);
-    const float inv = l > 0.f ? 1.f / l : 0.f;
+    const long u = u0 + m * 8 + min(part, a.n_split - 1) * 16;
+    const float mi = part < a.n_split ? a.pml[u * 2] : NEG_BIG;
+    float mx = mi;
 #pragma unroll
-    for (int p = 0; p < NP; ++p) {
+    for (int k = 1; k < 32; k <<= 1) mx = fmaxf(mx, __shfl_xor(mx, k));
+    w[m] = part < a.n_split ? fast_exp2(mi - mx) : 0.f;
+    float l = part < a.n_split ? a.pml[u * 2 + 1] * w[m] : 0.f;
+#pragma unroll
+    for (int k = 1; k < 32; k <<= 1) l += __shfl_xor(l, k);
+    w[m] = l > 0.f ? w[m] / l : 0.f;
+  }
+  float o[2][NP][4];
+#pragma unroll
+  for (int m = 0; m < 2; ++m)
+#pragma unroll
+    for (int p = 0; p < NP; ++p)
 #pragma unroll
       for (int r = 0; r < 4; ++r) o[m][p][r] = 0.f;
-      if (d0 + p * 128 >= a.dvp) continue;
-      for (int i = 0; i < a.n_split; ++i) {
-        const float c = fast_exp2(a.pml[(um + i * 16) * 2] - mx);
+#pragma unroll 4
+  for (int i = 0; i < a.n_split; ++i)
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const float c = __shfl(w[m], i, 32);
+#pragma unroll
+      for (int p = 0; p < NP; ++p) {
         const f32x4 v = *reinterpret_cast<const f32x4*>(
-            a.pacc + (um + i * 16) * a.dvp + d0 + p * 128);
+            a.pacc + (u0 + m * 8 + i * 16) * a.dvp + min(d0 + p * 128, a.dvp - 4));
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[m][p][r] += v[r] * c;
       }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[m][p][r] *= inv;
     }
-  }
   float ss = 0.f;
 #pragma unroll
   for (int p = 0; p < NP; ++p)

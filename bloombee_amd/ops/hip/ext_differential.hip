@@ -14,18 +14,27 @@ static void launch_tiled(DiffArgs& a, const Tensor& pre, const Tensor& dec,
   const int Hg = a.H / a.G;
   if (pre.numel() > 0) {
     a.list = pre.data_ptr<int>();
-    attn_diff_prefill_kernel<DK, DV>
-        <<<dim3((max_new * Hg + 63) / 64, a.G, pre.numel()), 256, 0,
-           cur_stream()>>>(a);
+    // half as many rows a workgroup where there are not enough of them
+    const long rows = max_new * Hg;
+    by_bool((rows + 127) / 128 * a.G * pre.numel() >= 256, [&](auto many) {
+      constexpr int NW = decltype(many)::value ? 8 : 4;
+      constexpr size_t lds = 2 * DiffTile<DK, DV>::BYTES;
+      auto k = attn_diff_prefill_kernel<DK, DV, NW>;
+      allow_lds(k, lds);
+      k<<<dim3((rows + 16 * NW - 1) / (16 * NW), a.G, pre.numel()), NW * 64, lds,
+          cur_stream()>>>(a);
+    });
     check_launch();
   }
   if (dec.numel() == 0) return;
   a.list = dec.data_ptr<int>();
   const long units = dec.numel() * a.G * ((Hg + 7) / 8);
-  // enough workgroups to fill the chip with at least two tiles for each wave
+  // enough workgroups to fill the chip with at least two tiles for each wave, one
+  // where there are few
   const long tiles = (seen_keys(a, max_ctx) + 31) / 32 + 1;
   a.n_split = (int)std::max<long>(
-      1, std::min<long>({32, 512 / std::max<long>(1, units), tiles / 8}));
+      1, std::min<long>({32, 512 / std::max<long>(1, units),
+                         tiles / (units < 32 ? 4 : 8)}));
   Tensor pml, pacc;
   if (a.n_split > 1) {
     auto o = like.options().dtype(at::kFloat);
@@ -97,6 +106,7 @@ void attn_differential(Tensor q, Tensor kp, Tensor vp, Tensor table,
   a.factor = (float)factor;
   a.eps = (float)eps;
 
+  while (1 << a.p_log2 < a.P) ++a.p_log2;
   auto size_ok = [](int d, int most) {
     return d <= most && (d == 32 || d == 64 || d == 128 || d == 256);
   };

@@ -248,13 +248,6 @@ __global__ __launch_bounds__(256) void moe_skinny_kernel(
 // tile: grid of column tiles * row tiles; K % 64 == 0
 // ---------------------------------------------------------------------------
 
-typedef const __attribute__((address_space(1))) void* gptr_t;
-typedef __attribute__((address_space(3))) void* lptr_t;
-
-DEVINL void copy16_to_lds(const unsigned short* g, unsigned char* l) {
-  __builtin_amdgcn_global_load_lds((gptr_t)g, (lptr_t)l, 16, 0, 0);
-}
-
 // UP: A row = sorted slot / top, out row = sorted position, N = activations
 //     (two planes: 128 per tile, 128 gate rows and 128 up rows of W; one: 256).
 // else: A row = sorted position, out row = slot, 256 columns per tile.

@@ -95,6 +95,15 @@ DEVINL void stv(float* p, const float* v) {
   }
 }
 
+// 16 B a lane from memory to LDS without registers; l is the wave's, lane i's piece
+// lands i * 16 behind it.
+typedef const __attribute__((address_space(1))) void* gptr_t;
+typedef __attribute__((address_space(3))) void* lptr_t;
+
+DEVINL void copy16_to_lds(const unsigned short* g, unsigned char* l) {
+  __builtin_amdgcn_global_load_lds((gptr_t)g, (lptr_t)l, 16, 0, 0);
+}
+
 // A GEMM's output as ks partial sums (N, ld).
 struct Parts {
   const void* p;  // (ks, N, ld)

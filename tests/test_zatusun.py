@@ -393,10 +393,24 @@ def test_layout_of_the_cache(models, monkeypatch):
     assert c.state(1).shape == c.state(7).shape == (2, 3, 32, 48)
     assert c.state(10).shape == (2, 5, 24, 40) and c.state(2) is None
     assert all(t.dtype == torch.float32 for t in c.states if t is not None)
-    # ... and the weights in common, but for the pass's own vector
+    # ... and the weights in common
     b = eng.stack.blocks
     assert b[1].in_w is b[4].in_w is b[7].in_w and b[3].out_w is b[9].out_w
-    assert b[1].step is not b[4].step and not torch.equal(b[1].step, b[4].step)
+    assert [x.enters for x in b[1:8:3]] == [0, 1, 2]
+    assert b[2].enters is None and b[10].enters is None
+
+
+def test_random_weights_do_not_depend_on_the_block_range(monkeypatch):
+    """A server that starts in the middle of the loop draws what one that holds
+    everything draws."""
+    monkeypatch.setenv("BBAMD_TORCH_DTYPE", "float32")
+    cfg = resolve_config("zatusun-tiny")
+    whole, part = BlockStack(cfg, 0, 6), BlockStack(cfg, 2, 6)
+    for i, blk in enumerate(part.blocks):
+        other = dict(whole.blocks[i + 2].named_parameters())
+        for name, w in blk.named_parameters():
+            assert torch.equal(w, other.pop(name)), (i, name)
+        assert not other
 
 
 def test_state_slots_are_admission(models, monkeypatch):
