@@ -48,7 +48,8 @@ DEVINL float forget_room(float lower, float z) {
 // log2 of the gate, accurate where it is nearly one. A gate below 2^-64 forgets
 // all there is.
 DEVINL float log2_forget(float lower, float z, float room) {
-  if (room < 0.01f) return -(room + 0.5f * room * room + room * room * room * (1.f / 3)) * LOG2E;
+  if (room < 0.01f)
+    return -room * (1.f + room * (0.5f + room * (1.f / 3))) * LOG2E;
   return __builtin_amdgcn_logf(fmaxf(lower + (1.f - lower) * sigmoid_f(z), 5.4e-20f));
 }
 

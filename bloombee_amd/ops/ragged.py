@@ -40,7 +40,7 @@ _hip_ragged = None   # loaded by the first device call
 # padded to the next one with zeros
 HEAD_SIZES = (32, 64, 128, 256)
 SKINNY_ROWS = 32   # up to here a GEMM is a weight stream (split-K kernel)
-ROUTER_COLS = 1024   # beyond, the vendor GEMM makes 32-bit columns, too
+ROUTER_COLS = 256   # beyond, the vendor GEMM makes 32-bit columns, too
 
 
 def _ext():
