@@ -89,7 +89,7 @@ ZATUSUN_PRESETS = {
     "zatusun-tiny": _preset(192, 320, [
         _latent(4, 32, 16, 40, 80, 96, _moe(5, 2, 64)),
         _hgrn2(3, 32, 40, _moe(6, 3, 64)),
-        _diff(4, 2, 24, 40, None, 16, rot=12), _hgrn2(2, 48, 64, None)],
+        _diff(4, 2, 24, 40, None, 16, rot=12), _hgrn2(2, 40, 56, None)],
         loop={"start": 1, "stop": 3, "times": 2}, positions=512),
 }
 

@@ -86,7 +86,7 @@ CONFIGS = {
     # no loop, no recurrence
     "attentions": model(128, 97, [
         (latent(4, 32, 32, 32, 64, 64), None),
-        (diff(4, 2, 32, 64, 24, 8), moe(4, 2, 32))], cap=None),
+        (diff(4, 2, 32, 40, 24, 10), moe(4, 2, 32))], cap=None),
     # recurrence only, one pass
     "recurrent": model(128, 97, [(hgrn(2, 32, 64), moe(3, 2, 64)),
                                  (hgrn(4, 32, 32), None)], loop=(1, 2, 1)),

@@ -230,7 +230,7 @@ class Diff:
 
 @kinds
 @pytest.mark.parametrize("H,G,D,V,rot", [
-    (4, 2, 32, 64, 8), (3, 3, 18, 21, 18), (6, 1, 24, 40, 12), (2, 1, 64, 32, 64),
+    (4, 2, 32, 56, 12), (3, 3, 18, 21, 18), (6, 1, 24, 40, 12), (2, 1, 64, 32, 64),
     (4, 2, 128, 256, 64), (20, 2, 48, 96, 32), (9, 1, 16, 16, 2),
     (2, 2, 150, 64, 100), (1, 1, 33, 300, 6)])
 @pytest.mark.parametrize("chunk", [0, 1, 37, 64])
@@ -512,7 +512,7 @@ def state_close(got, want, dt):
 
 @kinds
 @pytest.mark.parametrize("H,D,V", [
-    (2, 48, 64), (3, 32, 48), (2, 18, 21), (1, 64, 64), (2, 128, 256),
+    (2, 40, 56), (3, 32, 48), (2, 18, 21), (1, 64, 64), (2, 128, 256),
     (2, 96, 100), (1, 256, 32), (1, 260, 30), (1, 40, 400), (1, 128, 512),
     (5, 8, 530), (1, 200, 320)])
 def test_recurrence_portions(dev, dt, H, D, V):
@@ -624,7 +624,7 @@ def test_recurrence_splits_and_empty_slots(dev, dt, splits):
 # ---------------------------------------------------------------------------
 
 @kinds
-@pytest.mark.parametrize("N,E,top,scale", [(5, 12, 3, 1.0), (40, 7, 7, 1.0),
+@pytest.mark.parametrize("N,E,top,scale", [(5, 13, 4, 1.0), (40, 7, 7, 1.0),
                                            (33, 100, 1, 2.5), (3, 90, 70, 1.0)])
 def test_routing_over_the_chosen(dev, dt, N, E, top, scale):
     """Weights are a softmax over the chosen logits alone, also where those are
@@ -645,7 +645,7 @@ def test_routing_over_the_chosen(dev, dt, N, E, top, scale):
 
 @kinds
 @pytest.mark.parametrize("N,E,top,F,W,limit", [
-    (6, 5, 2, 64, 128, 0.8), (50, 12, 3, 40, 192, 1.5), (3, 4, 4, 200, 64, 7.0),
+    (6, 5, 2, 64, 128, 0.8), (50, 11, 3, 40, 192, 1.25), (3, 4, 4, 200, 64, 7.0),
     (300, 3, 2, 96, 256, 0.3), (32, 6, 1, 256, 256, 2.0)])
 def test_clamped_experts(dev, dt, N, E, top, F, W, limit):
     """Gates and ups on both sides of the limits, in the weight stream, the tiles
